@@ -70,10 +70,10 @@ def libraries():
         for s in srcs:
             if os.path.exists(os.path.join(CSRC, s)):
                 libs.setdefault(lib, []).append(_tu(s, os.path.basename(os.path.splitext(s)[0]) + ".o", decode_defs.get(s, ())))
-    # layer-list ("hybrid") decoders in their checkpoint dtype: a library of its own, so that serving such a model compiles six files, not the quantized stack.
+    # layer-list ("hybrid") decoders in their checkpoint dtype: a library of its own, so that serving such a model compiles seven files, not the quantized stack.
     # It carries the host-side cache bookkeeping too (the same objects libmrs_hip_ext.so links).
-    libs[HYBRID_LIB] = [_tu(s, os.path.basename(os.path.splitext(s)[0]) + ".o", PACKED_FP32_OFF if s.endswith(".hip") else ())
-                        for s in ("hyb_gemm.hip", "hyb_kernels.hip", "hyb_attn_talk.hip", "hyb_recur.hip", "host/kv_cache_manager.cpp", "host/state_pool.cpp")]
+    libs[HYBRID_LIB] = [_tu(s, os.path.basename(os.path.splitext(s)[0]) + ".o")
+                        for s in ("hyb_gemm.hip", "hyb_kernels.hip", "hyb_attn_talk.hip", "hyb_recur.hip", "hyb_linattn.hip", "host/kv_cache_manager.cpp", "host/state_pool.cpp")]
     return libs
 
 
@@ -108,7 +108,7 @@ def _compile(src, obj, defines, force, hdr_m):
     dep_m = max(hdr_m[0], hdr_m[1] if _includes_public_header(s) else 0.0)
     if not force and os.path.exists(o) and os.path.getmtime(o) >= max(os.path.getmtime(s), dep_m):
         return o, False
-    cmd = [HIPCC, *CXXFLAGS, *defines, "-c", s, "-o", o]
+    cmd = [HIPCC, *CXXFLAGS, *PACKED_FP32_OFF, *defines, "-c", s, "-o", o]
     if src.endswith(".cpp"):
         cmd = [HIPCC, "-x", "hip", *CXXFLAGS, *defines, "-c", s, "-o", o]
     r = subprocess.run(cmd, capture_output=True, text=True)
