@@ -270,8 +270,11 @@ __global__ void __launch_bounds__(256) gemm_tile_f32_kernel(GemmArgs a) {
 //   IN_GLU_CLAMP  A = f32 [M, 2 K] = gate | up: g = min(gate, p0), u = clamp(up, -p0, p0): x_k = round_T(g sigmoid(p1 g) (u + 1))
 //   IN_BIAS_XIELU A = f32 [M, K]: z = A + in_bias: x_k = round_T(z > 0 ? p0 z^2 + z / 2 : p1 (e^z - 1 - z) + z / 2)
 //   IN_RELU_SQ A = f32 [M, K]: x_k = round_T(max(A, 0)^2)
+//   IN_GLU_GELU A = f32 [M, 2 K] = gate | up: x_k = round_T(gelu(gate) * up), the tanh form
+//   IN_GELU    A = f32 [M, K]: x_k = round_T(gelu(A)), the erf form
+//   IN_SIG_GATE A = f32 [M, K], in_bias = f32 [M, gate_ld] gate logits: x_k = round_T(A * sigmoid(gate_k))
 // The batched form offsets A by columns: only IN_PLAIN reads it there.
-enum { IN_PLAIN = 0, IN_GLU = 1, IN_SCALED = 2, IN_GLU_CLAMP = 3, IN_BIAS_XIELU = 4, IN_RELU_SQ = 5 };
+enum { IN_PLAIN = 0, IN_GLU = 1, IN_SCALED = 2, IN_GLU_CLAMP = 3, IN_BIAS_XIELU = 4, IN_RELU_SQ = 5, IN_GLU_GELU = 6, IN_GELU = 7, IN_SIG_GATE = 8 };
 struct GemvArgs {
   const void *A;
   const void *W;
@@ -284,11 +287,12 @@ struct GemvArgs {
   const int *src_row;        // IN_SCALED
   const float *src_scale;
   int src_div;
-  const float *in_bias;      // IN_BIAS_XIELU
+  const float *in_bias;      // IN_BIAS_XIELU; IN_SIG_GATE: the gate logits
   float p0, p1;              // IN_GLU_CLAMP: limit, sigmoid factor; IN_BIAS_XIELU: the two coefficients
   int batch;                 // batched form (row_group null): blockIdx.z = b reads A at column offset b * a_bstride, the slab W + b * wstride, writes C at column offset b * c_bstride
   long long a_bstride, c_bstride;
   int c_is_T;                // C holds T instead of f32 (no accumulate)
+  int gate_ld;               // IN_SIG_GATE: values between the rows of gate logits
 };
 
 template <class T> struct Vec8;
@@ -320,6 +324,10 @@ __device__ __forceinline__ float glu_clamp_in(float gv, float uv, float limit, f
 }
 __device__ __forceinline__ float xielu_in(float z, float ap, float an) { return z > 0.f ? fmaf(ap * z, z, 0.5f * z) : fmaf(an, expm1f(z) - z, 0.5f * z); }
 
+__device__ __forceinline__ float gelu_tanh_in(float v) { return 0.5f * v * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * v * v, v, v))); }
+__device__ __forceinline__ float gelu_erf_in(float v) { return 0.5f * v * (1.0f + erff(v * 0.7071067811865476f)); }
+__device__ __forceinline__ float sigmoid_in(float v) { return 1.0f / (1.0f + expf(-v)); }
+
 // one activation value (element path) / eight (vector path) of row m at column k, as the product sees it
 template <class T, int IN> __device__ __forceinline__ float act1(const GemvArgs &a, int m, int k) {
   if (IN == IN_PLAIN) return to_f<T>(((const T *)a.A)[(size_t)blockIdx.z * a.a_bstride + (size_t)m * a.lda + k]);
@@ -328,6 +336,9 @@ template <class T, int IN> __device__ __forceinline__ float act1(const GemvArgs 
   if (IN == IN_GLU_CLAMP) return round_to<T>(glu_clamp_in(A[(size_t)m * a.lda + k], A[(size_t)m * a.lda + a.K + k], a.p0, a.p1));
   if (IN == IN_BIAS_XIELU) return round_to<T>(xielu_in(A[(size_t)m * a.lda + k] + (a.in_bias ? a.in_bias[k] : 0.f), a.p0, a.p1));
   if (IN == IN_RELU_SQ) { const float v = fmaxf(A[(size_t)m * a.lda + k], 0.f); return round_to<T>(v * v); }
+  if (IN == IN_GLU_GELU) return round_to<T>(gelu_tanh_in(A[(size_t)m * a.lda + k]) * A[(size_t)m * a.lda + a.K + k]);
+  if (IN == IN_GELU) return round_to<T>(gelu_erf_in(A[(size_t)m * a.lda + k]));
+  if (IN == IN_SIG_GATE) return round_to<T>(A[(size_t)m * a.lda + k] * sigmoid_in(a.in_bias[(size_t)m * a.gate_ld + k]));
   const int r = a.src_row[m];
   return round_to<T>((a.src_scale ? a.src_scale[r] : 1.0f) * A[(size_t)(r / a.src_div) * a.lda + k]);
 }
@@ -362,6 +373,28 @@ template <class T, int IN> __device__ __forceinline__ void act8(const GemvArgs &
     Vec8<float>::load(A + (size_t)m * a.lda + k, x);
 #pragma unroll
     for (int j = 0; j < 8; ++j) { const float v = fmaxf(x[j], 0.f); x[j] = round_to<T>(v * v); }
+    return;
+  }
+  if (IN == IN_GLU_GELU) {
+    float g[8], u[8];
+    Vec8<float>::load(A + (size_t)m * a.lda + k, g);
+    Vec8<float>::load(A + (size_t)m * a.lda + a.K + k, u);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] = round_to<T>(gelu_tanh_in(g[j]) * u[j]);
+    return;
+  }
+  if (IN == IN_GELU) {
+    Vec8<float>::load(A + (size_t)m * a.lda + k, x);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] = round_to<T>(gelu_erf_in(x[j]));
+    return;
+  }
+  if (IN == IN_SIG_GATE) {
+    float g[8];
+    Vec8<float>::load(A + (size_t)m * a.lda + k, x);
+    Vec8<float>::load(a.in_bias + (size_t)m * a.gate_ld + k, g);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] = round_to<T>(x[j] * sigmoid_in(g[j]));
     return;
   }
   const int r = a.src_row[m];
@@ -473,7 +506,7 @@ extern "C" int mrs_hyb_gemm_batched(const void *A, const void *W, void *C, int M
   const int esz = dtype == 1 ? 2 : 4;
   GemvArgs a{A, W, (float *)C, M, N, K, lda, ldw, ldc, 0, nullptr, wstride,
              (K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0 && (wstride * esz) % 16 == 0 && (a_bstride * esz) % 16 == 0) ? 1 : 0,
-             nullptr, nullptr, 1, nullptr, 0.f, 0.f, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T};
+             nullptr, nullptr, 1, nullptr, 0.f, 0.f, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T, 0};
   if (batch > 65535) return fail("mrs_hyb_gemm_batched: more than 65535 products in one batch");
   dim3 grid((N + 3) / 4, 1, batch > 0 ? batch : 1);
   hipStream_t s = (hipStream_t)stream;
@@ -485,24 +518,27 @@ extern "C" int mrs_hyb_gemm_batched(const void *A, const void *W, void *C, int M
 }
 
 /* in_mode: 0 plain (A in dtype), 1 GLU (A = f32 [M, 2 K] gate | up), 2 scaled rows (A = f32 source rows; row m = src_scale[r] * A[r / src_div], r = src_row[m]; no
- * src_scale: the rows are gathered as they are), 3 clamped GLU (A = f32 [M, 2 K]; p0 = limit, p1 = the sigmoid's factor), 4 xIELU(A + in_bias) (p0, p1 = its coefficients), 5 max(A, 0)^2 (A = f32 [M, K]) */
+ * src_scale: the rows are gathered as they are), 3 clamped GLU (A = f32 [M, 2 K]; p0 = limit, p1 = the sigmoid's factor), 4 xIELU(A + in_bias) (p0, p1 = its coefficients), 5 max(A, 0)^2 (A = f32 [M, K]),
+ * 6 GLU with the tanh gelu (A = f32 [M, 2 K] gate | up), 7 the erf gelu of A (f32 [M, K]), 8 A times sigmoid(gate) (A = f32 [M, K]; in_bias = gate logits, src_div = their row stride) */
 extern "C" int mrs_hyb_gemv_act(const void *A, const void *W, float *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate, const int *row_group,
                                 long long wstride, int in_mode, const int *src_row, const float *src_scale, int src_div, const float *in_bias, float p0, float p1, void *stream) {
   if (M <= 0 || N <= 0) return 0;
-  if (K <= 0 || lda < K || ldw < K || ldc < N || (dtype != 1 && dtype != 2) || in_mode < 0 || in_mode > 5) return fail("mrs_hyb_gemv: bad shape / dtype / input mode");
-  if ((in_mode == 1 || in_mode == 3) && lda < 2 * K) return fail("mrs_hyb_gemv: the gate | up operand needs rows of 2 K values");
+  if (K <= 0 || lda < K || ldw < K || ldc < N || (dtype != 1 && dtype != 2) || in_mode < 0 || in_mode > 8) return fail("mrs_hyb_gemv: bad shape / dtype / input mode");
+  if (in_mode == 8 && (!in_bias || src_div < K || row_group)) return fail("mrs_hyb_gemv: the gate logits need rows of K values");
+  if ((in_mode == 1 || in_mode == 3 || in_mode == 6) && lda < 2 * K) return fail("mrs_hyb_gemv: the gate | up operand needs rows of 2 K values");
   if (in_mode == 2 && (!src_row || src_div <= 0)) return fail("mrs_hyb_gemv: gathered rows need their source table");
   if (!row_group && M > 8) return fail("mrs_hyb_gemv: at most 8 rows share a weight");
   if (row_group && M > 65535) return fail("mrs_hyb_gemv: too many rows");
   const int esz = dtype == 1 ? 2 : 4;
   GemvArgs a{A, W, C, M, N, K, lda, ldw, ldc, accumulate, row_group, wstride,
              (K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0 && (wstride * esz) % 16 == 0 &&
-              (!in_bias || ((uintptr_t)in_bias % 16) == 0)) ? 1 : 0, src_row, src_scale, src_div, in_bias, p0, p1, 0, 0, 0, 0};
+              (!in_bias || ((uintptr_t)in_bias % 16) == 0) && (in_mode != 8 || src_div % 4 == 0)) ? 1 : 0, src_row, src_scale, src_div, in_bias, p0, p1, 0, 0, 0, 0, in_mode == 8 ? src_div : 0};
   dim3 grid((N + 3) / 4, row_group ? M : 1);
   hipStream_t s = (hipStream_t)stream;
 #define MRS_GEMV_(T, MR, IN) hipLaunchKernelGGL((gemv_rows_kernel<T, MR, IN>), grid, dim3(256), 0, s, a)
 #define MRS_GEMV(T, MR) do { if (in_mode == 0) MRS_GEMV_(T, MR, IN_PLAIN); else if (in_mode == 1) MRS_GEMV_(T, MR, IN_GLU); else if (in_mode == 2) MRS_GEMV_(T, MR, IN_SCALED); \
-                             else if (in_mode == 3) MRS_GEMV_(T, MR, IN_GLU_CLAMP); else if (in_mode == 4) MRS_GEMV_(T, MR, IN_BIAS_XIELU); else MRS_GEMV_(T, MR, IN_RELU_SQ); } while (0)
+                             else if (in_mode == 3) MRS_GEMV_(T, MR, IN_GLU_CLAMP); else if (in_mode == 4) MRS_GEMV_(T, MR, IN_BIAS_XIELU); else if (in_mode == 5) MRS_GEMV_(T, MR, IN_RELU_SQ); \
+                             else if (in_mode == 6) MRS_GEMV_(T, MR, IN_GLU_GELU); else if (in_mode == 7) MRS_GEMV_(T, MR, IN_GELU); else MRS_GEMV_(T, MR, IN_SIG_GATE); } while (0)
   const int mr = row_group ? 1 : M;
   if (dtype == 1) { if (mr <= 1) MRS_GEMV(mrs::bf16_t, 1); else if (mr <= 2) MRS_GEMV(mrs::bf16_t, 2); else if (mr <= 4) MRS_GEMV(mrs::bf16_t, 4); else MRS_GEMV(mrs::bf16_t, 8); }
   else { if (mr <= 1) MRS_GEMV(float, 1); else if (mr <= 2) MRS_GEMV(float, 2); else if (mr <= 4) MRS_GEMV(float, 4); else MRS_GEMV(float, 8); }

@@ -34,14 +34,22 @@ __device__ __forceinline__ float block_sum_256(float v, float *red) {
 }
 __device__ __forceinline__ float silu_f(float v) { return v / (1.0f + expf(-v)); }
 __device__ __forceinline__ float sigmoid_f(float v) { return 1.0f / (1.0f + expf(-v)); }
+__device__ __forceinline__ float gelu_tanh_f(float v) { return 0.5f * v * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * v * v, v, v))); }
+__device__ __forceinline__ float gelu_erf_f(float v) { return 0.5f * v * (1.0f + erff(v * 0.7071067811865476f)); }
 __device__ __forceinline__ float softplus_f(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
 
 // ---------------------------------------------------------------------------------- embedding rows -> f32 residual
-template <class T> __global__ void __launch_bounds__(256) embed_kernel(const int *__restrict__ tokens, const T *__restrict__ table, float *__restrict__ x, int W, int vocab) {
+// (times scale; out, nullable: the same rows rounded to T, the operand of a first sublayer that reads the residual stream as it is)
+template <class T> __global__ void __launch_bounds__(256) embed_kernel(const int *__restrict__ tokens, const T *__restrict__ table, float *__restrict__ x, int W, int vocab, float scale,
+                                                                       T *__restrict__ out) {
   const int t = blockIdx.x;
   int id = tokens[t];
   id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
-  for (int c = threadIdx.x; c < W; c += 256) x[(size_t)t * W + c] = to_f<T>(table[(size_t)id * W + c]);
+  for (int c = threadIdx.x; c < W; c += 256) {
+    const float v = to_f<T>(table[(size_t)id * W + c]) * scale;
+    x[(size_t)t * W + c] = v;
+    if (out) out[(size_t)t * W + c] = from_f<T>(v);
+  }
 }
 
 // ---------------------------------------------------------------------------------- x / sqrt(mean(x^2) + eps) * (w | 1 + w); grid.y = equal parts of the row
@@ -559,6 +567,7 @@ struct AttnArgs {
   int chunk;            // > 0: position i sees j <= i only inside its own chunk, floor(i / chunk) == floor(j / chunk), chunks counted from position 0 (window / keep_first unused)
   const float *sink_logit;  // [H], nullable: with `sink`, the extra term of head h is e^{sink_logit[h]} instead of e^0
   int gate_per_head;    // the gate holds ONE logit per (row, head) at column h (ldg >= H) instead of one per output value
+  int ldv;              // values between the rows of v_cache (Dv, or more when the value is the front part of a longer cached row)
 };
 __device__ __forceinline__ float sink_of(const AttnArgs &a, int h) { return a.sink_logit ? a.sink_logit[h] : 0.f; }
 __device__ __forceinline__ const float *gate_row(const AttnArgs &a, int t, int h) {
@@ -660,14 +669,14 @@ template <class T, int DVC, bool VEC> __global__ void __launch_bounds__(64) page
 #pragma unroll 4
           for (int j = 0; j < cnt; ++j) {
             float x, y;
-            Ld<T>::v2(vb + (size_t)rowbase[j] * a.Dv, x, y);
+            Ld<T>::v2(vb + (size_t)rowbase[j] * a.ldv, x, y);
             a0 = fmaf(ps[j], x, a0);
             a1 = fmaf(ps[j], y, a1);
           }
         } else {
           const bool two = d + 1 < a.Dv;
           for (int j = 0; j < cnt; ++j) {
-            const T *vr = vb + (size_t)rowbase[j] * a.Dv;
+            const T *vr = vb + (size_t)rowbase[j] * a.ldv;
             a0 = fmaf(ps[j], to_f<T>(vr[0]), a0);
             if (two) a1 = fmaf(ps[j], to_f<T>(vr[1]), a1);
           }
@@ -802,7 +811,7 @@ template <class T, int DVC, int NQ> __global__ void __launch_bounds__(64) paged_
 #pragma unroll 2
         for (int j = 0; j < cnt; ++j) {
           float x, y;
-          Ld<T>::v2(vb + (size_t)rowbase[j] * a.Dv, x, y);
+          Ld<T>::v2(vb + (size_t)rowbase[j] * a.ldv, x, y);
           float pj[NQ];
 #pragma unroll
           for (int q4 = 0; q4 < NQ; q4 += 4) {
@@ -956,6 +965,23 @@ template <class T> __global__ void __launch_bounds__(256) glu_silu_kernel(const 
   const float gv = gu[r * 2 * ff + c], uv = gu[r * 2 * ff + ff + c];
   out[i] = from_f<T>(silu_f(gv) * uv);
 }
+// gelu(gate) * up with the tanh form of gelu; gu [rows, 2 ff] = gate | up
+template <class T> __global__ void __launch_bounds__(256) glu_gelu_kernel(const float *__restrict__ gu, T *__restrict__ out, int rows, int ff) {
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= (size_t)rows * ff) return;
+  const size_t r = i / ff, c = i % ff;
+  out[i] = from_f<T>(gelu_tanh_f(gu[r * 2 * ff + c]) * gu[r * 2 * ff + ff + c]);
+}
+// the exact (erf) gelu of u [n]
+template <class T> __global__ void __launch_bounds__(256) gelu_erf_kernel(const float *__restrict__ u, T *__restrict__ out, size_t n) {
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i < n) out[i] = from_f<T>(gelu_erf_f(u[i]));
+}
+// y * sigmoid(gate): y [rows, n] f32 (contiguous), gate [rows, >= n] f32
+template <class T> __global__ void __launch_bounds__(256) sigmoid_gate_kernel(const float *__restrict__ y, const float *__restrict__ gate, int ldg, T *__restrict__ out, int n, size_t total) {
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i < total) out[i] = from_f<T>(y[i] * sigmoid_f(gate[(i / n) * ldg + i % n]));
+}
 // g = min(gate, limit), u = clamp(up, -limit, limit): g * sigmoid(alpha g) * (u + 1); gu [rows, 2 ff] = gate | up
 __device__ __forceinline__ float glu_clamped_f(float gv, float uv, float limit, float alpha) {
   const float g = fminf(gv, limit), u = fminf(fmaxf(uv, -limit), limit);
@@ -1045,6 +1071,58 @@ template <class T> __global__ void __launch_bounds__(256) layernorm_kernel(const
   }
 }
 
+// Designs whose sublayers read the residual stream as it is: resid += layer norm(y) * w (+ b), out (T, nullable) = the updated row rounded once, the next sublayer's operand.  y may
+// be given as routed experts' outputs instead: y = sum_k wts[t top + k] d[route_pos[t top + k]], summed while the row is read.  V: four values per access.
+template <class T, int V> __global__ void __launch_bounds__(256) layernorm_join_kernel(const float *__restrict__ y, int ldy, const float *__restrict__ d, const int *__restrict__ route_pos,
+                                                                                        const float *__restrict__ wts, int top, const float *__restrict__ w, const float *__restrict__ b,
+                                                                                        float *__restrict__ resid, int ldr, T *__restrict__ out, int width, float eps) {
+  __shared__ float red[4];
+  extern __shared__ __attribute__((aligned(16))) float row[];
+  const int t = blockIdx.x;
+  float s = 0.f;
+  for (int c = threadIdx.x * V; c < width; c += 256 * V) {
+    float v[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] = 0.f;
+    if (d) {
+      for (int k = 0; k < top; ++k) {
+        const float wk = wts[(size_t)t * top + k];
+        const float *dr = d + (size_t)route_pos[(size_t)t * top + k] * width + c;
+        float x[V];
+        if (V == 4) { const float4 q = *(const float4 *)dr; x[0] = q.x; x[V > 1 ? 1 : 0] = q.y; x[V > 2 ? 2 : 0] = q.z; x[V > 3 ? 3 : 0] = q.w; }
+        else x[0] = dr[0];
+#pragma unroll
+        for (int j = 0; j < V; ++j) v[j] = fmaf(wk, x[j], v[j]);
+      }
+    } else {
+      const float *yr = y + (size_t)t * ldy + c;
+      if (V == 4) { const float4 q = *(const float4 *)yr; v[0] = q.x; v[V > 1 ? 1 : 0] = q.y; v[V > 2 ? 2 : 0] = q.z; v[V > 3 ? 3 : 0] = q.w; }
+      else v[0] = yr[0];
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) { row[c + j] = v[j]; s += v[j]; }
+  }
+  const float mean = block_sum_256(s, red) / (float)width;
+  float q = 0.f;
+  for (int c = threadIdx.x * V; c < width; c += 256 * V)
+#pragma unroll
+    for (int j = 0; j < V; ++j) { const float dv = row[c + j] - mean; q = fmaf(dv, dv, q); }
+  const float inv = 1.0f / sqrtf(block_sum_256(q, red) / (float)width + eps);
+  for (int c = threadIdx.x * V; c < width; c += 256 * V) {
+    float *rp = resid + (size_t)t * ldr + c, x[V];
+    if (V == 4) { const float4 r4 = *(const float4 *)rp; x[0] = r4.x; x[V > 1 ? 1 : 0] = r4.y; x[V > 2 ? 2 : 0] = r4.z; x[V > 3 ? 3 : 0] = r4.w; }
+    else x[0] = rp[0];
+#pragma unroll
+    for (int j = 0; j < V; ++j) x[j] += (row[c + j] - mean) * inv * w[c + j] + (b ? b[c + j] : 0.f);
+    if (V == 4) *(float4 *)rp = make_float4(x[0], x[V > 1 ? 1 : 0], x[V > 2 ? 2 : 0], x[V > 3 ? 3 : 0]);
+    else rp[0] = x[0];
+    if (out) {
+#pragma unroll
+      for (int j = 0; j < V; ++j) out[(size_t)t * width + c + j] = from_f<T>(x[j]);
+    }
+  }
+}
+
 // ---------------------------------------------------------------------------------- projection biases, query temperature, K / V page write (no norm, no rotation)
 // q <- (q + qb) * (1 + coef ln(floor((pos + 1) / every) + 1)) in f32, rounded once to T; k + kb and v + vb go to the page slot of the row (no k_cache: the layer reads another
 // layer's pages and has no key / value columns)
@@ -1120,6 +1198,85 @@ template <class T> __global__ void __launch_bounds__(256) latent_norm_cache_kern
   for (int e = tid; e < R; e += 256) c_cache[(size_t)slot * R + e] = from_f<T>(c[e] * inv * w[e]);
 }
 
+// The general form: u [rows, ld] = [query latent qr (0: none) | latent R | rotated key part rot | ...] (f32, one product).  The query latent is RMS-normed (qw) and rounded to cq;
+// the latent is RMS-normed (cw) and goes, with the rotated key part (not normed) behind it, to the row's page slot of c_cache [blocks, 1, block_size, R + rot].
+// Rotation: in the first dims of the rot values, (x_i, x_{i + dims / 2}) turns by position * freq[i]; cos and sin times trig_mult.
+template <class T> __global__ void __launch_bounds__(256) latent_prep_kernel(const float *__restrict__ u, int ld, int qr, int R, int rot, int dims, const float *__restrict__ qw,
+                                                                             const float *__restrict__ cw, const float *__restrict__ freq, float trig_mult, const int *__restrict__ tok_pos,
+                                                                             const long long *__restrict__ slot_mapping, T *__restrict__ cq, T *__restrict__ c_cache, float eps) {
+  __shared__ float red[4];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const float *q = u + (size_t)t * ld, *c = q + qr, *k = c + R;
+  if (blockIdx.y == 1) {  // the query latent
+    float s = 0.f;
+    for (int e = tid; e < qr; e += 256) s = fmaf(q[e], q[e], s);
+    const float inv = 1.0f / sqrtf(block_sum_256(s, red) / (float)qr + eps);
+    for (int e = tid; e < qr; e += 256) cq[(size_t)t * qr + e] = from_f<T>(q[e] * inv * qw[e]);
+    return;
+  }
+  float s = 0.f;
+  for (int e = tid; e < R; e += 256) s = fmaf(c[e], c[e], s);
+  const float inv = 1.0f / sqrtf(block_sum_256(s, red) / (float)R + eps);
+  const long long slot = slot_mapping[t];
+  if (slot < 0) return;
+  T *row = c_cache + (size_t)slot * (R + rot);
+  for (int e = tid; e < R; e += 256) row[e] = from_f<T>(c[e] * inv * cw[e]);
+  const int half = dims >> 1;
+  const float pos = (float)tok_pos[t];
+  for (int e = tid; e < rot - half; e += 256) {  // `half` pairs, then the values that pass
+    if (e < half) {
+      float sn, cs;
+      sincosf(pos * freq[e], &sn, &cs);
+      sn *= trig_mult; cs *= trig_mult;
+      const float a = k[e], b = k[e + half];
+      row[R + e] = from_f<T>(a * cs - b * sn);
+      row[R + e + half] = from_f<T>(b * cs + a * sn);
+    } else {
+      row[R + e + half] = from_f<T>(k[e + half]);
+    }
+  }
+}
+// Queries of that attention: qf [rows, ldq] f32 holds per head D values and rot values behind them.  The D values go to q_out [rows, H * (D + rot)] (T) in the same layout; the
+// rotated part goes behind them there too, or (qa given) to the tail of qa [rows, H * (R + rot)] (T), whose front R values per head a product fills.
+template <class T> __global__ void __launch_bounds__(256) latent_query_kernel(const float *__restrict__ qf, int ldq, int H, int D, int R, int rot, int dims, const float *__restrict__ freq,
+                                                                              float trig_mult, const int *__restrict__ tok_pos, T *__restrict__ q_out, T *__restrict__ qa) {
+  extern __shared__ float trig[];  // cos [half] | sin [half] of the row's position
+  const int t = blockIdx.x, tid = threadIdx.x, half = dims >> 1, E = D + rot;
+  const float pos = (float)tok_pos[t];
+  for (int e = tid; e < half; e += 256) {
+    float sn, cs;
+    sincosf(pos * freq[e], &sn, &cs);
+    trig[e] = cs * trig_mult;
+    trig[half + e] = sn * trig_mult;
+  }
+  __syncthreads();
+  const float *q = qf + (size_t)t * ldq;
+  for (int e = tid; e < H * E; e += 256) {
+    const int h = e / E, j = e - h * E, i = j - D;
+    float v = q[e];
+    T *dst = q_out + (size_t)t * H * E + e;
+    if (i >= 0) {
+      if (i < half) v = v * trig[i] - q[e + half] * trig[half + i];
+      else if (i < dims) v = v * trig[i - half] + q[e - half] * trig[i];
+      if (qa) dst = qa + ((size_t)t * H + h) * (R + rot) + R + i;
+    }
+    *dst = from_f<T>(v);
+  }
+}
+// The cached rows of whole blocks on their way into keys and values of a prompt step: source [n blocks] of c_cache rows [c R | key part rot] -> c [n * block_size, R], and the key
+// part behind the D values of every head of k [n * block_size, H, D + rot]
+template <class T> __global__ void __launch_bounds__(256) latent_context_kernel(const T *__restrict__ c_cache, const int *__restrict__ source, T *__restrict__ c, T *__restrict__ k, int block_size,
+                                                                                int R, int rot, int H, int D) {
+  const int i = blockIdx.x;
+  const T *row = c_cache + ((size_t)source[i / block_size] * block_size + i % block_size) * (R + rot);
+  for (int e = threadIdx.x; e < R; e += 256) c[(size_t)i * R + e] = row[e];
+  const int E = D + rot;
+  for (int e = threadIdx.x; e < H * rot; e += 256) {
+    const int h = e / rot, j = e - h * rot;
+    k[((size_t)i * H + h) * E + D + j] = row[R + j];
+  }
+}
+
 // ---------------------------------------------------------------------------------- several residual streams (hyper-connections)
 // x [rows, S, W] f32.  One launch closes a sublayer and opens the next:
 //   write  (y given): new_r = sum_s mix[s, r] x_s + outw[r] y for every stream r, all from the old streams (mix null: new_r = outw[r] y -- the streams' start)
@@ -1189,12 +1346,16 @@ using namespace mrs::hyb;
 
 extern "C" const char *mrs_hyb_last_error() { return g_err; }
 
-extern "C" int mrs_hyb_embed(const int *tokens, const void *table, float *x, int rows, int W, int vocab, int dtype, void *stream) {
+/* x (f32) = table[token] * scale; out (dtype, nullable): the same rows rounded once */
+extern "C" int mrs_hyb_embed_scaled(const int *tokens, const void *table, float *x, void *out, int rows, int W, int vocab, float scale, int dtype, void *stream) {
   if (rows <= 0) return 0;
-  if (dtype == 1) hipLaunchKernelGGL(embed_kernel<mrs::bf16_t>, dim3(rows), dim3(256), 0, S_(stream), tokens, (const mrs::bf16_t *)table, x, W, vocab);
-  else if (dtype == 2) hipLaunchKernelGGL(embed_kernel<float>, dim3(rows), dim3(256), 0, S_(stream), tokens, (const float *)table, x, W, vocab);
+  if (dtype == 1) hipLaunchKernelGGL(embed_kernel<mrs::bf16_t>, dim3(rows), dim3(256), 0, S_(stream), tokens, (const mrs::bf16_t *)table, x, W, vocab, scale, (mrs::bf16_t *)out);
+  else if (dtype == 2) hipLaunchKernelGGL(embed_kernel<float>, dim3(rows), dim3(256), 0, S_(stream), tokens, (const float *)table, x, W, vocab, scale, (float *)out);
   else return fail("mrs_hyb_embed: dtype");
   return ok_or("mrs_hyb_embed");
+}
+extern "C" int mrs_hyb_embed(const int *tokens, const void *table, float *x, int rows, int W, int vocab, int dtype, void *stream) {
+  return mrs_hyb_embed_scaled(tokens, table, x, nullptr, rows, W, vocab, 1.0f, dtype, stream);
 }
 
 // parts > 1: every row is normed in `parts` equal pieces, each by its own root mean square.  out (dtype) and / or out32 (f32) receive the result, rstd [rows, parts] the 1 / rms.
@@ -1364,14 +1525,16 @@ extern "C" int mrs_hyb_qk_headnorm_rope_cache(const float *qkv, int ld, const fl
 static int attn_launch(const void *q, const void *k_cache, const void *v_cache, const int *block_tables, const int *tok_seq, const int *tok_pos, void *out,
                        int rows, int H, int G, int D, int Dv, int block_size, int max_blocks, int window, int keep_first, float scale, int dtype,
                        const int *seg_entry, const int *seg_row0, const int *seg_len, int segments, int seg_rows, float softcap, int sink, const float *gate, int ldg,
-                       float *scratch, int splits, int token_major, void *stream, int chunk = 0, const float *sink_logit = nullptr, int gate_per_head = 0) {
+                       float *scratch, int splits, int token_major, void *stream, int chunk = 0, const float *sink_logit = nullptr, int gate_per_head = 0, int ldv = 0) {
   if (rows <= 0) return 0;
   if (Dv > 512 || H % G) return fail("mrs_hyb_paged_window_attn: value size above 512 / heads % kv_heads");
   if (gate && ldg < (gate_per_head ? H : H * Dv)) return fail("mrs_hyb_paged_window_attn: gate rows shorter than heads (* value size)");
   if (chunk > 0 && (window > 0 || keep_first > 0)) return fail("mrs_hyb_paged_window_attn: chunks and a sliding window exclude each other");
+  if (ldv == 0) ldv = Dv;
+  if (ldv < Dv) return fail("mrs_hyb_paged_window_attn: value rows overlap");
   AttnArgs a{q, k_cache, v_cache, block_tables, tok_seq, tok_pos, out, H, G, D, Dv, block_size, max_blocks, window, keep_first, scale, softcap > 0.f ? softcap : 0.f, sink ? 1 : 0, gate, ldg, nullptr, 0, rows, token_major ? 1 : 0,
-             chunk > 0 ? chunk : 0, sink ? sink_logit : nullptr, gate_per_head ? 1 : 0};
-  const bool vec = D % 8 == 0 && Dv % 2 == 0 && ((uintptr_t)k_cache % 16) == 0 && ((uintptr_t)v_cache % 8) == 0;
+             chunk > 0 ? chunk : 0, sink ? sink_logit : nullptr, gate_per_head ? 1 : 0, ldv};
+  const bool vec = D % 8 == 0 && Dv % 2 == 0 && ldv % 2 == 0 && ((uintptr_t)k_cache % 16) == 0 && ((uintptr_t)v_cache % 8) == 0;
   const int c = (Dv + 127) / 128;
   if (vec && seg_entry && segments > 0 && rows > segments && segments <= 65535 && seg_rows > 0) {
     constexpr int NQ = 8;
@@ -1431,6 +1594,16 @@ extern "C" int mrs_hyb_paged_attn_chunked(const void *q, const void *k_cache, co
                                           int ldg, int gate_per_head, float *scratch, int splits, void *stream) {
   return attn_launch(q, k_cache, v_cache, block_tables, tok_seq, tok_pos, out, rows, H, G, D, Dv, block_size, max_blocks, 0, 0, scale, dtype, seg_entry, seg_row0, seg_len,
                      segments, seg_rows, softcap, sink, gate, ldg, scratch, splits, 0, stream, chunk, sink_logit, gate_per_head);
+}
+
+/* the same attention with a sliding window (and kept first tokens) next to a learned sink and an elementwise gate, over value rows of stride ldv (0: Dv): k_cache and v_cache may be
+ * ONE cache whose row is a key and whose front part is the value */
+extern "C" int mrs_hyb_paged_attn_sink_window(const void *q, const void *k_cache, const void *v_cache, const int *block_tables, const int *tok_seq, const int *tok_pos, void *out,
+                                              int rows, int H, int G, int D, int Dv, int block_size, int max_blocks, int window, int keep_first, float scale, int dtype,
+                                              const int *seg_entry, const int *seg_row0, const int *seg_len, int segments, int seg_rows, float softcap, int sink,
+                                              const float *sink_logit, const float *gate, int ldg, float *scratch, int splits, int token_major, int ldv, void *stream) {
+  return attn_launch(q, k_cache, v_cache, block_tables, tok_seq, tok_pos, out, rows, H, G, D, Dv, block_size, max_blocks, window, keep_first, scale, dtype, seg_entry, seg_row0, seg_len,
+                     segments, seg_rows, softcap, sink, gate, ldg, scratch, splits, token_major, stream, 0, sink_logit, 0, ldv);
 }
 
 /* h [rows, W] f32 (contiguous), wr [E (+ 1), W] f32 */
@@ -1496,6 +1669,35 @@ extern "C" int mrs_hyb_moe_combine_weighted(float *out, const float *d, const in
   return ok_or("mrs_hyb_moe_combine_weighted");
 }
 
+extern "C" int mrs_hyb_glu_gelu(const float *gu, void *out, int rows, int ff, int dtype, void *stream) {
+  if (rows <= 0) return 0;
+  const unsigned blocks = (unsigned)(((size_t)rows * ff + 255) / 256);
+  if (dtype == 1) hipLaunchKernelGGL(glu_gelu_kernel<mrs::bf16_t>, dim3(blocks), dim3(256), 0, S_(stream), gu, (mrs::bf16_t *)out, rows, ff);
+  else if (dtype == 2) hipLaunchKernelGGL(glu_gelu_kernel<float>, dim3(blocks), dim3(256), 0, S_(stream), gu, (float *)out, rows, ff);
+  else return fail("mrs_hyb_glu_gelu: dtype");
+  return ok_or("mrs_hyb_glu_gelu");
+}
+extern "C" int mrs_hyb_gelu_erf(const float *u, void *out, int rows, int ff, int dtype, void *stream) {
+  const size_t n = (size_t)rows * ff;
+  if (rows <= 0 || n == 0) return 0;
+  const unsigned blocks = (unsigned)((n + 255) / 256);
+  if (dtype == 1) hipLaunchKernelGGL(gelu_erf_kernel<mrs::bf16_t>, dim3(blocks), dim3(256), 0, S_(stream), u, (mrs::bf16_t *)out, n);
+  else if (dtype == 2) hipLaunchKernelGGL(gelu_erf_kernel<float>, dim3(blocks), dim3(256), 0, S_(stream), u, (float *)out, n);
+  else return fail("mrs_hyb_gelu_erf: dtype");
+  return ok_or("mrs_hyb_gelu_erf");
+}
+/* out (dtype) [rows, n] = y * sigmoid(gate) */
+extern "C" int mrs_hyb_sigmoid_gate(const float *y, const float *gate, int ldg, void *out, int rows, int n, int dtype, void *stream) {
+  const size_t total = (size_t)rows * n;
+  if (rows <= 0 || total == 0) return 0;
+  if (ldg < n) return fail("mrs_hyb_sigmoid_gate: gate rows shorter than the values");
+  const unsigned blocks = (unsigned)((total + 255) / 256);
+  if (dtype == 1) hipLaunchKernelGGL(sigmoid_gate_kernel<mrs::bf16_t>, dim3(blocks), dim3(256), 0, S_(stream), y, gate, ldg, (mrs::bf16_t *)out, n, total);
+  else if (dtype == 2) hipLaunchKernelGGL(sigmoid_gate_kernel<float>, dim3(blocks), dim3(256), 0, S_(stream), y, gate, ldg, (float *)out, n, total);
+  else return fail("mrs_hyb_sigmoid_gate: dtype");
+  return ok_or("mrs_hyb_sigmoid_gate");
+}
+
 extern "C" int mrs_hyb_glu_clamped(const float *gu, void *out, int rows, int ff, float limit, float alpha, int dtype, void *stream) {
   if (rows <= 0) return 0;
   const unsigned blocks = (unsigned)(((size_t)rows * ff + 255) / 256);
@@ -1542,6 +1744,24 @@ extern "C" int mrs_hyb_layernorm_pair(const float *y, int ldy, const float *in_b
   return ok_or("mrs_hyb_layernorm_pair");
 }
 
+/* resid [rows, ldr] += layer norm(y) * w (+ b, nullable); out (dtype, nullable) [rows, width] = the updated rows, rounded once.  y null: the rows are the routed experts' outputs
+ * d [rows * top, width], y[t] = sum_k wts[t top + k] d[route_pos[t top + k]] */
+extern "C" int mrs_hyb_layernorm_join(const float *y, int ldy, const float *d, const int *route_pos, const float *wts, int top, const float *w, const float *b, float *resid, int ldr,
+                                      void *out, int rows, int width, float eps, int dtype, void *stream) {
+  if (rows <= 0) return 0;
+  if (width <= 0 || width > 15000) return fail("mrs_hyb_layernorm_join: 1 .. 15000 values per row");
+  if (!resid || !w || ldr < width || (!y && (!d || !route_pos || !wts || top < 1)) || (y && ldy < width)) return fail("mrs_hyb_layernorm_join: the stream, the norm's weight and one input are needed");
+  if (dtype != 1 && dtype != 2) return fail("mrs_hyb_layernorm_join: dtype");
+  const size_t lds = (size_t)width * 4;
+  const bool v4 = width % 4 == 0 && ldr % 4 == 0 && (!y || (ldy % 4 == 0 && ((uintptr_t)y % 16) == 0)) && ((uintptr_t)resid % 16) == 0 && (y || ((uintptr_t)d % 16) == 0);
+  if (y) d = nullptr;
+#define MRS_LNJ(T, V) hipLaunchKernelGGL((layernorm_join_kernel<T, V>), dim3(rows), dim3(256), lds, S_(stream), y, ldy, d, route_pos, wts, top, w, b, resid, ldr, (T *)out, width, eps)
+  if (dtype == 1) { if (v4) MRS_LNJ(mrs::bf16_t, 4); else MRS_LNJ(mrs::bf16_t, 1); }
+  else { if (v4) MRS_LNJ(float, 4); else MRS_LNJ(float, 1); }
+#undef MRS_LNJ
+  return ok_or("mrs_hyb_layernorm_join");
+}
+
 /* temp_every <= 0: no query temperature.  k_cache null: the rows carry no key / value columns (a layer that reads another layer's pages) */
 extern "C" int mrs_hyb_qkv_bias_temp_cache(const float *qkv, int ld, const float *qb, const float *kb, const float *vb, const int *tok_pos, const long long *slot_mapping, void *q_out,
                                            void *k_cache, void *v_cache, int rows, int H, int G, int D, int Dv, int block_size, float temp_coef, int temp_every, int dtype,
@@ -1579,6 +1799,41 @@ extern "C" int mrs_hyb_latent_norm_cache(const float *u, int ld, int nq, int R, 
   else if (dtype == 2) hipLaunchKernelGGL(latent_norm_cache_kernel<float>, dim3(rows), dim3(256), 0, S_(stream), u, ld, nq, R, w, slot_mapping, (float *)q_out, (float *)c_cache, eps);
   else return fail("mrs_hyb_latent_norm_cache: dtype");
   return ok_or("mrs_hyb_latent_norm_cache");
+}
+
+/* u [rows, ld] = query latent [qr, 0: none] | latent [R] | rotated key part [rot]: cq [rows, qr] (dtype) = the normed query latent, c_cache[slot] (dtype, rows of R + rot) = the normed
+ * latent | the key part, its first dims values turned in half-split pairs (cos and sin times trig_mult) */
+extern "C" int mrs_hyb_latent_prep(const float *u, int ld, int qr, int R, int rot, int dims, const float *qw, const float *cw, const float *freq, float trig_mult, const int *tok_pos,
+                                   const long long *slot_mapping, void *cq, void *c_cache, float eps, int rows, int dtype, void *stream) {
+  if (rows <= 0) return 0;
+  if (qr < 0 || R <= 0 || rot < 0 || dims < 0 || (dims & 1) || dims > rot || ld < qr + R + rot || !cw || (qr > 0 && (!qw || !cq)) || (dims > 0 && !freq))
+    return fail("mrs_hyb_latent_prep: sizes (even rotated dimensions inside the key part), rows or weights");
+  dim3 grid(rows, qr > 0 ? 2 : 1);
+  if (dtype == 1) hipLaunchKernelGGL(latent_prep_kernel<mrs::bf16_t>, grid, dim3(256), 0, S_(stream), u, ld, qr, R, rot, dims, qw, cw, freq, trig_mult, tok_pos, slot_mapping, (mrs::bf16_t *)cq, (mrs::bf16_t *)c_cache, eps);
+  else if (dtype == 2) hipLaunchKernelGGL(latent_prep_kernel<float>, grid, dim3(256), 0, S_(stream), u, ld, qr, R, rot, dims, qw, cw, freq, trig_mult, tok_pos, slot_mapping, (float *)cq, (float *)c_cache, eps);
+  else return fail("mrs_hyb_latent_prep: dtype");
+  return ok_or("mrs_hyb_latent_prep");
+}
+/* qf [rows, ldq] f32 = H heads of D + rot values -> q_out (dtype, same layout), the last rot values of every head rotated; qa (nullable, dtype [rows, H * (R + rot)]): the rotated
+ * values go to its heads' tails instead */
+extern "C" int mrs_hyb_latent_query(const float *qf, int ldq, int H, int D, int R, int rot, int dims, const float *freq, float trig_mult, const int *tok_pos, void *q_out, void *qa,
+                                    int rows, int dtype, void *stream) {
+  if (rows <= 0) return 0;
+  if (H <= 0 || D <= 0 || rot < 0 || dims < 0 || (dims & 1) || dims > rot || dims > 8192 || ldq < H * (D + rot) || (dims > 0 && !freq) || (qa && R <= 0))
+    return fail("mrs_hyb_latent_query: head sizes (even rotated dimensions inside the rotated part) or rows");
+  if (dtype == 1) hipLaunchKernelGGL(latent_query_kernel<mrs::bf16_t>, dim3(rows), dim3(256), dims * 4, S_(stream), qf, ldq, H, D, R, rot, dims, freq, trig_mult, tok_pos, (mrs::bf16_t *)q_out, (mrs::bf16_t *)qa);
+  else if (dtype == 2) hipLaunchKernelGGL(latent_query_kernel<float>, dim3(rows), dim3(256), dims * 4, S_(stream), qf, ldq, H, D, R, rot, dims, freq, trig_mult, tok_pos, (float *)q_out, (float *)qa);
+  else return fail("mrs_hyb_latent_query: dtype");
+  return ok_or("mrs_hyb_latent_query");
+}
+/* blocks source [n] of c_cache (rows of R + rot) -> c [n * block_size, R] and, behind the D values of every head, k [n * block_size, H * (D + rot)] (all dtype) */
+extern "C" int mrs_hyb_latent_context(const void *c_cache, const int *source, void *c, void *k, int n, int block_size, int R, int rot, int H, int D, int dtype, void *stream) {
+  if (n <= 0) return 0;
+  if (block_size <= 0 || R <= 0 || rot < 0 || H <= 0 || D <= 0) return fail("mrs_hyb_latent_context: sizes");
+  if (dtype == 1) hipLaunchKernelGGL(latent_context_kernel<mrs::bf16_t>, dim3(n * block_size), dim3(256), 0, S_(stream), (const mrs::bf16_t *)c_cache, source, (mrs::bf16_t *)c, (mrs::bf16_t *)k, block_size, R, rot, H, D);
+  else if (dtype == 2) hipLaunchKernelGGL(latent_context_kernel<float>, dim3(n * block_size), dim3(256), 0, S_(stream), (const float *)c_cache, source, (float *)c, (float *)k, block_size, R, rot, H, D);
+  else return fail("mrs_hyb_latent_context: dtype");
+  return ok_or("mrs_hyb_latent_context");
 }
 
 /* x [rows, S, W] f32 residual streams.  y (nullable, [rows, W]): x_r <- sum_s mix[s, r] x_s + outw[r] y (mix null: x_r <- outw[r] y).  inw (nullable, [S]): v = sum_s inw[s] x_s of

@@ -1,0 +1,401 @@
+// hyb_linattn.hip -- gated linear attention with one decay per key channel (f32 state [slot, head, D, Dv], carried per sequence slot):
+//   alpha = sigmoid(z + bias)^(1 / tau);   S <- diag(alpha) S + k v^T;   o = S^T (q q_mult)
+// Same conventions as hyb_kernels.hip: a step's rows are one flat range, entry s owns rows [seq_start[s], seq_start[s + 1]) at positions seq_pos0[s] + i and state slot
+// seq_slot[s]; an entry whose first position is 0 reads its slot as zero.
+//
+//   scan   steps with portions: entries as chains, or the segments of long portions side by side (end states and decay products from zero, a carry, the outputs)
+//   step   steps of single rows: the second step of the decay's projection, the decays, the state update, the read-out, the per-head output norm and the SiLU gate in one launch
+//
+// Everything here is f32 arithmetic on f32 operands; T is only the type the results are rounded to for the next product (and the type of a weight).
+#include "common.cuh"
+#include <float.h>
+
+namespace mrs {
+namespace hybl {
+
+static thread_local char g_err[256];
+static int fail(const char *m) { snprintf(g_err, sizeof g_err, "%s", m); return 1; }
+static int ok_or(const char *what) {
+  if (hipGetLastError() == hipSuccess) return 0;
+  snprintf(g_err, sizeof g_err, "%s: launch failed", what);
+  return 1;
+}
+
+__device__ __forceinline__ float silu_f(float v) { return v / (1.0f + expf(-v)); }
+__device__ __forceinline__ float softplus_f(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
+// sigmoid(z)^(1 / tau) through its logarithm, -softplus(-z) / tau: no cancellation at either end
+__device__ __forceinline__ float channel_decay(float z, float inv_tau) { return expf(-softplus_f(-z) * inv_tau); }
+
+// sum over groups of R consecutive lanes (R = 4, 8, 16, groups aligned to R) with data-parallel-primitive moves inside a row of 16 lanes
+template <int CTRL> __device__ __forceinline__ float dpp_add(float x) {
+  return x + __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), CTRL, 0xf, 0xf, true));
+}
+template <int R> __device__ __forceinline__ float group_sum(float x) {
+  static_assert(R == 4 || R == 8 || R == 16, "groups of 4, 8 or 16 lanes");
+  x = dpp_add<0xB1>(x);               // quad_perm [1, 0, 3, 2]
+  x = dpp_add<0x4E>(x);               // quad_perm [2, 3, 0, 1]
+  if (R == 8) x = dpp_add<0x141>(x);  // row_half_mirror: the other quad of the eight
+  if (R == 16) {
+    x = dpp_add<0x124>(x);            // row_ror 4
+    x = dpp_add<0x128>(x);            // row_ror 8
+  }
+  return x;
+}
+
+struct GlaArgs {
+  const float *u;       // [rows, ldu]: v [H * Dv] at 0, k [H * D] at k_col, q [H * D] at q_col
+  const float *z;       // [rows, ldz]: decay logits [H * D], before the bias
+  const float *zb;      // [H * D]
+  float *state;         // [slots, H, D, Dv]
+  float *out;           // [rows, H * Dv]
+  const int *seq_pos0, *seq_slot;
+  const int *seg_entry, *seg_row0, *seg_len, *ent_seg0;  // segment table: entry, first row, rows; first segment of every entry (+ the total)
+  float *carry;         // [segments, H, D, Dv]: a segment's end state from zero, then the state the next segment starts from
+  float *decay;         // [segments, H, D]: the products of a segment's decays
+  int ldu, k_col, q_col, ldz, H, D, Dv;
+  float q_mult, inv_tau;
+};
+
+// The recurrence is linear in S and a row scales the state's rows by numbers of its own, so a long portion can run its segments side by side:
+//   A  every segment but an entry's last, from zero: its end state L_k and the channel products d_k                        (LOCAL; parallel over segments)
+//   B  init_(k+1) = diag(d_k) init_k + L_k, init_0 = the slot's state (zero for an entry that starts at position 0)      (gla_carry_kernel)
+//   C  every segment from its init state: the outputs; an entry's last segment leaves the slot's new state               (parallel over segments)
+// An entry of one segment is pass C alone.
+// A workgroup owns one (segment, head) and 64 / R * 4 value columns per wave.  A lane holds a register tile of the state: 4 columns times K = 4 J rows n = 4 (j R + r) + i (r = its
+// place in the group of R lanes): per row of tokens it reads 3 J + 1 16-byte groups (k, q, decays, v) from LDS for 12 K multiply-adds, lanes of a group at adjacent
+// addresses, and the four column sums close with data-parallel-primitive adds inside the group.  Token rows are staged TC at a time, key sizes and columns zero-padded to the tile
+// so that the loop has no guards; the next stage's values travel in registers while the current one is consumed, and the decays are evaluated on the way into LDS.
+template <int R, int J, bool LOCAL, int NT> __global__ void __launch_bounds__(NT) gla_scan_kernel(GlaArgs a, int TC, int vec) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];  // [2][TC][k Dp | q Dp | decay Dp | v PC]
+  constexpr int K = 4 * J, Dp = R * K, CW = 64 / R * 4, MAXV = 4;
+  const int tid = threadIdx.x, nthr = blockDim.x, wave = tid >> 6, lane = tid & 63, r = lane % R, pl = lane / R;
+  const int h = blockIdx.y, z = blockIdx.z, PC = (nthr >> 6) * CW, p0 = blockIdx.x * PC;
+  const int s = a.seg_entry[z], r0 = a.seg_row0[z], len = a.seg_len[z], D = a.D, Dv = a.Dv;
+  const bool first = z == a.ent_seg0[s], last = z == a.ent_seg0[s + 1] - 1;
+  if (len <= 0 || (LOCAL && last)) return;
+  const int pc = wave * CW + pl * 4, p = p0 + pc;    // this lane's first column: in the workgroup, in the head
+  const size_t np = (size_t)D * Dv;
+  float *st = a.state + ((size_t)a.seq_slot[s] * a.H + h) * np;
+  const float *init = LOCAL ? nullptr : (first ? (a.seq_pos0[s] > 0 ? st : nullptr) : a.carry + ((size_t)(z - 1) * a.H + h) * np);
+  float S[K][4], prod[LOCAL ? K : 1];
+#pragma unroll
+  for (int k = 0; k < K; ++k) {
+    const int n = 4 * ((k >> 2) * R + r) + (k & 3);
+#pragma unroll
+    for (int c = 0; c < 4; ++c) S[k][c] = (init && n < D && p + c < Dv) ? init[(size_t)n * Dv + p + c] : 0.f;
+    if (LOCAL) prod[k] = 1.0f;
+  }
+  // a stage = TC rows of U groups of four values, dealt to the threads flat; where a group comes from is worked out once
+  const int U = (3 * Dp + PC) >> 2, stage_n = TC * U, rowlen = 4 * U, stage = TC * rowlen;
+  float4 stg[MAXV];
+  const float *src[MAXV];
+  int what[MAXV], cnt4[MAXV], irow[MAXV], step[MAXV];   // 0: nothing, 1: plain, 2: query, 3: decay logit
+  float4 bias[MAXV];
+#pragma unroll
+  for (int m = 0; m < MAXV; ++m) {
+    const int e = tid + m * nthr;
+    what[m] = 0; cnt4[m] = 0; irow[m] = 0; step[m] = 0; src[m] = a.u;
+    bias[m] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (e >= stage_n) continue;
+    const int i = e / U, j = 4 * (e - i * U);
+    irow[m] = i;
+    const size_t row = (size_t)(r0 + i);
+    if (j < 3 * Dp) {
+      const int which = j / Dp, n = j - which * Dp;
+      cnt4[m] = D - n < 0 ? 0 : (D - n > 4 ? 4 : D - n);
+      if (which < 2) { src[m] = a.u + row * a.ldu + (which ? a.q_col : a.k_col) + h * D + n; step[m] = a.ldu; what[m] = 1 + which; }
+      else {
+        src[m] = a.z + row * a.ldz + h * D + n; step[m] = a.ldz; what[m] = 3;
+        const float *b = a.zb + h * D + n;
+        if (cnt4[m] > 0) bias[m].x = b[0];
+        if (cnt4[m] > 1) bias[m].y = b[1];
+        if (cnt4[m] > 2) bias[m].z = b[2];
+        if (cnt4[m] > 3) bias[m].w = b[3];
+      }
+    } else {
+      const int c = p0 + j - 3 * Dp;
+      cnt4[m] = Dv - c < 0 ? 0 : (Dv - c > 4 ? 4 : Dv - c);
+      src[m] = a.u + row * a.ldu + h * Dv + c; step[m] = a.ldu; what[m] = 1;
+    }
+    if (cnt4[m] == 0) what[m] = 0;
+  }
+  auto fetch = [&](int c0) {
+#pragma unroll
+    for (int m = 0; m < MAXV; ++m) {
+      float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (what[m] && c0 + irow[m] < len) {
+        const float *q = src[m] + (size_t)c0 * step[m];
+        if (vec && cnt4[m] == 4) v = *(const float4 *)q;
+        else {
+          v.x = q[0];
+          if (cnt4[m] > 1) v.y = q[1];
+          if (cnt4[m] > 2) v.z = q[2];
+          if (cnt4[m] > 3) v.w = q[3];
+        }
+      }
+      stg[m] = v;
+    }
+  };
+  auto put = [&](float *buf) {
+#pragma unroll
+    for (int m = 0; m < MAXV; ++m) {
+      const int e = tid + m * nthr;
+      if (e >= stage_n) continue;
+      float4 v = stg[m];
+      if (what[m] == 2) { v.x *= a.q_mult; v.y *= a.q_mult; v.z *= a.q_mult; v.w *= a.q_mult; }
+      else if (what[m] == 3) {  // (channels past the key size never see a key: whatever they decay by, they hold zero)
+        v.x = channel_decay(v.x + bias[m].x, a.inv_tau); v.y = channel_decay(v.y + bias[m].y, a.inv_tau);
+        v.z = channel_decay(v.z + bias[m].z, a.inv_tau); v.w = channel_decay(v.w + bias[m].w, a.inv_tau);
+      }
+      *(float4 *)(buf + 4 * e) = v;
+    }
+  };
+  fetch(0);
+  put(sm);
+  __syncthreads();
+  const bool out_vec = vec && p + 4 <= Dv;
+  int flip = 0;
+  for (int c0 = 0; c0 < len; c0 += TC, flip ^= 1) {
+    const float *cur = sm + flip * stage;
+    const bool more = c0 + TC < len;
+    if (more) fetch(c0 + TC);
+    const int cnt = len - c0 < TC ? len - c0 : TC;
+    for (int i = 0; i < cnt; ++i) {
+      const float *row = cur + i * rowlen;
+      const float4 v4 = *(const float4 *)(row + 3 * Dp + pc);
+      const float vv[4] = {v4.x, v4.y, v4.z, v4.w};
+      float o[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int j = 0; j < J; ++j) {
+        const int n = 4 * (j * R + r);
+        const float4 k4 = *(const float4 *)(row + n), a4 = *(const float4 *)(row + 2 * Dp + n);
+        float4 q4 = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (!LOCAL) q4 = *(const float4 *)(row + Dp + n);
+        const float kk[4] = {k4.x, k4.y, k4.z, k4.w}, aa[4] = {a4.x, a4.y, a4.z, a4.w}, qq[4] = {q4.x, q4.y, q4.z, q4.w};
+#pragma unroll
+        for (int i4 = 0; i4 < 4; ++i4) {
+          float *Sr = S[4 * j + i4];
+#pragma unroll
+          for (int c = 0; c < 4; ++c) {
+            Sr[c] = fmaf(aa[i4], Sr[c], kk[i4] * vv[c]);
+            if (!LOCAL) o[c] = fmaf(Sr[c], qq[i4], o[c]);
+          }
+          if (LOCAL) prod[LOCAL ? 4 * j + i4 : 0] *= aa[i4];
+        }
+      }
+      if (!LOCAL) {
+#pragma unroll
+        for (int c = 0; c < 4; ++c) o[c] = group_sum<R>(o[c]);
+        if (r == 0) {
+          float *op = a.out + (size_t)(r0 + c0 + i) * a.H * Dv + (size_t)h * Dv + p;
+          if (out_vec) *(float4 *)op = make_float4(o[0], o[1], o[2], o[3]);
+          else {
+#pragma unroll
+            for (int c = 0; c < 4; ++c)
+              if (p + c < Dv) op[c] = o[c];
+          }
+        }
+      }
+    }
+    if (more) put(sm + (flip ^ 1) * stage);
+    __syncthreads();
+  }
+  if (LOCAL) {
+    if (blockIdx.x == 0 && wave == 0 && pl == 0)
+#pragma unroll
+      for (int k = 0; k < K; ++k) {
+        const int n = 4 * ((k >> 2) * R + r) + (k & 3);
+        if (n < D) a.decay[((size_t)z * a.H + h) * D + n] = prod[LOCAL ? k : 0];
+      }
+    st = a.carry + ((size_t)z * a.H + h) * np;
+  }
+  if (LOCAL || last)
+#pragma unroll
+    for (int k = 0; k < K; ++k) {
+      const int n = 4 * ((k >> 2) * R + r) + (k & 3);
+      if (n >= D) continue;
+      float *d = st + (size_t)n * Dv + p;
+      if (out_vec) *(float4 *)d = make_float4(S[k][0], S[k][1], S[k][2], S[k][3]);
+      else {
+#pragma unroll
+        for (int c = 0; c < 4; ++c)
+          if (p + c < Dv) d[c] = S[k][c];
+      }
+    }
+}
+__global__ void __launch_bounds__(256) gla_carry_kernel(GlaArgs a) {
+  const int e = blockIdx.x * 256 + threadIdx.x, h = blockIdx.y, s = blockIdx.z;
+  const int np = a.D * a.Dv;
+  if (e >= np) return;
+  const int z0 = a.ent_seg0[s], z1 = a.ent_seg0[s + 1], n = e / a.Dv;
+  if (z1 - z0 < 2) return;
+  float cur = a.seq_pos0[s] > 0 ? a.state[((size_t)a.seq_slot[s] * a.H + h) * np + e] : 0.f;
+  for (int z = z0; z < z1 - 1; ++z) {
+    float *c = a.carry + ((size_t)z * a.H + h) * np + e;
+    cur = fmaf(a.decay[((size_t)z * a.H + h) * a.D + n], cur, *c);
+    *c = cur;
+  }
+}
+
+// Steps of single rows: one workgroup per (entry, head).  z = W_a2 a1 (a1: the row's `rank` values at a1_col of u, rounded to T as the product would read them), decays, then
+// thread (y, x) owns the columns 4 x .. 4 x + 3 (VP = 4) or x (VP = 1) of the state rows y, y + Y, ..: it updates them in place and adds up its part of the read-out; the parts
+// meet in LDS, the head is divided by its root mean square, multiplied by the weight `norm` [Dv] and by silu(gate).
+struct GlaStepArgs {
+  const float *u;           // [rows, ldu]: v | k | q | gate [H * Dv] at g_col | a1 [rank] at a1_col
+  const void *wa2;          // [H * D, rank] in T
+  const float *zb, *norm;
+  float *state;
+  const int *seq_start, *seq_pos0, *seq_slot;
+  void *out;                // [rows, H * Dv] in T
+  int ldu, k_col, q_col, g_col, a1_col, rank, H, D, Dv;
+  float q_mult, inv_tau, eps;
+};
+template <class T, int VP> __global__ void __launch_bounds__(1024) gla_step_kernel(GlaStepArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];  // k [Dq] | q [Dq] | decay [Dq] | a1 [rank padded] | o [Dv padded] | parts [Y][X * VP]
+  __shared__ float red[16];
+  const int s = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, nthr = blockDim.x, D = a.D, Dv = a.Dv, t = a.seq_start[s];
+  if (a.seq_start[s + 1] - t != 1) return;
+  const int Dq = (D + 3) & ~3, rp = (a.rank + 3) & ~3, vp = (Dv + 3) & ~3;
+  float *ks = sm, *qs = ks + Dq, *as = qs + Dq, *a1 = as + Dq, *os = a1 + rp, *parts = os + vp;
+  const float *ur = a.u + (size_t)t * a.ldu;
+  for (int j = tid; j < a.rank; j += nthr) a1[j] = round_to<T>(ur[a.a1_col + j]);
+  for (int n = tid; n < D; n += nthr) { ks[n] = ur[a.k_col + h * D + n]; qs[n] = ur[a.q_col + h * D + n] * a.q_mult; }
+  __syncthreads();
+  for (int n = tid; n < D; n += nthr) {
+    const T *w = (const T *)a.wa2 + (size_t)(h * D + n) * a.rank;
+    float z = 0.f;
+    for (int j = 0; j < a.rank; ++j) z = fmaf(a1[j], to_f<T>(w[j]), z);
+    as[n] = channel_decay(z + a.zb[h * D + n], a.inv_tau);
+  }
+  __syncthreads();
+  const bool carried = a.seq_pos0[s] > 0;
+  float *st = a.state + ((size_t)a.seq_slot[s] * a.H + h) * D * Dv;
+  const int cols = (Dv + VP - 1) / VP, X = cols < nthr ? cols : nthr, Y = nthr / X, x = tid % X, y = tid / X;
+  for (int cb = 0; cb < cols; cb += X) {
+    const int c = (cb + x) * VP;
+    float o[VP], v[VP];
+#pragma unroll
+    for (int j = 0; j < VP; ++j) o[j] = 0.f;
+    if (y < Y && cb + x < cols) {
+#pragma unroll
+      for (int j = 0; j < VP; ++j) v[j] = ur[h * Dv + c + j];
+#pragma unroll 4
+      for (int n = y; n < D; n += Y) {
+        float *sp = st + (size_t)n * Dv + c, S[VP];
+        if (VP == 4) {
+          const float4 s4 = carried ? *(const float4 *)sp : make_float4(0.f, 0.f, 0.f, 0.f);
+          S[0] = s4.x; S[VP > 1 ? 1 : 0] = s4.y; S[VP > 2 ? 2 : 0] = s4.z; S[VP > 3 ? 3 : 0] = s4.w;
+        } else {
+          S[0] = carried ? *sp : 0.f;
+        }
+        const float kn = ks[n], qn = qs[n], an = as[n];
+#pragma unroll
+        for (int j = 0; j < VP; ++j) {
+          S[j] = fmaf(an, S[j], kn * v[j]);
+          o[j] = fmaf(S[j], qn, o[j]);
+        }
+        if (VP == 4) *(float4 *)sp = make_float4(S[0], S[VP > 1 ? 1 : 0], S[VP > 2 ? 2 : 0], S[VP > 3 ? 3 : 0]);
+        else *sp = S[0];
+      }
+    }
+    __syncthreads();   // the previous column block's parts have been read
+    if (y < Y)
+#pragma unroll
+      for (int j = 0; j < VP; ++j) parts[(y * X + x) * VP + j] = o[j];
+    __syncthreads();
+    for (int e = tid; e < X * VP; e += nthr) {
+      if (cb * VP + e >= Dv) continue;
+      float sum = 0.f;
+      for (int q = 0; q < Y; ++q) sum += parts[q * X * VP + e];
+      os[cb * VP + e] = sum;
+    }
+  }
+  __syncthreads();
+  float ss = 0.f;
+  for (int d = tid; d < Dv; d += nthr) ss = fmaf(os[d], os[d], ss);
+  ss = wave_sum(ss);
+  if ((tid & 63) == 0) red[tid >> 6] = ss;
+  __syncthreads();
+  float tot = 0.f;
+  for (int w = 0; w < (nthr >> 6); ++w) tot += red[w];
+  const float inv = 1.0f / sqrtf(tot / (float)Dv + a.eps);
+  for (int d = tid; d < Dv; d += nthr) ((T *)a.out)[((size_t)t * a.H + h) * Dv + d] = from_f<T>(os[d] * inv * a.norm[d] * silu_f(ur[a.g_col + h * Dv + d]));
+}
+
+}  // namespace hybl
+}  // namespace mrs
+
+using namespace mrs::hybl;
+#define S_(s) ((hipStream_t)(s))
+
+extern "C" const char *mrs_hyb_linattn_last_error() { return g_err; }
+
+/* u [rows, ldu] = v [H * Dv] | ... with k [H * D] at k_col and q [H * D] at q_col; z [rows, ldz] decay logits [H * D], zb [H * D] their bias; alpha = sigmoid(z + zb)^inv_tau.
+ * Segment table as for the other scans; carry [segments, H, D, Dv] and decay [segments, H, D] are scratch, needed when segments > entries. */
+extern "C" int mrs_hyb_gla_scan(const float *u, int ldu, int k_col, int q_col, const float *z, int ldz, const float *zb, float *state, float *out, const int *seq_pos0,
+                                const int *seq_slot, const int *seg_entry, const int *seg_row0, const int *seg_len, const int *ent_seg0, float *carry, float *decay, int rows,
+                                int entries, int segments, int H, int D, int Dv, float q_mult, float inv_tau, void *stream) {
+  if (rows <= 0 || entries <= 0 || segments <= 0) return 0;
+  if (H <= 0 || D <= 0 || Dv <= 0 || D > 512) return fail("mrs_hyb_gla_scan: head sizes (key size 1 .. 512)");
+  if (entries > 65535 || segments > 65535 || H > 65535) return fail("mrs_hyb_gla_scan: more than 65535 entries, segments or heads");
+  if (k_col < H * Dv || q_col < H * Dv || ldu < k_col + H * D || ldu < q_col + H * D || ldz < H * D) return fail("mrs_hyb_gla_scan: rows shorter than v | k | q, or than the decay logits");
+  if (segments > entries && (!carry || !decay)) return fail("mrs_hyb_gla_scan: segmented entries need the carry scratch");
+  GlaArgs a{u, z, zb, state, out, seq_pos0, seq_slot, seg_entry, seg_row0, seg_len, ent_seg0, carry, decay, ldu, k_col, q_col, ldz, H, D, Dv, q_mult, inv_tau};
+  const int vec = (ldu % 4 == 0 && k_col % 4 == 0 && q_col % 4 == 0 && ldz % 4 == 0 && D % 4 == 0 && Dv % 4 == 0 && ((uintptr_t)u % 16) == 0 && ((uintptr_t)z % 16) == 0 &&
+                   ((uintptr_t)state % 16) == 0 && ((uintptr_t)out % 16) == 0 && ((uintptr_t)carry % 16) == 0) ? 1 : 0;
+  int R, J;
+  if (D <= 32) { R = 4; J = 2; } else if (D <= 64) { R = 8; J = 2; } else if (D <= 128) { R = 16; J = 2; } else if (D <= 256) { R = 16; J = 4; } else { R = 16; J = 8; }
+  const int Dp = 4 * R * J, CW = 64 / R * 4, all = (Dv + CW - 1) / CW;
+  // waves: a head's columns in workgroups of at most 16 waves (8 for the large register tiles), and enough of them that two rows fit a stage (4 groups of four values per thread)
+  const int most = J >= 4 ? 8 : 16;
+  int nblk = (all + most - 1) / most, nw = (all + nblk - 1) / nblk;
+  while (nw < most && 2 * (3 * Dp + nw * CW) / 4 > 4 * 64 * nw) ++nw;
+  const int U = (3 * Dp + nw * CW) / 4;
+  int TC = 4 * 64 * nw / U;
+  TC = TC > 16 ? 16 : TC;
+  while (TC > 1 && (size_t)2 * TC * U * 16 > 65536) --TC;
+  const size_t lds = (size_t)2 * TC * U * 16;
+  if (TC < 1 || lds > 65536) return fail("mrs_hyb_gla_scan: a row of operands does not fit the staging registers / 64 KB of LDS");
+  dim3 grid(nblk, H, segments), block(64 * nw);
+#define MRS_GLA__(R_, J_, L_, NT_) hipLaunchKernelGGL((gla_scan_kernel<R_, J_, L_, NT_>), grid, block, lds, S_(stream), a, TC, vec)
+#define MRS_GLA_(R_, J_, L_, MOST_) do { if (nw <= 4) MRS_GLA__(R_, J_, L_, 256); else if (nw <= 8) MRS_GLA__(R_, J_, L_, 512); else MRS_GLA__(R_, J_, L_, MOST_); } while (0)
+#define MRS_GLA(L_) do { if (D <= 32) MRS_GLA_(4, 2, L_, 1024); else if (D <= 64) MRS_GLA_(8, 2, L_, 1024); else if (D <= 128) MRS_GLA_(16, 2, L_, 1024); \
+                         else if (D <= 256) MRS_GLA_(16, 4, L_, 512); else MRS_GLA_(16, 8, L_, 512); } while (0)
+  if (segments > entries) {
+    MRS_GLA(true);
+    hipLaunchKernelGGL(gla_carry_kernel, dim3((unsigned)(((size_t)D * Dv + 255) / 256), H, entries), dim3(256), 0, S_(stream), a);
+  }
+  MRS_GLA(false);
+#undef MRS_GLA
+#undef MRS_GLA_
+#undef MRS_GLA__
+  return ok_or("mrs_hyb_gla_scan");
+}
+
+/* steps of single rows (rows == entries): u also holds the output gate [H * Dv] at g_col and the decay projection's first step [rank] at a1_col; wa2 [H * D, rank] (dtype);
+ * out (dtype) [rows, H * Dv] = o / rms(o) per head * norm [Dv] * silu(gate) */
+extern "C" int mrs_hyb_gla_step(const float *u, int ldu, int k_col, int q_col, int g_col, int a1_col, int rank, const void *wa2, const float *zb, const float *norm, float *state,
+                                void *out, const int *seq_start, const int *seq_pos0, const int *seq_slot, int rows, int entries, int H, int D, int Dv, float q_mult, float inv_tau,
+                                float eps, int dtype, void *stream) {
+  if (rows <= 0) return 0;
+  if (rows != entries || entries > 65535) return fail("mrs_hyb_gla_step: one row per entry");
+  if (H <= 0 || H > 65535 || D <= 0 || Dv <= 0 || rank <= 0) return fail("mrs_hyb_gla_step: head sizes / decay rank");
+  if (k_col < H * Dv || ldu < k_col + H * D || ldu < q_col + H * D || ldu < g_col + H * Dv || ldu < a1_col + rank) return fail("mrs_hyb_gla_step: rows shorter than their columns");
+  if (dtype != 1 && dtype != 2) return fail("mrs_hyb_gla_step: dtype");
+  const bool v4 = Dv % 4 == 0 && ((uintptr_t)state % 16) == 0;
+  const int VP = v4 ? 4 : 1, cols = Dv / VP;
+  // threads: at most eight state rows each where a head has that many, whole waves
+  long long want = (long long)cols * ((D + 7) / 8);
+  int nthr = want > 1024 ? 1024 : (int)((want + 63) / 64 * 64);
+  if (nthr < 64) nthr = 64;
+  const int X = cols < nthr ? cols : nthr, Y = nthr / X;
+  const size_t lds = (size_t)(3 * ((D + 3) & ~3) + ((rank + 3) & ~3) + ((Dv + 3) & ~3) + Y * X * VP) * 4;
+  if (lds > 65536 - 128) return fail("mrs_hyb_gla_step: the head does not fit 64 KB of LDS");
+  GlaStepArgs a{u, wa2, zb, norm, state, seq_start, seq_pos0, seq_slot, out, ldu, k_col, q_col, g_col, a1_col, rank, H, D, Dv, q_mult, inv_tau, eps};
+  dim3 grid(entries, H);
+#define MRS_GLAS(T) do { if (v4) hipLaunchKernelGGL((gla_step_kernel<T, 4>), grid, dim3(nthr), lds, S_(stream), a); else hipLaunchKernelGGL((gla_step_kernel<T, 1>), grid, dim3(nthr), lds, S_(stream), a); } while (0)
+  if (dtype == 1) MRS_GLAS(mrs::bf16_t);
+  else MRS_GLAS(float);
+#undef MRS_GLAS
+  return ok_or("mrs_hyb_gla_step");
+}

@@ -1,10 +1,10 @@
 """Layer-list ("hybrid") decoders served in their checkpoint dtype: every layer is `x += mixer(norm(x))` then optionally `x += feed_forward(norm(x))` (or both sublayers
 reading two norms of the same x: `parallel_sublayers`), the mixer being one of the registered kinds (`MIXERS`: state-space-duality recurrence, paged softmax attention with a
 sliding window / position chunks / kept first tokens / a learned sink, paged sigmoid attention with a distance bias and mixed head scores, sink attention with convolved
-projections, retention, latent attention, the gated delta rule, a matrix memory with exponential gates, two mixers side by side), the feed-forward one of `FEED_FORWARDS`
-(sigmoid-routed experts with a gated shared expert, softmax-routed clamped-GLU experts, routed squared-ReLU experts weighted over the chosen logits, dense xIELU and SiLU-GLU
-layers).  The norms are RMS norms (plain or one-plus weights) before every sublayer, or layer norms with bias before AND after every sublayer (`HybridSpec.norm`,
-`post_norms`).  The Gekilix, Sobunex, Setopel and Gifopel architectures (config.json `"architecture"`) are such lists.
+projections, retention, latent attention, the gated delta rule, gated linear attention, a matrix memory with exponential gates, two mixers side by side), the feed-forward one of
+`FEED_FORWARDS` (sigmoid-routed experts with a gated shared expert, softmax-routed clamped-GLU experts, routed squared-ReLU or GELU experts, dense xIELU, SiLU-GLU and GELU-GLU
+layers).  The norms are RMS norms (plain or one-plus weights) before every sublayer, layer norms with bias before AND after every sublayer (`HybridSpec.norm`, `post_norms`), or
+layer norms behind the sublayers only (`join_norms`).  The Gekilix, Sobunex, Setopel, Gifopel and Kebisun architectures (config.json `"architecture"`) are such lists.
 
 The step function is `HybridDecoder.forward_batch(batch)`: ONE ragged batch -- prompt portions of any length next to single decoded tokens -- through the HIP kernels of
 csrc/hyb_kernels.hip and csrc/hyb_gemm.hip (C ABI, this process's current stream; PyTorch owns buffers and the stream, nothing else).  What the sequences carry between
@@ -34,6 +34,7 @@ DTYPES = {"bfloat16": (1, torch.bfloat16), "float32": (2, torch.float32)}
 
 _SIGS = {
     "mrs_hyb_embed": [_vp, _vp, _vp, _i, _i, _i, _i, _vp],
+    "mrs_hyb_embed_scaled": [_vp] * 4 + [_i, _i, _i, _f, _i, _vp],
     "mrs_hyb_rmsnorm": [_vp, _i, _vp, _vp, _vp, _vp, _i, _i, _i, _f, _i, _i, _vp, _i, _i, _vp],
     "mrs_hyb_conv": [_vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp],
     "mrs_hyb_conv_qkv_cache": [_vp, _i] + [_vp] * 12 + [_i] * 8 + [_f, _i, _i, _vp],
@@ -74,12 +75,35 @@ _SIGS = {
     "mrs_hyb_norm_pair_add": [_vp, _i, _vp, _vp, _vp, _vp, _i, _i, _f, _f, _i, _vp],
     "mrs_hyb_round_cols": [_vp, _i, _vp, _i, _i, _i, _vp],
     "mrs_hyb_relu_sq": [_vp, _vp, _i, _i, _i, _vp],
+    "mrs_hyb_glu_gelu": [_vp, _vp, _i, _i, _i, _vp],
+    "mrs_hyb_gelu_erf": [_vp, _vp, _i, _i, _i, _vp],
+    "mrs_hyb_sigmoid_gate": [_vp, _vp, _i, _vp, _i, _i, _i, _vp],
+    "mrs_hyb_layernorm_join": [_vp, _i, _vp, _vp, _vp, _i, _vp, _vp, _vp, _i, _vp, _i, _i, _f, _i, _vp],
+    "mrs_hyb_paged_attn_sink_window": [_vp] * 7 + [_i] * 9 + [_f, _i, _vp, _vp, _vp, _i, _i, _f, _i, _vp, _vp, _i, _vp, _i, _i, _i, _vp],
+    "mrs_hyb_latent_prep": [_vp] + [_i] * 5 + [_vp, _vp, _vp, _f] + [_vp] * 4 + [_f, _i, _i, _vp],
+    "mrs_hyb_latent_query": [_vp] + [_i] * 6 + [_vp, _f, _vp, _vp, _vp, _i, _i, _vp],
+    "mrs_hyb_latent_context": [_vp] * 4 + [_i] * 7 + [_vp],
+    "mrs_hyb_gla_scan": [_vp, _i, _i, _i, _vp, _i] + [_vp] * 11 + [_i] * 6 + [_f, _f, _vp],
+    "mrs_hyb_gla_step": [_vp] + [_i] * 6 + [_vp] * 8 + [_i] * 5 + [_f, _f, _f, _i, _vp],
     "mrs_hyb_gemm": [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _l, _i, _vp],
     "mrs_hyb_gemv": [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _l, _i, _vp, _vp, _i, _vp],
     "mrs_hyb_gemv_act": [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _l, _i, _vp, _vp, _i, _vp, _f, _f, _vp],
 }
 _RECUR = {"mrs_hyb_rmsnorm_pair", "mrs_hyb_delta_prep", "mrs_hyb_delta_step_prep", "mrs_hyb_delta_scan", "mrs_hyb_exp_gates", "mrs_hyb_head_norm_gate", "mrs_hyb_norm_pair_add", "mrs_hyb_round_cols",
           "mrs_hyb_relu_sq"}   # launchers of csrc/hyb_recur.hip (their own error text)
+_LINATTN = {"mrs_hyb_gla_scan", "mrs_hyb_gla_step"}   # launchers of csrc/hyb_linattn.hip
+
+
+def _last_error(name: str) -> str:
+    if name in _RECUR:
+        return "mrs_hyb_recur_last_error"
+    if name in _LINATTN:
+        return "mrs_hyb_linattn_last_error"
+    if "gem" in name:
+        return "mrs_hyb_gemm_last_error"
+    return "mrs_hyb_talk_last_error" if "talk" in name else "mrs_hyb_last_error"
+
+
 _fns: dict = {}
 _step_stream: Optional[int] = None   # the stream handle of the step in progress (looked up once per forward_batch, not once per launch)
 
@@ -91,7 +115,7 @@ def _call(name: str, *args) -> None:
         fn = _fns[name] = _lib.sym("hybrid", name, _SIGS[name], C.c_int)
     conv = [a.data_ptr() if isinstance(a, torch.Tensor) else a for a in args]
     if fn(*conv, _step_stream if _step_stream is not None else torch.cuda.current_stream().cuda_stream) != 0:
-        err = _lib.sym("hybrid", "mrs_hyb_recur_last_error" if name in _RECUR else "mrs_hyb_gemm_last_error" if "gem" in name else ("mrs_hyb_talk_last_error" if "talk" in name else "mrs_hyb_last_error"), [], C.c_char_p)()
+        err = _lib.sym("hybrid", _last_error(name), [], C.c_char_p)()
         raise ValueError((err or b"").decode() or name)
 
 
@@ -120,7 +144,8 @@ class RaggedBatch:
     seg_rows: int = 0                          # rows of the longest segment (1: every entry brings one decoded token)
     host_blocks: Optional[List[Sequence[int]]] = None   # every entry's block ids covering its last position (host copy; `build` keeps it)
     host_lens: Optional[List[int]] = None               # rows of every entry (host copy; `build` keeps it)
-    _context: Optional[tuple] = None
+    host_pos0: Optional[List[int]] = None               # first position of every entry (host copy; `build` keeps it)
+    _context: Optional[dict] = None
     _entries: Optional[tuple] = None
     _long: Optional[dict] = None
 
@@ -156,21 +181,35 @@ class RaggedBatch:
             self._entries = (iota[:-1], self.seq_start[:-1], (self.seq_start[1:] - self.seq_start[:-1]).contiguous(), iota)
         return self._entries
 
-    def context_blocks(self):
-        """The blocks that hold the batch's whole contexts, renumbered densely: (tables i32 [entries, max_blocks] of dense ids, source i32 [n] = the pool block behind
-        dense block d, n).  A mixer that expands its cached rows for a prompt step (keys and values from latent rows) gathers the source blocks into a scratch and reads the
-        scratch through these tables."""
+    def context_blocks(self, window: int = 0, block_size: int = 0):
+        """The blocks that hold the batch's contexts, renumbered densely: (tables i32 [entries, max_blocks] of dense ids, source i32 [n] = the pool block behind dense block d,
+        n).  A mixer that expands its cached rows for a prompt step (keys and values from latent rows) gathers the source blocks into a scratch and reads the scratch
+        through these tables.  window > 0: blocks that lie wholly before an entry's first visible key (the window of its first row) are left out; their table entries are 0
+        and no kernel reads them."""
         if self._context is None:
+            self._context = {}
+        if window not in self._context:
             if self.host_blocks is None:
                 raise ValueError("RaggedBatch: this batch was not built from entries")
             tables = np.zeros((self.entries, self.max_blocks), dtype=np.int32)
             src: List[int] = []
             for s, blocks in enumerate(self.host_blocks):
-                tables[s, :len(blocks)] = np.arange(len(src), len(src) + len(blocks), dtype=np.int32)
-                src.extend(int(x) for x in blocks)
+                skip = max(0, self.host_pos0[s] - window + 1) // block_size if window > 0 else 0
+                kept = blocks[skip:]
+                tables[s, skip:skip + len(kept)] = np.arange(len(src), len(src) + len(kept), dtype=np.int32)
+                src.extend(int(x) for x in kept)
             dev = self.tokens.device
-            self._context = (torch.from_numpy(tables).to(dev), torch.tensor(src, dtype=torch.int32, device=dev), len(src))
-        return self._context
+            self._context[window] = (torch.from_numpy(tables).to(dev), torch.tensor(src, dtype=torch.int32, device=dev), len(src))
+        return self._context[window]
+
+    def visible_pairs(self, window: int = 0):
+        """(number of (row, visible key) pairs of the batch, number of context rows that hold those keys), with every earlier token visible or the last `window`."""
+        pairs = rows = 0
+        for n, p0 in zip(self.host_lens, self.host_pos0):
+            a = n if window <= 0 else min(n, max(0, window - p0))   # rows that still see everything before them
+            pairs += a * p0 + a * (a + 1) // 2 + (n - a) * window
+            rows += n + (p0 if window <= 0 else min(p0, window - 1))
+        return pairs, rows
 
     SEGMENT = int(os.environ.get("MRS_HYB_SEGMENT", "64"))   # rows per segment
 
@@ -228,15 +267,16 @@ class RaggedBatch:
             dv.append(dev_ints[o:o + n])
             o += n
         return RaggedBatch(T, S, mb, dv[0], dv[1], dv[2], dv[3], dv[4], dv[5], dv[6].view(S, mb), torch.from_numpy(slots).to(device),
-                           torch.tensor(want, dtype=torch.int32, device=device), nseg, dv[7], dv[8], dv[9], dv[10], max(1, min(L, max(lens, default=1))), host_blocks, lens)
+                           torch.tensor(want, dtype=torch.int32, device=device), nseg, dv[7], dv[8], dv[9], dv[10], max(1, min(L, max(lens, default=1))), host_blocks, lens, [int(e["pos0"]) for e in entries])
 
 
 # ------------------------------------------------------------------------------------------------------------------ layer descriptions
 @dataclass
 class RotarySpec:
-    """Rotary on the first `dims` dimensions of a head: a pair turns by position * f_i, f_i = base^(-2i / dims), optionally rescaled by wavelength (`scaling`: factor, low,
-    high, original -- wavelengths under original / high keep f, over original / low use f / factor, linear blend between).  `layout`: "interleaved" pairs (2i, 2i + 1) or
-    "half" pairs (i, i + dims / 2)."""
+    """Rotary on the first `dims` dimensions of a head: a pair turns by position * f_i, f_i = base^(-2i / dims), optionally rescaled (`scaling`): by wavelength (factor, low,
+    high, original -- wavelengths under original / high keep f, over original / low use f / factor, linear blend between), or by pair index (YaRN: factor, fast, slow,
+    original -- pairs that turn more than `fast` times over `original` positions keep f, fewer than `slow` times use f / factor, linear ramp over the index between; cos and
+    sin are then multiplied by `trig_mult`).  `layout`: "interleaved" pairs (2i, 2i + 1) or "half" pairs (i, i + dims / 2)."""
     dims: int
     base: float
     scaling: Optional[dict] = None
@@ -245,13 +285,23 @@ class RotarySpec:
     def frequencies(self) -> np.ndarray:
         i = np.arange(self.dims // 2, dtype=np.float64)
         f = np.float64(self.base) ** (-2.0 * i / self.dims)
-        if self.scaling:
+        if self.scaling and "fast" in self.scaling:
+            fac, fast, slow, orig = (float(self.scaling[k]) for k in ("factor", "fast", "slow", "original"))
+            index_of = lambda turns: self.dims * math.log(orig / (2.0 * math.pi * turns)) / (2.0 * math.log(self.base))   # where a pair makes that many turns
+            lo, hi = max(math.floor(index_of(fast)), 0), min(math.ceil(index_of(slow)), self.dims - 1)
+            ramp = np.clip((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+            f = f / fac * ramp + f * (1.0 - ramp)
+        elif self.scaling:
             fac, lo, hi, orig = (float(self.scaling[k]) for k in ("factor", "low", "high", "original"))
             wl = 2.0 * math.pi / f
             s = (orig / wl - lo) / (hi - lo)
             mid = (1.0 - s) * f / fac + s * f
             f = np.where(wl < orig / hi, f, np.where(wl > orig / lo, f / fac, mid))
         return f.astype(np.float32)
+
+    @property
+    def trig_mult(self) -> float:
+        return 0.1 * math.log(float(self.scaling["factor"])) + 1.0 if self.scaling and "fast" in self.scaling else 1.0
 
 
 @dataclass
@@ -351,6 +401,21 @@ class LatentAttentionSpec:
     vdim: int
     kv_rank: int
     scale: float
+    q_rank: int = 0            # > 0: queries come from a normed latent of this size (tensors dq, dq.norm, uq) instead of one projection
+    rot_dim: int = 0           # > 0: every head has that many more query dimensions, scored against ONE key part shared by the heads (further rows of dkv, cached behind the latent)
+    rotary: Optional[RotarySpec] = None   # rotation of the rot_dim parts (half-split pairs)
+    window: int = 0            # 0: every earlier token
+    sink: bool = False         # the softmax's denominator has one more term e^{sink_h}, a learned number per head (tensor `sink`)
+    gate: bool = False         # the concatenated heads are multiplied by sigmoid(Wg h) element by element (tensor `g` [heads * vdim, width])
+
+
+@dataclass
+class GlaSpec:
+    """Gated linear attention (GlaMixer): S <- diag(sigmoid(z)^(1 / tau)) S + k v^T, o = S^T q, one decay per head and key channel from the two-step projection `a1`, `a2`."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
 
 
 @dataclass
@@ -401,6 +466,20 @@ class TopkSoftmaxMoeSpec:
     ff: int
     shared_ff: int = 0
     kind = "moe_topk_softmax_relu2"
+    act = "relu2"
+    routing = "chosen"
+
+
+@dataclass
+class UngatedMoeSpec:
+    """Routed experts without gates, down(act(up h)) (UngatedMoe).  `act`: "gelu" (erf form) or "relu2".  `routing`: the weights are the chosen experts' scores of a softmax over
+    "all" logits, or of a softmax over the "chosen" ones (with a router bias)."""
+    experts: int
+    top: int
+    ff: int
+    act: str = "gelu"
+    routing: str = "all"
+    kind = "moe_ungated"
 
 
 @dataclass
@@ -412,8 +491,9 @@ class DenseSpec:
 
 @dataclass
 class GluSpec:
-    """down(silu(gate h) * (up h)) (GluFeedForward)."""
+    """down(act(gate h) * (up h)) (GluFeedForward); `act`: "silu" or "gelu_tanh"."""
     ff: int
+    act: str = "silu"
     kind = "dense_glu_silu"
 
 
@@ -435,11 +515,14 @@ class HybridSpec:
     embed: str = "embed"
     final_norm: str = "final.norm"
     head: str = "head"
-    norm: str = "rms_one_plus"   # "rms_one_plus": x / rms * (1 + w);  "rms": x / rms * w;  "layer": (x - mean) / sqrt(var + eps) * w + b, the bias being the tensor `<name>.b`
+    norm: str = "rms_one_plus"   # "rms_one_plus": x / rms * (1 + w);  "rms": x / rms * w;  "layer": (x - mean) / sqrt(var + eps) * w + b, the bias being the tensor `<name>.b`;  "layer_plain": without the bias
     parallel_sublayers: bool = False   # x += mixer(norm1(x)) + feed_forward(norm2(x)), both norms of the same x (else one sublayer after the other)
     post_norms: bool = False     # every sublayer's output is normed (`norm1b` / `norm2b`) before it joins the residual stream
     embed_norm: Optional[str] = None   # tensor of a norm (of the model's kind) applied to the embedding rows
     residual_mult: float = 1.0   # every sublayer's output is multiplied by this before it joins the residual stream(s)
+    join_norms: bool = False     # sublayers read the residual row as it is; their outputs are normed (`norm1` / `norm2`) on the way into it: x += norm(sublayer(x))
+    layer_scale: bool = False    # a sublayer's (normed) output is multiplied element by element by the tensors `ls1` / `ls2`
+    embed_scale: float = 1.0     # the embedding rows are multiplied by this
     streams: int = 0             # > 0: that many residual streams with per-sublayer read / write / mixing weights (`hc1.*` / `hc2.*`: in [S], out [S], mix [S, S] from -> to)
 
 
@@ -592,10 +675,43 @@ def gifopel_spec(cfg: dict) -> HybridSpec:
     return HybridSpec(int(cfg["vocab"]), int(cfg["width"]), float(cfg["norm"]["eps"]), layers, head="embed", norm="rms", parallel_sublayers=True)
 
 
+def kebisun_spec(cfg: dict) -> HybridSpec:
+    """config.json of a Kebisun checkpoint -> the layer list: a scaled embedding, sublayers that read the residual row itself and join it through a layer norm (no bias) and a
+    per-channel scale, mixers `gla` (gated linear attention) and `latent_attention` (query latent, shared rotated key part, sliding window, learned sink, output gate), dense
+    GELU-GLU or routed GELU feed-forwards.  Every size and every model-dependent constant comes from the file; a key that is absent switches its mechanism off."""
+    layers = []
+    for i, L in enumerate(cfg["layers"]):
+        m, kind = L["mixer"], L["type"]
+        if kind == "gla":
+            mixer = GlaSpec(int(m["heads"]), int(m["dim"]), int(m["vdim"]), float(m["tau"]))
+        elif kind == "latent_attention":
+            rot, mask, rot_dim = m.get("rot") or {}, m.get("mask") or {}, int(m.get("rot_dim", 0) or 0)
+            dims = int(rot.get("dims", 0) or 0)
+            if dims > rot_dim or dims % 2:
+                raise ValueError(f"Kebisun: layer {i} rotates {dims} of {rot_dim} dimensions")
+            mixer = LatentAttentionSpec(int(m["heads"]), int(m["dim"]), int(m["vdim"]), int(m["kv_rank"]), float(m["scale"]), int(m.get("q_rank", 0) or 0), rot_dim,
+                                        RotarySpec(dims, float(rot["base"]), rot.get("scaling"), "half") if dims else None, int(mask.get("size", 0) or 0), True, True)
+        else:
+            raise ValueError(f"Kebisun: unknown layer type {kind!r}")
+        f = L.get("mlp")
+        ff = None
+        if f:
+            if f.get("kind") == "dense":
+                ff = GluSpec(int(f["ff"]), "gelu_tanh")
+            elif f.get("kind") == "moe":
+                ff = UngatedMoeSpec(int(f["router"]["experts"]), int(f["router"]["top"]), int(f["expert"]["ff"]), "gelu", "all")
+            else:
+                raise ValueError(f"Kebisun: unknown feed-forward kind {f.get('kind')!r}")
+        layers.append(LayerSpec(kind, mixer, ff, f"l{i}."))
+    return HybridSpec(int(cfg["vocab"]), int(cfg["width"]), float(cfg["norm"]["eps"]), layers, norm="layer_plain", join_norms=True, layer_scale=True,
+                      embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)))
+
+
 # ------------------------------------------------------------------------------------------------------------------ mixers and feed-forwards
 class _Module:
     out_bias = None            # f32 bias of the module's last product, left to the caller (a norm that follows adds it while it reads the product)
     wants_f32_input = False    # feed-forwards: the normed rows are needed in f32 too (routers)
+    defers_combine = False     # feed-forwards: `forward(defer=True)` returns routed outputs for the next launch to sum instead of summing them
 
     def __init__(self, model: "HybridDecoder"):
         self.m = model
@@ -1066,82 +1182,209 @@ class RetentionMixer(_Module):
 class LatentAttention(_Module):
     """q | latent in one product; the latent row c = norm(W_dkv h) (plain weight) is the only thing paged.  Head h's keys W_uk,h c and values W_uv,h c are never
     materialised: q'_h = W_uk,h^T q_h scores against the cached rows (one shared key / value head of kv_rank dimensions for all query heads), the weighted sum of cached
-    rows is expanded by W_uv,h afterwards -- the same sums, reassociated.  Causal softmax, s = scale (q . k); no positions."""
+    rows is expanded by W_uv,h afterwards -- the same sums, reassociated.  Causal softmax, s = scale (q . k); no positions.
+
+    Options: queries from a normed latent of their own (q_rank: q = W_uq norm(W_dq h)); rot_dim further dimensions per query head scored against one rotated key part that all
+    heads share (the last rows of W_dkv, not normed, cached behind the latent: a page row is [latent | key part]); a sliding window; a learned sink per head; sigmoid(W_g h) on
+    the concatenated heads."""
 
     def __init__(self, model, spec: LatentAttentionSpec, prefix: str):
         super().__init__(model)
         self.s, self.p = spec, prefix
-        self.c_cache = torch.zeros(model.num_blocks, 1, model.block_size, spec.kv_rank, dtype=model.torch_dtype, device=model.device)
+        if spec.rotary and (spec.rotary.layout != "half" or spec.rotary.dims > spec.rot_dim):
+            raise ValueError(f"{prefix}: latent attention rotates half-split pairs inside rot_dim")
+        self.row = spec.kv_rank + spec.rot_dim
+        self.c_cache = torch.zeros(model.num_blocks, 1, model.block_size, self.row, dtype=model.torch_dtype, device=model.device)
+        self.freq = torch.from_numpy(spec.rotary.frequencies()).to(model.device) if spec.rotary else None
+        self.dims, self.trig_mult = (spec.rotary.dims, float(np.float32(spec.rotary.trig_mult))) if spec.rotary else (0, 1.0)
+        self.plain = not (spec.q_rank or spec.rot_dim)   # the query is one product and the row is the latent alone
 
     def carried(self):
         return (self.c_cache,)
 
     def kv_bytes_per_token(self) -> int:
-        return self.c_cache.element_size() * self.s.kv_rank
+        return self.c_cache.element_size() * self.row
 
     def load(self, get):
         s, p, W = self.s, self.p, self.m.spec.width
         dev, dt = self.m.device, self.m.torch_dtype
-        q, dkv, uk, uv = (get(p + n) for n in ("q", "dkv", "uk", "uv"))
-        if tuple(q.shape) != (s.heads * s.dim, W) or tuple(dkv.shape) != (s.kv_rank, W) or tuple(uk.shape) != (s.heads * s.dim, s.kv_rank) or \
-                tuple(uv.shape) != (s.heads * s.vdim, s.kv_rank):
+        H, D, Dr, Dv, R = s.heads, s.dim, s.rot_dim, s.vdim, s.kv_rank
+        q, dkv, uk, uv = (get(p + n) for n in ("dq" if s.q_rank else "q", "dkv", "uk", "uv"))
+        if tuple(q.shape) != (s.q_rank or H * (D + Dr), W) or tuple(dkv.shape) != (R + Dr, W) or tuple(uk.shape) != (H * D, R) or tuple(uv.shape) != (H * Dv, R):
             raise ValueError(f"{p}: projection shapes do not match the mixer's sizes")
-        self.w_in = torch.cat([q, dkv], 0).to(dev, dt).contiguous()                                       # [q | latent, W]
-        self.w_ukT = uk.reshape(s.heads, s.dim, s.kv_rank).transpose(1, 2).to(dev, dt).contiguous()       # [H, kv_rank, dim]: q' = this . q
-        self.w_uv = uv.reshape(s.heads, s.vdim, s.kv_rank).to(dev, dt).contiguous()                       # [H, vdim, kv_rank]
+        parts = [q, dkv]
+        if s.gate:
+            parts.append(get(p + "g"))
+            if tuple(parts[-1].shape) != (H * Dv, W):
+                raise ValueError(f"{p}: the gate projection has one row per output value")
+        self.w_in = torch.cat(parts, 0).to(dev, dt).contiguous()                                          # [q (query latent) | latent | key part | gate, W]
+        self.gate_col = q.shape[0] + R + Dr
+        self.w_uq = self.q_norm = None
+        if s.q_rank:
+            self.w_uq, self.q_norm = self.w(get, p + "uq", True), self.w(get, p + "dq.norm", False).reshape(-1)
+            if tuple(self.w_uq.shape) != (H * (D + Dr), s.q_rank) or self.q_norm.numel() != s.q_rank:
+                raise ValueError(f"{p}: query latent shapes do not match the mixer's sizes")
+        self.w_ukT = uk.reshape(H, D, R).transpose(1, 2).to(dev, dt).contiguous()                         # [H, kv_rank, dim]: q' = this . q
+        self.w_uv = uv.reshape(H, Dv, R).to(dev, dt).contiguous()                                         # [H, vdim, kv_rank]
         self.w_uk = uk.to(dev, dt).contiguous()                                                           # [H * dim, kv_rank]: the keys themselves (prompt steps)
         self.c_norm = self.w(get, p + "dkv.norm", False)
+        self.sink = self.w(get, p + "sink", False).reshape(-1) if s.sink else None
         self.w_o = self.w(get, p + "o", True)
-        if self.c_norm.numel() != s.kv_rank or tuple(self.w_o.shape) != (W, s.heads * s.vdim):
-            raise ValueError(f"{p}: norm / output shapes do not match the mixer's sizes")
+        if self.c_norm.numel() != R or tuple(self.w_o.shape) != (W, H * Dv) or (s.sink and self.sink.numel() != H):
+            raise ValueError(f"{p}: norm / sink / output shapes do not match the mixer's sizes")
+
+    def queries(self, u, b: RaggedBatch, absorbed: bool):
+        """The batch's latent rows into their pages and its queries: q [T, H * (dim + rot_dim)], or (absorbed) qa [T, H * (kv_rank + rot_dim)] ready for the cached rows."""
+        s, m, T = self.s, self.m, b.rows
+        H, D, Dr, R = s.heads, s.dim, s.rot_dim, s.kv_rank
+        dt, dev = m.torch_dtype, m.device
+        q = torch.empty(T, H * (D + Dr), dtype=dt, device=dev)
+        qa = torch.empty(T, H * (R + Dr), dtype=dt, device=dev) if absorbed else None
+        if self.plain:
+            _call("mrs_hyb_latent_norm_cache", u, u.stride(0), H * D, R, self.c_norm, b.slot_mapping, q, self.c_cache, m.spec.eps, T, m.dt)
+        else:
+            cq = torch.empty(T, s.q_rank, dtype=dt, device=dev) if s.q_rank else None
+            c_col = 0 if s.q_rank else H * (D + Dr)
+            _call("mrs_hyb_latent_prep", u[:, c_col:], u.stride(0), s.q_rank, R, Dr, self.dims, self.q_norm, self.c_norm, self.freq, self.trig_mult, b.tok_pos, b.slot_mapping, cq,
+                  self.c_cache, m.spec.eps, T, m.dt)
+            qf = m.linear(cq, self.w_uq) if s.q_rank else u
+            _call("mrs_hyb_latent_query", qf, qf.stride(0), H, D, R, Dr, self.dims, self.freq, self.trig_mult, b.tok_pos, q, qa, T, m.dt)
+        if absorbed:
+            m.batched_linear(q, self.w_ukT, H, a_block=D + Dr, out=qa, c_block=R + Dr)
+        return qa if absorbed else q
 
     def forward(self, h, x, b: RaggedBatch, accumulate: bool = True):
         s, m = self.s, self.m
         T, dev, dt = b.rows, m.device, m.torch_dtype
-        H, D, Dv, R = s.heads, s.dim, s.vdim, s.kv_rank
-        u = m.linear(h, self.w_in)                                         # f32 [T, q | latent]
-        q = torch.empty(T, H * D, dtype=dt, device=dev)
-        _call("mrs_hyb_latent_norm_cache", u, u.stride(0), H * D, R, self.c_norm, b.slot_mapping, q, self.c_cache, m.spec.eps, T, m.dt)
+        H, D, Dr, Dv, R = s.heads, s.dim, s.rot_dim, s.vdim, s.kv_rank
+        u = m.linear(h, self.w_in)                                         # f32 [T, q (query latent) | latent | key part | gate logits]
+        gate, ldg = (u[:, self.gate_col:], u.stride(0)) if s.gate else (None, 0)
+        seg = (b.seg_entry, b.seg_row0, b.seg_len, b.segments, RaggedBatch.SEGMENT)
         if self.expands(b):
-            # a step with prompt portions: the contexts' latent rows are gathered block by block and expanded into keys and values of `dim` / `vdim` per head (two products
-            # on the matrix cores); attention then costs dim + vdim per (query, key) pair instead of 2 kv_rank
-            tables, source, n = b.context_blocks()
+            # a step with prompt portions: the contexts' latent rows are gathered block by block and expanded into keys and values of `dim` (+ rot_dim) / `vdim` per head (two
+            # products on the matrix cores); attention then costs dim + rot_dim + vdim per (query, key) pair instead of 2 kv_rank + rot_dim
+            q = self.queries(u, b, False)
             bs = m.block_size
-            per = bs * R * self.c_cache.element_size() // 4
+            tables, source, n = b.context_blocks(s.window, bs)
             c = torch.empty(n * bs, R, dtype=dt, device=dev)
-            _call("mrs_hyb_gather_rows", self.c_cache, source, c, n, per)
-            k = m.linear_rounded(c, self.w_uk)                              # [n * bs, H * dim]: block, slot, head -- the attention kernel's token-major layout
+            if Dr:
+                k = torch.empty(n * bs, H * (D + Dr), dtype=dt, device=dev)
+                _call("mrs_hyb_latent_context", self.c_cache, source, c, k, n, bs, R, Dr, H, D, m.dt)
+                m.batched_linear(c, self.w_uk.view(H, D, R), H, a_block=0, out=k, c_block=D + Dr)
+            else:
+                _call("mrs_hyb_gather_rows", self.c_cache, source, c, n, bs * R * self.c_cache.element_size() // 4)
+                k = m.linear_rounded(c, self.w_uk)                          # [n * bs, H * dim]: block, slot, head -- the attention kernel's token-major layout
             v = m.linear_rounded(c, self.w_uv.view(H * Dv, R))
             ov = torch.empty(T, H * Dv, dtype=dt, device=dev)
-            _call("mrs_hyb_paged_attn_opts", q, k, v, tables, b.tok_seq, b.tok_pos, ov, T, H, H, D, Dv, bs, b.max_blocks, 0, 0, s.scale, m.dt, b.seg_entry, b.seg_row0, b.seg_len,
-                  b.segments, RaggedBatch.SEGMENT, 0.0, 0, None, 0, None, 0, 1)
-        else:
-            qa = m.batched_linear(q, self.w_ukT, H)                        # [T, H * kv_rank] in the serving dtype
-            oa = torch.empty(T, H * R, dtype=dt, device=dev)
-            _call("mrs_hyb_paged_attn_opts", qa, self.c_cache, self.c_cache, b.block_tables, b.tok_seq, b.tok_pos, oa, T, H, 1, R, R, m.block_size, b.max_blocks, 0, 0, s.scale,
-                  m.dt, b.seg_entry, b.seg_row0, b.seg_len, b.segments, RaggedBatch.SEGMENT, 0.0, 0, None, 0, *m.key_splits(b, H, R), 0)
-            ov = m.batched_linear(oa, self.w_uv, H)                        # [T, H * vdim]
-        m.linear(ov, self.w_o, out=x, accumulate=accumulate)
+            _call("mrs_hyb_paged_attn_sink_window", q, k, v, tables, b.tok_seq, b.tok_pos, ov, T, H, H, D + Dr, Dv, bs, b.max_blocks, s.window, 0, s.scale, m.dt, *seg, 0.0,
+                  int(s.sink), self.sink, gate, ldg, None, 0, 1, 0)
+            m.linear(ov, self.w_o, out=x, accumulate=accumulate)
+            return
+        qa = self.queries(u, b, True)                                      # [T, H * (kv_rank + rot_dim)] in the serving dtype
+        oa = torch.empty(T, H * R, dtype=dt, device=dev)
+        _call("mrs_hyb_paged_attn_sink_window", qa, self.c_cache, self.c_cache, b.block_tables, b.tok_seq, b.tok_pos, oa, T, H, 1, self.row, R, m.block_size, b.max_blocks, s.window, 0,
+              s.scale, m.dt, *seg, 0.0, int(s.sink), self.sink, None, 0, *m.key_splits(b, H, R, s.window), 0, self.row)
+        if not s.gate:
+            m.linear(m.batched_linear(oa, self.w_uv, H), self.w_o, out=x, accumulate=accumulate)
+            return
+        ov = m.batched_linear(oa, self.w_uv, H, f32=True)                  # [T, H * vdim]
+        if T <= m.GEMV_ROWS:   # decode-sized steps: the gate in the output product's operand load
+            m.gemv_act(ov, self.w_o, x, T, x.shape[1], H * Dv, H * Dv, H * Dv, None, 0, 8, src_div=ldg, bias=gate, accumulate=accumulate)
+            return
+        og = torch.empty(T, H * Dv, dtype=dt, device=dev)
+        _call("mrs_hyb_sigmoid_gate", ov, gate, ldg, og, T, H * Dv, m.dt)
+        m.linear(og, self.w_o, out=x, accumulate=accumulate)
 
     MATRIX_TO_VECTOR_RATE = 6.0   # products on the matrix cores against attention arithmetic on the vector ALU, per operation
 
     def expands(self, b: RaggedBatch) -> bool:
-        """Whether this step materialises keys and values.  Reading latent rows directly costs 2 kv_rank multiply-adds per (query, key) pair and head, expanded ones dim + vdim
-        plus the expansion of every context row (kv_rank (dim + vdim) per head, on the matrix cores).  With about rows / 2 queries per context row the expansion pays from
-        rows > 2 kv_rank (dim + vdim) / (rate (2 kv_rank - dim - vdim)) on; steps of single rows never expand."""
+        """Whether this step materialises keys and values.  Reading latent rows directly costs 2 kv_rank (+ rot_dim) multiply-adds per (query, key) pair and head, expanded ones
+        dim + vdim (+ rot_dim) plus the expansion of every context row (kv_rank (dim + vdim) per head, on the matrix cores): it pays from
+        pairs / context rows > kv_rank (dim + vdim) / (rate (2 kv_rank - dim - vdim)) on; steps of single rows never expand."""
         s = self.s
         gain = 2 * s.kv_rank - s.dim - s.vdim
-        if b.seg_rows <= 1 or b.host_blocks is None or gain <= 0 or (self.m.block_size * s.kv_rank * self.c_cache.element_size()) % 4:
+        if b.seg_rows <= 1 or b.host_blocks is None or gain <= 0 or (not s.rot_dim and (self.m.block_size * s.kv_rank * self.c_cache.element_size()) % 4):
             return False
-        return b.rows * self.MATRIX_TO_VECTOR_RATE * gain > 2 * s.kv_rank * (s.dim + s.vdim)
+        pairs, rows = b.visible_pairs(s.window)
+        return pairs * self.MATRIX_TO_VECTOR_RATE * gain > rows * s.kv_rank * (s.dim + s.vdim)
+
+
+class GlaMixer(_Module):
+    """v | k | q | gate | the decay projection's first step in one product; z = W_a2 (first step, rounded once) + bias, one logit per head and key channel;
+    alpha = sigmoid(z)^(1 / tau); q times dim^(-1/2).  Per head the f32 state S [dim, vdim] (carried per slot): S <- diag(alpha) S + k v^T, o = S^T q; o / rms(o) per head times
+    the weight `norm` [vdim] times silu(gate), output projection.  Long portions run their segments side by side (csrc/hyb_linattn.hip)."""
+
+    SCAN_WAVES = int(os.environ.get("MRS_GLA_WAVES", "4096"))   # waves per pass that a scan aims at: enough segments for that, no more (each costs dim x vdim of carry)
+
+    def __init__(self, model, spec: GlaSpec, prefix: str):
+        super().__init__(model)
+        self.s, self.p = spec, prefix
+        self.state = torch.zeros(model.state_slots, spec.heads, spec.dim, spec.vdim, dtype=torch.float32, device=model.device)
+        self.q_mult, self.inv_tau = float(np.float32(spec.dim) ** np.float32(-0.5)), float(np.float32(1.0) / np.float32(spec.tau))
+
+    def carried(self):
+        return (self.state,)
+
+    def state_bytes_per_slot(self) -> int:
+        return 4 * self.state[0].numel()
+
+    def load(self, get):
+        s, p, W = self.s, self.p, self.m.spec.width
+        nv, nk = s.heads * s.vdim, s.heads * s.dim
+        parts = [get(p + n) for n in ("v", "k", "q", "g", "a1")]
+        self.rank = parts[4].shape[0]
+        if [t.shape[0] for t in parts[:4]] != [nv, nk, nk, nv] or any(t.shape[1] != W for t in parts):
+            raise ValueError(f"{p}: projection shapes do not match the mixer's sizes")
+        self.w_in = torch.cat(parts, 0).to(self.m.device, self.m.torch_dtype).contiguous()     # [v | k | q | gate | a1, W]
+        self.k_col, self.q_col, self.g_col, self.a_col = nv, nv + nk, nv + 2 * nk, 2 * nv + 2 * nk
+        self.w_a2, self.w_o = self.w(get, p + "a2", True), self.w(get, p + "o", True)
+        self.b_a, self.norm = self.w(get, p + "a2.b", False).reshape(-1), self.w(get, p + "norm", False).reshape(-1)
+        if tuple(self.w_a2.shape) != (nk, self.rank) or self.b_a.numel() != nk or self.norm.numel() != s.vdim or tuple(self.w_o.shape) != (W, nv):
+            raise ValueError(f"{p}: decay / norm / output shapes do not match the mixer's sizes")
+
+    def segments(self, b: RaggedBatch):
+        """(segment table, segments) of this step's scan: one chain per entry when the entries fill the chip, else segments of 64 .. 512 rows, as short as SCAN_WAVES asks for"""
+        s = self.s
+        columns = 64 if s.dim <= 32 else 32 if s.dim <= 64 else 16                             # value columns per wave of the scan
+        per = s.heads * -(-s.vdim // columns)
+        if b.host_lens is None or b.seg_rows <= 1 or b.entries * per >= self.SCAN_WAVES:
+            return b.entry_table(), b.entries
+        rows = 64
+        while rows < 512 and per * sum(-(-n // rows) for n in b.host_lens) > self.SCAN_WAVES:
+            rows *= 2
+        *table, n = b.segment_table(rows)
+        return table, n
+
+    def forward(self, h, x, b: RaggedBatch, accumulate: bool = True):
+        s, m = self.s, self.m
+        T, dev = b.rows, m.device
+        f32 = dict(dtype=torch.float32, device=dev)
+        nv = s.heads * s.vdim
+        u = m.linear(h, self.w_in)                                          # f32 [T, v | k | q | gate | a1]
+        o = torch.empty(T, nv, dtype=m.torch_dtype, device=dev)
+        if T == b.entries and b.seg_rows == 1:   # every entry brings one row: decays, state, read-out, head norm and gate in one launch
+            _call("mrs_hyb_gla_step", u, u.stride(0), self.k_col, self.q_col, self.g_col, self.a_col, self.rank, self.w_a2, self.b_a, self.norm, self.state, o, b.seq_start,
+                  b.seq_pos0, b.seq_slot, T, b.entries, s.heads, s.dim, s.vdim, self.q_mult, self.inv_tau, m.spec.eps, m.dt)
+        else:
+            z = m.linear(m.round_cols(u[:, self.a_col:], self.rank), self.w_a2)
+            table, nseg = self.segments(b)
+            y, carry, decay = torch.empty(T, nv, **f32), None, None
+            if nseg > b.entries:
+                carry, decay = torch.empty(nseg, s.heads, s.dim, s.vdim, **f32), torch.empty(nseg, s.heads, s.dim, **f32)
+            _call("mrs_hyb_gla_scan", u, u.stride(0), self.k_col, self.q_col, z, z.stride(0), self.b_a, self.state, y, b.seq_pos0, b.seq_slot, *table, carry, decay, T, b.entries, nseg,
+                  s.heads, s.dim, s.vdim, self.q_mult, self.inv_tau)
+            _call("mrs_hyb_head_norm_gate", y, s.vdim, None, self.norm, 0, u[:, self.g_col:], u.stride(0), 2, o, T, s.heads, s.vdim, m.spec.eps, m.dt)
+        m.linear(o, self.w_o, out=x, accumulate=accumulate)
 
 
 class GluFeedForward(_Module):
-    """down(silu(gate h) * (up h)), no biases; gate | up are one product."""
+    """down(act(gate h) * (up h)), no biases; gate | up are one product.  act: SiLU or the tanh form of GELU."""
+    ACTS = {"silu": (1, "mrs_hyb_glu_silu"), "gelu_tanh": (6, "mrs_hyb_glu_gelu")}   # operand mode of the row kernel, the launch between prompt-sized products
 
     def __init__(self, model, spec: GluSpec, prefix: str):
         super().__init__(model)
         self.s, self.p = spec, prefix
+        self.in_mode, self.act = self.ACTS[spec.act]
 
     def load(self, get):
         s, p, W = self.s, self.p, self.m.spec.width
@@ -1156,10 +1399,10 @@ class GluFeedForward(_Module):
         T = b.rows
         gu = m.linear(h, self.w_gu)
         if T <= m.GEMV_ROWS:   # decode-sized steps: the GLU in the down product's operand load
-            _call("mrs_hyb_gemv", gu, self.w_down, x, T, x.shape[1], s.ff, 2 * s.ff, s.ff, x.stride(0), m.dt, int(accumulate), None, 0, 1, None, None, 1)
+            m.gemv_act(gu, self.w_down, x, T, x.shape[1], s.ff, 2 * s.ff, s.ff, None, 0, self.in_mode, accumulate=accumulate)
             return
         a = torch.empty(T, s.ff, dtype=m.torch_dtype, device=m.device)
-        _call("mrs_hyb_glu_silu", gu, a, T, s.ff, m.dt)
+        _call(self.act, gu, a, T, s.ff, m.dt)
         m.linear(a, self.w_down, out=x, accumulate=accumulate)
 
 
@@ -1357,55 +1600,67 @@ class ParallelMixer(_Module):
         _call("mrs_hyb_norm_pair_add", x, x.stride(0), yl, self.w_left, yr, self.w_right, b.rows, m.spec.width, m.spec.eps, 0.5, int(accumulate))
 
 
-class TopkSoftmaxReluSqMoe(_Module):
-    """Router logits (weight and bias) in f32; the `top` largest are chosen, their weights are the softmax over the chosen logits only, applied to the experts' OUTPUTS.
-    Expert (no biases, no gate): down(max(up h, 0)^2).  All experts of a step run as grouped products over expert-sorted rows."""
+class UngatedMoe(_Module):
+    """Router logits in f32; the `top` largest are chosen.  Weights (on the experts' OUTPUTS): the softmax over the chosen logits only (routing "chosen", the router has a bias), or
+    the chosen scores of the softmax over all of them, un-renormalised ("all").  Expert (no biases, no gate): down(act(up h)), act = max(., 0)^2 or the erf form of GELU.  All
+    experts of a step run as grouped products over expert-sorted rows."""
     wants_f32_input = True
+    ACTS = {"relu2": (5, "mrs_hyb_relu_sq"), "gelu": (7, "mrs_hyb_gelu_erf")}   # operand mode of the row kernel, the launch between prompt-sized products
+    defers_combine = True   # `forward(defer=True)` hands the weighted sum to the launch that norms it into the stream
 
-    def __init__(self, model, spec: TopkSoftmaxMoeSpec, prefix: str):
+    def __init__(self, model, spec, prefix: str):
         super().__init__(model)
         self.s, self.p = spec, prefix
+        self.in_mode, self.act = self.ACTS[spec.act]
+        if spec.routing not in ("all", "chosen"):
+            raise ValueError(f"{prefix}: routing all | chosen")
 
     def load(self, get):
         s, p, m = self.s, self.p, self.m
         dev, dt = m.device, m.torch_dtype
         self.w_up = torch.stack([get(f"{p}e{e}.up") for e in range(s.experts)]).to(dev, dt).contiguous()       # [E, ff, W]
         self.w_down = torch.stack([get(f"{p}e{e}.down") for e in range(s.experts)]).to(dev, dt).contiguous()   # [E, W, ff]
-        self.w_router, self.b_router = self.w(get, p + "router", False), self.w(get, p + "router.b", False).reshape(-1)
+        self.w_router = self.w(get, p + "router", False)
+        self.b_router = self.w(get, p + "router.b", False).reshape(-1) if s.routing == "chosen" else None
         if tuple(self.w_up.shape[1:]) != (s.ff, m.spec.width) or tuple(self.w_down.shape[1:]) != (m.spec.width, s.ff) or \
-                tuple(self.w_router.shape) != (s.experts, m.spec.width) or self.b_router.numel() != s.experts:
+                tuple(self.w_router.shape) != (s.experts, m.spec.width) or (self.b_router is not None and self.b_router.numel() != s.experts):
             raise ValueError(f"{p}: expert / router shapes do not match the layer's sizes")
 
-    def forward(self, h, h32, x, b: RaggedBatch, accumulate: bool = True):
+    def forward(self, h, h32, x, b: RaggedBatch, accumulate: bool = True, defer: bool = False):
         s, m = self.s, self.m
         T, W, dev = b.rows, m.spec.width, m.device
         R = T * s.top
         ids = torch.empty(R, dtype=torch.int32, device=dev)
         wts = torch.empty(R, dtype=torch.float32, device=dev)
-        _call("mrs_hyb_route_topk_softmax", h32, self.w_router, self.b_router, T, W, s.experts, s.top, 1.0, ids, wts)
+        if s.routing == "chosen":
+            _call("mrs_hyb_route_topk_softmax", h32, self.w_router, self.b_router, T, W, s.experts, s.top, 1.0, ids, wts)
+        else:
+            _call("mrs_hyb_route_softmax_topk", h32, self.w_router, T, W, s.experts, s.top, 1.0, ids, wts)
         meta = torch.empty(s.experts + 1 + 3 * R, dtype=torch.int32, device=dev)
         bounds, sorted_route, route_pos, sorted_expert = meta[:s.experts + 1], meta[s.experts + 1:][:R], meta[s.experts + 1 + R:][:R], meta[s.experts + 1 + 2 * R:][:R]
         _call("mrs_hyb_moe_dispatch", ids, R, s.experts, bounds, sorted_route, route_pos, sorted_expert)
         f32 = dict(dtype=torch.float32, device=dev)
         if R <= m.GROUPED_GEMV_ROWS:
-            # decode-sized steps: every route streams its expert's slabs; the row gather and the squared ReLU happen in the consuming product's operand load (same roundings)
+            # decode-sized steps: every route streams its expert's slabs; the row gather and the activation happen in the consuming product's operand load (same roundings)
             up = torch.empty(R, s.ff, **f32)
             m.gemv_act(h32, self.w_up, up, R, s.ff, W, h32.stride(0), W, sorted_expert, self.w_up.stride(0), 2, sorted_route, s.top)
             d = torch.empty(R, W, **f32)
-            m.gemv_act(up, self.w_down, d, R, W, s.ff, s.ff, s.ff, sorted_expert, self.w_down.stride(0), 5)
+            m.gemv_act(up, self.w_down, d, R, W, s.ff, s.ff, s.ff, sorted_expert, self.w_down.stride(0), self.in_mode)
         else:
             xs = torch.empty(R, W, dtype=m.torch_dtype, device=dev)
             _call("mrs_hyb_moe_gather", h32, sorted_route, None, s.top, xs, R, W, m.dt)
             up = m.grouped_linear(xs, self.w_up, bounds, sorted_expert)
             act = torch.empty(R, s.ff, dtype=m.torch_dtype, device=dev)
-            _call("mrs_hyb_relu_sq", up, act, R, s.ff, m.dt)
+            _call(self.act, up, act, R, s.ff, m.dt)
             d = m.grouped_linear(act, self.w_down, bounds, sorted_expert)
+        if defer:
+            return d, route_pos, wts, s.top
         _call("mrs_hyb_moe_combine_weighted", x, d, route_pos, wts, s.top, None, T, W, int(accumulate))
 
 
 MIXERS: Dict[str, Callable] = {"delta_rule": DeltaRuleMixer, "mlstm": MlstmMixer, "parallel": ParallelMixer, "mamba2": Mamba2Mixer, "attention": WindowAttention, "talk_attention": TalkSigmoidAttention, "sink_attention": GatedSinkAttention,
-                               "retention": RetentionMixer, "latent_attention": LatentAttention}
-FEED_FORWARDS: Dict[str, Callable] = {"moe_topk_softmax_relu2": TopkSoftmaxReluSqMoe, "moe": SigmoidMoe, "moe_softmax_clamped": ClampedSoftmaxMoe, "dense_xielu": XieluFeedForward, "dense_glu_silu": GluFeedForward}
+                               "retention": RetentionMixer, "latent_attention": LatentAttention, "gla": GlaMixer}
+FEED_FORWARDS: Dict[str, Callable] = {"moe_topk_softmax_relu2": UngatedMoe, "moe_ungated": UngatedMoe, "moe": SigmoidMoe, "moe_softmax_clamped": ClampedSoftmaxMoe, "dense_xielu": XieluFeedForward, "dense_glu_silu": GluFeedForward}
 
 
 class _Layer:
@@ -1450,6 +1705,14 @@ class HybridDecoder:
         self.embed = get(sp.embed).to(self.device, self.torch_dtype).contiguous()
         self.head = self.embed if sp.head == sp.embed else get(sp.head).to(self.device, self.torch_dtype).contiguous()   # a head tied to the embedding is the same tensor
         norm = lambda n: (f32(n), f32(n + ".b") if sp.norm == "layer" else None)
+
+        def join_norm(n, scale):
+            """the norm behind a sublayer, its per-channel scale folded in (the product of two bf16 numbers is exact in f32)"""
+            w, bias = norm(n)
+            if not sp.layer_scale:
+                return w, bias
+            ls = f32(scale)
+            return (w * ls).contiguous(), None if bias is None else (bias * ls).contiguous()
         self.final_norm = norm(sp.final_norm)
         if tuple(self.embed.shape) != (sp.vocab, sp.width) or tuple(self.head.shape) != (sp.vocab, sp.width):
             raise ValueError("embedding / head shapes do not match vocab x width")
@@ -1472,11 +1735,11 @@ class HybridDecoder:
             if self.multi_stream:
                 l.hc1 = hyper(l.spec.prefix + "hc1")
                 l.hc2 = hyper(l.spec.prefix + "hc2") if l.ff else None
-            l.norm1 = norm(l.spec.prefix + "norm1")
+            l.norm1 = join_norm(l.spec.prefix + "norm1", l.spec.prefix + "ls1") if sp.join_norms else norm(l.spec.prefix + "norm1")
             l.norm1b = norm(l.spec.prefix + "norm1b") if sp.post_norms else None
             l.mixer.load(get)
             if l.ff:
-                l.norm2 = norm(l.spec.prefix + "norm2")
+                l.norm2 = join_norm(l.spec.prefix + "norm2", l.spec.prefix + "ls2") if sp.join_norms else norm(l.spec.prefix + "norm2")
                 l.norm2b = norm(l.spec.prefix + "norm2b") if sp.post_norms else None
                 l.ff.load(get)
         for l in self.layers:   # layers that use another layer's tensors: the same norms and feed-forward, the same mixer weights around pages / taps / states of their own
@@ -1540,13 +1803,16 @@ class HybridDecoder:
         _call("mrs_hyb_gemm_batched", a, w, out, M, w.shape[0], K, a.stride(0), w.stride(0), out.stride(0), self.dt, 0, 0, 0, 0, 1)
         return out
 
-    def batched_linear(self, a, w, heads: int):
-        """a [M, heads * K] (column block h = the operand of head h), w [heads, N, K] -> [M, heads * N] in the serving dtype, rounded once: per-head products whose
-        consumer is another product or the attention kernel."""
+    def batched_linear(self, a, w, heads: int, a_block: Optional[int] = None, out=None, c_block: Optional[int] = None, f32: bool = False):
+        """a [M, heads * K] (column block h = the operand of head h), w [heads, N, K] -> [M, heads * N] in the serving dtype, rounded once (f32: unrounded): per-head products
+        whose consumer is another product or the attention kernel.  a_block: columns from one head's operand to the next (0: all heads read the same K columns); out, c_block:
+        a given result whose head blocks lie c_block columns apart."""
         M = a.shape[0]
         _, N, K = w.shape
-        out = torch.empty(M, heads * N, dtype=self.torch_dtype, device=self.device)
-        _call("mrs_hyb_gemm_batched", a, w, out, M, N, K, a.stride(0), K, out.stride(0), self.dt, heads, K, N * K, N, 1)
+        if out is None:
+            out = torch.empty(M, heads * N, dtype=torch.float32 if f32 else self.torch_dtype, device=self.device)
+        _call("mrs_hyb_gemm_batched", a, w, out, M, N, K, a.stride(0), K, out.stride(0), self.dt, heads, K if a_block is None else a_block, N * K, N if c_block is None else c_block,
+              int(not f32))
         return out
 
     def layer_norm(self, x, wb, want32: bool = False):
@@ -1559,7 +1825,7 @@ class HybridDecoder:
 
     def pre_norm(self, x, wb, want32: bool = False):
         """The norm in front of a sublayer (and of the head), of the kind the model's description names."""
-        if self.spec.norm == "layer":
+        if self.spec.norm in ("layer", "layer_plain"):
             return self.layer_norm(x, wb, want32)
         return self.norm(x, wb[0], one_plus=self.spec.norm == "rms_one_plus", want32=want32)
 
@@ -1594,10 +1860,20 @@ class HybridDecoder:
         _call("mrs_hyb_layernorm_pair", y, y.stride(0), in_bias, wb[0], wb[1], x, x.stride(0), then[0], then[1], out, out32, rows, width, self.spec.eps, self.dt)
         return (out, out32) if want32 else out
 
+    def join(self, x, y, wb, deferred=None):
+        """x += norm(y) through the norm behind a sublayer; deferred = (expert outputs, places, weights, experts per row): y is their weighted sum, taken in the same launch.
+        Returns the updated rows in the serving dtype, the next sublayer's operand."""
+        rows, width = x.shape
+        out = torch.empty(rows, width, dtype=self.torch_dtype, device=self.device) if self.torch_dtype != torch.float32 else None
+        d, route_pos, wts, top = deferred or (None, None, None, 0)
+        _call("mrs_hyb_layernorm_join", None if deferred else y, y.stride(0), d, route_pos, wts, top, wb[0], wb[1], x, x.stride(0), out, rows, width, self.spec.eps, self.dt)
+        return out if out is not None else x
+
     def gemv_act(self, a, w, out, M, N, K, lda, ldw, row_group, wstride, in_mode, src_row=None, src_div=1, bias=None, p0=0.0, p1=0.0, accumulate=False, src_scale=None):
         """out [M, N] (+)= act(a) . w^T for at most GEMV_ROWS rows (or one weight slab per row with `row_group`), the activation evaluated in the operand load.  in_mode:
         0 plain, 1 silu(gate) * up of a = f32 [gate | up], 2 gathered (and scaled) f32 source rows, 3 clamped GLU of a = f32 [gate | up] (p0 = limit, p1 = the sigmoid's
-        factor), 4 xIELU(a + bias) (p0, p1 = its two coefficients)."""
+        factor), 4 xIELU(a + bias) (p0, p1 = its two coefficients), 5 max(a, 0)^2, 6 gelu(gate) * up (tanh form), 7 gelu(a) (erf form), 8 a * sigmoid(bias) (bias = gate
+        logits of row stride src_div)."""
         _call("mrs_hyb_gemv_act", a, w, out, M, N, K, lda, ldw, out.stride(0), self.dt, int(accumulate), row_group, wstride, in_mode, src_row, src_scale, src_div, bias, p0, p1)
 
     def linear(self, a, w, out=None, accumulate: bool = False, dtype_code: Optional[int] = None):
@@ -1640,7 +1916,9 @@ class HybridDecoder:
         if T == 0:
             return torch.empty(0, sp.vocab, dtype=torch.float32, device=self.device)
         x = torch.empty(T, sp.width, dtype=torch.float32, device=self.device)
-        _call("mrs_hyb_embed", b.tokens, self.embed, x, T, sp.width, sp.vocab, self.dt)
+        if sp.join_norms:
+            return self._forward_joined(b, x)
+        _call("mrs_hyb_embed_scaled", b.tokens, self.embed, x, None, T, sp.width, sp.vocab, sp.embed_scale, self.dt)
         if self.embed_norm is not None:
             e = torch.empty_like(x)
             if sp.norm == "layer":
@@ -1671,6 +1949,33 @@ class HybridDecoder:
                 if l.ff:
                     h, h32 = self.pre_norm(x, l.norm2, want32=True)
                     l.ff.forward(h, h32, x, b)
+            if self.trace_layers is not None:
+                self.trace_layers.append(x.clone())
+        n = b.want.numel()
+        if n == 0:
+            return torch.empty(0, sp.vocab, dtype=torch.float32, device=self.device)
+        xs = torch.empty(n, sp.width, dtype=torch.float32, device=self.device)
+        _call("mrs_hyb_gather_rows", x, b.want, xs, n, sp.width)
+        return self.linear(self.pre_norm(xs, self.final_norm), self.head)
+
+    def _forward_joined(self, b: RaggedBatch, x: torch.Tensor) -> torch.Tensor:
+        """Designs whose sublayers read the residual rows themselves: one launch per sublayer norms its product, adds it to the f32 stream and rounds the updated rows for the
+        next sublayer (routed experts' outputs are summed in that launch too)."""
+        sp, T = self.spec, b.rows
+        if sp.post_norms or sp.parallel_sublayers or sp.embed_norm or self.multi_stream or sp.norm not in ("layer", "layer_plain"):
+            raise NotImplementedError("norms on the way into the stream are built for layer norms, one stream and nothing in front of the sublayers")
+        h = torch.empty(T, sp.width, dtype=self.torch_dtype, device=self.device) if self.torch_dtype != torch.float32 else None
+        _call("mrs_hyb_embed_scaled", b.tokens, self.embed, x, h, T, sp.width, sp.vocab, sp.embed_scale, self.dt)
+        h = x if h is None else h
+        y = torch.empty_like(x)
+        for l in self.layers:
+            if l.mixer.out_bias is not None or (l.ff and l.ff.out_bias is not None):
+                raise NotImplementedError("a sublayer with an output bias behind a norm that joins the stream")
+            l.mixer.forward(h, y, b, accumulate=False)
+            h = self.join(x, y, l.norm1)
+            if l.ff:
+                deferred = l.ff.forward(h, x, y, b, accumulate=False, **({"defer": True} if l.ff.defers_combine else {}))
+                h = self.join(x, y, l.norm2, deferred)
             if self.trace_layers is not None:
                 self.trace_layers.append(x.clone())
         n = b.want.numel()
@@ -1836,6 +2141,9 @@ def synthetic_weights(spec: HybridSpec, device, seed: int = 0) -> Callable[[str]
             continue
         for n in ["norm1"] + (["norm2"] if ls.ff else []) + ((["norm1b"] + (["norm2b"] if ls.ff else [])) if spec.post_norms else []):
             norm_names.add(p + n)
+        if spec.layer_scale:
+            norm_like.update({p + q for q in (("ls1", "ls2") if ls.ff else ("ls1",))})
+            shapes.update({p + q: (W,) for q in (("ls1", "ls2") if ls.ff else ("ls1",))})
         if spec.streams:
             for q in ("hc1", "hc2") if ls.ff else ("hc1",):
                 shapes.update({f"{p}{q}.in": (spec.streams,), f"{p}{q}.out": (spec.streams,), f"{p}{q}.mix": (spec.streams, spec.streams)})
@@ -1853,8 +2161,18 @@ def synthetic_weights(spec: HybridSpec, device, seed: int = 0) -> Callable[[str]
             shapes.update({p + "mix.q": (m.heads * m.dim, W), p + "mix.k": (m.heads * m.dim, W), p + "mix.v": (m.heads * m.vdim, W), p + "mix.g": (m.heads * m.vdim, W),
                            p + "mix.o": (W, m.heads * m.vdim)})
         elif isinstance(m, LatentAttentionSpec):
-            shapes.update({p + "mix.q": (m.heads * m.dim, W), p + "mix.dkv": (m.kv_rank, W), p + "mix.dkv.norm": (m.kv_rank,), p + "mix.uk": (m.heads * m.dim, m.kv_rank),
+            nq = m.heads * (m.dim + m.rot_dim)
+            shapes.update({p + "mix.dkv": (m.kv_rank + m.rot_dim, W), p + "mix.dkv.norm": (m.kv_rank,), p + "mix.uk": (m.heads * m.dim, m.kv_rank),
                            p + "mix.uv": (m.heads * m.vdim, m.kv_rank), p + "mix.o": (W, m.heads * m.vdim)})
+            shapes.update({p + "mix.dq": (m.q_rank, W), p + "mix.dq.norm": (m.q_rank,), p + "mix.uq": (nq, m.q_rank)} if m.q_rank else {p + "mix.q": (nq, W)})
+            if m.sink:
+                shapes[p + "mix.sink"] = (m.heads,)
+            if m.gate:
+                shapes[p + "mix.g"] = (m.heads * m.vdim, W)
+        elif isinstance(m, GlaSpec):
+            nk, nv, rank = m.heads * m.dim, m.heads * m.vdim, max(8, min(128, W // 16))
+            shapes.update({p + "mix.q": (nk, W), p + "mix.k": (nk, W), p + "mix.v": (nv, W), p + "mix.g": (nv, W), p + "mix.o": (W, nv), p + "mix.norm": (m.vdim,),
+                           p + "mix.a1": (rank, W), p + "mix.a2": (nk, rank), p + "mix.a2.b": (nk,)})
         elif isinstance(m, TalkAttentionSpec):
             shapes.update({p + "mix.q": (m.heads * m.dim, W), p + "mix.q.b": (m.heads * m.dim,), p + "mix.g": (m.heads, W), p + "mix.talk": (m.heads, m.heads),
                            p + "mix.pb": (m.heads,), p + "mix.o": (W, m.heads * m.vdim), p + "mix.o.b": (W,)})
@@ -1870,8 +2188,10 @@ def synthetic_weights(spec: HybridSpec, device, seed: int = 0) -> Callable[[str]
             shapes.update({p + "mlp.gate": (ls.ff.ff, W), p + "mlp.up": (ls.ff.ff, W), p + "mlp.down": (W, ls.ff.ff)})
         elif isinstance(ls.ff, DenseSpec):
             shapes.update({p + "mlp.up": (ls.ff.ff, W), p + "mlp.up.b": (ls.ff.ff,), p + "mlp.down": (W, ls.ff.ff), p + "mlp.down.b": (W,), p + "mlp.act": (2,)})
-        elif isinstance(ls.ff, TopkSoftmaxMoeSpec):
-            shapes.update({p + "mlp.router": (ls.ff.experts, W), p + "mlp.router.b": (ls.ff.experts,)})
+        elif isinstance(ls.ff, (TopkSoftmaxMoeSpec, UngatedMoeSpec)):
+            shapes[p + "mlp.router"] = (ls.ff.experts, W)
+            if ls.ff.routing == "chosen":
+                shapes[p + "mlp.router.b"] = (ls.ff.experts,)
             for e in range(ls.ff.experts):
                 shapes.update({f"{p}mlp.e{e}.up": (ls.ff.ff, W), f"{p}mlp.e{e}.down": (W, ls.ff.ff)})
         elif ls.ff:
@@ -1892,8 +2212,8 @@ def synthetic_weights(spec: HybridSpec, device, seed: int = 0) -> Callable[[str]
         shape = shapes[name]
         r = torch.randn(*shape, device=device, generator=g)
         last = name.rsplit(".", 1)[-1]
-        if name.endswith(("q.norm", "k.norm", "dkv.norm")) or last == "D" or name.endswith(("mix.norm", "left.norm", "right.norm")) or name in norm_like or \
-                (name in norm_names and spec.norm in ("layer", "rms")):
+        if name.endswith(("q.norm", "k.norm", "dkv.norm", "dq.norm")) or last == "D" or name.endswith(("mix.norm", "left.norm", "right.norm")) or name in norm_like or \
+                (name in norm_names and spec.norm in ("layer", "layer_plain", "rms")):
             r = 1.0 + 0.1 * r
         elif name.endswith("f.b"):
             r = 3.0 + 0.5 * r      # forget gates mostly open
@@ -1925,7 +2245,7 @@ def synthetic_weights(spec: HybridSpec, device, seed: int = 0) -> Callable[[str]
     return get
 
 
-SPEC_READERS: Dict[str, Callable[[dict], HybridSpec]] = {"Gekilix": gekilix_spec, "Sobunex": sobunex_spec, "Setopel": setopel_spec, "Gifopel": gifopel_spec}
+SPEC_READERS: Dict[str, Callable[[dict], HybridSpec]] = {"Gekilix": gekilix_spec, "Sobunex": sobunex_spec, "Setopel": setopel_spec, "Gifopel": gifopel_spec, "Kebisun": kebisun_spec}
 
 
 class HybridCache:
