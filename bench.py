@@ -1294,6 +1294,264 @@ def gifopel_leg(a, dev):
                       "config": {"model": f"gifopel-{a.gifopel}", "global_batch": 1, "seq_len": 512, "parallelism": "tp1"}, "gifopel": out}), flush=True)
 
 
+KEBISUN_SIZES = {
+    # layer lists that resemble a small, a mid-size and a large decoder: latent attention and gated linear attention in turn
+    "s": dict(width=1024, layers=6, heads=16, dim=64, rot=32, vdim=64, kv_rank=256, q_rank=384, window=2048, g_heads=8, g_dim=64, g_vdim=128, ff=2816, experts=32, top=4, eff=512, vocab=32000),
+    "m": dict(width=2048, layers=6, heads=16, dim=128, rot=64, vdim=128, kv_rank=512, q_rank=768, window=2048, g_heads=8, g_dim=128, g_vdim=256, ff=5632, experts=64, top=6, eff=768,
+              vocab=32000),
+    "l": dict(width=4096, layers=3, heads=32, dim=128, rot=64, vdim=128, kv_rank=512, q_rank=1536, window=2048, g_heads=16, g_dim=128, g_vdim=256, ff=11008, experts=64, top=6, eff=1408,
+              vocab=32000),
+}
+
+
+def kebisun_leg(a, dev):
+    """`--kebisun SIZE`: prefill and decode throughput of a Kebisun layer list (norms on the way into the stream; latent attention with a query latent, a shared rotated key part,
+    window, sink and gate; gated linear attention; dense GELU-GLU and routed GELU feed-forwards; bf16 weights, random) beside the closest model of the package at equal size:
+    latent attention with plain queries of the same key size, retention of equal state size, dense SiLU-GLU and routed squared-ReLU experts of equal weight bytes behind RMS
+    norms.  Then the kernels of the two designs that do like work, at the model's shapes: time and the fraction of the roofline (8 TB/s for what must be read and written;
+    prompt attention and the recurrences run on the f32 vector ALU in both designs and are priced in FLOP/s of the work done)."""
+    import torch
+    from mistralrs_amd.hybrid import (GlaSpec, GluSpec, HybridCache, HybridDecoder, HybridSpec, LatentAttentionSpec, LayerSpec, RaggedBatch, RetentionSpec, RotarySpec,
+                                      TopkSoftmaxMoeSpec, UngatedMoeSpec, _call, synthetic_weights)
+    z = KEBISUN_SIZES[a.kebisun]
+    W, H, D, Dr, Dv, R = z["width"], z["heads"], z["dim"], z["rot"], z["vdim"], z["kv_rank"]
+    gH, gD, gDv = z["g_heads"], z["g_dim"], z["g_vdim"]
+    scale = (D + Dr) ** -0.5
+    new_layers, old_layers = [], []
+    for i in range(z["layers"]):
+        ff_new = GluSpec(z["ff"], "gelu_tanh") if i == 0 else UngatedMoeSpec(z["experts"], z["top"], z["eff"])
+        ff_old = GluSpec(z["ff"]) if i == 0 else TopkSoftmaxMoeSpec(z["experts"], z["top"], z["eff"])
+        if i % 2 == 0:
+            rot = RotarySpec(Dr, 10000.0, {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}, "half")
+            new_layers.append(LayerSpec("latent_attention", LatentAttentionSpec(H, D, Dv, R, scale, z["q_rank"], Dr, rot, z["window"], True, True), ff_new, f"l{i}."))
+            old_layers.append(LayerSpec("latent_attention", LatentAttentionSpec(H, D + Dr, Dv, R, scale), ff_old, f"l{i}."))
+        else:
+            new_layers.append(LayerSpec("gla", GlaSpec(gH, gD, gDv, 16.0), ff_new, f"l{i}."))
+            old_layers.append(LayerSpec("retention", RetentionSpec(gH, gD, gDv, [1.0 - 2.0 ** (-5 - h % 8) for h in range(gH)], RotarySpec(gD, 10000.0, None, "half")), ff_old, f"l{i}."))
+    specs = {"kebisun": HybridSpec(z["vocab"], W, 1e-6, new_layers, norm="layer_plain", join_norms=True, layer_scale=True, embed_scale=W ** 0.5),
+             "latent_attention_retention_moe": HybridSpec(z["vocab"], W, 1e-6, old_layers, norm="rms")}
+    prompts, batches, bs, ctx = [512, 2048], [1, 8], 32, 512
+    max_tok = max(prompts) + a.warmup + a.steps + 64
+
+    def timed(fn, reps):
+        fn()
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        for _ in range(reps):
+            fn()
+        torch.cuda.synchronize()
+        return (time.perf_counter() - t0) / reps
+
+    def graphed(fn, reps=20):
+        """a launch (or a few) of a decode step as it runs in a step: from a HIP graph, so that host time does not hide the kernels"""
+        fn()
+        torch.cuda.synchronize()
+        g = torch.cuda.CUDAGraph()
+        with torch.cuda.graph(g):
+            for _ in range(reps):
+                fn()
+        t = timed(g.replay, 5)
+        return t / reps
+
+    out = {"sizes": z, "dtype": "bf16", "weights": "random, drawn on the device", "models": {}, "kernels": {}}
+    keep = {}
+    with torch.no_grad():
+        for name, spec in specs.items():
+            model = HybridDecoder(spec, dev, "bfloat16", num_blocks=max(batches) * (-(-max_tok // bs) + 1) + 2, block_size=bs, state_slots=max(batches))
+            model.load_weights(synthetic_weights(spec, dev, 0))
+            cache = HybridCache(model)
+            r = {"prefill": {}, "decode": {}}
+            for T in prompts:
+                assert cache.reserve(1, T)
+                b = RaggedBatch.build([cache.entry(1, [(1000 + i) % z["vocab"] for i in range(T)], 0, [T - 1])], bs, dev)
+                t = timed(lambda: model.forward_batch(b), 3)
+                r["prefill"][str(T)] = {"tokens_per_sec": round(T / t, 1), "ms": round(1e3 * t, 3)}
+                cache.release(1)
+            for nb in batches:
+                for q in range(nb):
+                    assert cache.reserve(q + 1, ctx + a.warmup + a.steps + 2)
+                model.forward_batch(RaggedBatch.build([cache.entry(q + 1, [(1000 + i + q) % z["vocab"] for i in range(ctx)], 0, []) for q in range(nb)], bs, dev))
+                g = model.capture_decode(nb, -(-(ctx + a.warmup + a.steps + 2) // bs))
+                pos = ctx
+
+                def step():
+                    nonlocal pos
+                    g.replay([cache.entry(q + 1, [7 + q], pos) for q in range(nb)])
+                    pos += 1
+                for _ in range(a.warmup):
+                    step()
+                torch.cuda.synchronize()
+                t0 = time.perf_counter()
+                for _ in range(a.steps):
+                    step()
+                torch.cuda.synchronize()
+                t = (time.perf_counter() - t0) / a.steps
+                r["decode"][f"batch{nb}"] = {"tokens_per_sec": round(nb / t, 1), "ms_per_step": round(1e3 * t, 4)}
+                del g
+                for q in range(nb):
+                    cache.release(q + 1)
+            out["models"][name] = r
+            keep[name] = model
+            torch.cuda.empty_cache()
+        if a.kebisun_models_only:
+            d1 = out["models"]["kebisun"]["decode"]["batch1"]
+            print(json.dumps({"metric": "kebisun_decode_tokens_per_sec", "value": d1["tokens_per_sec"], "unit": "tokens/s", "kebisun": out}), flush=True)
+            return
+        # ---- like kernels of the two designs
+        new, old = keep["kebisun"], keep["latent_attention_retention_moe"]
+        kern = out["kernels"]
+        e = 2
+        f32, bf = dict(dtype=torch.float32, device=dev), dict(dtype=torch.bfloat16, device=dev)
+
+        def pair(label, t_new, t_old, nbytes=None, flops=None, **extra):
+            d = {"kebisun_us": round(1e6 * t_new, 1), "other_us": round(1e6 * t_old, 1), "time_ratio": round(t_new / t_old, 2), **extra}
+            if nbytes is not None:
+                d.update(min_bytes=nbytes[0], other_min_bytes=nbytes[1], kebisun_hbm_frac=round(nbytes[0] / t_new / HBM_PEAK, 4), other_hbm_frac=round(nbytes[1] / t_old / HBM_PEAK, 4))
+            if flops is not None:
+                d.update(flops=flops[0], other_flops=flops[1], kebisun_tflops=round(flops[0] / t_new / 1e12, 2), other_tflops=round(flops[1] / t_old / 1e12, 2))
+            kern[label] = d
+        lat, gla = new.layers[0].mixer, new.layers[1].mixer
+        olat, ret = old.layers[0].mixer, old.layers[1].mixer
+
+        def batch(ents):
+            bps = -(-(2048 + 64) // bs)
+            return RaggedBatch.build([{"tokens": [0] * n, "pos0": p0, "slot": q, "blocks": list(range(1 + q * bps, 1 + q * bps + -(-(p0 + n) // bs))), "want": []}
+                                      for q, (p0, n) in enumerate(ents)], bs, dev)
+        # the recurrences
+        nv, nk = gH * gDv, gH * gD
+        st = nk * gDv
+        for label, ents in (("prompt_2048", [(0, 2048)]), ("prompt_8x256", [(0, 256)] * 8), ("decode_batch8", [(600, 1)] * 8), ("decode_batch1", [(600, 1)])):
+            b = batch(ents)
+            T = b.rows
+            u = torch.randn(T, gla.w_in.shape[0], **f32) * 0.1
+            uo = torch.randn(T, ret.w_in.shape[0], **f32) * 0.1
+            y, steps, yo = torch.empty(T, nv, **f32), torch.empty(T, gH, 2, **f32), torch.empty(T, nv, **bf)
+            carry, dk = torch.empty(b.segments, gH, gD, gDv, **f32), torch.empty(b.segments, gH, **f32)
+
+            def old_scan():
+                _call("mrs_hyb_decay_scan", uo, uo.stride(0), ret.decay, ret.state, y, b.seq_pos0, b.seq_slot, b.seg_entry, b.seg_row0, b.seg_len, b.ent_seg0, steps, carry, dk,
+                      T, b.entries, b.segments, gH, gDv, gD, gH)
+            if T == b.entries:
+                o = torch.empty(T, nv, **bf)
+
+                def new_step():
+                    _call("mrs_hyb_gla_step", u, u.stride(0), gla.k_col, gla.q_col, gla.g_col, gla.a_col, gla.rank, gla.w_a2, gla.b_a, gla.norm, gla.state, o, b.seq_start, b.seq_pos0,
+                          b.seq_slot, T, b.entries, gH, gD, gDv, gla.q_mult, gla.inv_tau, 1e-6, 1)
+
+                def old_step():
+                    old_scan()
+                    _call("mrs_hyb_rmsnorm", y, nv, None, yo, None, None, T, nv, gH, 1e-6, 0, 1, uo[:, ret.gate_col:], uo.stride(0), 1)
+                t_new, t_old = graphed(new_step), graphed(old_step)
+                pair(f"linear_attention_step_with_decays_norm_gate_vs_retention_scan_norm_gate_{label}", t_new, t_old, (T * 8 * st, T * 8 * st))
+            else:
+                zz = torch.randn(T, nk, **f32)
+                table, nseg = gla.segments(b)
+                cy, dy = (torch.empty(nseg, gH, gD, gDv, **f32), torch.empty(nseg, gH, gD, **f32)) if nseg > b.entries else (None, None)
+                t_new = timed(lambda: _call("mrs_hyb_gla_scan", u, u.stride(0), gla.k_col, gla.q_col, zz, nk, gla.b_a, gla.state, y, b.seq_pos0, b.seq_slot, *table, cy, dy, T, b.entries,
+                                            nseg, gH, gD, gDv, gla.q_mult, gla.inv_tau), 10)
+                t_old = timed(old_scan, 10)
+                pair(f"linear_attention_scan_vs_retention_scan_{label}", t_new, t_old, None, (6.0 * T * st, 6.0 * T * st), segments=nseg)
+        # attention
+        for c_ in (lat.c_cache, olat.c_cache):
+            c_.normal_()
+        for label, ents, win in (("prompt_2048", [(0, 2048)], z["window"]), ("prompt_2048_window_512", [(0, 2048)], 512), ("prompt_512_after_1536", [(1536, 512)], z["window"]),
+                                 ("decode_batch8_ctx2048", [(2047, 1)] * 8, z["window"]), ("decode_batch1_ctx2048", [(2047, 1)], z["window"])):
+            b = batch(ents)
+            T = b.rows
+            seg = (b.seg_entry, b.seg_row0, b.seg_len, b.segments, RaggedBatch.SEGMENT)
+            pairs, opairs = b.visible_pairs(win)[0], b.visible_pairs(0)[0]
+            gate = torch.randn(T, H * Dv, **f32)
+            if T > b.entries:
+                tables, source, n = b.context_blocks(win, bs)
+                otables, osource, on = b.context_blocks()
+                q = torch.randn(T, H * (D + Dr), device=dev).to(torch.bfloat16)
+                k, v = torch.randn(on * bs, H * (D + Dr), device=dev).to(torch.bfloat16), torch.randn(on * bs, H * Dv, device=dev).to(torch.bfloat16)
+                o = torch.empty(T, H * Dv, **bf)
+                vt = v.t().contiguous()
+                kw, vw = k[:n * bs], vt[:, :n * bs].contiguous()
+                t_new = timed(lambda: lat.attend_expanded(q, kw, vw, tables, b, o, gate, H * Dv, win), 10)
+                t_old = timed(lambda: olat.attend_expanded(q, k, vt, otables, b, o, None, 0, 0), 10)
+                t_gen = timed(lambda: _call("mrs_hyb_paged_attn_opts", q, k, v, otables, b.tok_seq, b.tok_pos, o, T, H, H, D + Dr, Dv, bs, b.max_blocks, 0, 0, scale, 1, *seg, 0.0, 0,
+                                            None, 0, None, 0, 1), 10)
+                per = 2.0 * H * (D + Dr + Dv)
+            else:
+                qa = torch.randn(T, H * (R + Dr), device=dev).to(torch.bfloat16)
+                oa, ov = torch.empty(T, H * R, **bf), torch.empty(T, H * Dv, **bf)
+                t_new = graphed(lambda: lat.attend_latent(qa, b, ov, gate, H * Dv, win))
+                t_old = graphed(lambda: olat.attend_latent(qa, b, ov, None, 0, 0))
+                sp = old.key_splits(b, H, R)
+                t_gen = graphed(lambda: _call("mrs_hyb_paged_attn_opts", qa, olat.c_cache, olat.c_cache, b.block_tables, b.tok_seq, b.tok_pos, oa, T, H, 1, R, R, bs, b.max_blocks, 0, 0,
+                                              scale, 1, *seg, 0.0, 0, None, 0, *sp, 0))
+                per = 2.0 * H * (2 * R + Dr)
+            byt = e * (b.visible_pairs(win)[1] * (R + Dr)), e * (b.visible_pairs(0)[1] * R)
+            pair("latent_attention_" + label, t_new, t_old, byt if T == b.entries else None, (per * pairs, (per if T > b.entries else 4.0 * H * R) * opairs), general_paged_kernel_us=round(1e6 * t_gen, 1))
+        # expansion of the context and the operands of latent attention
+        b = batch([(0, 2048)])
+        T = 2048
+        tables, source, n = b.context_blocks(z["window"], bs)
+        c = torch.empty(n * bs, R, **bf)
+
+        def expand_new():
+            return lat.expand_context(b, z["window"])
+
+        def expand_old():
+            _call("mrs_hyb_gather_rows", olat.c_cache, source, c, n, bs * R * e // 4)
+            return old.linear_rounded(c, olat.w_uk), old.linear_rounded(c, olat.w_uv.view(H * Dv, R))
+        t_new, t_old = timed(expand_new, 10), timed(expand_old, 10)
+        pair("context_expansion_2048_rows", t_new, t_old, None, (2.0 * T * R * H * (D + Dv), 2.0 * T * R * H * (D + Dr + Dv)))
+        for label, rows in (("2048_rows", 2048), ("decode_batch8", 8)):
+            b = batch([(0, 2048)] if rows == 2048 else [(600, 1)] * rows)
+            u, uo = torch.randn(rows, lat.w_in.shape[0], **f32), torch.randn(rows, olat.w_in.shape[0], **f32)
+            qf = torch.randn(rows, H * (D + Dr), **f32)
+            cq, qo, qa = torch.empty(rows, z["q_rank"], **bf), torch.empty(rows, H * (D + Dr), **bf), torch.empty(rows, H * (R + Dr), **bf)
+
+            def prep():
+                _call("mrs_hyb_latent_prep", u, u.stride(0), z["q_rank"], R, Dr, lat.dims, lat.q_norm, lat.c_norm, lat.freq, lat.trig_mult, b.tok_pos, b.slot_mapping, cq, lat.c_cache,
+                      1e-6, rows, 1)
+                _call("mrs_hyb_latent_query", qf, H * (D + Dr), H, D, R, Dr, lat.dims, lat.freq, lat.trig_mult, b.tok_pos, qo, qa if rows == 8 else None, rows, 1)
+            tm = (lambda f: timed(f, 10)) if rows == 2048 else graphed
+            t_new = tm(prep)
+            t_old = tm(lambda: _call("mrs_hyb_latent_norm_cache", uo, uo.stride(0), H * (D + Dr), R, olat.c_norm, b.slot_mapping, qo, olat.c_cache, 1e-6, rows, 1))
+            pair(f"latent_operands_two_launches_vs_one_{label}", t_new, t_old, (rows * (6 * (z["q_rank"] + R + Dr) + 6 * H * (D + Dr)), rows * (6 * R + 6 * H * (D + Dr))))
+        # row-wise kernels
+        for label, T in (("2048_rows", 2048), ("decode_batch8", 8)):
+            tm = (lambda f: timed(f, 10)) if T == 2048 else graphed
+            x, y, wv = torch.randn(T, W, **f32), torch.randn(T, W, **f32), torch.randn(W, **f32)
+            ob, o32 = torch.empty(T, W, **bf), torch.empty(T, W, **f32)
+            t_new = tm(lambda: _call("mrs_hyb_layernorm_join", y, W, None, None, None, 0, wv, None, x, W, ob, T, W, 1e-6, 1))
+            t_old = tm(lambda: _call("mrs_hyb_layernorm_pair", y, W, None, wv, wv, x, W, wv, wv, ob, o32, T, W, 1e-6, 1))
+            pair("norm_into_the_stream_vs_two_norms_in_one_launch_" + label, t_new, t_old, (T * W * 14, T * W * 18))
+            top, ff = z["top"], z["eff"]
+            R_ = T * top
+            d, rp, wt = torch.randn(R_, W, **f32), torch.randperm(R_, device=dev).to(torch.int32), torch.rand(R_, **f32)
+            t_new = tm(lambda: _call("mrs_hyb_layernorm_join", None, W, d, rp, wt, top, wv, None, x, W, ob, T, W, 1e-6, 1))
+
+            def old_combine():
+                _call("mrs_hyb_moe_combine_weighted", x, d, rp, wt, top, None, T, W, 1)
+                _call("mrs_hyb_rmsnorm", x, W, wv, ob, None, None, T, W, 1, 1e-6, 0, 1, None, 0, 0)
+            t_old = tm(old_combine)
+            pair("expert_sum_norm_into_the_stream_vs_expert_sum_and_norm_" + label, t_new, t_old, (T * W * (4 * top + 10), T * W * (4 * top + 8 + 6)))
+            if T == 2048:
+                gu, act2 = torch.randn(T, 2 * z["ff"], **f32), torch.empty(T, z["ff"], **bf)
+                pair("glu_activation_prompt", tm(lambda: _call("mrs_hyb_glu_gelu", gu, act2, T, z["ff"], 1)), tm(lambda: _call("mrs_hyb_glu_silu", gu, act2, T, z["ff"], 1)),
+                     (T * z["ff"] * 10, T * z["ff"] * 10))
+        # feed-forwards as units
+        y = torch.randn(2048, W, **f32)
+        for rows in (1, 8, 2048):
+            tm = (lambda f: timed(f, 5)) if rows == 2048 else graphed
+            b = batch([(0, 2048)] if rows == 2048 else [(600, 1)] * rows)
+            x = torch.randn(rows, W, **f32)
+            h = x.to(torch.bfloat16)
+            for name, li, nbytes in (("dense", 0, 3 * W * z["ff"] * 2), ("routed", 1, min(rows * z["top"], z["experts"]) * 2 * W * z["eff"] * 2)):
+                fn, fo = new.layers[li].ff, old.layers[li].ff
+                t_new, t_old = tm(lambda: fn.forward(h, x, y[:rows], b, accumulate=False)), tm(lambda: fo.forward(h, x, y[:rows], b, accumulate=False))
+                pair(f"{name}_feed_forward_{rows}_rows", t_new, t_old, (nbytes, nbytes) if rows <= 8 else None)
+    d1 = out["models"]["kebisun"]["decode"]["batch1"]
+    print(json.dumps({"metric": "kebisun_decode_tokens_per_sec", "value": d1["tokens_per_sec"], "unit": "tokens/s", "n_gpus": 1, "steps": a.steps, "warmup": a.warmup,
+                      "ms_per_step": d1["ms_per_step"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+                      "config": {"model": f"kebisun-{a.kebisun}", "global_batch": 1, "seq_len": 512, "parallelism": "tp1"}, "kebisun": out}), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -1326,11 +1584,22 @@ def main():
     ap.add_argument("--setopel", choices=sorted(SETOPEL_SIZES), default=None,
                     help="instead of the default workload: a Setopel layer list (residual streams; latent / sink attention, retention; SiLU-GLU feed-forwards; bf16) of the given size "
                          "beside an attention + state-space list of the package at equal size, and the like kernels of the two one by one")
+    ap.add_argument("--kebisun", choices=sorted(KEBISUN_SIZES), default=None,
+                    help="instead of the default workload: a Kebisun layer list (latent attention with a rotated key part / window / sink / gate, gated linear attention; dense / routed GELU "
+                         "feed-forwards) beside the package's closest model at equal size, and the like kernels of the two")
+    ap.add_argument("--kebisun-models-only", action="store_true", help="--kebisun: without the like kernels (profiling runs)")
     ap.add_argument("--gifopel", choices=sorted(GIFOPEL_SIZES), default=None,
                     help="instead of the default workload: a Gifopel layer list (matrix memory, chunked sink attention beside a delta rule, delta rule with channel decays; dense / routed "
                          "squared-ReLU feed-forwards; bf16) of the given size beside a state-space + windowed-attention + routed-experts list of the package at equal size, and the like "
                          "kernels of the two one by one")
     a = ap.parse_args()
+    if a.kebisun:
+        import torch
+        dev = torch.device("cuda", 0)
+        torch.cuda.set_device(dev)
+        if a.steps == 256:
+            a.steps = 128
+        return kebisun_leg(a, dev)
     if a.gifopel:
         import torch
         dev = torch.device("cuda", 0)

@@ -30,9 +30,19 @@ struct GemmArgs {
   int batch;
   long long a_bstride, c_bstride;
   int c_is_T;                // C holds T (bf16 | f32 as the operands), rounded once in the epilogue, instead of f32 (no accumulate then): the consumer is another product
+  int ep;                    // with c_is_T: EP_RELU_SQ | EP_GELU of the sums before they are rounded
 };
+// What a product that writes operands (T, rounded once) applies to its f32 sums first; the last two join two columns, n and n + N of a [gate | up] weight, into one.
+enum { EP_NONE = 0, EP_RELU_SQ = 1, EP_GELU = 2, EP_GLU_SILU = 3, EP_GLU_GELU = 4 };
+__device__ __forceinline__ float ep_act(int ep, float v) {
+  if (ep == EP_RELU_SQ) { v = fmaxf(v, 0.f); return v * v; }
+  if (ep == EP_GELU) return 0.5f * v * (1.0f + erff(v * 0.7071067811865476f));                // the erf form
+  if (ep == EP_GLU_SILU) return v / (1.0f + expf(-v));
+  if (ep == EP_GLU_GELU) return 0.5f * v * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * v * v, v, v)));   // the tanh form
+  return v;
+}
 template <class T> __device__ __forceinline__ void store_c(const GemmArgs &a, size_t idx, float v) {
-  if (a.c_is_T) ((T *)a.C)[idx] = from_f<T>(v);
+  if (a.c_is_T) ((T *)a.C)[idx] = from_f<T>(a.ep ? ep_act(a.ep, v) : v);
   else a.C[idx] = a.accumulate ? a.C[idx] + v : v;
 }
 
@@ -270,11 +280,8 @@ __global__ void __launch_bounds__(256) gemm_tile_f32_kernel(GemmArgs a) {
 //   IN_GLU_CLAMP  A = f32 [M, 2 K] = gate | up: g = min(gate, p0), u = clamp(up, -p0, p0): x_k = round_T(g sigmoid(p1 g) (u + 1))
 //   IN_BIAS_XIELU A = f32 [M, K]: z = A + in_bias: x_k = round_T(z > 0 ? p0 z^2 + z / 2 : p1 (e^z - 1 - z) + z / 2)
 //   IN_RELU_SQ A = f32 [M, K]: x_k = round_T(max(A, 0)^2)
-//   IN_GLU_GELU A = f32 [M, 2 K] = gate | up: x_k = round_T(gelu(gate) * up), the tanh form
-//   IN_GELU    A = f32 [M, K]: x_k = round_T(gelu(A)), the erf form
-//   IN_SIG_GATE A = f32 [M, K], in_bias = f32 [M, gate_ld] gate logits: x_k = round_T(A * sigmoid(gate_k))
 // The batched form offsets A by columns: only IN_PLAIN reads it there.
-enum { IN_PLAIN = 0, IN_GLU = 1, IN_SCALED = 2, IN_GLU_CLAMP = 3, IN_BIAS_XIELU = 4, IN_RELU_SQ = 5, IN_GLU_GELU = 6, IN_GELU = 7, IN_SIG_GATE = 8 };
+enum { IN_PLAIN = 0, IN_GLU = 1, IN_SCALED = 2, IN_GLU_CLAMP = 3, IN_BIAS_XIELU = 4, IN_RELU_SQ = 5 };
 struct GemvArgs {
   const void *A;
   const void *W;
@@ -287,12 +294,11 @@ struct GemvArgs {
   const int *src_row;        // IN_SCALED
   const float *src_scale;
   int src_div;
-  const float *in_bias;      // IN_BIAS_XIELU; IN_SIG_GATE: the gate logits
+  const float *in_bias;      // IN_BIAS_XIELU
   float p0, p1;              // IN_GLU_CLAMP: limit, sigmoid factor; IN_BIAS_XIELU: the two coefficients
   int batch;                 // batched form (row_group null): blockIdx.z = b reads A at column offset b * a_bstride, the slab W + b * wstride, writes C at column offset b * c_bstride
   long long a_bstride, c_bstride;
   int c_is_T;                // C holds T instead of f32 (no accumulate)
-  int gate_ld;               // IN_SIG_GATE: values between the rows of gate logits
 };
 
 template <class T> struct Vec8;
@@ -324,10 +330,6 @@ __device__ __forceinline__ float glu_clamp_in(float gv, float uv, float limit, f
 }
 __device__ __forceinline__ float xielu_in(float z, float ap, float an) { return z > 0.f ? fmaf(ap * z, z, 0.5f * z) : fmaf(an, expm1f(z) - z, 0.5f * z); }
 
-__device__ __forceinline__ float gelu_tanh_in(float v) { return 0.5f * v * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * v * v, v, v))); }
-__device__ __forceinline__ float gelu_erf_in(float v) { return 0.5f * v * (1.0f + erff(v * 0.7071067811865476f)); }
-__device__ __forceinline__ float sigmoid_in(float v) { return 1.0f / (1.0f + expf(-v)); }
-
 // one activation value (element path) / eight (vector path) of row m at column k, as the product sees it
 template <class T, int IN> __device__ __forceinline__ float act1(const GemvArgs &a, int m, int k) {
   if (IN == IN_PLAIN) return to_f<T>(((const T *)a.A)[(size_t)blockIdx.z * a.a_bstride + (size_t)m * a.lda + k]);
@@ -336,9 +338,6 @@ template <class T, int IN> __device__ __forceinline__ float act1(const GemvArgs 
   if (IN == IN_GLU_CLAMP) return round_to<T>(glu_clamp_in(A[(size_t)m * a.lda + k], A[(size_t)m * a.lda + a.K + k], a.p0, a.p1));
   if (IN == IN_BIAS_XIELU) return round_to<T>(xielu_in(A[(size_t)m * a.lda + k] + (a.in_bias ? a.in_bias[k] : 0.f), a.p0, a.p1));
   if (IN == IN_RELU_SQ) { const float v = fmaxf(A[(size_t)m * a.lda + k], 0.f); return round_to<T>(v * v); }
-  if (IN == IN_GLU_GELU) return round_to<T>(gelu_tanh_in(A[(size_t)m * a.lda + k]) * A[(size_t)m * a.lda + a.K + k]);
-  if (IN == IN_GELU) return round_to<T>(gelu_erf_in(A[(size_t)m * a.lda + k]));
-  if (IN == IN_SIG_GATE) return round_to<T>(A[(size_t)m * a.lda + k] * sigmoid_in(a.in_bias[(size_t)m * a.gate_ld + k]));
   const int r = a.src_row[m];
   return round_to<T>((a.src_scale ? a.src_scale[r] : 1.0f) * A[(size_t)(r / a.src_div) * a.lda + k]);
 }
@@ -375,28 +374,6 @@ template <class T, int IN> __device__ __forceinline__ void act8(const GemvArgs &
     for (int j = 0; j < 8; ++j) { const float v = fmaxf(x[j], 0.f); x[j] = round_to<T>(v * v); }
     return;
   }
-  if (IN == IN_GLU_GELU) {
-    float g[8], u[8];
-    Vec8<float>::load(A + (size_t)m * a.lda + k, g);
-    Vec8<float>::load(A + (size_t)m * a.lda + a.K + k, u);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) x[j] = round_to<T>(gelu_tanh_in(g[j]) * u[j]);
-    return;
-  }
-  if (IN == IN_GELU) {
-    Vec8<float>::load(A + (size_t)m * a.lda + k, x);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) x[j] = round_to<T>(gelu_erf_in(x[j]));
-    return;
-  }
-  if (IN == IN_SIG_GATE) {
-    float g[8];
-    Vec8<float>::load(A + (size_t)m * a.lda + k, x);
-    Vec8<float>::load(a.in_bias + (size_t)m * a.gate_ld + k, g);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) x[j] = round_to<T>(x[j] * sigmoid_in(g[j]));
-    return;
-  }
   const int r = a.src_row[m];
   const float w = a.src_scale ? a.src_scale[r] : 1.0f;
   Vec8<float>::load(A + (size_t)(r / a.src_div) * a.lda + k, x);
@@ -404,7 +381,8 @@ template <class T, int IN> __device__ __forceinline__ void act8(const GemvArgs &
   for (int j = 0; j < 8; ++j) x[j] = round_to<T>(w * x[j]);
 }
 
-template <class T, int MR, int IN> __global__ void __launch_bounds__(256) gemv_rows_kernel(GemvArgs a) {
+template <class T, int MR, int IN, int EP = EP_NONE> __global__ void __launch_bounds__(256) gemv_rows_kernel(GemvArgs a) {
+  constexpr bool GLU = EP == EP_GLU_SILU || EP == EP_GLU_GELU;   // W holds 2 N rows, gate | up
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int n = blockIdx.x * 4 + wave;
   if (n >= a.N) return;
@@ -417,34 +395,47 @@ template <class T, int MR, int IN> __global__ void __launch_bounds__(256) gemv_r
   } else if (a.batch > 0) {
     W += (size_t)blockIdx.z * a.wstride;
   }
-  const T *wr = W + (size_t)n * a.ldw;
-  float acc[MR];
+  const T *wr = W + (size_t)n * a.ldw, *wu = GLU ? wr + (size_t)a.N * a.ldw : wr;
+  float acc[MR], up[GLU ? MR : 1];
 #pragma unroll
   for (int m = 0; m < MR; ++m) acc[m] = 0.f;
+#pragma unroll
+  for (int m = 0; m < (GLU ? MR : 1); ++m) up[m] = 0.f;
   if (a.vec_ok) {
     for (int k = lane * 8; k < a.K; k += 512) {
-      float w[8], x[8];
+      float w[8], x[8], w2[8];
       Vec8<T>::load_nt(wr + k, w);
+      if (GLU) Vec8<T>::load_nt(wu + k, w2);
 #pragma unroll
       for (int m = 0; m < MR; ++m)
         if (m < m_cnt) {
           act8<T, IN>(a, m_lo + m, k, x);
 #pragma unroll
           for (int j = 0; j < 8; ++j) acc[m] = fmaf(w[j], x[j], acc[m]);
+          if (GLU) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) up[GLU ? m : 0] = fmaf(w2[j], x[j], up[GLU ? m : 0]);
+          }
         }
     }
   } else {
     for (int k = lane; k < a.K; k += 64) {
-      const float w = to_f<T>(wr[k]);
+      const float w = to_f<T>(wr[k]), w2 = GLU ? to_f<T>(wu[k]) : 0.f;
 #pragma unroll
       for (int m = 0; m < MR; ++m)
-        if (m < m_cnt) acc[m] = fmaf(w, act1<T, IN>(a, m_lo + m, k), acc[m]);
+        if (m < m_cnt) {
+          const float x = act1<T, IN>(a, m_lo + m, k);
+          acc[m] = fmaf(w, x, acc[m]);
+          if (GLU) up[GLU ? m : 0] = fmaf(w2, x, up[GLU ? m : 0]);
+        }
     }
   }
 #pragma unroll
   for (int m = 0; m < MR; ++m) {
     if (m >= m_cnt) break;
-    const float s = wave_sum(acc[m]);
+    float s = wave_sum(acc[m]);
+    if (EP != EP_NONE) s = ep_act(EP, s);
+    if (GLU) s *= wave_sum(up[GLU ? m : 0]);
     if (lane == 0) {
       const size_t idx = (size_t)blockIdx.z * a.c_bstride + (size_t)(m_lo + m) * a.ldc + n;
       if (a.c_is_T) ((T *)a.C)[idx] = from_f<T>(s);
@@ -465,7 +456,7 @@ extern "C" const char *mrs_hyb_gemm_last_error() { return g_err; }
 
 // dtype: 1 bf16, 2 f32.  groups > 0: grouped form (bounds [groups + 1] on the device, max_rows = the largest number of rows a group can have).
 static int gemm_launch(const void *A, const void *W, void *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate,
-                       const int *bounds, int groups, long long wstride, int max_rows, int batch, long long a_bstride, long long c_bstride, int c_is_T, void *stream) {
+                       const int *bounds, int groups, long long wstride, int max_rows, int batch, long long a_bstride, long long c_bstride, int c_is_T, void *stream, int ep = 0) {
   if (M <= 0 || N <= 0) return 0;
   if (batch > 0 && groups > 0) return fail("mrs_hyb_gemm: grouped and batched at once");
   if (c_is_T && accumulate) return fail("mrs_hyb_gemm: a product that writes operands does not accumulate");
@@ -474,7 +465,7 @@ static int gemm_launch(const void *A, const void *W, void *C, int M, int N, int 
   const int esz = dtype == 1 ? 2 : 4, vq = 8;
   GemmArgs a{A, W, (float *)C, M, N, K, lda, ldw, ldc, accumulate, groups > 0 ? bounds : nullptr, wstride,
              (K % vq == 0 && lda % vq == 0 && ldw % vq == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0 && (wstride * esz) % 16 == 0 &&
-              (batch <= 0 || (a_bstride * esz) % 16 == 0)) ? 1 : 0, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T};
+              (batch <= 0 || (a_bstride * esz) % 16 == 0)) ? 1 : 0, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T, ep};
   const int gz = groups > 0 ? groups : (batch > 0 ? batch : 1);
   const int rows = groups > 0 ? max_rows : M;
   if (rows <= 0) return 0;
@@ -496,6 +487,12 @@ extern "C" int mrs_hyb_gemm(const void *A, const void *W, float *C, int M, int N
                             const int *bounds, int groups, long long wstride, int max_rows, void *stream) {
   return gemm_launch(A, W, C, M, N, K, lda, ldw, ldc, dtype, accumulate, bounds, groups, wstride, max_rows, 0, 0, 0, 0, stream);
 }
+/* the same with C in dtype, an activation of the f32 sums first: ep 1 = max(., 0)^2, 2 = the erf form of gelu */
+extern "C" int mrs_hyb_gemm_act(const void *A, const void *W, void *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, const int *bounds, int groups, long long wstride,
+                                int max_rows, int ep, void *stream) {
+  if (ep != EP_RELU_SQ && ep != EP_GELU) return fail("mrs_hyb_gemm_act: activation");
+  return gemm_launch(A, W, C, M, N, K, lda, ldw, ldc, dtype, 0, bounds, groups, wstride, max_rows, 0, 0, 0, 1, stream, ep);
+}
 /* `batch` products in one launch: product b multiplies A + b * a_bstride [M, K] (row stride lda) with W + b * wstride [N, K] into C + b * c_bstride (row stride ldc): the heads'
  * operands as column blocks of row-major buffers.  c_is_T: C holds dtype values (rounded once) instead of f32.  batch 0: one product.  At most 8 rows take the row kernel. */
 extern "C" int mrs_hyb_gemm_batched(const void *A, const void *W, void *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int batch, long long a_bstride,
@@ -506,7 +503,7 @@ extern "C" int mrs_hyb_gemm_batched(const void *A, const void *W, void *C, int M
   const int esz = dtype == 1 ? 2 : 4;
   GemvArgs a{A, W, (float *)C, M, N, K, lda, ldw, ldc, 0, nullptr, wstride,
              (K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0 && (wstride * esz) % 16 == 0 && (a_bstride * esz) % 16 == 0) ? 1 : 0,
-             nullptr, nullptr, 1, nullptr, 0.f, 0.f, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T, 0};
+             nullptr, nullptr, 1, nullptr, 0.f, 0.f, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T};
   if (batch > 65535) return fail("mrs_hyb_gemm_batched: more than 65535 products in one batch");
   dim3 grid((N + 3) / 4, 1, batch > 0 ? batch : 1);
   hipStream_t s = (hipStream_t)stream;
@@ -518,27 +515,24 @@ extern "C" int mrs_hyb_gemm_batched(const void *A, const void *W, void *C, int M
 }
 
 /* in_mode: 0 plain (A in dtype), 1 GLU (A = f32 [M, 2 K] gate | up), 2 scaled rows (A = f32 source rows; row m = src_scale[r] * A[r / src_div], r = src_row[m]; no
- * src_scale: the rows are gathered as they are), 3 clamped GLU (A = f32 [M, 2 K]; p0 = limit, p1 = the sigmoid's factor), 4 xIELU(A + in_bias) (p0, p1 = its coefficients), 5 max(A, 0)^2 (A = f32 [M, K]),
- * 6 GLU with the tanh gelu (A = f32 [M, 2 K] gate | up), 7 the erf gelu of A (f32 [M, K]), 8 A times sigmoid(gate) (A = f32 [M, K]; in_bias = gate logits, src_div = their row stride) */
+ * src_scale: the rows are gathered as they are), 3 clamped GLU (A = f32 [M, 2 K]; p0 = limit, p1 = the sigmoid's factor), 4 xIELU(A + in_bias) (p0, p1 = its coefficients), 5 max(A, 0)^2 (A = f32 [M, K]) */
 extern "C" int mrs_hyb_gemv_act(const void *A, const void *W, float *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate, const int *row_group,
                                 long long wstride, int in_mode, const int *src_row, const float *src_scale, int src_div, const float *in_bias, float p0, float p1, void *stream) {
   if (M <= 0 || N <= 0) return 0;
-  if (K <= 0 || lda < K || ldw < K || ldc < N || (dtype != 1 && dtype != 2) || in_mode < 0 || in_mode > 8) return fail("mrs_hyb_gemv: bad shape / dtype / input mode");
-  if (in_mode == 8 && (!in_bias || src_div < K || row_group)) return fail("mrs_hyb_gemv: the gate logits need rows of K values");
-  if ((in_mode == 1 || in_mode == 3 || in_mode == 6) && lda < 2 * K) return fail("mrs_hyb_gemv: the gate | up operand needs rows of 2 K values");
+  if (K <= 0 || lda < K || ldw < K || ldc < N || (dtype != 1 && dtype != 2) || in_mode < 0 || in_mode > 5) return fail("mrs_hyb_gemv: bad shape / dtype / input mode");
+  if ((in_mode == 1 || in_mode == 3) && lda < 2 * K) return fail("mrs_hyb_gemv: the gate | up operand needs rows of 2 K values");
   if (in_mode == 2 && (!src_row || src_div <= 0)) return fail("mrs_hyb_gemv: gathered rows need their source table");
   if (!row_group && M > 8) return fail("mrs_hyb_gemv: at most 8 rows share a weight");
   if (row_group && M > 65535) return fail("mrs_hyb_gemv: too many rows");
   const int esz = dtype == 1 ? 2 : 4;
   GemvArgs a{A, W, C, M, N, K, lda, ldw, ldc, accumulate, row_group, wstride,
              (K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0 && (wstride * esz) % 16 == 0 &&
-              (!in_bias || ((uintptr_t)in_bias % 16) == 0) && (in_mode != 8 || src_div % 4 == 0)) ? 1 : 0, src_row, src_scale, src_div, in_bias, p0, p1, 0, 0, 0, 0, in_mode == 8 ? src_div : 0};
+              (!in_bias || ((uintptr_t)in_bias % 16) == 0)) ? 1 : 0, src_row, src_scale, src_div, in_bias, p0, p1, 0, 0, 0, 0};
   dim3 grid((N + 3) / 4, row_group ? M : 1);
   hipStream_t s = (hipStream_t)stream;
 #define MRS_GEMV_(T, MR, IN) hipLaunchKernelGGL((gemv_rows_kernel<T, MR, IN>), grid, dim3(256), 0, s, a)
 #define MRS_GEMV(T, MR) do { if (in_mode == 0) MRS_GEMV_(T, MR, IN_PLAIN); else if (in_mode == 1) MRS_GEMV_(T, MR, IN_GLU); else if (in_mode == 2) MRS_GEMV_(T, MR, IN_SCALED); \
-                             else if (in_mode == 3) MRS_GEMV_(T, MR, IN_GLU_CLAMP); else if (in_mode == 4) MRS_GEMV_(T, MR, IN_BIAS_XIELU); else if (in_mode == 5) MRS_GEMV_(T, MR, IN_RELU_SQ); \
-                             else if (in_mode == 6) MRS_GEMV_(T, MR, IN_GLU_GELU); else if (in_mode == 7) MRS_GEMV_(T, MR, IN_GELU); else MRS_GEMV_(T, MR, IN_SIG_GATE); } while (0)
+                             else if (in_mode == 3) MRS_GEMV_(T, MR, IN_GLU_CLAMP); else if (in_mode == 4) MRS_GEMV_(T, MR, IN_BIAS_XIELU); else MRS_GEMV_(T, MR, IN_RELU_SQ); } while (0)
   const int mr = row_group ? 1 : M;
   if (dtype == 1) { if (mr <= 1) MRS_GEMV(mrs::bf16_t, 1); else if (mr <= 2) MRS_GEMV(mrs::bf16_t, 2); else if (mr <= 4) MRS_GEMV(mrs::bf16_t, 4); else MRS_GEMV(mrs::bf16_t, 8); }
   else { if (mr <= 1) MRS_GEMV(float, 1); else if (mr <= 2) MRS_GEMV(float, 2); else if (mr <= 4) MRS_GEMV(float, 4); else MRS_GEMV(float, 8); }
@@ -552,4 +546,36 @@ extern "C" int mrs_hyb_gemv(const void *A, const void *W, float *C, int M, int N
   if (in_mode < 0 || in_mode > 2) return fail("mrs_hyb_gemv: bad shape / dtype / input mode");
   if (in_mode == 2 && !src_scale) return fail("mrs_hyb_gemv: scaled rows need their source table");
   return mrs_hyb_gemv_act(A, W, C, M, N, K, lda, ldw, ldc, dtype, accumulate, row_group, wstride, in_mode, src_row, src_scale, src_div, nullptr, 0.f, 0.f, stream);
+}
+
+/* out (dtype) [M, N] = activation of the rows' products with W, rounded once, ready to be the next product's operand.  ep 1 max(., 0)^2, 2 gelu (erf form): W [N, K];
+ * 3 silu(gate) * up, 4 gelu(gate) * up (tanh form): W [2 N, K] = gate | up.  in_mode 0: A in dtype; 2: A = f32 source rows, row m reads row src_row[m] / src_div (rounded to dtype).
+ * row_group (nullable): row m multiplies the slab W + row_group[m] * wstride; without it at most 8 rows. */
+extern "C" int mrs_hyb_gemv_ep(const void *A, const void *W, void *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, const int *row_group, long long wstride, int in_mode,
+                               const int *src_row, int src_div, int ep, void *stream) {
+  if (M <= 0 || N <= 0) return 0;
+  if (K <= 0 || lda < K || ldw < K || ldc < N || (dtype != 1 && dtype != 2) || (in_mode != 0 && in_mode != 2) || ep < 1 || ep > 4) return fail("mrs_hyb_gemv_ep: bad shape / dtype / mode");
+  if (in_mode == 2 && (!src_row || src_div <= 0)) return fail("mrs_hyb_gemv_ep: gathered rows need their source table");
+  if (!row_group && M > 8) return fail("mrs_hyb_gemv_ep: at most 8 rows share a weight");
+  if (row_group && (M > 65535 || ep > 2)) return fail("mrs_hyb_gemv_ep: too many rows, or a gated activation with a weight per row");
+  if (in_mode == 2 && !row_group) return fail("mrs_hyb_gemv_ep: gathered rows come with a weight each");
+  const int esz = dtype == 1 ? 2 : 4;
+  GemvArgs a{A, W, (float *)C, M, N, K, lda, ldw, ldc, 0, row_group, wstride,
+             (K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0 && (wstride * esz) % 16 == 0) ? 1 : 0, src_row, nullptr, src_div, nullptr,
+             0.f, 0.f, 0, 0, 0, 1};
+  dim3 grid((N + 3) / 4, row_group ? M : 1);
+  hipStream_t s = (hipStream_t)stream;
+#define MRS_GEP_(T, MR, IN, EP) hipLaunchKernelGGL((gemv_rows_kernel<T, MR, IN, EP>), grid, dim3(256), 0, s, a)
+#define MRS_GEP1(T, IN) do { if (ep == 1) MRS_GEP_(T, 1, IN, EP_RELU_SQ); else MRS_GEP_(T, 1, IN, EP_GELU); } while (0)
+#define MRS_GEPM(T, MR) do { if (ep == 1) MRS_GEP_(T, MR, IN_PLAIN, EP_RELU_SQ); else if (ep == 2) MRS_GEP_(T, MR, IN_PLAIN, EP_GELU); \
+                             else if (ep == 3) MRS_GEP_(T, MR, IN_PLAIN, EP_GLU_SILU); else MRS_GEP_(T, MR, IN_PLAIN, EP_GLU_GELU); } while (0)
+#define MRS_GEP(T) do { if (row_group) { if (in_mode == 2) MRS_GEP1(T, IN_SCALED); else MRS_GEP1(T, IN_PLAIN); } \
+                        else if (M <= 1) MRS_GEPM(T, 1); else if (M <= 2) MRS_GEPM(T, 2); else if (M <= 4) MRS_GEPM(T, 4); else MRS_GEPM(T, 8); } while (0)
+  if (dtype == 1) MRS_GEP(mrs::bf16_t);
+  else MRS_GEP(float);
+#undef MRS_GEP
+#undef MRS_GEPM
+#undef MRS_GEP1
+#undef MRS_GEP_
+  return hipGetLastError() == hipSuccess ? 0 : fail("mrs_hyb_gemv_ep: launch failed");
 }

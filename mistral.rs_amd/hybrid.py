@@ -76,13 +76,17 @@ _SIGS = {
     "mrs_hyb_round_cols": [_vp, _i, _vp, _i, _i, _i, _vp],
     "mrs_hyb_relu_sq": [_vp, _vp, _i, _i, _i, _vp],
     "mrs_hyb_glu_gelu": [_vp, _vp, _i, _i, _i, _vp],
-    "mrs_hyb_gelu_erf": [_vp, _vp, _i, _i, _i, _vp],
     "mrs_hyb_sigmoid_gate": [_vp, _vp, _i, _vp, _i, _i, _i, _vp],
     "mrs_hyb_layernorm_join": [_vp, _i, _vp, _vp, _vp, _i, _vp, _vp, _vp, _i, _vp, _i, _i, _f, _i, _vp],
     "mrs_hyb_paged_attn_sink_window": [_vp] * 7 + [_i] * 9 + [_f, _i, _vp, _vp, _vp, _i, _i, _f, _i, _vp, _vp, _i, _vp, _i, _i, _i, _vp],
     "mrs_hyb_latent_prep": [_vp] + [_i] * 5 + [_vp, _vp, _vp, _f] + [_vp] * 4 + [_f, _i, _i, _vp],
     "mrs_hyb_latent_query": [_vp] + [_i] * 6 + [_vp, _f, _vp, _vp, _vp, _i, _i, _vp],
     "mrs_hyb_latent_context": [_vp] * 4 + [_i] * 7 + [_vp],
+    "mrs_hyb_latent_mfma_prompt": [_vp] * 8 + [_i, _i, _vp, _vp, _i, _vp] + [_i] * 8 + [_f, _vp],
+    "mrs_hyb_latent_mfma_decode": [_vp] * 7 + [_i] * 8 + [_f, _vp],
+    "mrs_hyb_latent_mfma_merge": [_vp] * 5 + [_i, _vp] + [_i] * 5 + [_vp],
+    "mrs_hyb_gemm_act": [_vp] * 3 + [_i] * 7 + [_vp, _i, _l, _i, _i, _vp],
+    "mrs_hyb_gemv_ep": [_vp] * 3 + [_i] * 7 + [_vp, _l, _i, _vp, _i, _i, _vp],
     "mrs_hyb_gla_scan": [_vp, _i, _i, _i, _vp, _i] + [_vp] * 11 + [_i] * 6 + [_f, _f, _vp],
     "mrs_hyb_gla_step": [_vp] + [_i] * 6 + [_vp] * 8 + [_i] * 5 + [_f, _f, _f, _i, _vp],
     "mrs_hyb_gemm": [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _l, _i, _vp],
@@ -99,6 +103,8 @@ def _last_error(name: str) -> str:
         return "mrs_hyb_recur_last_error"
     if name in _LINATTN:
         return "mrs_hyb_linattn_last_error"
+    if "latent_mfma" in name:
+        return "mrs_hyb_latent_mfma_last_error"
     if "gem" in name:
         return "mrs_hyb_gemm_last_error"
     return "mrs_hyb_talk_last_error" if "talk" in name else "mrs_hyb_last_error"
@@ -1253,47 +1259,85 @@ class LatentAttention(_Module):
             m.batched_linear(q, self.w_ukT, H, a_block=D + Dr, out=qa, c_block=R + Dr)
         return qa if absorbed else q
 
+    # bf16 serving: attention on the matrix cores (csrc/hyb_latent.hip) at the sizes its tiles cover, else (and in f32) the general paged kernels
+    @property
+    def mfma_prompt(self) -> bool:
+        s, m = self.s, self.m
+        return self.USE_MFMA and m.dt == 1 and (s.dim + s.rot_dim) % 8 == 0 and s.dim + s.rot_dim <= 256 and s.vdim % 8 == 0 and s.vdim <= 128 and m.block_size % 8 == 0 and \
+            RaggedBatch.SEGMENT <= 64
+
+    @property
+    def mfma_decode(self) -> bool:
+        s, m = self.s, self.m
+        return self.USE_MFMA and m.dt == 1 and s.kv_rank % 16 == 0 and s.kv_rank <= 512 and self.row % 8 == 0 and self.row <= 640
+
+    USE_MFMA = os.environ.get("MRS_LATENT_MFMA", "1") != "0"
+    DECODE_GROUPS = 512   # workgroups a decode step's attention aims at (two per compute unit)
+
+    def expand_context(self, b: RaggedBatch, window: int):
+        """The contexts' latent rows, gathered block by block and expanded (two products on the matrix cores): (block tables, keys [n * block_size, H * (dim + rot_dim)], values
+        [n * block_size, H * vdim], or transposed [H * vdim, n * block_size] for the matrix-core attention)."""
+        s, m = self.s, self.m
+        H, D, Dr, Dv, R, bs = s.heads, s.dim, s.rot_dim, s.vdim, s.kv_rank, m.block_size
+        tables, source, n = b.context_blocks(window, bs)
+        c = torch.empty(n * bs, R, dtype=m.torch_dtype, device=m.device)
+        if Dr:
+            k = torch.empty(n * bs, H * (D + Dr), dtype=m.torch_dtype, device=m.device)
+            _call("mrs_hyb_latent_context", self.c_cache, source, c, k, n, bs, R, Dr, H, D, m.dt)
+            m.batched_linear(c, self.w_uk.view(H, D, R), H, a_block=0, out=k, c_block=D + Dr)
+        else:
+            _call("mrs_hyb_gather_rows", self.c_cache, source, c, n, bs * R * self.c_cache.element_size() // 4)
+            k = m.linear_rounded(c, self.w_uk)
+        w_uv = self.w_uv.view(H * Dv, R)
+        return tables, k, m.linear_rounded(w_uv, c) if self.mfma_prompt else m.linear_rounded(c, w_uv)
+
+    def attend_expanded(self, q, k, v, tables, b: RaggedBatch, out, gate, ldg: int, window: int) -> None:
+        """Attention over expanded keys and values: dim + rot_dim + vdim multiply-adds per (query, key) pair and head instead of 2 kv_rank + rot_dim."""
+        s, m = self.s, self.m
+        H, E, Dv = s.heads, s.dim + s.rot_dim, s.vdim
+        seg = (b.seg_entry, b.seg_row0, b.seg_len, b.segments, RaggedBatch.SEGMENT)
+        if self.mfma_prompt:
+            _call("mrs_hyb_latent_mfma_prompt", q, k, v, tables, b.tok_pos, *seg, self.sink, gate, ldg, out, b.rows, H, E, Dv, k.shape[0], b.max_blocks, m.block_size, window, s.scale)
+        else:
+            _call("mrs_hyb_paged_attn_sink_window", q, k, v, tables, b.tok_seq, b.tok_pos, out, b.rows, H, H, E, Dv, m.block_size, b.max_blocks, window, 0, s.scale, m.dt, *seg, 0.0,
+                  int(s.sink), self.sink, gate, ldg, None, 0, 1, 0)
+
+    def decode_shares(self, b: RaggedBatch, window: int) -> int:
+        """How many workgroups share a row's keys in a step of single rows: enough to fill the chip, at least 64 keys each"""
+        keys = b.max_blocks * self.m.block_size
+        keys = min(keys, window) if window > 0 else keys
+        return max(1, min(64, keys // 64, self.DECODE_GROUPS // max(1, b.rows * -(-self.s.heads // 16))))
+
+    def attend_latent(self, qa, b: RaggedBatch, out, gate, ldg: int, window: int) -> None:
+        """Attention over the cached rows themselves (a row is the key of every head, its first kv_rank values are the value), expanded to value size and gated: out [T, H * vdim]"""
+        s, m = self.s, self.m
+        T, H, R, Dv, dev = b.rows, s.heads, s.kv_rank, s.vdim, m.device
+        if b.seg_rows == 1 and self.mfma_decode:
+            n = self.decode_shares(b, window)
+            part, ml = torch.empty(n, T, H, R, dtype=torch.float32, device=dev), torch.empty(n, T, H, 2, dtype=torch.float32, device=dev)
+            _call("mrs_hyb_latent_mfma_decode", qa, self.c_cache, b.block_tables, b.tok_seq, b.tok_pos, part, ml, T, H, R, self.row, m.block_size, b.max_blocks, window, n, s.scale)
+            _call("mrs_hyb_latent_mfma_merge", part, ml, self.sink, self.w_uv, gate, ldg, out, T, H, R, Dv, n)
+            return
+        oa = torch.empty(T, H * R, dtype=m.torch_dtype, device=dev)
+        _call("mrs_hyb_paged_attn_sink_window", qa, self.c_cache, self.c_cache, b.block_tables, b.tok_seq, b.tok_pos, oa, T, H, 1, self.row, R, m.block_size, b.max_blocks, window, 0,
+              s.scale, m.dt, b.seg_entry, b.seg_row0, b.seg_len, b.segments, RaggedBatch.SEGMENT, 0.0, int(s.sink), self.sink, None, 0, *m.key_splits(b, H, R, window), 0, self.row)
+        if gate is None:
+            m.batched_linear(oa, self.w_uv, H, out=out)
+        else:
+            _call("mrs_hyb_sigmoid_gate", m.batched_linear(oa, self.w_uv, H, f32=True), gate, ldg, out, T, H * Dv, m.dt)
+
     def forward(self, h, x, b: RaggedBatch, accumulate: bool = True):
         s, m = self.s, self.m
-        T, dev, dt = b.rows, m.device, m.torch_dtype
-        H, D, Dr, Dv, R = s.heads, s.dim, s.rot_dim, s.vdim, s.kv_rank
         u = m.linear(h, self.w_in)                                         # f32 [T, q (query latent) | latent | key part | gate logits]
         gate, ldg = (u[:, self.gate_col:], u.stride(0)) if s.gate else (None, 0)
-        seg = (b.seg_entry, b.seg_row0, b.seg_len, b.segments, RaggedBatch.SEGMENT)
-        if self.expands(b):
-            # a step with prompt portions: the contexts' latent rows are gathered block by block and expanded into keys and values of `dim` (+ rot_dim) / `vdim` per head (two
-            # products on the matrix cores); attention then costs dim + rot_dim + vdim per (query, key) pair instead of 2 kv_rank + rot_dim
+        ov = torch.empty(b.rows, s.heads * s.vdim, dtype=m.torch_dtype, device=m.device)
+        if self.expands(b):   # a step with prompt portions
             q = self.queries(u, b, False)
-            bs = m.block_size
-            tables, source, n = b.context_blocks(s.window, bs)
-            c = torch.empty(n * bs, R, dtype=dt, device=dev)
-            if Dr:
-                k = torch.empty(n * bs, H * (D + Dr), dtype=dt, device=dev)
-                _call("mrs_hyb_latent_context", self.c_cache, source, c, k, n, bs, R, Dr, H, D, m.dt)
-                m.batched_linear(c, self.w_uk.view(H, D, R), H, a_block=0, out=k, c_block=D + Dr)
-            else:
-                _call("mrs_hyb_gather_rows", self.c_cache, source, c, n, bs * R * self.c_cache.element_size() // 4)
-                k = m.linear_rounded(c, self.w_uk)                          # [n * bs, H * dim]: block, slot, head -- the attention kernel's token-major layout
-            v = m.linear_rounded(c, self.w_uv.view(H * Dv, R))
-            ov = torch.empty(T, H * Dv, dtype=dt, device=dev)
-            _call("mrs_hyb_paged_attn_sink_window", q, k, v, tables, b.tok_seq, b.tok_pos, ov, T, H, H, D + Dr, Dv, bs, b.max_blocks, s.window, 0, s.scale, m.dt, *seg, 0.0,
-                  int(s.sink), self.sink, gate, ldg, None, 0, 1, 0)
-            m.linear(ov, self.w_o, out=x, accumulate=accumulate)
-            return
-        qa = self.queries(u, b, True)                                      # [T, H * (kv_rank + rot_dim)] in the serving dtype
-        oa = torch.empty(T, H * R, dtype=dt, device=dev)
-        _call("mrs_hyb_paged_attn_sink_window", qa, self.c_cache, self.c_cache, b.block_tables, b.tok_seq, b.tok_pos, oa, T, H, 1, self.row, R, m.block_size, b.max_blocks, s.window, 0,
-              s.scale, m.dt, *seg, 0.0, int(s.sink), self.sink, None, 0, *m.key_splits(b, H, R, s.window), 0, self.row)
-        if not s.gate:
-            m.linear(m.batched_linear(oa, self.w_uv, H), self.w_o, out=x, accumulate=accumulate)
-            return
-        ov = m.batched_linear(oa, self.w_uv, H, f32=True)                  # [T, H * vdim]
-        if T <= m.GEMV_ROWS:   # decode-sized steps: the gate in the output product's operand load
-            m.gemv_act(ov, self.w_o, x, T, x.shape[1], H * Dv, H * Dv, H * Dv, None, 0, 8, src_div=ldg, bias=gate, accumulate=accumulate)
-            return
-        og = torch.empty(T, H * Dv, dtype=dt, device=dev)
-        _call("mrs_hyb_sigmoid_gate", ov, gate, ldg, og, T, H * Dv, m.dt)
-        m.linear(og, self.w_o, out=x, accumulate=accumulate)
+            tables, k, v = self.expand_context(b, s.window)
+            self.attend_expanded(q, k, v, tables, b, ov, gate, ldg, s.window)
+        else:
+            self.attend_latent(self.queries(u, b, True), b, ov, gate, ldg, s.window)
+        m.linear(ov, self.w_o, out=x, accumulate=accumulate)
 
     MATRIX_TO_VECTOR_RATE = 6.0   # products on the matrix cores against attention arithmetic on the vector ALU, per operation
 
@@ -1379,12 +1423,12 @@ class GlaMixer(_Module):
 
 class GluFeedForward(_Module):
     """down(act(gate h) * (up h)), no biases; gate | up are one product.  act: SiLU or the tanh form of GELU."""
-    ACTS = {"silu": (1, "mrs_hyb_glu_silu"), "gelu_tanh": (6, "mrs_hyb_glu_gelu")}   # operand mode of the row kernel, the launch between prompt-sized products
+    ACTS = {"silu": (3, "mrs_hyb_glu_silu"), "gelu_tanh": (4, "mrs_hyb_glu_gelu")}   # what the row kernel applies as it writes, the launch between prompt-sized products
 
     def __init__(self, model, spec: GluSpec, prefix: str):
         super().__init__(model)
         self.s, self.p = spec, prefix
-        self.in_mode, self.act = self.ACTS[spec.act]
+        self.ep, self.act = self.ACTS[spec.act]
 
     def load(self, get):
         s, p, W = self.s, self.p, self.m.spec.width
@@ -1397,12 +1441,11 @@ class GluFeedForward(_Module):
     def forward(self, h, h32, x, b: RaggedBatch, accumulate: bool = True):
         s, m = self.s, self.m
         T = b.rows
-        gu = m.linear(h, self.w_gu)
-        if T <= m.GEMV_ROWS:   # decode-sized steps: the GLU in the down product's operand load
-            m.gemv_act(gu, self.w_down, x, T, x.shape[1], s.ff, 2 * s.ff, s.ff, None, 0, self.in_mode, accumulate=accumulate)
-            return
         a = torch.empty(T, s.ff, dtype=m.torch_dtype, device=m.device)
-        _call(self.act, gu, a, T, s.ff, m.dt)
+        if T <= m.GEMV_ROWS:   # decode-sized steps: a wave makes one gate and one up value and writes their GLU
+            m.gemv_ep(h, self.w_gu, a, self.ep)
+        else:
+            _call(self.act, m.linear(h, self.w_gu), a, T, s.ff, m.dt)
         m.linear(a, self.w_down, out=x, accumulate=accumulate)
 
 
@@ -1605,13 +1648,13 @@ class UngatedMoe(_Module):
     the chosen scores of the softmax over all of them, un-renormalised ("all").  Expert (no biases, no gate): down(act(up h)), act = max(., 0)^2 or the erf form of GELU.  All
     experts of a step run as grouped products over expert-sorted rows."""
     wants_f32_input = True
-    ACTS = {"relu2": (5, "mrs_hyb_relu_sq"), "gelu": (7, "mrs_hyb_gelu_erf")}   # operand mode of the row kernel, the launch between prompt-sized products
+    ACTS = {"relu2": 1, "gelu": 2}   # what the up product applies to its sums as it writes the down product's operand
     defers_combine = True   # `forward(defer=True)` hands the weighted sum to the launch that norms it into the stream
 
     def __init__(self, model, spec, prefix: str):
         super().__init__(model)
         self.s, self.p = spec, prefix
-        self.in_mode, self.act = self.ACTS[spec.act]
+        self.ep = self.ACTS[spec.act]
         if spec.routing not in ("all", "chosen"):
             raise ValueError(f"{prefix}: routing all | chosen")
 
@@ -1641,17 +1684,16 @@ class UngatedMoe(_Module):
         _call("mrs_hyb_moe_dispatch", ids, R, s.experts, bounds, sorted_route, route_pos, sorted_expert)
         f32 = dict(dtype=torch.float32, device=dev)
         if R <= m.GROUPED_GEMV_ROWS:
-            # decode-sized steps: every route streams its expert's slabs; the row gather and the activation happen in the consuming product's operand load (same roundings)
-            up = torch.empty(R, s.ff, **f32)
-            m.gemv_act(h32, self.w_up, up, R, s.ff, W, h32.stride(0), W, sorted_expert, self.w_up.stride(0), 2, sorted_route, s.top)
+            # decode-sized steps: every route streams its expert's slabs, the rows gathered in the up product's operand load (same roundings)
+            act = torch.empty(R, s.ff, dtype=m.torch_dtype, device=dev)
+            m.gemv_ep(h32, self.w_up, act, self.ep, sorted_expert, sorted_route, s.top)
             d = torch.empty(R, W, **f32)
-            m.gemv_act(up, self.w_down, d, R, W, s.ff, s.ff, s.ff, sorted_expert, self.w_down.stride(0), self.in_mode)
+            m.gemv_act(act, self.w_down, d, R, W, s.ff, s.ff, s.ff, sorted_expert, self.w_down.stride(0), 0)
         else:
             xs = torch.empty(R, W, dtype=m.torch_dtype, device=dev)
             _call("mrs_hyb_moe_gather", h32, sorted_route, None, s.top, xs, R, W, m.dt)
-            up = m.grouped_linear(xs, self.w_up, bounds, sorted_expert)
             act = torch.empty(R, s.ff, dtype=m.torch_dtype, device=dev)
-            _call(self.act, up, act, R, s.ff, m.dt)
+            _call("mrs_hyb_gemm_act", xs, self.w_up, act, R, s.ff, W, W, W, s.ff, m.dt, bounds, s.experts, self.w_up.stride(0), R, self.ep)
             d = m.grouped_linear(act, self.w_down, bounds, sorted_expert)
         if defer:
             return d, route_pos, wts, s.top
@@ -1872,9 +1914,15 @@ class HybridDecoder:
     def gemv_act(self, a, w, out, M, N, K, lda, ldw, row_group, wstride, in_mode, src_row=None, src_div=1, bias=None, p0=0.0, p1=0.0, accumulate=False, src_scale=None):
         """out [M, N] (+)= act(a) . w^T for at most GEMV_ROWS rows (or one weight slab per row with `row_group`), the activation evaluated in the operand load.  in_mode:
         0 plain, 1 silu(gate) * up of a = f32 [gate | up], 2 gathered (and scaled) f32 source rows, 3 clamped GLU of a = f32 [gate | up] (p0 = limit, p1 = the sigmoid's
-        factor), 4 xIELU(a + bias) (p0, p1 = its two coefficients), 5 max(a, 0)^2, 6 gelu(gate) * up (tanh form), 7 gelu(a) (erf form), 8 a * sigmoid(bias) (bias = gate
-        logits of row stride src_div)."""
+        factor), 4 xIELU(a + bias) (p0, p1 = its two coefficients), 5 max(a, 0)^2."""
         _call("mrs_hyb_gemv_act", a, w, out, M, N, K, lda, ldw, out.stride(0), self.dt, int(accumulate), row_group, wstride, in_mode, src_row, src_scale, src_div, bias, p0, p1)
+
+    def gemv_ep(self, a, w, out, ep: int, row_group=None, src_row=None, src_div: int = 1):
+        """out [M, N] (serving dtype, rounded once) = an activation of a . w^T for at most GEMV_ROWS rows, or one weight slab w[row_group[m]] per row with the f32 rows a
+        gathered by src_row / src_div.  ep: 1 max(., 0)^2, 2 gelu (erf form), 3 silu(gate) * up, 4 gelu(gate) * up (tanh form; w = [gate | up], 2 N rows)."""
+        M, N = out.shape
+        _call("mrs_hyb_gemv_ep", a, w, out, M, N, w.shape[-1], a.stride(0), w.stride(-2), out.stride(0), self.dt, row_group, w.stride(0) if row_group is not None else 0,
+              2 if src_row is not None else 0, src_row, src_div, ep)
 
     def linear(self, a, w, out=None, accumulate: bool = False, dtype_code: Optional[int] = None):
         """out (f32 [M, N]) (+)= a [M, K] . w [N, K]^T"""
