@@ -30,19 +30,9 @@ struct GemmArgs {
   int batch;
   long long a_bstride, c_bstride;
   int c_is_T;                // C holds T (bf16 | f32 as the operands), rounded once in the epilogue, instead of f32 (no accumulate then): the consumer is another product
-  int ep;                    // with c_is_T: EP_RELU_SQ | EP_GELU of the sums before they are rounded
 };
-// What a product that writes operands (T, rounded once) applies to its f32 sums first; the last two join two columns, n and n + N of a [gate | up] weight, into one.
-enum { EP_NONE = 0, EP_RELU_SQ = 1, EP_GELU = 2, EP_GLU_SILU = 3, EP_GLU_GELU = 4 };
-__device__ __forceinline__ float ep_act(int ep, float v) {
-  if (ep == EP_RELU_SQ) { v = fmaxf(v, 0.f); return v * v; }
-  if (ep == EP_GELU) return 0.5f * v * (1.0f + erff(v * 0.7071067811865476f));                // the erf form
-  if (ep == EP_GLU_SILU) return v / (1.0f + expf(-v));
-  if (ep == EP_GLU_GELU) return 0.5f * v * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * v * v, v, v)));   // the tanh form
-  return v;
-}
 template <class T> __device__ __forceinline__ void store_c(const GemmArgs &a, size_t idx, float v) {
-  if (a.c_is_T) ((T *)a.C)[idx] = from_f<T>(a.ep ? ep_act(a.ep, v) : v);
+  if (a.c_is_T) ((T *)a.C)[idx] = from_f<T>(v);
   else a.C[idx] = a.accumulate ? a.C[idx] + v : v;
 }
 
@@ -381,6 +371,16 @@ template <class T, int IN> __device__ __forceinline__ void act8(const GemvArgs &
   for (int j = 0; j < 8; ++j) x[j] = round_to<T>(w * x[j]);
 }
 
+// What a row product that writes operands (T, rounded once) applies to its f32 sums first; the last two join two columns, n and n + N of a [gate | up] weight, into one.
+// (Prompt tiles leave the activation to a launch of its own: sixty-four evaluations of erf per lane in the epilogue measured 2 - 3x the product's time.)
+enum { EP_NONE = 0, EP_RELU_SQ = 1, EP_GELU = 2, EP_GLU_SILU = 3, EP_GLU_GELU = 4 };
+__device__ __forceinline__ float ep_act(int ep, float v) {
+  if (ep == EP_RELU_SQ) { v = fmaxf(v, 0.f); return v * v; }
+  if (ep == EP_GELU) return 0.5f * v * (1.0f + erff(v * 0.7071067811865476f));                // the erf form
+  if (ep == EP_GLU_SILU) return v / (1.0f + expf(-v));
+  if (ep == EP_GLU_GELU) return 0.5f * v * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * v * v, v, v)));   // the tanh form
+  return v;
+}
 template <class T, int MR, int IN, int EP = EP_NONE> __global__ void __launch_bounds__(256) gemv_rows_kernel(GemvArgs a) {
   constexpr bool GLU = EP == EP_GLU_SILU || EP == EP_GLU_GELU;   // W holds 2 N rows, gate | up
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -456,7 +456,7 @@ extern "C" const char *mrs_hyb_gemm_last_error() { return g_err; }
 
 // dtype: 1 bf16, 2 f32.  groups > 0: grouped form (bounds [groups + 1] on the device, max_rows = the largest number of rows a group can have).
 static int gemm_launch(const void *A, const void *W, void *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate,
-                       const int *bounds, int groups, long long wstride, int max_rows, int batch, long long a_bstride, long long c_bstride, int c_is_T, void *stream, int ep = 0) {
+                       const int *bounds, int groups, long long wstride, int max_rows, int batch, long long a_bstride, long long c_bstride, int c_is_T, void *stream) {
   if (M <= 0 || N <= 0) return 0;
   if (batch > 0 && groups > 0) return fail("mrs_hyb_gemm: grouped and batched at once");
   if (c_is_T && accumulate) return fail("mrs_hyb_gemm: a product that writes operands does not accumulate");
@@ -465,7 +465,7 @@ static int gemm_launch(const void *A, const void *W, void *C, int M, int N, int 
   const int esz = dtype == 1 ? 2 : 4, vq = 8;
   GemmArgs a{A, W, (float *)C, M, N, K, lda, ldw, ldc, accumulate, groups > 0 ? bounds : nullptr, wstride,
              (K % vq == 0 && lda % vq == 0 && ldw % vq == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0 && (wstride * esz) % 16 == 0 &&
-              (batch <= 0 || (a_bstride * esz) % 16 == 0)) ? 1 : 0, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T, ep};
+              (batch <= 0 || (a_bstride * esz) % 16 == 0)) ? 1 : 0, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T};
   const int gz = groups > 0 ? groups : (batch > 0 ? batch : 1);
   const int rows = groups > 0 ? max_rows : M;
   if (rows <= 0) return 0;
@@ -486,12 +486,6 @@ static int gemm_launch(const void *A, const void *W, void *C, int M, int N, int 
 extern "C" int mrs_hyb_gemm(const void *A, const void *W, float *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate,
                             const int *bounds, int groups, long long wstride, int max_rows, void *stream) {
   return gemm_launch(A, W, C, M, N, K, lda, ldw, ldc, dtype, accumulate, bounds, groups, wstride, max_rows, 0, 0, 0, 0, stream);
-}
-/* the same with C in dtype, an activation of the f32 sums first: ep 1 = max(., 0)^2, 2 = the erf form of gelu */
-extern "C" int mrs_hyb_gemm_act(const void *A, const void *W, void *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, const int *bounds, int groups, long long wstride,
-                                int max_rows, int ep, void *stream) {
-  if (ep != EP_RELU_SQ && ep != EP_GELU) return fail("mrs_hyb_gemm_act: activation");
-  return gemm_launch(A, W, C, M, N, K, lda, ldw, ldc, dtype, 0, bounds, groups, wstride, max_rows, 0, 0, 0, 1, stream, ep);
 }
 /* `batch` products in one launch: product b multiplies A + b * a_bstride [M, K] (row stride lda) with W + b * wstride [N, K] into C + b * c_bstride (row stride ldc): the heads'
  * operands as column blocks of row-major buffers.  c_is_T: C holds dtype values (rounded once) instead of f32.  batch 0: one product.  At most 8 rows take the row kernel. */

@@ -971,6 +971,11 @@ template <class T> __global__ void __launch_bounds__(256) glu_gelu_kernel(const 
   const size_t r = i / ff, c = i % ff;
   out[i] = from_f<T>(gelu_tanh_f(gu[r * 2 * ff + c]) * gu[r * 2 * ff + ff + c]);
 }
+// the exact (erf) gelu of u [n]
+template <class T> __global__ void __launch_bounds__(256) gelu_erf_kernel(const float *__restrict__ u, T *__restrict__ out, size_t n) {
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i < n) out[i] = from_f<T>(0.5f * u[i] * (1.0f + erff(u[i] * 0.7071067811865476f)));
+}
 // y * sigmoid(gate): y [rows, n] f32 (contiguous), gate [rows, >= n] f32
 template <class T> __global__ void __launch_bounds__(256) sigmoid_gate_kernel(const float *__restrict__ y, const float *__restrict__ gate, int ldg, T *__restrict__ out, int n, size_t total) {
   const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
@@ -1670,6 +1675,16 @@ extern "C" int mrs_hyb_glu_gelu(const float *gu, void *out, int rows, int ff, in
   else if (dtype == 2) hipLaunchKernelGGL(glu_gelu_kernel<float>, dim3(blocks), dim3(256), 0, S_(stream), gu, (float *)out, rows, ff);
   else return fail("mrs_hyb_glu_gelu: dtype");
   return ok_or("mrs_hyb_glu_gelu");
+}
+/* the erf form of gelu */
+extern "C" int mrs_hyb_gelu_erf(const float *u, void *out, int rows, int ff, int dtype, void *stream) {
+  const size_t n = (size_t)rows * ff;
+  if (rows <= 0 || n == 0) return 0;
+  const unsigned blocks = (unsigned)((n + 255) / 256);
+  if (dtype == 1) hipLaunchKernelGGL(gelu_erf_kernel<mrs::bf16_t>, dim3(blocks), dim3(256), 0, S_(stream), u, (mrs::bf16_t *)out, n);
+  else if (dtype == 2) hipLaunchKernelGGL(gelu_erf_kernel<float>, dim3(blocks), dim3(256), 0, S_(stream), u, (float *)out, n);
+  else return fail("mrs_hyb_gelu_erf: dtype");
+  return ok_or("mrs_hyb_gelu_erf");
 }
 /* out (dtype) [rows, n] = y * sigmoid(gate) */
 extern "C" int mrs_hyb_sigmoid_gate(const float *y, const float *gate, int ldg, void *out, int rows, int n, int dtype, void *stream) {

@@ -377,7 +377,7 @@ struct LatentMergeArgs {
   uint16_t *out;
   int rows, H, R, Dv, splits, ldg;
 };
-__global__ void __launch_bounds__(256) latent_merge_kernel(LatentMergeArgs a) {
+__global__ void __launch_bounds__(1024) latent_merge_kernel(LatentMergeArgs a) {
   extern __shared__ __attribute__((aligned(16))) float sm[];  // o [R] | weight of every share
   const int h = blockIdx.x, t = blockIdx.y, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   float *o = sm, *ws = sm + a.R;
@@ -389,17 +389,19 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(LatentMergeArgs a) {
   const float L = wave_sum(lane < a.splits ? a.ml[(lane * step + at) * 2 + 1] * e : 0.f) + (a.sink ? exp2_f(sv - M) : 0.f);
   if (wave == 0 && lane < a.splits) ws[lane] = e / L;
   __syncthreads();
-  for (int r = tid; r < a.R; r += 256) {
+  const int nthr = blockDim.x, nw = nthr >> 6;
+  for (int r = tid; r < a.R; r += nthr) {
     float acc = 0.f;
-    for (int s = 0; s < a.splits; ++s) {
-      const float w = ws[s];
-      if (w != 0.f) acc = fmaf(w, a.part[(s * step + at) * a.R + r], acc);
+#pragma unroll 8
+    for (int s = 0; s < a.splits; ++s) {   // (an empty share's sums were never written: whatever is read there is dropped)
+      const float w = ws[s], v = a.part[(s * step + at) * a.R + r];
+      acc = w != 0.f ? fmaf(w, v, acc) : acc;
     }
     o[r] = round_to<bf16_t>(acc);
   }
   __syncthreads();
 #pragma unroll 4
-  for (int dv = wave; dv < a.Dv; dv += 4) {
+  for (int dv = wave; dv < a.Dv; dv += nw) {
     const uint16_t *w = a.w_uv + ((size_t)h * a.Dv + dv) * a.R;
     float acc = 0.f;
     for (int r = lane * 8; r < a.R; r += 512) {
@@ -478,6 +480,7 @@ extern "C" int mrs_hyb_latent_mfma_merge(const float *part, const float *ml, con
   if (gate && ldg < H * Dv) return fail("mrs_hyb_latent_mfma_merge: gate rows shorter than heads * value size");
   if (((uintptr_t)w_uv) % 16) return fail("mrs_hyb_latent_mfma_merge: unaligned operands");
   LatentMergeArgs a{part, ml, sink, gate, (const uint16_t *)w_uv, (uint16_t *)out, rows, H, R, Dv, splits, ldg};
-  hipLaunchKernelGGL(latent_merge_kernel, dim3(H, rows), dim3(256), (size_t)(a.R + 64) * 4, S_(stream), a);
+  const int nthr = (long long)rows * H >= 1024 ? 256 : 1024;   // few (row, head) pairs: more loads of the expansion in flight per compute unit
+  hipLaunchKernelGGL(latent_merge_kernel, dim3(H, rows), dim3(nthr), (size_t)(a.R + 64) * 4, S_(stream), a);
   return ok_or("mrs_hyb_latent_mfma_merge");
 }

@@ -44,17 +44,30 @@ template <int R> __device__ __forceinline__ float group_sum(float x) {
 
 struct GlaArgs {
   const float *u;       // [rows, ldu]: v [H * Dv] at 0, k [H * D] at k_col, q [H * D] at q_col
-  const float *z;       // [rows, ldz]: decay logits [H * D], before the bias
-  const float *zb;      // [H * D]
+  const float *dec;     // [rows, H * D]: the decays
   float *state;         // [slots, H, D, Dv]
   float *out;           // [rows, H * Dv]
   const int *seq_pos0, *seq_slot;
   const int *seg_entry, *seg_row0, *seg_len, *ent_seg0;  // segment table: entry, first row, rows; first segment of every entry (+ the total)
   float *carry;         // [segments, H, D, Dv]: a segment's end state from zero, then the state the next segment starts from
   float *decay;         // [segments, H, D]: the products of a segment's decays
-  int ldu, k_col, q_col, ldz, H, D, Dv;
-  float q_mult, inv_tau;
+  int ldu, k_col, q_col, H, D, Dv;
+  float q_mult;
 };
+// decays of all rows, in place: z [rows, n] (the products W_a2 a1) -> sigmoid(z + b)^(1 / tau); V values per access
+template <int V> __global__ void __launch_bounds__(256) gla_decays_kernel(float *__restrict__ z, const float *__restrict__ b, int n, size_t total, float inv_tau) {
+  const size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * V;
+  if (i >= total) return;
+  const int c = (int)(i % n);
+  if (V == 4) {
+    float4 v = *(const float4 *)(z + i);
+    v.x = channel_decay(v.x + b[c], inv_tau); v.y = channel_decay(v.y + b[c + 1], inv_tau);
+    v.z = channel_decay(v.z + b[c + 2], inv_tau); v.w = channel_decay(v.w + b[c + 3], inv_tau);
+    *(float4 *)(z + i) = v;
+  } else {
+    z[i] = channel_decay(z[i] + b[c], inv_tau);
+  }
+}
 
 // The recurrence is linear in S and a row scales the state's rows by numbers of its own, so a long portion can run its segments side by side:
 //   A  every segment but an entry's last, from zero: its end state L_k and the channel products d_k                        (LOCAL; parallel over segments)
@@ -64,7 +77,7 @@ struct GlaArgs {
 // A workgroup owns one (segment, head) and 64 / R * 4 value columns per wave.  A lane holds a register tile of the state: 4 columns times K = 4 J rows n = 4 (j R + r) + i (r = its
 // place in the group of R lanes): per row of tokens it reads 3 J + 1 16-byte groups (k, q, decays, v) from LDS for 12 K multiply-adds, lanes of a group at adjacent
 // addresses, and the four column sums close with data-parallel-primitive adds inside the group.  Token rows are staged TC at a time, key sizes and columns zero-padded to the tile
-// so that the loop has no guards; the next stage's values travel in registers while the current one is consumed, and the decays are evaluated on the way into LDS.
+// so that the loop has no guards; the next stage's values travel in registers while the current one is consumed.
 template <int R, int J, bool LOCAL, int NT> __global__ void __launch_bounds__(NT) gla_scan_kernel(GlaArgs a, int TC, int vec) {
   extern __shared__ __attribute__((aligned(16))) float sm[];  // [2][TC][k Dp | q Dp | decay Dp | v PC]
   constexpr int K = 4 * J, Dp = R * K, CW = 64 / R * 4, MAXV = 4;
@@ -88,49 +101,40 @@ template <int R, int J, bool LOCAL, int NT> __global__ void __launch_bounds__(NT
   // a stage = TC rows of U groups of four values, dealt to the threads flat; where a group comes from is worked out once
   const int U = (3 * Dp + PC) >> 2, stage_n = TC * U, rowlen = 4 * U, stage = TC * rowlen;
   float4 stg[MAXV];
-  const float *src[MAXV];
-  int what[MAXV], cnt4[MAXV], irow[MAXV], step[MAXV];   // 0: nothing, 1: plain, 2: query, 3: decay logit
-  float4 bias[MAXV];
+  int src[MAXV], info[MAXV];   // offset in u or z of the group in the first stage; what (0 nothing, 1 plain, 2 query, 3 decay) | values << 2 | row << 5
 #pragma unroll
   for (int m = 0; m < MAXV; ++m) {
     const int e = tid + m * nthr;
-    what[m] = 0; cnt4[m] = 0; irow[m] = 0; step[m] = 0; src[m] = a.u;
-    bias[m] = make_float4(0.f, 0.f, 0.f, 0.f);
+    src[m] = info[m] = 0;
     if (e >= stage_n) continue;
-    const int i = e / U, j = 4 * (e - i * U);
-    irow[m] = i;
-    const size_t row = (size_t)(r0 + i);
+    const int i = e / U, j = 4 * (e - i * U), row = r0 + i;
+    int what = 1, left;
     if (j < 3 * Dp) {
       const int which = j / Dp, n = j - which * Dp;
-      cnt4[m] = D - n < 0 ? 0 : (D - n > 4 ? 4 : D - n);
-      if (which < 2) { src[m] = a.u + row * a.ldu + (which ? a.q_col : a.k_col) + h * D + n; step[m] = a.ldu; what[m] = 1 + which; }
-      else {
-        src[m] = a.z + row * a.ldz + h * D + n; step[m] = a.ldz; what[m] = 3;
-        const float *b = a.zb + h * D + n;
-        if (cnt4[m] > 0) bias[m].x = b[0];
-        if (cnt4[m] > 1) bias[m].y = b[1];
-        if (cnt4[m] > 2) bias[m].z = b[2];
-        if (cnt4[m] > 3) bias[m].w = b[3];
-      }
+      left = D - n;
+      what = 1 + which;
+      src[m] = which < 2 ? row * a.ldu + (which ? a.q_col : a.k_col) + h * D + n : row * a.H * D + h * D + n;
     } else {
       const int c = p0 + j - 3 * Dp;
-      cnt4[m] = Dv - c < 0 ? 0 : (Dv - c > 4 ? 4 : Dv - c);
-      src[m] = a.u + row * a.ldu + h * Dv + c; step[m] = a.ldu; what[m] = 1;
+      left = Dv - c;
+      src[m] = row * a.ldu + h * Dv + c;
     }
-    if (cnt4[m] == 0) what[m] = 0;
+    left = left > 4 ? 4 : left;
+    if (left > 0) info[m] = what | (left << 2) | (i << 5);
   }
   auto fetch = [&](int c0) {
 #pragma unroll
     for (int m = 0; m < MAXV; ++m) {
       float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (what[m] && c0 + irow[m] < len) {
-        const float *q = src[m] + (size_t)c0 * step[m];
-        if (vec && cnt4[m] == 4) v = *(const float4 *)q;
+      const int what = info[m] & 3, left = (info[m] >> 2) & 7, i = info[m] >> 5;
+      if (what && c0 + i < len) {
+        const float *q = what == 3 ? a.dec + (src[m] + c0 * a.H * D) : a.u + (src[m] + c0 * a.ldu);
+        if (vec && left == 4) v = *(const float4 *)q;
         else {
           v.x = q[0];
-          if (cnt4[m] > 1) v.y = q[1];
-          if (cnt4[m] > 2) v.z = q[2];
-          if (cnt4[m] > 3) v.w = q[3];
+          if (left > 1) v.y = q[1];
+          if (left > 2) v.z = q[2];
+          if (left > 3) v.w = q[3];
         }
       }
       stg[m] = v;
@@ -139,14 +143,10 @@ template <int R, int J, bool LOCAL, int NT> __global__ void __launch_bounds__(NT
   auto put = [&](float *buf) {
 #pragma unroll
     for (int m = 0; m < MAXV; ++m) {
-      const int e = tid + m * nthr;
+      const int e = tid + m * nthr, what = info[m] & 3;
       if (e >= stage_n) continue;
       float4 v = stg[m];
-      if (what[m] == 2) { v.x *= a.q_mult; v.y *= a.q_mult; v.z *= a.q_mult; v.w *= a.q_mult; }
-      else if (what[m] == 3) {  // (channels past the key size never see a key: whatever they decay by, they hold zero)
-        v.x = channel_decay(v.x + bias[m].x, a.inv_tau); v.y = channel_decay(v.y + bias[m].y, a.inv_tau);
-        v.z = channel_decay(v.z + bias[m].z, a.inv_tau); v.w = channel_decay(v.w + bias[m].w, a.inv_tau);
-      }
+      if (what == 2) { v.x *= a.q_mult; v.y *= a.q_mult; v.z *= a.q_mult; v.w *= a.q_mult; }
       *(float4 *)(buf + 4 * e) = v;
     }
   };
@@ -330,18 +330,26 @@ using namespace mrs::hybl;
 
 extern "C" const char *mrs_hyb_linattn_last_error() { return g_err; }
 
-/* u [rows, ldu] = v [H * Dv] | ... with k [H * D] at k_col and q [H * D] at q_col; z [rows, ldz] decay logits [H * D], zb [H * D] their bias; alpha = sigmoid(z + zb)^inv_tau.
+/* z [rows, n] -> sigmoid(z + b [n])^inv_tau, in place */
+extern "C" int mrs_hyb_gla_decays(float *z, const float *b, int rows, int n, float inv_tau, void *stream) {
+  const size_t total = (size_t)rows * n;
+  if (rows <= 0 || n <= 0) return 0;
+  if (n % 4 == 0 && ((uintptr_t)z % 16) == 0) hipLaunchKernelGGL(gla_decays_kernel<4>, dim3((unsigned)((total / 4 + 255) / 256)), dim3(256), 0, S_(stream), z, b, n, total, inv_tau);
+  else hipLaunchKernelGGL(gla_decays_kernel<1>, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, S_(stream), z, b, n, total, inv_tau);
+  return ok_or("mrs_hyb_gla_decays");
+}
+/* u [rows, ldu] = v [H * Dv] | ... with k [H * D] at k_col and q [H * D] at q_col; dec [rows, H * D] the decays.
  * Segment table as for the other scans; carry [segments, H, D, Dv] and decay [segments, H, D] are scratch, needed when segments > entries. */
-extern "C" int mrs_hyb_gla_scan(const float *u, int ldu, int k_col, int q_col, const float *z, int ldz, const float *zb, float *state, float *out, const int *seq_pos0,
-                                const int *seq_slot, const int *seg_entry, const int *seg_row0, const int *seg_len, const int *ent_seg0, float *carry, float *decay, int rows,
-                                int entries, int segments, int H, int D, int Dv, float q_mult, float inv_tau, void *stream) {
+extern "C" int mrs_hyb_gla_scan(const float *u, int ldu, int k_col, int q_col, const float *dec, float *state, float *out, const int *seq_pos0, const int *seq_slot,
+                                const int *seg_entry, const int *seg_row0, const int *seg_len, const int *ent_seg0, float *carry, float *decay, int rows, int entries, int segments,
+                                int H, int D, int Dv, float q_mult, void *stream) {
   if (rows <= 0 || entries <= 0 || segments <= 0) return 0;
   if (H <= 0 || D <= 0 || Dv <= 0 || D > 512) return fail("mrs_hyb_gla_scan: head sizes (key size 1 .. 512)");
   if (entries > 65535 || segments > 65535 || H > 65535) return fail("mrs_hyb_gla_scan: more than 65535 entries, segments or heads");
-  if (k_col < H * Dv || q_col < H * Dv || ldu < k_col + H * D || ldu < q_col + H * D || ldz < H * D) return fail("mrs_hyb_gla_scan: rows shorter than v | k | q, or than the decay logits");
+  if (k_col < H * Dv || q_col < H * Dv || ldu < k_col + H * D || ldu < q_col + H * D) return fail("mrs_hyb_gla_scan: rows shorter than v | k | q");
   if (segments > entries && (!carry || !decay)) return fail("mrs_hyb_gla_scan: segmented entries need the carry scratch");
-  GlaArgs a{u, z, zb, state, out, seq_pos0, seq_slot, seg_entry, seg_row0, seg_len, ent_seg0, carry, decay, ldu, k_col, q_col, ldz, H, D, Dv, q_mult, inv_tau};
-  const int vec = (ldu % 4 == 0 && k_col % 4 == 0 && q_col % 4 == 0 && ldz % 4 == 0 && D % 4 == 0 && Dv % 4 == 0 && ((uintptr_t)u % 16) == 0 && ((uintptr_t)z % 16) == 0 &&
+  GlaArgs a{u, dec, state, out, seq_pos0, seq_slot, seg_entry, seg_row0, seg_len, ent_seg0, carry, decay, ldu, k_col, q_col, H, D, Dv, q_mult};
+  const int vec = (ldu % 4 == 0 && k_col % 4 == 0 && q_col % 4 == 0 && D % 4 == 0 && Dv % 4 == 0 && ((uintptr_t)u % 16) == 0 && ((uintptr_t)dec % 16) == 0 &&
                    ((uintptr_t)state % 16) == 0 && ((uintptr_t)out % 16) == 0 && ((uintptr_t)carry % 16) == 0) ? 1 : 0;
   int R, J;
   if (D <= 32) { R = 4; J = 2; } else if (D <= 64) { R = 8; J = 2; } else if (D <= 128) { R = 16; J = 2; } else if (D <= 256) { R = 16; J = 4; } else { R = 16; J = 8; }
@@ -355,6 +363,7 @@ extern "C" int mrs_hyb_gla_scan(const float *u, int ldu, int k_col, int q_col, c
   TC = TC > 16 ? 16 : TC;
   while (TC > 1 && (size_t)2 * TC * U * 16 > 65536) --TC;
   const size_t lds = (size_t)2 * TC * U * 16;
+  if ((long long)rows * ldu > 0x7fffffffLL) return fail("mrs_hyb_gla_scan: more than 2^31 projected values in one step");
   if (TC < 1 || lds > 65536) return fail("mrs_hyb_gla_scan: a row of operands does not fit the staging registers / 64 KB of LDS");
   dim3 grid(nblk, H, segments), block(64 * nw);
 #define MRS_GLA__(R_, J_, L_, NT_) hipLaunchKernelGGL((gla_scan_kernel<R_, J_, L_, NT_>), grid, block, lds, S_(stream), a, TC, vec)

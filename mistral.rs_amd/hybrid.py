@@ -85,9 +85,10 @@ _SIGS = {
     "mrs_hyb_latent_mfma_prompt": [_vp] * 8 + [_i, _i, _vp, _vp, _i, _vp] + [_i] * 8 + [_f, _vp],
     "mrs_hyb_latent_mfma_decode": [_vp] * 7 + [_i] * 8 + [_f, _vp],
     "mrs_hyb_latent_mfma_merge": [_vp] * 5 + [_i, _vp] + [_i] * 5 + [_vp],
-    "mrs_hyb_gemm_act": [_vp] * 3 + [_i] * 7 + [_vp, _i, _l, _i, _i, _vp],
+    "mrs_hyb_gelu_erf": [_vp, _vp, _i, _i, _i, _vp],
     "mrs_hyb_gemv_ep": [_vp] * 3 + [_i] * 7 + [_vp, _l, _i, _vp, _i, _i, _vp],
-    "mrs_hyb_gla_scan": [_vp, _i, _i, _i, _vp, _i] + [_vp] * 11 + [_i] * 6 + [_f, _f, _vp],
+    "mrs_hyb_gla_decays": [_vp, _vp, _i, _i, _f, _vp],
+    "mrs_hyb_gla_scan": [_vp, _i, _i, _i] + [_vp] * 11 + [_i] * 6 + [_f, _vp],
     "mrs_hyb_gla_step": [_vp] + [_i] * 6 + [_vp] * 8 + [_i] * 5 + [_f, _f, _f, _i, _vp],
     "mrs_hyb_gemm": [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _l, _i, _vp],
     "mrs_hyb_gemv": [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _l, _i, _vp, _vp, _i, _vp],
@@ -95,7 +96,7 @@ _SIGS = {
 }
 _RECUR = {"mrs_hyb_rmsnorm_pair", "mrs_hyb_delta_prep", "mrs_hyb_delta_step_prep", "mrs_hyb_delta_scan", "mrs_hyb_exp_gates", "mrs_hyb_head_norm_gate", "mrs_hyb_norm_pair_add", "mrs_hyb_round_cols",
           "mrs_hyb_relu_sq"}   # launchers of csrc/hyb_recur.hip (their own error text)
-_LINATTN = {"mrs_hyb_gla_scan", "mrs_hyb_gla_step"}   # launchers of csrc/hyb_linattn.hip
+_LINATTN = {"mrs_hyb_gla_decays", "mrs_hyb_gla_scan", "mrs_hyb_gla_step"}   # launchers of csrc/hyb_linattn.hip
 
 
 def _last_error(name: str) -> str:
@@ -1387,13 +1388,13 @@ class GlaMixer(_Module):
             raise ValueError(f"{p}: decay / norm / output shapes do not match the mixer's sizes")
 
     def segments(self, b: RaggedBatch):
-        """(segment table, segments) of this step's scan: one chain per entry when the entries fill the chip, else segments of 64 .. 512 rows, as short as SCAN_WAVES asks for"""
+        """(segment table, segments) of this step's scan: one chain per entry when the entries fill the chip, else segments of 32 .. 512 rows, as short as SCAN_WAVES asks for"""
         s = self.s
         columns = 64 if s.dim <= 32 else 32 if s.dim <= 64 else 16                             # value columns per wave of the scan
         per = s.heads * -(-s.vdim // columns)
         if b.host_lens is None or b.seg_rows <= 1 or b.entries * per >= self.SCAN_WAVES:
             return b.entry_table(), b.entries
-        rows = 64
+        rows = 32
         while rows < 512 and per * sum(-(-n // rows) for n in b.host_lens) > self.SCAN_WAVES:
             rows *= 2
         *table, n = b.segment_table(rows)
@@ -1411,12 +1412,13 @@ class GlaMixer(_Module):
                   b.seq_pos0, b.seq_slot, T, b.entries, s.heads, s.dim, s.vdim, self.q_mult, self.inv_tau, m.spec.eps, m.dt)
         else:
             z = m.linear(m.round_cols(u[:, self.a_col:], self.rank), self.w_a2)
+            _call("mrs_hyb_gla_decays", z, self.b_a, T, z.shape[1], self.inv_tau)
             table, nseg = self.segments(b)
             y, carry, decay = torch.empty(T, nv, **f32), None, None
             if nseg > b.entries:
                 carry, decay = torch.empty(nseg, s.heads, s.dim, s.vdim, **f32), torch.empty(nseg, s.heads, s.dim, **f32)
-            _call("mrs_hyb_gla_scan", u, u.stride(0), self.k_col, self.q_col, z, z.stride(0), self.b_a, self.state, y, b.seq_pos0, b.seq_slot, *table, carry, decay, T, b.entries, nseg,
-                  s.heads, s.dim, s.vdim, self.q_mult, self.inv_tau)
+            _call("mrs_hyb_gla_scan", u, u.stride(0), self.k_col, self.q_col, z, self.state, y, b.seq_pos0, b.seq_slot, *table, carry, decay, T, b.entries, nseg,
+                  s.heads, s.dim, s.vdim, self.q_mult)
             _call("mrs_hyb_head_norm_gate", y, s.vdim, None, self.norm, 0, u[:, self.g_col:], u.stride(0), 2, o, T, s.heads, s.vdim, m.spec.eps, m.dt)
         m.linear(o, self.w_o, out=x, accumulate=accumulate)
 
@@ -1648,13 +1650,13 @@ class UngatedMoe(_Module):
     the chosen scores of the softmax over all of them, un-renormalised ("all").  Expert (no biases, no gate): down(act(up h)), act = max(., 0)^2 or the erf form of GELU.  All
     experts of a step run as grouped products over expert-sorted rows."""
     wants_f32_input = True
-    ACTS = {"relu2": 1, "gelu": 2}   # what the up product applies to its sums as it writes the down product's operand
+    ACTS = {"relu2": (1, "mrs_hyb_relu_sq"), "gelu": (2, "mrs_hyb_gelu_erf")}   # what the row kernel applies as it writes, the launch between prompt-sized products
     defers_combine = True   # `forward(defer=True)` hands the weighted sum to the launch that norms it into the stream
 
     def __init__(self, model, spec, prefix: str):
         super().__init__(model)
         self.s, self.p = spec, prefix
-        self.ep = self.ACTS[spec.act]
+        self.ep, self.act = self.ACTS[spec.act]
         if spec.routing not in ("all", "chosen"):
             raise ValueError(f"{prefix}: routing all | chosen")
 
@@ -1693,7 +1695,7 @@ class UngatedMoe(_Module):
             xs = torch.empty(R, W, dtype=m.torch_dtype, device=dev)
             _call("mrs_hyb_moe_gather", h32, sorted_route, None, s.top, xs, R, W, m.dt)
             act = torch.empty(R, s.ff, dtype=m.torch_dtype, device=dev)
-            _call("mrs_hyb_gemm_act", xs, self.w_up, act, R, s.ff, W, W, W, s.ff, m.dt, bounds, s.experts, self.w_up.stride(0), R, self.ep)
+            _call(self.act, m.grouped_linear(xs, self.w_up, bounds, sorted_expert), act, R, s.ff, m.dt)
             d = m.grouped_linear(act, self.w_down, bounds, sorted_expert)
         if defer:
             return d, route_pos, wts, s.top
