@@ -377,7 +377,7 @@ __global__ void __launch_bounds__(GT) gemm_qi_kernel(const GemmArgs a) {
         for (int v = 0; v < 16; ++v) zero[v] = 0.f;
         const f16v M = __builtin_amdgcn_mfma_f32_32x32x16_f16(bsf, wm, zero, 0, 0, 0);
 #pragma unroll
-        for (int q4 = 0; q4 < 4; ++q4) {  // two outputs per instruction (v_pk_*_f32: the same IEEE operations per lane)
+        for (int q4 = 0; q4 < 4; ++q4) {  // outputs in pairs
           const float4 y4 = *(const float4 *)(yd_s + wt * 64 + tt * 32 + 8 * q4 + 4 * hf);
 #pragma unroll
           for (int k = 0; k < 4; k += 2) {

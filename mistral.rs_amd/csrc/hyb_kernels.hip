@@ -1526,7 +1526,7 @@ static int attn_launch(const void *q, const void *k_cache, const void *v_cache, 
                        const int *seg_entry, const int *seg_row0, const int *seg_len, int segments, int seg_rows, float softcap, int sink, const float *gate, int ldg,
                        float *scratch, int splits, int token_major, void *stream, int chunk = 0, const float *sink_logit = nullptr, int gate_per_head = 0, int ldv = 0) {
   if (rows <= 0) return 0;
-  if (Dv > 512 || H % G) return fail("mrs_hyb_paged_window_attn: value size above 512 / heads % kv_heads");
+  if (Dv > 1024 || H % G) return fail("mrs_hyb_paged_window_attn: value size above 1024 / heads % kv_heads");
   if (gate && ldg < (gate_per_head ? H : H * Dv)) return fail("mrs_hyb_paged_window_attn: gate rows shorter than heads (* value size)");
   if (chunk > 0 && (window > 0 || keep_first > 0)) return fail("mrs_hyb_paged_window_attn: chunks and a sliding window exclude each other");
   if (ldv == 0) ldv = Dv;
@@ -1541,8 +1541,8 @@ static int attn_launch(const void *q, const void *k_cache, const void *v_cache, 
     if (lds <= 65536) {
       dim3 grid((seg_rows + NQ - 1) / NQ, H, segments);
 #define MRS_ATTN_T(T, C) hipLaunchKernelGGL((paged_window_attn_tile_kernel<T, C, NQ>), grid, dim3(64), lds, S_(stream), a, seg_entry, seg_row0, seg_len)
-      if (dtype == 1) { if (c <= 1) MRS_ATTN_T(mrs::bf16_t, 1); else if (c <= 2) MRS_ATTN_T(mrs::bf16_t, 2); else MRS_ATTN_T(mrs::bf16_t, 4); }
-      else if (dtype == 2) { if (c <= 1) MRS_ATTN_T(float, 1); else if (c <= 2) MRS_ATTN_T(float, 2); else MRS_ATTN_T(float, 4); }
+      if (dtype == 1) { if (c <= 1) MRS_ATTN_T(mrs::bf16_t, 1); else if (c <= 2) MRS_ATTN_T(mrs::bf16_t, 2); else if (c <= 4) MRS_ATTN_T(mrs::bf16_t, 4); else MRS_ATTN_T(mrs::bf16_t, 8); }
+      else if (dtype == 2) { if (c <= 1) MRS_ATTN_T(float, 1); else if (c <= 2) MRS_ATTN_T(float, 2); else if (c <= 4) MRS_ATTN_T(float, 4); else MRS_ATTN_T(float, 8); }
       else return fail("mrs_hyb_paged_window_attn: dtype");
 #undef MRS_ATTN_T
       return ok_or("mrs_hyb_paged_window_attn");
@@ -1557,8 +1557,8 @@ static int attn_launch(const void *q, const void *k_cache, const void *v_cache, 
   dim3 grid(rows, H, a.splits > 1 ? a.splits : 1);
 #define MRS_ATTN(T, C) do { if (vec) hipLaunchKernelGGL((paged_window_attn_kernel<T, C, true>), grid, dim3(64), lds, S_(stream), a); \
                             else hipLaunchKernelGGL((paged_window_attn_kernel<T, C, false>), grid, dim3(64), lds, S_(stream), a); } while (0)
-  if (dtype == 1) { if (c <= 1) MRS_ATTN(mrs::bf16_t, 1); else if (c <= 2) MRS_ATTN(mrs::bf16_t, 2); else MRS_ATTN(mrs::bf16_t, 4); }
-  else if (dtype == 2) { if (c <= 1) MRS_ATTN(float, 1); else if (c <= 2) MRS_ATTN(float, 2); else MRS_ATTN(float, 4); }
+  if (dtype == 1) { if (c <= 1) MRS_ATTN(mrs::bf16_t, 1); else if (c <= 2) MRS_ATTN(mrs::bf16_t, 2); else if (c <= 4) MRS_ATTN(mrs::bf16_t, 4); else MRS_ATTN(mrs::bf16_t, 8); }
+  else if (dtype == 2) { if (c <= 1) MRS_ATTN(float, 1); else if (c <= 2) MRS_ATTN(float, 2); else if (c <= 4) MRS_ATTN(float, 4); else MRS_ATTN(float, 8); }
   else return fail("mrs_hyb_paged_window_attn: dtype");
 #undef MRS_ATTN
   if (a.splits > 1) {
