@@ -1,4 +1,4 @@
-/* mrs_hybrid.h -- C ABI of libmrs_hybrid.so: the kernels of layer-list ("hybrid") decoders served in their checkpoint dtype (csrc/hyb_kernels.hip, csrc/hyb_gemm.hip) and
+/* mrs_hybrid.h -- C ABI of libmrs_hybrid.so: the kernels of layer-list ("hybrid") decoders served in their checkpoint dtype (csrc/hyb_*.hip) and
  * the host-side state slot pool (csrc/host/state_pool.cpp; the paged KV cache manager's mrs_kv_* of mrs_hip_ext.h is linked into this library as well).
  *
  * Conventions: every launcher runs on the stream handed in as its last argument and returns 0, or 1 after storing a message for mrs_hyb_last_error() /
@@ -65,6 +65,28 @@ int mrs_hyb_gemm(const void *A, const void *W, float *C, int M, int N, int K, in
 int mrs_hyb_gemm_batched(const void *A, const void *W, void *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int batch, long long a_bstride, long long wstride, long long c_bstride, int c_is_T, void *stream);
 int mrs_hyb_gemv(const void *A, const void *W, float *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate, const int *row_group, long long wstride, int in_mode, const int *src_row, const float *src_scale, int src_div, void *stream);
 int mrs_hyb_gemv_act(const void *A, const void *W, float *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate, const int *row_group, long long wstride, int in_mode, const int *src_row, const float *src_scale, int src_div, const float *in_bias, float p0, float p1, void *stream);
+/* ---- hyb_kernels.hip: scaled embedding, norms that join the stream, latent attention with a rotated key part, window + sink + gate */
+int mrs_hyb_embed_scaled(const int *tokens, const void *table, float *x, void *out, int rows, int W, int vocab, float scale, int dtype, void *stream);
+int mrs_hyb_paged_attn_sink_window(const void *q, const void *k_cache, const void *v_cache, const int *block_tables, const int *tok_seq, const int *tok_pos, void *out, int rows, int H, int G, int D, int Dv, int block_size, int max_blocks, int window, int keep_first, float scale, int dtype, const int *seg_entry, const int *seg_row0, const int *seg_len, int segments, int seg_rows, float softcap, int sink, const float *sink_logit, const float *gate, int ldg, float *scratch, int splits, int token_major, int ldv, void *stream);
+int mrs_hyb_glu_gelu(const float *gu, void *out, int rows, int ff, int dtype, void *stream);
+int mrs_hyb_gelu_erf(const float *u, void *out, int rows, int ff, int dtype, void *stream);
+int mrs_hyb_sigmoid_gate(const float *y, const float *gate, int ldg, void *out, int rows, int n, int dtype, void *stream);
+int mrs_hyb_layernorm_join(const float *y, int ldy, const float *d, const int *route_pos, const float *wts, int top, const float *w, const float *b, float *resid, int ldr, void *out, int rows, int width, float eps, int dtype, void *stream);
+int mrs_hyb_latent_prep(const float *u, int ld, int qr, int R, int rot, int dims, const float *qw, const float *cw, const float *freq, float trig_mult, const int *tok_pos, const long long *slot_mapping, void *cq, void *c_cache, float eps, int rows, int dtype, void *stream);
+int mrs_hyb_latent_query(const float *qf, int ldq, int H, int D, int R, int rot, int dims, const float *freq, float trig_mult, const int *tok_pos, void *q_out, void *qa, int rows, int dtype, void *stream);
+int mrs_hyb_latent_context(const void *c_cache, const int *source, void *c, void *k, int n, int block_size, int R, int rot, int H, int D, int dtype, void *stream);
+/* ---- hyb_gemm.hip: row products that write activated operands */
+int mrs_hyb_gemv_ep(const void *A, const void *W, void *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, const int *row_group, long long wstride, int in_mode, const int *src_row, int src_div, int ep, void *stream);
+/* ---- hyb_linattn.hip: gated linear attention */
+const char *mrs_hyb_linattn_last_error();
+int mrs_hyb_gla_decays(float *z, const float *b, int rows, int n, float inv_tau, void *stream);
+int mrs_hyb_gla_scan(const float *u, int ldu, int k_col, int q_col, const float *dec, float *state, float *out, const int *seq_pos0, const int *seq_slot, const int *seg_entry, const int *seg_row0, const int *seg_len, const int *ent_seg0, float *carry, float *decay, int rows, int entries, int segments, int H, int D, int Dv, float q_mult, void *stream);
+int mrs_hyb_gla_step(const float *u, int ldu, int k_col, int q_col, int g_col, int a1_col, int rank, const void *wa2, const float *zb, const float *norm, float *state, void *out, const int *seq_start, const int *seq_pos0, const int *seq_slot, int rows, int entries, int H, int D, int Dv, float q_mult, float inv_tau, float eps, int dtype, void *stream);
+/* ---- hyb_latent.hip: latent attention on the matrix cores (bf16) */
+const char *mrs_hyb_latent_mfma_last_error();
+int mrs_hyb_latent_mfma_prompt(const void *q, const void *k, const void *vt, const int *tables, const int *tok_pos, const int *seg_entry, const int *seg_row0, const int *seg_len, int segments, int seg_rows, const float *sink, const float *gate, int ldg, void *out, int rows, int H, int DK, int Dv, int n_rows, int max_blocks, int block_size, int window, float scale, void *stream);
+int mrs_hyb_latent_mfma_decode(const void *q, const void *cache, const int *block_tables, const int *tok_seq, const int *tok_pos, float *part, float *ml, int rows, int H, int R, int E, int block_size, int max_blocks, int window, int splits, float scale, void *stream);
+int mrs_hyb_latent_mfma_merge(const float *part, const float *ml, const float *sink, const void *w_uv, const float *gate, int ldg, void *out, int rows, int H, int R, int Dv, int splits, void *stream);
 void *mrs_state_pool_create(size_t num_slots);
 void mrs_state_pool_destroy(void *h);
 size_t mrs_state_pool_capacity(void *h);
