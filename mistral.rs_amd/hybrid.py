@@ -7,7 +7,7 @@ layers).  The norms are RMS norms (plain or one-plus weights) before every subla
 layer norms behind the sublayers only (`join_norms`).  The Gekilix, Sobunex, Setopel, Gifopel and Kebisun architectures (config.json `"architecture"`) are such lists.
 
 The step function is `HybridDecoder.forward_batch(batch)`: ONE ragged batch -- prompt portions of any length next to single decoded tokens -- through the HIP kernels of
-csrc/hyb_kernels.hip and csrc/hyb_gemm.hip (C ABI, this process's current stream; PyTorch owns buffers and the stream, nothing else).  What the sequences carry between
+csrc/hyb_*.hip (C ABI, this process's current stream; PyTorch owns buffers and the stream, nothing else).  What the sequences carry between
 steps lives outside the step: K / V pages addressed through the block tables of `KVCacheManager`, convolution taps and recurrent states in the slots of `StateSlotPool`
 (kv_cache_manager.py).  The scheduler's engine (scheduler.PagedEngine) and the trace runner (bin/trace_run) both drive this function.
 
