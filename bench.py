@@ -1445,7 +1445,7 @@ def kebisun_leg(a, dev):
                 pair(f"linear_attention_step_with_decays_norm_gate_vs_retention_scan_norm_gate_{label}", t_new, t_old, (T * 8 * st, T * 8 * st))
             else:
                 zz = 1.0 - 0.1 * torch.rand(T, nk, **f32)
-                table, nseg = gla.segments(b)
+                table, nseg = scan_segments(b, gla.s.heads, gla.s.dim, gla.s.vdim)
                 cy, dy = (torch.empty(nseg, gH, gD, gDv, **f32), torch.empty(nseg, gH, gD, **f32)) if nseg > b.entries else (None, None)
                 t_new = timed(lambda: _call("mrs_hyb_gla_scan", u, u.stride(0), gla.k_col, gla.q_col, zz, gla.state, y, b.seq_pos0, b.seq_slot, *table, cy, dy, T, b.entries,
                                             nseg, gH, gD, gDv, gla.q_mult), 10)

@@ -30,8 +30,10 @@ struct GemmArgs {
   int batch;
   long long a_bstride, c_bstride;
   int c_is_T;                // C holds T (bf16 | f32 as the operands), rounded once in the epilogue, instead of f32 (no accumulate then): the consumer is another product
+  float alpha;               // the product is multiplied by this before it is added or stored
 };
 template <class T> __device__ __forceinline__ void store_c(const GemmArgs &a, size_t idx, float v) {
+  v *= a.alpha;
   if (a.c_is_T) ((T *)a.C)[idx] = from_f<T>(v);
   else a.C[idx] = a.accumulate ? a.C[idx] + v : v;
 }
@@ -289,6 +291,7 @@ struct GemvArgs {
   int batch;                 // batched form (row_group null): blockIdx.z = b reads A at column offset b * a_bstride, the slab W + b * wstride, writes C at column offset b * c_bstride
   long long a_bstride, c_bstride;
   int c_is_T;                // C holds T instead of f32 (no accumulate)
+  float alpha;               // the product is multiplied by this before it is added or stored (before an activation)
 };
 
 template <class T> struct Vec8;
@@ -433,7 +436,7 @@ template <class T, int MR, int IN, int EP = EP_NONE> __global__ void __launch_bo
 #pragma unroll
   for (int m = 0; m < MR; ++m) {
     if (m >= m_cnt) break;
-    float s = wave_sum(acc[m]);
+    float s = wave_sum(acc[m]) * a.alpha;
     if (EP != EP_NONE) s = ep_act(EP, s);
     if (GLU) s *= wave_sum(up[GLU ? m : 0]);
     if (lane == 0) {
@@ -456,7 +459,8 @@ extern "C" const char *mrs_hyb_gemm_last_error() { return g_err; }
 
 // dtype: 1 bf16, 2 f32.  groups > 0: grouped form (bounds [groups + 1] on the device, max_rows = the largest number of rows a group can have).
 static int gemm_launch(const void *A, const void *W, void *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate,
-                       const int *bounds, int groups, long long wstride, int max_rows, int batch, long long a_bstride, long long c_bstride, int c_is_T, void *stream) {
+                       const int *bounds, int groups, long long wstride, int max_rows, int batch, long long a_bstride, long long c_bstride, int c_is_T, void *stream,
+                       float alpha = 1.0f) {
   if (M <= 0 || N <= 0) return 0;
   if (batch > 0 && groups > 0) return fail("mrs_hyb_gemm: grouped and batched at once");
   if (c_is_T && accumulate) return fail("mrs_hyb_gemm: a product that writes operands does not accumulate");
@@ -465,7 +469,7 @@ static int gemm_launch(const void *A, const void *W, void *C, int M, int N, int 
   const int esz = dtype == 1 ? 2 : 4, vq = 8;
   GemmArgs a{A, W, (float *)C, M, N, K, lda, ldw, ldc, accumulate, groups > 0 ? bounds : nullptr, wstride,
              (K % vq == 0 && lda % vq == 0 && ldw % vq == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0 && (wstride * esz) % 16 == 0 &&
-              (batch <= 0 || (a_bstride * esz) % 16 == 0)) ? 1 : 0, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T};
+              (batch <= 0 || (a_bstride * esz) % 16 == 0)) ? 1 : 0, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T, alpha};
   const int gz = groups > 0 ? groups : (batch > 0 ? batch : 1);
   const int rows = groups > 0 ? max_rows : M;
   if (rows <= 0) return 0;
@@ -497,7 +501,7 @@ extern "C" int mrs_hyb_gemm_batched(const void *A, const void *W, void *C, int M
   const int esz = dtype == 1 ? 2 : 4;
   GemvArgs a{A, W, (float *)C, M, N, K, lda, ldw, ldc, 0, nullptr, wstride,
              (K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0 && (wstride * esz) % 16 == 0 && (a_bstride * esz) % 16 == 0) ? 1 : 0,
-             nullptr, nullptr, 1, nullptr, 0.f, 0.f, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T};
+             nullptr, nullptr, 1, nullptr, 0.f, 0.f, batch > 0 ? batch : 0, a_bstride, c_bstride, c_is_T, 1.0f};
   if (batch > 65535) return fail("mrs_hyb_gemm_batched: more than 65535 products in one batch");
   dim3 grid((N + 3) / 4, 1, batch > 0 ? batch : 1);
   hipStream_t s = (hipStream_t)stream;
@@ -508,10 +512,9 @@ extern "C" int mrs_hyb_gemm_batched(const void *A, const void *W, void *C, int M
   return hipGetLastError() == hipSuccess ? 0 : fail("mrs_hyb_gemm_batched: launch failed");
 }
 
-/* in_mode: 0 plain (A in dtype), 1 GLU (A = f32 [M, 2 K] gate | up), 2 scaled rows (A = f32 source rows; row m = src_scale[r] * A[r / src_div], r = src_row[m]; no
- * src_scale: the rows are gathered as they are), 3 clamped GLU (A = f32 [M, 2 K]; p0 = limit, p1 = the sigmoid's factor), 4 xIELU(A + in_bias) (p0, p1 = its coefficients), 5 max(A, 0)^2 (A = f32 [M, K]) */
-extern "C" int mrs_hyb_gemv_act(const void *A, const void *W, float *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate, const int *row_group,
-                                long long wstride, int in_mode, const int *src_row, const float *src_scale, int src_div, const float *in_bias, float p0, float p1, void *stream) {
+static int gemv_launch(const void *A, const void *W, float *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate, const int *row_group,
+                       long long wstride, int in_mode, const int *src_row, const float *src_scale, int src_div, const float *in_bias, float p0, float p1, float alpha,
+                       void *stream) {
   if (M <= 0 || N <= 0) return 0;
   if (K <= 0 || lda < K || ldw < K || ldc < N || (dtype != 1 && dtype != 2) || in_mode < 0 || in_mode > 5) return fail("mrs_hyb_gemv: bad shape / dtype / input mode");
   if ((in_mode == 1 || in_mode == 3) && lda < 2 * K) return fail("mrs_hyb_gemv: the gate | up operand needs rows of 2 K values");
@@ -521,7 +524,7 @@ extern "C" int mrs_hyb_gemv_act(const void *A, const void *W, float *C, int M, i
   const int esz = dtype == 1 ? 2 : 4;
   GemvArgs a{A, W, C, M, N, K, lda, ldw, ldc, accumulate, row_group, wstride,
              (K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0 && (wstride * esz) % 16 == 0 &&
-              (!in_bias || ((uintptr_t)in_bias % 16) == 0)) ? 1 : 0, src_row, src_scale, src_div, in_bias, p0, p1, 0, 0, 0, 0};
+              (!in_bias || ((uintptr_t)in_bias % 16) == 0)) ? 1 : 0, src_row, src_scale, src_div, in_bias, p0, p1, 0, 0, 0, 0, alpha};
   dim3 grid((N + 3) / 4, row_group ? M : 1);
   hipStream_t s = (hipStream_t)stream;
 #define MRS_GEMV_(T, MR, IN) hipLaunchKernelGGL((gemv_rows_kernel<T, MR, IN>), grid, dim3(256), 0, s, a)
@@ -535,6 +538,18 @@ extern "C" int mrs_hyb_gemv_act(const void *A, const void *W, float *C, int M, i
   return hipGetLastError() == hipSuccess ? 0 : fail("mrs_hyb_gemv: launch failed");
 }
 
+/* in_mode: 0 plain (A in dtype), 1 GLU (A = f32 [M, 2 K] gate | up), 2 scaled rows (A = f32 source rows; row m = src_scale[r] * A[r / src_div], r = src_row[m]; no
+ * src_scale: the rows are gathered as they are), 3 clamped GLU (A = f32 [M, 2 K]; p0 = limit, p1 = the sigmoid's factor), 4 xIELU(A + in_bias) (p0, p1 = its coefficients), 5 max(A, 0)^2 (A = f32 [M, K]) */
+extern "C" int mrs_hyb_gemv_act(const void *A, const void *W, float *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate, const int *row_group,
+                                long long wstride, int in_mode, const int *src_row, const float *src_scale, int src_div, const float *in_bias, float p0, float p1, void *stream) {
+  return gemv_launch(A, W, C, M, N, K, lda, ldw, ldc, dtype, accumulate, row_group, wstride, in_mode, src_row, src_scale, src_div, in_bias, p0, p1, 1.0f, stream);
+}
+/* C[M, N] (+)= alpha * A . W^T (A in dtype): a sublayer that joins the residual stream with a factor of its own.  At most 8 rows take the row kernel. */
+extern "C" int mrs_hyb_gemm_scaled(const void *A, const void *W, float *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate, float alpha, void *stream) {
+  if (M <= 0 || N <= 0) return 0;
+  if (M > 8) return gemm_launch(A, W, C, M, N, K, lda, ldw, ldc, dtype, accumulate, nullptr, 0, 0, 0, 0, 0, 0, 0, stream, alpha);
+  return gemv_launch(A, W, C, M, N, K, lda, ldw, ldc, dtype, accumulate, nullptr, 0, 0, nullptr, nullptr, 1, nullptr, 0.f, 0.f, alpha, stream);
+}
 extern "C" int mrs_hyb_gemv(const void *A, const void *W, float *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate,
                             const int *row_group, long long wstride, int in_mode, const int *src_row, const float *src_scale, int src_div, void *stream) {
   if (in_mode < 0 || in_mode > 2) return fail("mrs_hyb_gemv: bad shape / dtype / input mode");
@@ -556,7 +571,7 @@ extern "C" int mrs_hyb_gemv_ep(const void *A, const void *W, void *C, int M, int
   const int esz = dtype == 1 ? 2 : 4;
   GemvArgs a{A, W, (float *)C, M, N, K, lda, ldw, ldc, 0, row_group, wstride,
              (K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0 && (wstride * esz) % 16 == 0) ? 1 : 0, src_row, nullptr, src_div, nullptr,
-             0.f, 0.f, 0, 0, 0, 1};
+             0.f, 0.f, 0, 0, 0, 1, 1.0f};
   dim3 grid((N + 3) / 4, row_group ? M : 1);
   hipStream_t s = (hipStream_t)stream;
 #define MRS_GEP_(T, MR, IN, EP) hipLaunchKernelGGL((gemv_rows_kernel<T, MR, IN, EP>), grid, dim3(256), 0, s, a)

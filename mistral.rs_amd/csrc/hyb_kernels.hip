@@ -53,7 +53,7 @@ template <class T> __global__ void __launch_bounds__(256) embed_kernel(const int
 
 // ---------------------------------------------------------------------------------- x / sqrt(mean(x^2) + eps) * (w | 1 + w); grid.y = equal parts of the row
 // w null: no weight.  gate (optional, [rows, ldg]): gate_after 0: the row is multiplied by silu(gate) BEFORE its root mean square is taken; gate_after 1: the normed row is
-// multiplied by silu(gate)
+// multiplied by silu(gate), 2: by sigmoid(gate)
 template <class T> __global__ void __launch_bounds__(256) rmsnorm_kernel(const float *__restrict__ x, int ldx, const float *__restrict__ w, T *__restrict__ out, float *__restrict__ out32,
                                                                           float *__restrict__ rstd, int part, float eps, int one_plus, int ldo, const float *__restrict__ gate, int ldg,
                                                                           int gate_after) {
@@ -75,7 +75,7 @@ template <class T> __global__ void __launch_bounds__(256) rmsnorm_kernel(const f
   for (int c = threadIdx.x; c < part; c += 256) {
     const float wv = w ? w[(size_t)g * part + c] : (one_plus ? 0.f : 1.0f);
     float v = (pre ? row[c] : xr[c]) * inv * (one_plus ? 1.0f + wv : wv);
-    if (gr && gate_after) v *= silu_f(gr[c]);
+    if (gr && gate_after) v *= gate_after == 2 ? sigmoid_f(gr[c]) : silu_f(gr[c]);
     if (out) out[(size_t)t * ldo + (size_t)g * part + c] = from_f<T>(v);
     if (out32) out32[(size_t)t * ldo + (size_t)g * part + c] = v;
   }
@@ -1157,6 +1157,89 @@ template <class T> __global__ void __launch_bounds__(256) qkv_bias_temp_cache_ke
     ((T *)a.v_cache)[(((size_t)blk * a.G + g) * a.block_size + off) * a.Dv + d] = from_f<T>(v[e] + (a.vb ? a.vb[e] : 0.f));
   }
 }
+// ---------------------------------------------------------------------------------- layers that run again: what joins the stream in front of a pass, with the norm behind it
+// x += scale * table[token] (table null: not) + step (null: not), in this order; out = x / rms(x) * (w | 1 + w), out32 (nullable) the same in f32
+template <class T> __global__ void __launch_bounds__(256) pass_norm_kernel(float *__restrict__ x, const int *__restrict__ tokens, const T *__restrict__ table, int vocab, float scale,
+                                                                           const float *__restrict__ step, const float *__restrict__ w, T *__restrict__ out, float *__restrict__ out32, int W,
+                                                                           float eps, int one_plus) {
+  __shared__ float red[4];
+  const int t = blockIdx.x;
+  float *xr = x + (size_t)t * W;
+  const T *er = nullptr;
+  if (table) {
+    int id = tokens[t];
+    id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+    er = table + (size_t)id * W;
+  }
+  float s = 0.f;
+  for (int c = threadIdx.x; c < W; c += 256) {
+    float v = xr[c];
+    if (er) v += to_f<T>(er[c]) * scale;
+    if (step) v += step[c];
+    xr[c] = v;
+    s = fmaf(v, v, s);
+  }
+  const float inv = 1.0f / sqrtf(block_sum_256(s, red) / (float)W + eps);
+  for (int c = threadIdx.x; c < W; c += 256) {   // (every thread reads back what it wrote)
+    const float v = xr[c] * inv * (one_plus ? 1.0f + w[c] : w[c]);
+    out[(size_t)t * W + c] = from_f<T>(v);
+    if (out32) out32[(size_t)t * W + c] = v;
+  }
+}
+
+// ---------------------------------------------------------------------------------- q | k | v + bias, half-split rotary on queries and keys, page write
+// The pair (d, d + rot / 2) of a head's first rot values turns by position * freq[d], cos and sin times trig_mult; the values (columns from v_col, which may be the key columns: the
+// values are then the keys before rotation) pass.  A row's angles are worked out once for all heads.
+struct RopeHalfArgs {
+  const float *u;             // [rows, ld]: q [H * D] at 0, k [G * D] at H * D, v [G * Dv] at v_col
+  const float *qb, *kb, *vb;  // nullable
+  const float *freq;          // [rot / 2]
+  const int *tok_pos;
+  const long long *slot_mapping;
+  void *q_out, *k_cache, *v_cache;
+  int ld, v_col, H, G, D, Dv, rot, block_size;
+  float trig_mult;
+};
+template <class T> __global__ void __launch_bounds__(256) rope_half_cache_kernel(RopeHalfArgs a) {
+  extern __shared__ float trig[];  // cos [rot / 2] | sin [rot / 2]
+  const int t = blockIdx.x, tid = threadIdx.x, half = a.rot >> 1, per = a.D - half, nq = a.H * a.D;
+  const float pos = (float)a.tok_pos[t];
+  for (int i = tid; i < half; i += 256) {
+    float sn, cs;
+    sincosf(pos * a.freq[i], &sn, &cs);
+    trig[i] = cs * a.trig_mult;
+    trig[half + i] = sn * a.trig_mult;
+  }
+  __syncthreads();
+  const float *row = a.u + (size_t)t * a.ld;
+  const long long slot = a.slot_mapping[t];
+  const long long blk = slot / a.block_size;
+  const int off = (int)(slot % a.block_size);
+  const int items = (a.H + (slot >= 0 ? a.G : 0)) * per;   // of a head: `half` pairs, then the D - rot values that pass
+  for (int e = tid; e < items; e += 256) {
+    const int h = e / per, i = e - h * per;
+    const bool is_q = h < a.H;
+    const int g = h - a.H;
+    const float *x = row + (size_t)h * a.D;   // (key heads follow the query heads)
+    const float *b = is_q ? (a.qb ? a.qb + h * a.D : nullptr) : (a.kb ? a.kb + g * a.D : nullptr);
+    T *o = is_q ? (T *)a.q_out + (size_t)t * nq + (size_t)h * a.D : (T *)a.k_cache + (((size_t)blk * a.G + g) * a.block_size + off) * a.D;
+    const int j = i + half;
+    const float xj = x[j] + (b ? b[j] : 0.f);
+    if (i < half) {
+      const float xi = x[i] + (b ? b[i] : 0.f), cs = trig[i], sn = trig[half + i];
+      o[i] = from_f<T>(xi * cs - xj * sn);
+      o[j] = from_f<T>(xj * cs + xi * sn);
+    } else {
+      o[j] = from_f<T>(xj);
+    }
+  }
+  if (slot < 0) return;
+  const float *v = row + a.v_col;
+  for (int e = tid; e < a.G * a.Dv; e += 256) {
+    const int g = e / a.Dv, d = e - g * a.Dv;
+    ((T *)a.v_cache)[(((size_t)blk * a.G + g) * a.block_size + off) * a.Dv + d] = from_f<T>(v[e] + (a.vb ? a.vb[e] : 0.f));
+  }
+}
 // ---------------------------------------------------------------------------------- half-split rotary on f32 rows, in place (queries and keys of a recurrence)
 // u [rows, ld]: `heads` heads of D values from column col.  In the first `rot` dimensions of a head, (x_i, x_{i + rot / 2}) turns by position * freq[i]; then every value of
 // the head is multiplied by mult.  grid.y = 0: the range at q_col (mult 1), 1: the range at k_col (mult k_mult).
@@ -1773,6 +1856,31 @@ extern "C" int mrs_hyb_qkv_bias_temp_cache(const float *qkv, int ld, const float
   else if (dtype == 2) hipLaunchKernelGGL(qkv_bias_temp_cache_kernel<float>, dim3(rows), dim3(256), 0, S_(stream), a);
   else return fail("mrs_hyb_qkv_bias_temp_cache: dtype");
   return ok_or("mrs_hyb_qkv_bias_temp_cache");
+}
+
+/* x [rows, W] += scale * table[token] (table nullable, dtype) + step [W] (nullable); out (dtype) / out32 (f32, nullable) = the RMS norm of the new rows */
+extern "C" int mrs_hyb_pass_norm(float *x, const int *tokens, const void *table, int vocab, float scale, const float *step, const float *w, void *out, float *out32, int rows, int W,
+                                 float eps, int one_plus, int dtype, void *stream) {
+  if (rows <= 0) return 0;
+  if (!w || !out || (table && (!tokens || vocab <= 0))) return fail("mrs_hyb_pass_norm: a norm weight, an output and tokens beside a table");
+  if (dtype == 1) hipLaunchKernelGGL(pass_norm_kernel<mrs::bf16_t>, dim3(rows), dim3(256), 0, S_(stream), x, tokens, (const mrs::bf16_t *)table, vocab, scale, step, w, (mrs::bf16_t *)out, out32, W, eps, one_plus);
+  else if (dtype == 2) hipLaunchKernelGGL(pass_norm_kernel<float>, dim3(rows), dim3(256), 0, S_(stream), x, tokens, (const float *)table, vocab, scale, step, w, (float *)out, out32, W, eps, one_plus);
+  else return fail("mrs_hyb_pass_norm: dtype");
+  return ok_or("mrs_hyb_pass_norm");
+}
+/* u [rows, ld]: q [H * D] | k [G * D] and v [G * Dv] from column v_col (G * D columns at H * D: the values are the keys before rotation); biases nullable */
+extern "C" int mrs_hyb_rope_half_cache(const float *u, int ld, int v_col, const float *qb, const float *kb, const float *vb, const float *freq, float trig_mult, const int *tok_pos,
+                                       const long long *slot_mapping, void *q_out, void *k_cache, void *v_cache, int rows, int H, int G, int D, int Dv, int rot, int block_size,
+                                       int dtype, void *stream) {
+  if (rows <= 0) return 0;
+  if (H <= 0 || G <= 0 || H % G || D <= 0 || Dv <= 0 || rot < 0 || (rot & 1) || rot > D || block_size <= 0) return fail("mrs_hyb_rope_half_cache: head sizes (even rot <= dim, heads % kv_heads == 0)");
+  if (v_col < 0 || ld < (H + G) * D || ld < v_col + G * Dv) return fail("mrs_hyb_rope_half_cache: rows shorter than q | k | v");
+  if (rot > 8192) return fail("mrs_hyb_rope_half_cache: more than 8192 rotated dimensions");
+  RopeHalfArgs a{u, qb, kb, vb, freq, tok_pos, slot_mapping, q_out, k_cache, v_cache, ld, v_col, H, G, D, Dv, rot, block_size, trig_mult};
+  if (dtype == 1) hipLaunchKernelGGL(rope_half_cache_kernel<mrs::bf16_t>, dim3(rows), dim3(256), (size_t)rot * 4, S_(stream), a);
+  else if (dtype == 2) hipLaunchKernelGGL(rope_half_cache_kernel<float>, dim3(rows), dim3(256), (size_t)rot * 4, S_(stream), a);
+  else return fail("mrs_hyb_rope_half_cache: dtype");
+  return ok_or("mrs_hyb_rope_half_cache");
 }
 
 extern "C" int mrs_hyb_gather_rows(const float *x, const int *idx, float *out, int n, int W, void *stream) {

@@ -9,7 +9,7 @@
 //                        every entry one chain, or the segments of long portions side by side (end states and transitions from zero | identity, a carry, the outputs)
 //   exponential gates    capped log gates, the running maximum m, the step values e^{i - m'}, e^{f + m - m'} and e^{-m'} of every row
 //   head norm + gate     per-head output norm (optionally behind a normaliser column), shared or full weight, sigmoid / SiLU gate, rounded once for the out-projection
-//   normed average       x (+)= c (y1 / rms(y1) w1 + y2 / rms(y2) w2)
+//   normed average       x (+)= c (y1 / rms(y1) w1 + y2 / rms(y2) w2), optionally with the norm in front of the next sublayer
 //   squared ReLU, rounded column blocks
 //
 // Everything here is f32 arithmetic on f32 operands; T is only the type the results are rounded to for the next product.
@@ -485,8 +485,10 @@ template <class T> __global__ void __launch_bounds__(64) head_norm_gate_kernel(c
 }
 
 // ---------------------------------------------------------------------------------- x (+)= c (y1 / rms(y1) w1 + y2 / rms(y2) w2)
-__global__ void __launch_bounds__(256) norm_pair_add_kernel(float *__restrict__ x, int ldx, const float *__restrict__ y1, const float *__restrict__ w1, const float *__restrict__ y2,
-                                                            const float *__restrict__ w2, int W, float eps, float c, int accumulate) {
+// then (nullable, with NEXT): the norm weight in front of the next sublayer; the updated row leaves normed as well, rounded (out) and in f32 (out32, nullable)
+template <class T, bool NEXT> __global__ void __launch_bounds__(256) norm_pair_add_kernel(float *__restrict__ x, int ldx, const float *__restrict__ y1, const float *__restrict__ w1,
+                                                            const float *__restrict__ y2, const float *__restrict__ w2, int W, float eps, float c, int accumulate,
+                                                            const float *__restrict__ then, int one_plus, T *__restrict__ out, float *__restrict__ out32) {
   __shared__ float red[4];
   const int t = blockIdx.x;
   const float *a = y1 + (size_t)t * W, *b = y2 + (size_t)t * W;
@@ -494,10 +496,20 @@ __global__ void __launch_bounds__(256) norm_pair_add_kernel(float *__restrict__ 
   for (int k = threadIdx.x; k < W; k += 256) { s1 = fmaf(a[k], a[k], s1); s2 = fmaf(b[k], b[k], s2); }
   const float i1 = 1.0f / sqrtf(block_sum_256(s1, red) / (float)W + eps);
   const float i2 = 1.0f / sqrtf(block_sum_256(s2, red) / (float)W + eps);
+  float s3 = 0.f;
   for (int k = threadIdx.x; k < W; k += 256) {
     const float v = c * (a[k] * i1 * w1[k] + b[k] * i2 * w2[k]);
     float *xp = x + (size_t)t * ldx + k;
-    *xp = accumulate ? *xp + v : v;
+    const float n = accumulate ? *xp + v : v;
+    *xp = n;
+    if (NEXT) s3 = fmaf(n, n, s3);
+  }
+  if (!NEXT) return;
+  const float i3 = 1.0f / sqrtf(block_sum_256(s3, red) / (float)W + eps);
+  for (int k = threadIdx.x; k < W; k += 256) {   // (every thread reads back what it wrote)
+    const float v = x[(size_t)t * ldx + k] * i3 * (one_plus ? 1.0f + then[k] : then[k]);
+    out[(size_t)t * W + k] = from_f<T>(v);
+    if (out32) out32[(size_t)t * W + k] = v;
   }
 }
 
@@ -642,8 +654,18 @@ extern "C" int mrs_hyb_head_norm_gate(const float *y, int ldp, const float *mexp
 extern "C" int mrs_hyb_norm_pair_add(float *x, int ldx, const float *y1, const float *w1, const float *y2, const float *w2, int rows, int W, float eps, float c, int accumulate,
                                      void *stream) {
   if (rows <= 0) return 0;
-  hipLaunchKernelGGL(norm_pair_add_kernel, dim3(rows), dim3(256), 0, S_(stream), x, ldx, y1, w1, y2, w2, W, eps, c, accumulate);
+  hipLaunchKernelGGL((norm_pair_add_kernel<float, false>), dim3(rows), dim3(256), 0, S_(stream), x, ldx, y1, w1, y2, w2, W, eps, c, accumulate, nullptr, 0, nullptr, nullptr);
   return ok_or("mrs_hyb_norm_pair_add");
+}
+/* the same, and the norm in front of the next sublayer in the same launch: out (dtype) [rows, W] = x / rms(x) * (then | 1 + then) of the updated rows, out32 (nullable) in f32 */
+extern "C" int mrs_hyb_norm_pair_add_norm(float *x, int ldx, const float *y1, const float *w1, const float *y2, const float *w2, int rows, int W, float eps, float c, int accumulate,
+                                          const float *then, int one_plus, void *out, float *out32, int dtype, void *stream) {
+  if (rows <= 0) return 0;
+  if (!then || !out) return fail("mrs_hyb_norm_pair_add_norm: the next norm's weight and an output are needed");
+  if (dtype == 1) hipLaunchKernelGGL((norm_pair_add_kernel<mrs::bf16_t, true>), dim3(rows), dim3(256), 0, S_(stream), x, ldx, y1, w1, y2, w2, W, eps, c, accumulate, then, one_plus, (mrs::bf16_t *)out, out32);
+  else if (dtype == 2) hipLaunchKernelGGL((norm_pair_add_kernel<float, true>), dim3(rows), dim3(256), 0, S_(stream), x, ldx, y1, w1, y2, w2, W, eps, c, accumulate, then, one_plus, (float *)out, out32);
+  else return fail("mrs_hyb_norm_pair_add_norm: dtype");
+  return ok_or("mrs_hyb_norm_pair_add_norm");
 }
 
 extern "C" int mrs_hyb_round_cols(const float *u, int ldu, void *out, int rows, int n, int dtype, void *stream) {

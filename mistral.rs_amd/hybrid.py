@@ -21,7 +21,7 @@ import ctypes as C
 import json
 import math
 import os
-from dataclasses import dataclass, field
+from dataclasses import dataclass, field, replace
 from typing import Callable, Dict, List, Optional, Sequence
 
 import numpy as np
@@ -88,6 +88,18 @@ _SIGS = {
     "mrs_hyb_gelu_erf": [_vp, _vp, _i, _i, _i, _vp],
     "mrs_hyb_gemv_ep": [_vp] * 3 + [_i] * 7 + [_vp, _l, _i, _vp, _i, _i, _vp],
     "mrs_hyb_gla_decays": [_vp, _vp, _i, _i, _f, _vp],
+    "mrs_hyb_bonus_scan": [_vp, _i, _i, _i] + [_vp] * 12 + [_i] * 6 + [_vp],
+    "mrs_hyb_lightning_scan": [_vp, _i, _i, _i] + [_vp] * 11 + [_i] * 6 + [_vp],
+    "mrs_hyb_bonus_step": [_vp, _i, _i, _i, _i, _vp, _i] + [_vp] * 9 + [_i] * 5 + [_f, _i, _vp],
+    "mrs_hyb_lightning_step": [_vp, _i, _i, _i] + [_vp] * 6 + [_i] * 5 + [_vp],
+    "mrs_hyb_token_shift": [_vp] * 8 + [_i] * 4 + [_vp],
+    "mrs_hyb_tanh_round": [_vp, _vp, _i, _i, _i, _vp],
+    "mrs_hyb_rglru_scan": [_vp] * 7 + [_i] + [_vp] * 11 + [_i] * 7 + [_vp],
+    "mrs_hyb_rglru_step": [_vp] * 7 + [_i] + [_vp] * 6 + [_i] * 5 + [_vp],
+    "mrs_hyb_pass_norm": [_vp, _vp, _vp, _i, _f, _vp, _vp, _vp, _vp, _i, _i, _f, _i, _i, _vp],
+    "mrs_hyb_rope_half_cache": [_vp, _i, _i, _vp, _vp, _vp, _vp, _f] + [_vp] * 5 + [_i] * 8 + [_vp],
+    "mrs_hyb_norm_pair_add_norm": [_vp, _i, _vp, _vp, _vp, _vp, _i, _i, _f, _f, _i, _vp, _i, _vp, _vp, _i, _vp],
+    "mrs_hyb_gemm_scaled": [_vp, _vp, _vp] + [_i] * 8 + [_f, _vp],
     "mrs_hyb_gla_scan": [_vp, _i, _i, _i] + [_vp] * 11 + [_i] * 6 + [_f, _vp],
     "mrs_hyb_gla_step": [_vp] + [_i] * 6 + [_vp] * 8 + [_i] * 5 + [_f, _f, _f, _i, _vp],
     "mrs_hyb_gemm": [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _l, _i, _vp],
@@ -95,8 +107,9 @@ _SIGS = {
     "mrs_hyb_gemv_act": [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _l, _i, _vp, _vp, _i, _vp, _f, _f, _vp],
 }
 _RECUR = {"mrs_hyb_rmsnorm_pair", "mrs_hyb_delta_prep", "mrs_hyb_delta_step_prep", "mrs_hyb_delta_scan", "mrs_hyb_exp_gates", "mrs_hyb_head_norm_gate", "mrs_hyb_norm_pair_add", "mrs_hyb_round_cols",
-          "mrs_hyb_relu_sq"}   # launchers of csrc/hyb_recur.hip (their own error text)
-_LINATTN = {"mrs_hyb_gla_decays", "mrs_hyb_gla_scan", "mrs_hyb_gla_step"}   # launchers of csrc/hyb_linattn.hip
+          "mrs_hyb_relu_sq", "mrs_hyb_norm_pair_add_norm"}   # launchers of csrc/hyb_recur.hip (their own error text)
+_LINATTN = {"mrs_hyb_gla_decays", "mrs_hyb_gla_scan", "mrs_hyb_gla_step", "mrs_hyb_bonus_scan", "mrs_hyb_bonus_step", "mrs_hyb_lightning_scan", "mrs_hyb_lightning_step",
+            "mrs_hyb_token_shift", "mrs_hyb_tanh_round"}   # launchers of csrc/hyb_linattn.hip
 
 
 def _last_error(name: str) -> str:
@@ -104,6 +117,8 @@ def _last_error(name: str) -> str:
         return "mrs_hyb_recur_last_error"
     if name in _LINATTN:
         return "mrs_hyb_linattn_last_error"
+    if "rglru" in name:
+        return "mrs_hyb_rglru_last_error"
     if "latent_mfma" in name:
         return "mrs_hyb_latent_mfma_last_error"
     if "gem" in name:
@@ -326,6 +341,8 @@ class AttentionSpec:
     head_norm: bool = False    # the query / key norm runs per head with weights [dim] shared by the heads
     sink: bool = False         # the softmax's denominator has one more term e^{sink_h}, a learned number per head (tensor `sink`)
     head_gate: bool = False    # head h's output is multiplied by sigmoid(Wg h)_h, one logit per head (tensor `g` [heads, width])
+    bias: bool = False         # the projections have biases (tensors `q.b`, `k.b`, `v.b`)
+    values_are_keys: bool = False   # there is no value projection: the values are the keys as projected, before rotation (vdim = dim)
 
 
 @dataclass
@@ -353,11 +370,13 @@ class MlstmSpec:
 
 @dataclass
 class ParallelSpec:
-    """Two mixers side by side on the same input; the result is half the sum of their outputs, each normed over the model width (ParallelMixer)."""
+    """Two mixers side by side on the same input (ParallelMixer).  scales None: the result is half the sum of their outputs, each normed over the model width; else their outputs times
+    the two scales."""
     left_kind: str
     left: object
     right_kind: str
     right: object
+    scales: Optional[tuple] = None
 
 
 @dataclass
@@ -423,6 +442,30 @@ class GlaSpec:
     dim: int
     vdim: int
     tau: float
+
+
+@dataclass
+class LightningSpec:
+    """Decayed linear attention with SiLU operands and a norm over all heads (LightningMixer): S <- decay_h S + k v^T, o = S^T q."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: List[float]
+
+
+@dataclass
+class TimeMixSpec:
+    """Time mixing (TimeMixMixer): operands mixed with the row before, one decay per key channel from the data, a bonus for the current row."""
+    heads: int
+    dim: int
+
+
+@dataclass
+class RgLruSpec:
+    """A real-gated linear recurrent unit behind a short convolution, next to a GELU branch (RgLruMixer)."""
+    width: int
+    blocks: int
+    conv: int
 
 
 @dataclass
@@ -511,6 +554,7 @@ class LayerSpec:
     ff: Optional[object]       # MoeSpec | ClampedMoeSpec | DenseSpec | None
     prefix: str                # tensor-name prefix of the layer
     weights_of: Optional[int] = None   # index of the layer whose tensors (mixer, feed-forward, norms) this layer uses; its pages and state slots are its own
+    enter: Optional[int] = None        # number of the pass that starts with this layer: row `enter` of HybridSpec.step joins the stream in front of it (from pass 1 on behind the embedding rows)
 
 
 @dataclass
@@ -530,6 +574,7 @@ class HybridSpec:
     join_norms: bool = False     # sublayers read the residual row as it is; their outputs are normed (`norm1` / `norm2`) on the way into it: x += norm(sublayer(x))
     layer_scale: bool = False    # a sublayer's (normed) output is multiplied element by element by the tensors `ls1` / `ls2`
     embed_scale: float = 1.0     # the embedding rows are multiplied by this
+    step: Optional[str] = None   # tensor [passes, width]: one vector per pass through the layers that run several times (LayerSpec.enter)
     streams: int = 0             # > 0: that many residual streams with per-sublayer read / write / mixing weights (`hc1.*` / `hc2.*`: in [S], out [S], mix [S, S] from -> to)
 
 
@@ -714,10 +759,63 @@ def kebisun_spec(cfg: dict) -> HybridSpec:
                       embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)))
 
 
+def zumuzen_spec(cfg: dict) -> HybridSpec:
+    """config.json of a Zumuzen checkpoint -> the layer list in running order (a looped layer once per pass, with the first pass's tensors and pages / states of its own): plain-weight
+    RMS norms in front of the sublayers, mixers `rglru`, `parallel` (chunked attention beside decayed linear attention) and `parallel_2` (chunked attention with a sink whose values
+    are its keys, beside time mixing), dense SiLU-GLU feed-forwards.  Every size and every model-dependent constant comes from the file; a key that is absent switches its mechanism
+    off."""
+    def attention(i, m, values_are_keys, sink):
+        rot, mask = m.get("rot") or {}, m.get("mask") or {}
+        dims = int(rot.get("dims", 0) or 0)
+        H, G, D = int(m["heads"]), int(m.get("kv_heads", m["heads"])), int(m["dim"])
+        if dims % 2 or dims > D or H % G:
+            raise ValueError(f"Zumuzen: layer {i} rotates {dims} of {D} dimensions, {H} query heads read {G}")
+        return AttentionSpec(H, G, D, D if values_are_keys else int(m["vdim"]), float(m["scale"]), 0, 0, RotarySpec(dims, float(rot["base"]), rot.get("scaling"), "half") if dims else None,
+                             False, chunk=int(mask.get("size", 0) or 0), sink=sink, bias=True, values_are_keys=values_are_keys)
+    layers = []
+    for i, L in enumerate(cfg["layers"]):
+        m, kind = L["mixer"], L["type"]
+        if kind == "rglru":
+            mixer = RgLruSpec(int(m["width"]), int(m["blocks"]), int(m["conv"]))
+        elif kind == "parallel":
+            r = m["right"]
+            decay = [float(d) for d in r["decay"]]
+            if len(decay) != int(r["heads"]):
+                raise ValueError(f"Zumuzen: layer {i} lists {len(decay)} decays for {r['heads']} heads")
+            mixer = ParallelSpec("attention", attention(i, m["left"], False, False), "lightning", LightningSpec(int(r["heads"]), int(r["dim"]), int(r["vdim"]), decay))
+        elif kind == "parallel_2":
+            r = m["right"]
+            mixer = ParallelSpec("attention", attention(i, m["left"], True, True), "time_mix", TimeMixSpec(int(r["heads"]), int(r["dim"])),
+                                 (float(m["left_scale"]), float(m["right_scale"])))
+        else:
+            raise ValueError(f"Zumuzen: unknown layer type {kind!r}")
+        f = L.get("mlp")
+        ff = None
+        if f:
+            if f.get("kind") != "dense":
+                raise ValueError(f"Zumuzen: unknown feed-forward kind {f.get('kind')!r}")
+            ff = GluSpec(int(f["ff"]))
+        layers.append(LayerSpec("rglru" if kind == "rglru" else "parallel", mixer, ff, f"l{i}."))
+    loop = cfg.get("loop") or {}
+    start, stop, times = int(loop.get("start", 0)), int(loop.get("stop", 0)), int(loop.get("times", 1))
+    if not loop:
+        return HybridSpec(int(cfg["vocab"]), int(cfg["width"]), float(cfg["norm"]["eps"]), layers, norm="rms")
+    if not 0 <= start < stop <= len(layers) or times < 1:
+        raise ValueError(f"Zumuzen: layers {start} .. {stop} of {len(layers)} cannot run {times} times")
+    run = [replace(ls) for ls in layers[:start]]
+    for t in range(times):
+        for i in range(start, stop):
+            run.append(replace(layers[i], weights_of=i if t else None, enter=t if i == start else None))   # (the first pass's layers keep their indices)
+    return HybridSpec(int(cfg["vocab"]), int(cfg["width"]), float(cfg["norm"]["eps"]), run + layers[stop:], norm="rms", step="loop.step")
+
+
 # ------------------------------------------------------------------------------------------------------------------ mixers and feed-forwards
 class _Module:
     out_bias = None            # f32 bias of the module's last product, left to the caller (a norm that follows adds it while it reads the product)
-    wants_f32_input = False    # feed-forwards: the normed rows are needed in f32 too (routers)
+    wants_f32_input = False    # the normed rows are needed in f32 too (routers, token shifts): `h32` of `forward`
+    product = None             # mixers: attribute that holds the weight of the one product that makes everything of the input; `forward(u=)` takes that product's rows then
+    norms_next = False         # mixers: `forward(then=)` takes the norm weight in front of the next sublayer and returns that sublayer's input (rounded, f32 | None)
+    out_scale = 1.0            # mixers: the out-projection's result is multiplied by this
     defers_combine = False     # feed-forwards: `forward(defer=True)` returns routed outputs for the next launch to sum instead of summing them
 
     def __init__(self, model: "HybridDecoder"):
@@ -789,28 +887,44 @@ class Mamba2Mixer(_Module):
 class WindowAttention(_Module):
     """q, k, v projections (one product); plain-weight RMS norm over the WHOLE query and key projections; interleaved rotary on the first dims of every head; K / V into
     pages; softmax over the keys j <= i with i - j < window or j < keep_first (true positions throughout); out-projection.  Grouped heads: query head h reads key / value
-    head h // (heads / kv_heads); key and value head sizes are independent."""
+    head h // (heads / kv_heads); key and value head sizes are independent.  Options: biases on the projections, half-split rotary pairs (with a ramp over pair indices), values that
+    are the keys before rotation (no value projection), position chunks, a learned sink, a gate per head."""
+    product = "w_qkv"
 
     def __init__(self, model, spec: AttentionSpec, prefix: str):
         super().__init__(model)
         self.s, self.p = spec, prefix
         dev, bs, nb = model.device, model.block_size, model.num_blocks
+        self.half = spec.bias or spec.values_are_keys or (spec.rotary is not None and spec.rotary.layout == "half")   # rows go through the half-split rotary launch
+        if self.half and (spec.qk_norm or spec.head_norm or (spec.rotary is not None and spec.rotary.layout != "half")):
+            raise NotImplementedError(f"{prefix}: biases / keys as values / half-split rotary beside query and key norms or interleaved pairs")
+        if spec.heads % spec.kv_heads or (spec.values_are_keys and spec.vdim != spec.dim):
+            raise ValueError(f"{prefix}: heads % kv_heads must be 0, values that are keys have the keys' size")
         self.k_cache = torch.zeros(nb, spec.kv_heads, bs, spec.dim, dtype=model.torch_dtype, device=dev)
         self.v_cache = torch.zeros(nb, spec.kv_heads, bs, spec.vdim, dtype=model.torch_dtype, device=dev)
+        self.trig_mult = float(np.float32(spec.rotary.trig_mult)) if spec.rotary else 1.0
         self.freq = torch.from_numpy(spec.rotary.frequencies()).to(dev) if spec.rotary else torch.zeros(1, dtype=torch.float32, device=dev)
 
     def load(self, get):
         s, p = self.s, self.p
-        q, k, v = (get(p + n) for n in ("q", "k", "v"))
+        q, k = get(p + "q"), get(p + "k")
+        v = k if s.values_are_keys else get(p + "v")
         if q.shape[0] != s.heads * s.dim or k.shape[0] != s.kv_heads * s.dim or v.shape[0] != s.kv_heads * s.vdim:
             raise ValueError(f"{p}: projection shapes do not match the mixer's sizes")
-        parts = [q, k, v]
+        parts = [q, k] if s.values_are_keys else [q, k, v]
+        self.v_col = s.heads * s.dim + (0 if s.values_are_keys else s.kv_heads * s.dim)
+        self.qb = self.kb = self.vb = None
+        if s.bias:
+            self.qb, self.kb = self.w(get, p + "q.b", False).reshape(-1), self.w(get, p + "k.b", False).reshape(-1)
+            self.vb = self.kb if s.values_are_keys else self.w(get, p + "v.b", False).reshape(-1)
+            if (self.qb.numel(), self.kb.numel(), self.vb.numel()) != (q.shape[0], k.shape[0], v.shape[0]):
+                raise ValueError(f"{p}: projection biases do not match the mixer's sizes")
         if s.head_gate:
             parts.append(get(p + "g"))
             if tuple(parts[-1].shape) != (s.heads, q.shape[1]):
                 raise ValueError(f"{p}: the gate projection has one row per head")
         self.w_qkv = torch.cat(parts, 0).to(self.m.device, self.m.torch_dtype).contiguous()   # [q | k | v (| gate logits), W]
-        self.gate_col = s.heads * s.dim + s.kv_heads * (s.dim + s.vdim)
+        self.gate_col = sum(t.shape[0] for t in parts[:2 if s.values_are_keys else 3])
         self.w_o = self.w(get, p + "o", True)
         self.q_norm = self.w(get, p + "q.norm", False) if s.qk_norm else None
         self.k_norm = self.w(get, p + "k.norm", False) if s.qk_norm else None
@@ -828,13 +942,17 @@ class WindowAttention(_Module):
     def kv_bytes_per_token(self) -> int:
         return self.k_cache.element_size() * self.s.kv_heads * (self.s.dim + self.s.vdim)
 
-    def forward(self, h, x, b: RaggedBatch, accumulate: bool = True):
+    def forward(self, h, x, b: RaggedBatch, accumulate: bool = True, u=None):
         s, m = self.s, self.m
         T = b.rows
-        qkv = m.linear(h, self.w_qkv)
+        qkv = m.linear(h, self.w_qkv) if u is None else u
         q = torch.empty(T, s.heads * s.dim, dtype=m.torch_dtype, device=m.device)
-        _call("mrs_hyb_qk_headnorm_rope_cache" if s.head_norm else "mrs_hyb_qk_norm_rope_cache", qkv, qkv.stride(0), self.q_norm, self.k_norm, self.freq, b.tok_pos,
-              b.slot_mapping, q, self.k_cache, self.v_cache, T, s.heads, s.kv_heads, s.dim, s.vdim, s.rotary.dims if s.rotary else 0, m.block_size, m.spec.eps, m.dt)
+        if self.half:
+            _call("mrs_hyb_rope_half_cache", qkv, qkv.stride(0), self.v_col, self.qb, self.kb, self.vb, self.freq, self.trig_mult, b.tok_pos, b.slot_mapping, q, self.k_cache,
+                  self.v_cache, T, s.heads, s.kv_heads, s.dim, s.vdim, s.rotary.dims if s.rotary else 0, m.block_size, m.dt)
+        else:
+            _call("mrs_hyb_qk_headnorm_rope_cache" if s.head_norm else "mrs_hyb_qk_norm_rope_cache", qkv, qkv.stride(0), self.q_norm, self.k_norm, self.freq, b.tok_pos,
+                  b.slot_mapping, q, self.k_cache, self.v_cache, T, s.heads, s.kv_heads, s.dim, s.vdim, s.rotary.dims if s.rotary else 0, m.block_size, m.spec.eps, m.dt)
         o = torch.empty(T, s.heads * s.vdim, dtype=m.torch_dtype, device=m.device)
         if s.chunk or s.sink or s.head_gate:
             if s.window or s.keep_first:
@@ -846,7 +964,7 @@ class WindowAttention(_Module):
         else:
             _call("mrs_hyb_paged_window_attn", q, self.k_cache, self.v_cache, b.block_tables, b.tok_seq, b.tok_pos, o, T, s.heads, s.kv_heads, s.dim, s.vdim, m.block_size,
                   b.max_blocks, s.window, s.keep_first, s.scale, m.dt, b.seg_entry, b.seg_row0, b.seg_len, b.segments, RaggedBatch.SEGMENT)
-        m.linear(o, self.w_o, out=x, accumulate=accumulate)
+        m.linear(o, self.w_o, out=x, accumulate=accumulate, scale=self.out_scale)
 
 
 class TalkSigmoidAttention(_Module):
@@ -1354,12 +1472,26 @@ class LatentAttention(_Module):
         return pairs * self.MATRIX_TO_VECTOR_RATE * gain > rows * s.kv_rank * (s.dim + s.vdim)
 
 
+SCAN_WAVES = int(os.environ.get("MRS_GLA_WAVES", "4096"))   # waves per pass that a linear-attention scan aims at: enough segments for that, no more (each costs dim x vdim of carry)
+
+
+def scan_segments(b: RaggedBatch, heads: int, dim: int, vdim: int):
+    """(segment table, segments) of a linear-attention scan: one chain per entry when the entries fill the chip, else segments of 32 .. 512 rows, as short as SCAN_WAVES asks for"""
+    columns = 64 if dim <= 32 else 32 if dim <= 64 else 16                                 # value columns per wave of the scan
+    per = heads * -(-vdim // columns)
+    if b.host_lens is None or b.seg_rows <= 1 or b.entries * per >= SCAN_WAVES:
+        return b.entry_table(), b.entries
+    rows = 32
+    while rows < 512 and per * sum(-(-n // rows) for n in b.host_lens) > SCAN_WAVES:
+        rows *= 2
+    *table, n = b.segment_table(rows)
+    return table, n
+
+
 class GlaMixer(_Module):
     """v | k | q | gate | the decay projection's first step in one product; z = W_a2 (first step, rounded once) + bias, one logit per head and key channel;
     alpha = sigmoid(z)^(1 / tau); q times dim^(-1/2).  Per head the f32 state S [dim, vdim] (carried per slot): S <- diag(alpha) S + k v^T, o = S^T q; o / rms(o) per head times
     the weight `norm` [vdim] times silu(gate), output projection.  Long portions run their segments side by side (csrc/hyb_linattn.hip)."""
-
-    SCAN_WAVES = int(os.environ.get("MRS_GLA_WAVES", "4096"))   # waves per pass that a scan aims at: enough segments for that, no more (each costs dim x vdim of carry)
 
     def __init__(self, model, spec: GlaSpec, prefix: str):
         super().__init__(model)
@@ -1387,19 +1519,6 @@ class GlaMixer(_Module):
         if tuple(self.w_a2.shape) != (nk, self.rank) or self.b_a.numel() != nk or self.norm.numel() != s.vdim or tuple(self.w_o.shape) != (W, nv):
             raise ValueError(f"{p}: decay / norm / output shapes do not match the mixer's sizes")
 
-    def segments(self, b: RaggedBatch):
-        """(segment table, segments) of this step's scan: one chain per entry when the entries fill the chip, else segments of 32 .. 512 rows, as short as SCAN_WAVES asks for"""
-        s = self.s
-        columns = 64 if s.dim <= 32 else 32 if s.dim <= 64 else 16                             # value columns per wave of the scan
-        per = s.heads * -(-s.vdim // columns)
-        if b.host_lens is None or b.seg_rows <= 1 or b.entries * per >= self.SCAN_WAVES:
-            return b.entry_table(), b.entries
-        rows = 32
-        while rows < 512 and per * sum(-(-n // rows) for n in b.host_lens) > self.SCAN_WAVES:
-            rows *= 2
-        *table, n = b.segment_table(rows)
-        return table, n
-
     def forward(self, h, x, b: RaggedBatch, accumulate: bool = True):
         s, m = self.s, self.m
         T, dev = b.rows, m.device
@@ -1413,7 +1532,7 @@ class GlaMixer(_Module):
         else:
             z = m.linear(m.round_cols(u[:, self.a_col:], self.rank), self.w_a2)
             _call("mrs_hyb_gla_decays", z, self.b_a, T, z.shape[1], self.inv_tau)
-            table, nseg = self.segments(b)
+            table, nseg = scan_segments(b, s.heads, s.dim, s.vdim)
             y, carry, decay = torch.empty(T, nv, **f32), None, None
             if nseg > b.entries:
                 carry, decay = torch.empty(nseg, s.heads, s.dim, s.vdim, **f32), torch.empty(nseg, s.heads, s.dim, **f32)
@@ -1421,6 +1540,163 @@ class GlaMixer(_Module):
                   s.heads, s.dim, s.vdim, self.q_mult)
             _call("mrs_hyb_head_norm_gate", y, s.vdim, None, self.norm, 0, u[:, self.g_col:], u.stride(0), 2, o, T, s.heads, s.vdim, m.spec.eps, m.dt)
         m.linear(o, self.w_o, out=x, accumulate=accumulate)
+
+
+class LightningMixer(_Module):
+    """v | k | q | gate in one product; q, k, v through SiLU (as the scan reads them); per head the f32 state S [dim, vdim] (carried per slot): S <- decay_h S + k v^T, o = S^T q; the
+    concatenated heads over their common root mean square, times `norm` [heads * vdim], times sigmoid(gate), output projection.  The scan is csrc/hyb_linattn.hip's with one
+    decay per head."""
+    product = "w_in"
+
+    def __init__(self, model, spec: LightningSpec, prefix: str):
+        super().__init__(model)
+        self.s, self.p = spec, prefix
+        self.state = torch.zeros(model.state_slots, spec.heads, spec.dim, spec.vdim, dtype=torch.float32, device=model.device)
+        self.decay = torch.tensor(spec.decay, dtype=torch.float64).to(model.device, torch.float32)
+
+    def carried(self):
+        return (self.state,)
+
+    def state_bytes_per_slot(self) -> int:
+        return 4 * self.state[0].numel()
+
+    def load(self, get):
+        s, p, W = self.s, self.p, self.m.spec.width
+        nv, nk = s.heads * s.vdim, s.heads * s.dim
+        parts = [get(p + n) for n in ("v", "k", "q", "g")]
+        if [t.shape[0] for t in parts] != [nv, nk, nk, nv] or any(t.shape[1] != W for t in parts):
+            raise ValueError(f"{p}: projection shapes do not match the mixer's sizes")
+        self.w_in = torch.cat(parts, 0).to(self.m.device, self.m.torch_dtype).contiguous()     # [v | k | q | gate, W]
+        self.k_col, self.q_col, self.g_col = nv, nv + nk, nv + 2 * nk
+        self.norm, self.w_o = self.w(get, p + "norm", False).reshape(-1), self.w(get, p + "o", True)
+        if self.norm.numel() != nv or tuple(self.w_o.shape) != (W, nv):
+            raise ValueError(f"{p}: norm / output shapes do not match the mixer's sizes")
+
+    def forward(self, h, x, b: RaggedBatch, accumulate: bool = True, u=None):
+        s, m = self.s, self.m
+        T, f32 = b.rows, dict(dtype=torch.float32, device=m.device)
+        if u is None:
+            u = m.linear(h, self.w_in)                                      # f32 [T, v | k | q | gate]
+        y = torch.empty(T, s.heads * s.vdim, **f32)
+        if T == b.entries and b.seg_rows == 1:
+            _call("mrs_hyb_lightning_step", u, u.stride(0), self.k_col, self.q_col, self.decay, self.state, y, b.seq_start, b.seq_pos0, b.seq_slot, T, b.entries, s.heads, s.dim, s.vdim)
+        else:
+            table, nseg = scan_segments(b, s.heads, s.dim, s.vdim)
+            carry = decay = None
+            if nseg > b.entries:
+                carry, decay = torch.empty(nseg, s.heads, s.dim, s.vdim, **f32), torch.empty(nseg, s.heads, s.dim, **f32)
+            _call("mrs_hyb_lightning_scan", u, u.stride(0), self.k_col, self.q_col, self.decay, self.state, y, b.seq_pos0, b.seq_slot, *table, carry, decay, T, b.entries, nseg,
+                  s.heads, s.dim, s.vdim)
+        yn = m.norm(y, self.norm, one_plus=False, gate=u[:, self.g_col:], gate_after=2)
+        m.linear(yn, self.w_o, out=x, accumulate=accumulate, scale=self.out_scale)
+
+
+class TimeMixMixer(_Module):
+    """Every operand reads a mix of its own of the row and the row before it (the slot's row at an entry's start): h + (h' - h) mu_s.  v, k, r, gate are four products in one launch, the
+    decay a two-step projection: w = exp(-exp(W_w2 tanh(W_w1 mix) + w0)) per head and key channel.  Per head the f32 state S [dim, dim]: o = (S + diag(u) k v^T)^T r, then
+    S <- diag(w) S + k v^T.  o / rms(o) per head, times `norm` [heads * dim], times silu(gate), output projection.  Carries S and the last row (f32) per slot."""
+    wants_f32_input = True
+
+    def __init__(self, model, spec: TimeMixSpec, prefix: str):
+        super().__init__(model)
+        self.s, self.p = spec, prefix
+        self.state = torch.zeros(model.state_slots, spec.heads, spec.dim, spec.dim, dtype=torch.float32, device=model.device)
+        self.last = torch.zeros(model.state_slots, model.spec.width, dtype=torch.float32, device=model.device)
+
+    def carried(self):
+        return (self.state, self.last)
+
+    def state_bytes_per_slot(self) -> int:
+        return 4 * (self.state[0].numel() + self.last[0].numel())
+
+    def load(self, get):
+        s, p, W = self.s, self.p, self.m.spec.width
+        n = s.heads * s.dim
+        names = ("v", "k", "r", "g")
+        parts = [get(p + q) for q in names]
+        if any(tuple(t.shape) != (n, W) for t in parts):
+            raise ValueError(f"{p}: projection shapes do not match the mixer's sizes")
+        self.w_in = torch.stack(parts).to(self.m.device, self.m.torch_dtype).contiguous()      # [4, heads * dim, W]: v, k, r, gate
+        self.mu = torch.stack([get(f"{p}mu.{q}").reshape(-1) for q in names + ("w",)]).to(self.m.device, torch.float32).contiguous()
+        self.w1, self.w2, self.w_o = self.w(get, p + "w1", True), self.w(get, p + "w2", True), self.w(get, p + "o", True)
+        self.w0, self.bonus, self.norm = (self.w(get, p + q, False).reshape(-1) for q in ("w0", "u", "norm"))
+        if self.mu.shape[1] != W or self.w1.shape[1] != W or tuple(self.w2.shape) != (n, self.w1.shape[0]) or tuple(self.w_o.shape) != (W, n) or \
+                any(t.numel() != n for t in (self.w0, self.bonus, self.norm)):
+            raise ValueError(f"{p}: mix / decay / bonus / norm / output shapes do not match the mixer's sizes")
+
+    def forward(self, h, x, b: RaggedBatch, accumulate: bool = True, h32=None):
+        s, m = self.s, self.m
+        T, W, n, f32 = b.rows, m.spec.width, self.s.heads * self.s.dim, dict(dtype=torch.float32, device=self.m.device)
+        mix = torch.empty(5, T, W, dtype=m.torch_dtype, device=m.device)
+        _call("mrs_hyb_token_shift", h32, self.mu, self.last, mix, b.tok_seq, b.seq_start, b.seq_pos0, b.seq_slot, T, W, 5, m.dt)
+        u = torch.empty(T, 4 * n, **f32)                                    # v | k | r | gate
+        _call("mrs_hyb_gemm_batched", mix, self.w_in, u, T, n, W, W, W, 4 * n, m.dt, 4, T * W, n * W, n, 0)
+        a1 = m.linear(mix[4], self.w1)
+        o = torch.empty(T, n, dtype=m.torch_dtype, device=m.device)
+        if T == b.entries and b.seg_rows == 1:   # every entry brings one row: decays, read-out, state, head norm and gate in one launch
+            _call("mrs_hyb_bonus_step", u, u.stride(0), n, 2 * n, 3 * n, a1, a1.shape[1], self.w2, self.w0, self.bonus, self.norm, self.state, o, b.seq_start, b.seq_pos0, b.seq_slot,
+                  T, b.entries, s.heads, s.dim, s.dim, m.spec.eps, m.dt)
+        else:
+            t1 = torch.empty(T, a1.shape[1], dtype=m.torch_dtype, device=m.device)
+            _call("mrs_hyb_tanh_round", a1, t1, T, a1.shape[1], m.dt)
+            z = m.linear(t1, self.w2)
+            _call("mrs_hyb_gla_decays", z, self.w0, T, n, 0.0)
+            table, nseg = scan_segments(b, s.heads, s.dim, s.dim)
+            y, carry, decay = torch.empty(T, n, **f32), None, None
+            if nseg > b.entries:
+                carry, decay = torch.empty(nseg, s.heads, s.dim, s.dim, **f32), torch.empty(nseg, s.heads, s.dim, **f32)
+            _call("mrs_hyb_bonus_scan", u, u.stride(0), n, 2 * n, z, self.bonus, self.state, y, b.seq_pos0, b.seq_slot, *table, carry, decay, T, b.entries, nseg, s.heads, s.dim, s.dim)
+            _call("mrs_hyb_head_norm_gate", y, s.dim, None, self.norm, 1, u[:, 3 * n:], u.stride(0), 2, o, T, s.heads, s.dim, m.spec.eps, m.dt)
+        m.linear(o, self.w_o, out=x, accumulate=accumulate, scale=self.out_scale)
+
+
+class RgLruMixer(_Module):
+    """y | x branches in one product; u = causal convolution of x + bias (its own bias, no activation; the last taps - 1 inputs ride in the slot); per channel part the gates
+    r = sigmoid(ra u + ra.b), i = sigmoid(ri u + ri.b); a = exp(-8 r softplus(lam)); S <- a S + sqrt(1 - a^2) i u per channel, f32, carried per slot; the states times
+    gelu_tanh(y + bias), output projection.  Segments of a portion run side by side (csrc/hyb_rglru.hip)."""
+    ROWS = 64   # rows per segment of the scan
+
+    def __init__(self, model, spec: RgLruSpec, prefix: str):
+        super().__init__(model)
+        self.s, self.p = spec, prefix
+        if spec.width % spec.blocks or spec.conv < 1:
+            raise ValueError(f"{prefix}: width % blocks must be 0; at least one tap")
+        self.conv_state = torch.zeros(model.state_slots, spec.width, max(spec.conv - 1, 1), dtype=torch.float32, device=model.device)
+        self.state = torch.zeros(model.state_slots, spec.width, dtype=torch.float32, device=model.device)
+
+    def carried(self):
+        return (self.conv_state, self.state)
+
+    def state_bytes_per_slot(self) -> int:
+        return 4 * (self.conv_state[0].numel() + self.state[0].numel())
+
+    def load(self, get):
+        s, p, W, C = self.s, self.p, self.m.spec.width, self.s.width
+        y, xw = get(p + "y"), get(p + "x")
+        part = C // s.blocks
+        self.w_in = torch.cat([y, xw], 0).to(self.m.device, self.m.torch_dtype).contiguous()    # [y | x, W]
+        self.ra, self.ri, self.w_o = self.w(get, p + "ra", True), self.w(get, p + "ri", True), self.w(get, p + "o", True)
+        self.conv_w = self.w(get, p + "conv", False)
+        self.yb, self.xb, self.conv_b, self.ba, self.bi, self.lam = (self.w(get, p + q, False).reshape(-1) for q in ("y.b", "x.b", "conv.b", "ra.b", "ri.b", "lam"))
+        if tuple(y.shape) != (C, W) or tuple(xw.shape) != (C, W) or tuple(self.ra.shape) != (s.blocks, part, part) or self.ra.shape != self.ri.shape or \
+                tuple(self.conv_w.shape) != (C, s.conv) or tuple(self.w_o.shape) != (W, C) or any(t.numel() != C for t in (self.yb, self.xb, self.conv_b, self.ba, self.bi, self.lam)):
+            raise ValueError(f"{p}: projection / convolution / gate shapes do not match the mixer's sizes")
+
+    def forward(self, h, x, b: RaggedBatch, accumulate: bool = True):
+        s, m, C = self.s, self.m, self.s.width
+        T, f32 = b.rows, dict(dtype=torch.float32, device=self.m.device)
+        yx = m.linear(h, self.w_in)                                         # f32 [T, y | x]
+        u = torch.empty(T, C, **f32)
+        _call("mrs_hyb_conv", yx[:, C:], yx.stride(0), self.xb, self.conv_w, self.conv_b, self.conv_state, b.tok_seq, b.seq_start, b.seq_pos0, b.seq_slot, u, T, b.entries, C, s.conv, 0)
+        o = torch.empty(T, C, dtype=m.torch_dtype, device=m.device)
+        gates = (self.ra, self.ri, self.ba, self.bi, self.lam, yx, yx.stride(0), self.yb, self.state)
+        if T == b.entries and b.seg_rows == 1:
+            _call("mrs_hyb_rglru_step", u, *gates, o, b.seq_start, b.seq_pos0, b.seq_slot, T, b.entries, C, s.blocks, m.dt)
+        else:
+            _, row0, length, ent0, n = b.segment_table(self.ROWS)
+            local, prod, start = torch.empty(T, C, **f32), torch.empty(T, C, **f32), torch.empty(n, C, **f32)
+            _call("mrs_hyb_rglru_scan", u, *gates, local, prod, start, o, b.seq_pos0, b.seq_slot, row0, length, ent0, T, b.entries, n, min(self.ROWS, max(b.host_lens)), C, s.blocks, m.dt)
+        m.linear(o, self.w_o, out=x, accumulate=accumulate, scale=self.out_scale)
 
 
 class GluFeedForward(_Module):
@@ -1606,14 +1882,20 @@ class MlstmMixer(_Module):
 
 
 class ParallelMixer(_Module):
-    """Two registered mixers (tensors under `left.` / `right.`) read the same input; result = (left / rms(left) * w_left + right / rms(right) * w_right) / 2, the norms over
-    the model width with plain weights `left.out` / `right.out`.  Pages, taps and states are the sub-mixers' own."""
+    """Two registered mixers (tensors under `left.` / `right.`) read the same input.  Result: (left / rms(left) * w_left + right / rms(right) * w_right) / 2, the norms over the model
+    width with plain weights `left.out` / `right.out`; or (ParallelSpec.scales) scale_left left + scale_right right, each out-projection adding its share to the stream.  Pages,
+    taps and states are the sub-mixers' own.  When both make everything from one product of the input, the two products are one."""
 
     def __init__(self, model, spec: ParallelSpec, prefix: str):
         super().__init__(model)
         self.s, self.p = spec, prefix
         self.left = MIXERS[spec.left_kind](model, spec.left, prefix + "left.")
         self.right = MIXERS[spec.right_kind](model, spec.right, prefix + "right.")
+        self.wants_f32_input = self.left.wants_f32_input or self.right.wants_f32_input
+        self.norms_next = spec.scales is None
+        self.joint = self.left.product is not None and self.right.product is not None
+        if spec.scales is not None:
+            self.left.out_scale, self.right.out_scale = (float(v) for v in spec.scales)
 
     def carried(self):
         return tuple(self.left.carried()) + tuple(self.right.carried())
@@ -1627,22 +1909,45 @@ class ParallelMixer(_Module):
     def load(self, get):
         self.left.load(get)
         self.right.load(get)
-        self.w_left, self.w_right = self.w(get, self.p + "left.out", False), self.w(get, self.p + "right.out", False)
-        if self.w_left.numel() != self.m.spec.width or self.w_right.numel() != self.m.spec.width:
-            raise ValueError(f"{self.p}: the output norms run over the model width")
+        if self.joint:
+            wl, wr = getattr(self.left, self.left.product), getattr(self.right, self.right.product)
+            self.w_in, self.cut = torch.cat([wl, wr], 0), wl.shape[0]
+            setattr(self.left, self.left.product, self.w_in[:self.cut])
+            setattr(self.right, self.right.product, self.w_in[self.cut:])
+        if self.s.scales is None:
+            self.w_left, self.w_right = self.w(get, self.p + "left.out", False), self.w(get, self.p + "right.out", False)
+            if self.w_left.numel() != self.m.spec.width or self.w_right.numel() != self.m.spec.width:
+                raise ValueError(f"{self.p}: the output norms run over the model width")
 
     def share_from(self, other: "ParallelMixer") -> None:
+        for k, v in other.__dict__.items():
+            if k not in ("left", "right", "m"):
+                setattr(self, k, v)
         self.left.share_from(other.left)
         self.right.share_from(other.right)
-        self.w_left, self.w_right = other.w_left, other.w_right
 
-    def forward(self, h, x, b: RaggedBatch, accumulate: bool = True):
+    def forward(self, h, x, b: RaggedBatch, accumulate: bool = True, h32=None, then=None):
         m = self.m
+        kl, kr = ({"h32": h32} if c.wants_f32_input else {} for c in (self.left, self.right))
+        if self.joint:
+            u = m.linear(h, self.w_in)
+            kl["u"], kr["u"] = u[:, :self.cut], u[:, self.cut:]
+        if self.s.scales is not None:
+            self.left.forward(h, x, b, accumulate=accumulate, **kl)
+            self.right.forward(h, x, b, accumulate=True, **kr)
+            return None
         yl = torch.empty(b.rows, m.spec.width, dtype=torch.float32, device=m.device)
         yr = torch.empty_like(yl)
-        self.left.forward(h, yl, b, accumulate=False)
-        self.right.forward(h, yr, b, accumulate=False)
-        _call("mrs_hyb_norm_pair_add", x, x.stride(0), yl, self.w_left, yr, self.w_right, b.rows, m.spec.width, m.spec.eps, 0.5, int(accumulate))
+        self.left.forward(h, yl, b, accumulate=False, **kl)
+        self.right.forward(h, yr, b, accumulate=False, **kr)
+        if then is None:
+            _call("mrs_hyb_norm_pair_add", x, x.stride(0), yl, self.w_left, yr, self.w_right, b.rows, m.spec.width, m.spec.eps, 0.5, int(accumulate))
+            return None
+        weight, one_plus, want32 = then
+        out = torch.empty(b.rows, m.spec.width, dtype=m.torch_dtype, device=m.device)
+        out32 = torch.empty_like(yl) if want32 else None
+        _call("mrs_hyb_norm_pair_add_norm", x, x.stride(0), yl, self.w_left, yr, self.w_right, b.rows, m.spec.width, m.spec.eps, 0.5, int(accumulate), weight, int(one_plus), out, out32, m.dt)
+        return out, out32
 
 
 class UngatedMoe(_Module):
@@ -1703,7 +2008,7 @@ class UngatedMoe(_Module):
 
 
 MIXERS: Dict[str, Callable] = {"delta_rule": DeltaRuleMixer, "mlstm": MlstmMixer, "parallel": ParallelMixer, "mamba2": Mamba2Mixer, "attention": WindowAttention, "talk_attention": TalkSigmoidAttention, "sink_attention": GatedSinkAttention,
-                               "retention": RetentionMixer, "latent_attention": LatentAttention, "gla": GlaMixer}
+                               "retention": RetentionMixer, "latent_attention": LatentAttention, "gla": GlaMixer, "lightning": LightningMixer, "time_mix": TimeMixMixer, "rglru": RgLruMixer}
 FEED_FORWARDS: Dict[str, Callable] = {"moe_topk_softmax_relu2": UngatedMoe, "moe_ungated": UngatedMoe, "moe": SigmoidMoe, "moe_softmax_clamped": ClampedSoftmaxMoe, "dense_xielu": XieluFeedForward, "dense_glu_silu": GluFeedForward}
 
 
@@ -1761,6 +2066,13 @@ class HybridDecoder:
         if tuple(self.embed.shape) != (sp.vocab, sp.width) or tuple(self.head.shape) != (sp.vocab, sp.width):
             raise ValueError("embedding / head shapes do not match vocab x width")
         self.embed_norm = norm(sp.embed_norm) if sp.embed_norm else None
+        passes = [ls.enter for ls in sp.layers if ls.enter is not None]
+        if passes:
+            if sp.embed_norm or sp.post_norms or sp.join_norms or sp.parallel_sublayers or sp.streams or sp.residual_mult != 1.0 or sp.norm not in ("rms", "rms_one_plus"):
+                raise NotImplementedError("layers that run several times are built for RMS norms in front of the sublayers of one plain stream")
+            self.step = f32(sp.step)
+            if self.step.dim() != 2 or self.step.shape[0] <= max(passes) or self.step.shape[1] != sp.width:
+                raise ValueError(f"{sp.step}: one vector of the model's width per pass")
         S = max(1, sp.streams)
         self.ones = torch.ones(S, dtype=torch.float32, device=self.device)
 
@@ -1804,9 +2116,9 @@ class HybridDecoder:
         return model
 
     # ---- building blocks on the current stream
-    def norm(self, x, w, one_plus: bool, parts: int = 1, want32: bool = False, gate=None, gate_after: bool = False):
-        """RMS norm of every row (in `parts` equal pieces; w None: no weight); gate [rows, >= width]: the row is multiplied by silu(gate) first, or (gate_after) the
-        normed row is."""
+    def norm(self, x, w, one_plus: bool, parts: int = 1, want32: bool = False, gate=None, gate_after: int = 0):
+        """RMS norm of every row (in `parts` equal pieces; w None: no weight); gate [rows, >= width]: the row is multiplied by silu(gate) first (gate_after 0), or the normed row is
+        (1), or by sigmoid(gate) (2)."""
         rows, width = x.shape
         out = torch.empty(rows, width, dtype=self.torch_dtype, device=self.device)
         out32 = torch.empty(rows, width, dtype=torch.float32, device=self.device) if want32 else None
@@ -1873,6 +2185,16 @@ class HybridDecoder:
             return self.layer_norm(x, wb, want32)
         return self.norm(x, wb[0], one_plus=self.spec.norm == "rms_one_plus", want32=want32)
 
+    def enter_pass(self, x, t: int, b: RaggedBatch, wb, want32: bool = False):
+        """What joins the stream in front of pass t through the layers that run several times (from the second pass on the embedding rows, then the pass's step vector), and the norm in
+        front of the pass's first sublayer, in one launch; returns like `pre_norm`."""
+        rows, width = x.shape
+        out = torch.empty(rows, width, dtype=self.torch_dtype, device=self.device)
+        out32 = torch.empty(rows, width, dtype=torch.float32, device=self.device) if want32 else None
+        _call("mrs_hyb_pass_norm", x, b.tokens, self.embed if t else None, self.spec.vocab, self.spec.embed_scale, self.step[t], wb[0], out, out32, rows, width, self.spec.eps,
+              int(self.spec.norm == "rms_one_plus"), self.dt)
+        return (out, out32) if want32 else out
+
     def pre_norm_pair(self, x, wb1, wb2, want32: bool = False):
         """The norms in front of two sublayers that read the same rows: one pass, one root mean square, two weights.  Returns (first, second, second in f32 | None)."""
         if self.spec.norm == "layer":
@@ -1926,14 +2248,16 @@ class HybridDecoder:
         _call("mrs_hyb_gemv_ep", a, w, out, M, N, w.shape[-1], a.stride(0), w.stride(-2), out.stride(0), self.dt, row_group, w.stride(0) if row_group is not None else 0,
               2 if src_row is not None else 0, src_row, src_div, ep)
 
-    def linear(self, a, w, out=None, accumulate: bool = False, dtype_code: Optional[int] = None):
-        """out (f32 [M, N]) (+)= a [M, K] . w [N, K]^T"""
+    def linear(self, a, w, out=None, accumulate: bool = False, dtype_code: Optional[int] = None, scale: float = 1.0):
+        """out (f32 [M, N]) (+)= scale * a [M, K] . w [N, K]^T"""
         M, K = a.shape
         N = w.shape[0]
         if out is None:
             out = torch.empty(M, N, dtype=torch.float32, device=self.device)
         dt = dtype_code or self.dt
-        if M <= self.GEMV_ROWS:
+        if scale != 1.0:
+            _call("mrs_hyb_gemm_scaled", a, w, out, M, N, K, a.stride(0), w.stride(0), out.stride(0), dt, int(accumulate), scale)
+        elif M <= self.GEMV_ROWS:
             _call("mrs_hyb_gemv", a, w, out, M, N, K, a.stride(0), w.stride(0), out.stride(0), dt, int(accumulate), None, 0, 0, None, None, 1)
         else:
             _call("mrs_hyb_gemm", a, w, out, M, N, K, a.stride(0), w.stride(0), out.stride(0), dt, int(accumulate), None, 0, 0, 0)
@@ -1995,9 +2319,16 @@ class HybridDecoder:
                 l.mixer.forward(h1, x, b)
                 l.ff.forward(h2, h32, x, b)
             else:
-                l.mixer.forward(self.pre_norm(x, l.norm1), x, b)
+                want32 = l.mixer.wants_f32_input
+                h = self.enter_pass(x, l.spec.enter, b, l.norm1, want32) if l.spec.enter is not None else self.pre_norm(x, l.norm1, want32)
+                h, kw = (h[0], {"h32": h[1]}) if want32 else (h, {})
+                if l.ff and l.mixer.norms_next:   # the launch that adds the mixer's result to the stream norms the new rows for the feed-forward
+                    h, h32 = l.mixer.forward(h, x, b, then=(l.norm2[0], sp.norm == "rms_one_plus", l.ff.wants_f32_input), **kw)
+                else:
+                    l.mixer.forward(h, x, b, **kw)
+                    if l.ff:
+                        h, h32 = self.pre_norm(x, l.norm2, want32=True) if l.ff.wants_f32_input else (self.pre_norm(x, l.norm2), None)
                 if l.ff:
-                    h, h32 = self.pre_norm(x, l.norm2, want32=True)
                     l.ff.forward(h, h32, x, b)
             if self.trace_layers is not None:
                 self.trace_layers.append(x.clone())
@@ -2154,11 +2485,12 @@ def synthetic_weights(spec: HybridSpec, device, seed: int = 0) -> Callable[[str]
     def new_mixer_shapes(p, m) -> bool:
         """delta-rule, matrix-memory, parallel and chunked / gated attention mixers; False: `m` is of another kind"""
         if isinstance(m, ParallelSpec):
-            shapes.update({p + "left.out": (W,), p + "right.out": (W,)})
-            norm_like.update({p + "left.out", p + "right.out"})
+            if m.scales is None:
+                shapes.update({p + "left.out": (W,), p + "right.out": (W,)})
+                norm_like.update({p + "left.out", p + "right.out"})
             for side, sub in (("left.", m.left), ("right.", m.right)):
                 if not new_mixer_shapes(p + side, sub):
-                    raise ValueError("synthetic_weights: a parallel mixer's sides are attention, delta-rule or matrix-memory mixers")
+                    raise ValueError("synthetic_weights: a parallel mixer's sides are attention, delta-rule, matrix-memory, decayed linear attention or time mixing")
         elif isinstance(m, DeltaRuleSpec):
             nqk, nv, rank = m.kv_heads * m.dim, m.heads * m.vdim, max(8, min(128, W // 16))
             for n, rows in (("q", nqk), ("k", nqk), ("v", nv)):
@@ -2173,9 +2505,30 @@ def synthetic_weights(spec: HybridSpec, device, seed: int = 0) -> Callable[[str]
             nk, nv = m.heads * m.dim, m.heads * m.vdim
             shapes.update({p + "q": (nk, W), p + "k": (nk, W), p + "v": (nv, W), p + "g": (nv, W), p + "o": (W, nv), p + "norm": (nv,), p + "i": (m.heads, W), p + "i.b": (m.heads,),
                            p + "f": (m.heads, W), p + "f.b": (m.heads,)})
-        elif isinstance(m, AttentionSpec) and (m.head_norm or m.sink or m.head_gate):
-            shapes.update({p + "q": (m.heads * m.dim, W), p + "k": (m.kv_heads * m.dim, W), p + "v": (m.kv_heads * m.vdim, W), p + "o": (W, m.heads * m.vdim),
-                           p + "q.norm": (m.dim if m.head_norm else m.heads * m.dim,), p + "k.norm": (m.dim if m.head_norm else m.kv_heads * m.dim,)})
+        elif isinstance(m, LightningSpec):
+            nk, nv = m.heads * m.dim, m.heads * m.vdim
+            shapes.update({p + "q": (nk, W), p + "k": (nk, W), p + "v": (nv, W), p + "g": (nv, W), p + "o": (W, nv), p + "norm": (nv,)})
+        elif isinstance(m, TimeMixSpec):
+            n, rank = m.heads * m.dim, max(8, min(128, W // 16))
+            for q in ("r", "k", "v", "g"):
+                shapes.update({p + q: (n, W), p + "mu." + q: (W,)})
+            shapes.update({p + "mu.w": (W,), p + "w1": (rank, W), p + "w2": (n, rank), p + "w0": (n,), p + "u": (m.heads, m.dim), p + "norm": (n,), p + "o": (W, n)})
+            step_like.add(p + "w0")
+            norm_like.add(p + "norm")
+        elif isinstance(m, RgLruSpec):
+            part = m.width // m.blocks
+            shapes.update({p + "y": (m.width, W), p + "y.b": (m.width,), p + "x": (m.width, W), p + "x.b": (m.width,), p + "conv": (m.width, m.conv), p + "conv.b": (m.width,),
+                           p + "ra": (m.blocks, part, part), p + "ra.b": (m.blocks, part), p + "ri": (m.blocks, part, part), p + "ri.b": (m.blocks, part), p + "lam": (m.width,),
+                           p + "o": (W, m.width)})
+            step_like.add(p + "lam")
+        elif isinstance(m, AttentionSpec) and (m.head_norm or m.sink or m.head_gate or m.bias or m.values_are_keys):
+            shapes.update({p + "q": (m.heads * m.dim, W), p + "k": (m.kv_heads * m.dim, W), p + "o": (W, m.heads * m.vdim)})
+            if not m.values_are_keys:
+                shapes[p + "v"] = (m.kv_heads * m.vdim, W)
+            if m.qk_norm:
+                shapes.update({p + "q.norm": (m.dim if m.head_norm else m.heads * m.dim,), p + "k.norm": (m.dim if m.head_norm else m.kv_heads * m.dim,)})
+            if m.bias:
+                shapes.update({p + n + ".b": (shapes[p + n][0],) for n in (("q", "k") if m.values_are_keys else ("q", "k", "v"))})
             if m.sink:
                 shapes[p + "sink"] = (m.heads,)
             if m.head_gate:
@@ -2185,6 +2538,9 @@ def synthetic_weights(spec: HybridSpec, device, seed: int = 0) -> Callable[[str]
         return True
 
     norm_like = set()   # plain-weight norms besides the layers' own: drawn around one
+    step_like = set()   # logarithms of slow decays
+    if spec.step:
+        shapes[spec.step] = (1 + max(ls.enter for ls in spec.layers if ls.enter is not None), W)
     for ls in spec.layers:
         p, m = ls.prefix, ls.mixer
         if ls.weights_of is not None:
@@ -2265,6 +2621,10 @@ def synthetic_weights(spec: HybridSpec, device, seed: int = 0) -> Callable[[str]
         if name.endswith(("q.norm", "k.norm", "dkv.norm", "dq.norm")) or last == "D" or name.endswith(("mix.norm", "left.norm", "right.norm")) or name in norm_like or \
                 (name in norm_names and spec.norm in ("layer", "layer_plain", "rms")):
             r = 1.0 + 0.1 * r
+        elif name == spec.step or ".mu." in name:
+            r = 0.5 + 0.1 * r if ".mu." in name else 0.1 * r
+        elif name in step_like:
+            r = -3.0 + 0.5 * r
         elif name.endswith("f.b"):
             r = 3.0 + 0.5 * r      # forget gates mostly open
         elif last == "mix" and len(shape) == 2 and shape[0] == shape[1] == spec.streams:
@@ -2295,7 +2655,7 @@ def synthetic_weights(spec: HybridSpec, device, seed: int = 0) -> Callable[[str]
     return get
 
 
-SPEC_READERS: Dict[str, Callable[[dict], HybridSpec]] = {"Gekilix": gekilix_spec, "Sobunex": sobunex_spec, "Setopel": setopel_spec, "Gifopel": gifopel_spec, "Kebisun": kebisun_spec}
+SPEC_READERS: Dict[str, Callable[[dict], HybridSpec]] = {"Gekilix": gekilix_spec, "Sobunex": sobunex_spec, "Setopel": setopel_spec, "Gifopel": gifopel_spec, "Kebisun": kebisun_spec, "Zumuzen": zumuzen_spec}
 
 
 class HybridCache:

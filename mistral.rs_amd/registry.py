@@ -46,6 +46,12 @@ def _load_kebisun(path: str, device, dtype: str = "bfloat16", **kw):
     return HybridDecoder.from_pretrained(path, device, dtype, **kw)
 
 
+@register("Zumuzen")
+def _load_zumuzen(path: str, device, dtype: str = "bfloat16", **kw):
+    from .hybrid import HybridDecoder
+    return HybridDecoder.from_pretrained(path, device, dtype, **kw)
+
+
 @register("llama")
 def _load_llama_gguf(path: str, device, dtype: str = "bfloat16", **kw):
     from .gguf.archive import load_llama
