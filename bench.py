@@ -1312,7 +1312,7 @@ def kebisun_leg(a, dev):
     prompt attention and the recurrences run on the f32 vector ALU in both designs and are priced in FLOP/s of the work done)."""
     import torch
     from mistralrs_amd.hybrid import (GlaSpec, GluSpec, HybridCache, HybridDecoder, HybridSpec, LatentAttentionSpec, LayerSpec, RaggedBatch, RetentionSpec, RotarySpec,
-                                      TopkSoftmaxMoeSpec, UngatedMoeSpec, _call, synthetic_weights)
+                                      TopkSoftmaxMoeSpec, UngatedMoeSpec, _call, scan_segments, synthetic_weights)
     z = KEBISUN_SIZES[a.kebisun]
     W, H, D, Dr, Dv, R = z["width"], z["heads"], z["dim"], z["rot"], z["vdim"], z["kv_rank"]
     gH, gD, gDv = z["g_heads"], z["g_dim"], z["g_vdim"]
@@ -1552,6 +1552,260 @@ def kebisun_leg(a, dev):
                       "config": {"model": f"kebisun-{a.kebisun}", "global_batch": 1, "seq_len": 512, "parallelism": "tp1"}, "kebisun": out}), flush=True)
 
 
+ZUMUZEN_SIZES = {
+    # layer lists that resemble a small, a mid-size and a large decoder: a recurrent block, then two passes through attention beside decayed linear attention / time mixing
+    "s": dict(width=1024, heads=8, kv=4, dim=128, vdim=128, chunk=2048, r_width=1024, blocks=8, conv=4, l_heads=8, l_dim=128, l_vdim=128, t_heads=16, t_dim=64, ff=2816, vocab=32000),
+    "m": dict(width=2048, heads=16, kv=4, dim=128, vdim=128, chunk=2048, r_width=2048, blocks=8, conv=4, l_heads=16, l_dim=128, l_vdim=128, t_heads=32, t_dim=64, ff=5632, vocab=32000),
+    "l": dict(width=4096, heads=32, kv=8, dim=128, vdim=128, chunk=2048, r_width=4096, blocks=16, conv=4, l_heads=32, l_dim=128, l_vdim=128, t_heads=64, t_dim=64, ff=11008, vocab=32000),
+}
+
+
+def zumuzen_leg(a, dev):
+    """`--zumuzen SIZE`: prefill and decode throughput of a Zumuzen layer list (a real-gated linear recurrent unit; chunked attention beside decayed linear attention; chunked sink
+    attention over keys as values beside time mixing; the last three layers run twice; bf16 weights, random) beside the closest model of the package at equal size: a state-space
+    layer of equal width, chunked sink attention with head norms and gates next to retention of equal state size, the same next to gated linear attention, the same feed-forwards,
+    the same layers run twice.  Then the kernels of the two designs that do like work, at the model's shapes, replayed from HIP graphs: time and the fraction of the roofline
+    (8 TB/s for what must be read and written; attention and the recurrences are priced in FLOP/s of the work done)."""
+    import torch
+    from mistralrs_amd.hybrid import (AttentionSpec, GlaSpec, GluSpec, HybridCache, HybridDecoder, HybridSpec, LayerSpec, LightningSpec, Mamba2Spec, ParallelSpec, RaggedBatch,
+                                      RetentionSpec, RgLruSpec, RotarySpec, TimeMixSpec, _call, scan_segments, synthetic_weights)
+    z = ZUMUZEN_SIZES[a.zumuzen]
+    W, H, G, D, Dv, C = z["width"], z["heads"], z["kv"], z["dim"], z["vdim"], z["r_width"]
+    lH, lD, lDv, tH, tD = z["l_heads"], z["l_dim"], z["l_vdim"], z["t_heads"], z["t_dim"]
+    scale, ff = D ** -0.5, GluSpec(z["ff"])
+    yarn = {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}
+    decays = [1.0 - 2.0 ** (-5 - h % 8) for h in range(lH)]
+    both = ParallelSpec("attention", AttentionSpec(H, G, D, Dv, scale, 0, 0, RotarySpec(D, 500000.0, None, "half"), False, chunk=z["chunk"], bias=True), "lightning",
+                        LightningSpec(lH, lD, lDv, decays))
+    both2 = ParallelSpec("attention", AttentionSpec(H, G, D, D, scale, 0, 0, RotarySpec(D // 2, 250000.0, yarn, "half"), False, chunk=z["chunk"], sink=True, bias=True, values_are_keys=True),
+                         "time_mix", TimeMixSpec(tH, tD), (0.75, 1.25))
+    oattn = AttentionSpec(H, G, D, Dv, scale, 0, 0, RotarySpec(D // 2, 500000.0), True, chunk=z["chunk"], head_norm=True, sink=True, head_gate=True)
+    new = [LayerSpec("rglru", RgLruSpec(C, z["blocks"], z["conv"]), ff, "l0.")]
+    old = [LayerSpec("mamba2", Mamba2Spec(C // 64, 64, 16, 1, z["conv"], 1), ff, "l0.")]
+    for t in range(2):   # two passes with the same weights
+        for i, (mn, right) in enumerate(((both, ("retention", RetentionSpec(lH, lD, lDv, decays, RotarySpec(lD, 10000.0, None, "half")))), (both2, ("gla", GlaSpec(tH, tD, tD, 16.0))),
+                                         (both, ("retention", RetentionSpec(lH, lD, lDv, decays, RotarySpec(lD, 10000.0, None, "half"))))), 1):
+            new.append(LayerSpec("parallel", mn, ff, f"l{i}.", i if t else None, t if i == 1 else None))
+            old.append(LayerSpec("attention", oattn, None, f"l{i}a.", 2 * i - 1 if t else None))
+            old.append(LayerSpec(right[0], right[1], ff, f"l{i}.", 2 * i if t else None))
+    specs = {"zumuzen": HybridSpec(z["vocab"], W, 1e-6, new, norm="rms", step="loop.step"), "state_space_attention_retention_gla": HybridSpec(z["vocab"], W, 1e-6, old, norm="rms")}
+    prompts, batches, bs, ctx = [512, 2048], [1, 8], 32, 512
+    max_tok = max(prompts) + a.warmup + a.steps + 64
+
+    def timed(fn, reps):
+        fn()
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        for _ in range(reps):
+            fn()
+        torch.cuda.synchronize()
+        return (time.perf_counter() - t0) / reps
+
+    def graphed(fn, reps=20):
+        """a launch (or a few) from a HIP graph, so that host time does not hide the kernels"""
+        fn()
+        torch.cuda.synchronize()
+        g = torch.cuda.CUDAGraph()
+        with torch.cuda.graph(g):
+            for _ in range(reps):
+                fn()
+        return timed(g.replay, 5) / reps
+
+    out = {"sizes": z, "dtype": "bf16", "weights": "random, drawn on the device", "models": {}, "kernels": {}}
+    keep = {}
+    with torch.no_grad():
+        for name, spec in specs.items():
+            model = HybridDecoder(spec, dev, "bfloat16", num_blocks=max(batches) * (-(-max_tok // bs) + 1) + 2, block_size=bs, state_slots=max(batches))
+            model.load_weights(synthetic_weights(spec, dev, 0))
+            cache = HybridCache(model)
+            r = {"prefill": {}, "decode": {}}
+            for T in prompts:
+                assert cache.reserve(1, T)
+                b = RaggedBatch.build([cache.entry(1, [(1000 + i) % z["vocab"] for i in range(T)], 0, [T - 1])], bs, dev)
+                model.forward_batch(b)
+                t = timed(lambda: model.forward_batch(b), 10)
+                r["prefill"][str(T)] = {"tokens_per_sec": round(T / t, 1), "ms": round(1e3 * t, 3)}
+                cache.release(1)
+            for nb in batches:
+                for q in range(nb):
+                    assert cache.reserve(q + 1, ctx + a.warmup + a.steps + 2)
+                model.forward_batch(RaggedBatch.build([cache.entry(q + 1, [(1000 + i + q) % z["vocab"] for i in range(ctx)], 0, []) for q in range(nb)], bs, dev))
+                g = model.capture_decode(nb, -(-(ctx + a.warmup + a.steps + 2) // bs))
+                pos = ctx
+
+                def step():
+                    nonlocal pos
+                    g.replay([cache.entry(q + 1, [7 + q], pos) for q in range(nb)])
+                    pos += 1
+                for _ in range(a.warmup):
+                    step()
+                torch.cuda.synchronize()
+                t0 = time.perf_counter()
+                for _ in range(a.steps):
+                    step()
+                torch.cuda.synchronize()
+                t = (time.perf_counter() - t0) / a.steps
+                r["decode"][f"batch{nb}"] = {"tokens_per_sec": round(nb / t, 1), "ms_per_step": round(1e3 * t, 4)}
+                del g
+                for q in range(nb):
+                    cache.release(q + 1)
+            out["models"][name] = r
+            keep[name] = model
+            torch.cuda.empty_cache()
+            print(f"# {name}: {json.dumps(r)}", file=sys.stderr, flush=True)
+        d1 = out["models"]["zumuzen"]["decode"]["batch1"]
+        line = {"metric": "zumuzen_decode_tokens_per_sec", "value": d1["tokens_per_sec"], "unit": "tokens/s", "n_gpus": 1, "steps": a.steps, "warmup": a.warmup,
+                "ms_per_step": d1["ms_per_step"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+                "config": {"model": f"zumuzen-{a.zumuzen}", "global_batch": 1, "seq_len": 512, "parallelism": "tp1"}, "zumuzen": out}
+        if a.zumuzen_models_only:
+            print(json.dumps(line), flush=True)
+            return
+        # ---- like kernels of the two designs
+        nm, om = keep["zumuzen"], keep["state_space_attention_retention_gla"]
+        lru, att, lit, att2, tmx = nm.layers[0].mixer, nm.layers[1].mixer.left, nm.layers[1].mixer.right, nm.layers[2].mixer.left, nm.layers[2].mixer.right
+        ssm, oat, ret, gla = om.layers[0].mixer, om.layers[1].mixer, om.layers[2].mixer, om.layers[4].mixer
+        kern = out["kernels"]
+        f32, bf = dict(dtype=torch.float32, device=dev), dict(dtype=torch.bfloat16, device=dev)
+
+        def pair(label, t_new, t_old, nbytes=None, flops=None, **extra):
+            d = {"zumuzen_us": round(1e6 * t_new, 1), "other_us": round(1e6 * t_old, 1), "time_ratio": round(t_new / t_old, 2), **extra}
+            if nbytes is not None:
+                d.update(min_bytes=nbytes[0], other_min_bytes=nbytes[1], zumuzen_hbm_frac=round(nbytes[0] / t_new / HBM_PEAK, 4), other_hbm_frac=round(nbytes[1] / t_old / HBM_PEAK, 4))
+            if flops is not None:
+                d.update(flops=flops[0], other_flops=flops[1], zumuzen_tflops=round(flops[0] / t_new / 1e12, 2), other_tflops=round(flops[1] / t_old / 1e12, 2))
+            kern[label] = d
+            print(f"# {label}: {json.dumps(d)}", file=sys.stderr, flush=True)
+
+        def batch(ents):
+            bps = -(-(2048 + 64) // bs)
+            return RaggedBatch.build([{"tokens": [0] * n, "pos0": p0, "slot": q, "blocks": list(range(1 + q * bps, 1 + q * bps + -(-(p0 + n) // bs))), "want": []}
+                                      for q, (p0, n) in enumerate(ents)], bs, dev)
+        for label, ents in (("prompt_2048", [(0, 2048)]), ("prompt_8x256", [(0, 256)] * 8), ("decode_batch8", [(600, 1)] * 8), ("decode_batch1", [(600, 1)])):
+            b = batch(ents)
+            T, single = b.rows, b.seg_rows == 1
+            seg = (b.seg_entry, b.seg_row0, b.seg_len, b.ent_seg0)
+            who = (b.seq_pos0, b.seq_slot)
+            # the recurrent block: gates, recurrence, GELU branch | step sizes, scan, gated norm (convolution and products are the same launches)
+            u, yx, o = torch.randn(T, C, **f32), torch.randn(T, 2 * C, **f32), torch.empty(T, C, **bf)
+            gates = (lru.ra, lru.ri, lru.ba, lru.bi, lru.lam, yx, 2 * C, lru.yb, lru.state)
+            loc, prd, sta = torch.empty(T, C, **f32), torch.empty(T, C, **f32), torch.empty(b.segments, C, **f32)
+
+            def new_lru():
+                if single:
+                    _call("mrs_hyb_rglru_step", u, *gates, o, b.seq_start, *who, T, b.entries, C, z["blocks"], 1)
+                else:
+                    _call("mrs_hyb_rglru_scan", u, *gates, loc, prd, sta, o, *who, b.seg_row0, b.seg_len, b.ent_seg0, T, b.entries, b.segments, 64, C, z["blocks"], 1)
+            ms = ssm.s
+            uo, xbc, yy = torch.randn(T, ssm.w_in.shape[0], **f32), torch.randn(T, ms.conv_channels, **f32) * 0.1, torch.empty(T, ms.inner, **f32)
+            steps, cy, dk = torch.empty(T, ms.heads, 2, **f32), torch.empty(b.segments, ms.heads, ms.state, ms.vdim, **f32), torch.empty(b.segments, ms.heads, **f32)
+
+            def old_ssm():
+                _call("mrs_hyb_ssd_scan", xbc, uo, ssm.dt_bias, ssm.A_log, ssm.D, ssm.ssm_state, yy, *who, *seg, steps, cy, dk, T, b.entries, b.segments, ms.conv_channels, uo.stride(0),
+                      ms.inner + ms.conv_channels, ms.heads, ms.vdim, ms.state, ms.groups)
+                _call("mrs_hyb_rmsnorm", yy, ms.inner, ssm.norm, o, None, None, T, ms.inner, 1, 1e-6, 0, 1, uo, uo.stride(0), 0)
+            part = C // z["blocks"]
+            pair(f"gated_recurrence_vs_state_space_scan_and_norm_{label}", graphed(new_lru), graphed(old_ssm),
+                 (T * C * (4 + 4 + 2) + 4 * C * part + b.entries * 8 * C, T * (4 * (2 * C + 32) + 2 * C) + b.entries * 8 * C * ms.state), (4.0 * T * C * part, 4.0 * T * C * ms.state))
+            # decayed linear attention | retention (rotation is a launch of its own there and left out)
+            st = lH * lD * lDv
+            nv, nk = lH * lDv, lH * lD
+            ul, uo, y, yo = torch.randn(T, lit.w_in.shape[0], **f32) * 0.3, torch.randn(T, ret.w_in.shape[0], **f32) * 0.3, torch.empty(T, nv, **f32), torch.empty(T, nv, **bf)
+            cy, dk, steps = torch.empty(b.segments, lH, lD, lDv, **f32), torch.empty(b.segments, lH, **f32), torch.empty(T, lH, 2, **f32)
+            table, nseg = scan_segments(b, lH, lD, lDv)
+            ncy, ndk = (torch.empty(nseg, lH, lD, lDv, **f32), torch.empty(nseg, lH, lD, **f32)) if nseg > b.entries else (None, None)
+
+            def new_lit():
+                if single:
+                    _call("mrs_hyb_lightning_step", ul, ul.stride(0), lit.k_col, lit.q_col, lit.decay, lit.state, y, b.seq_start, *who, T, b.entries, lH, lD, lDv)
+                else:
+                    _call("mrs_hyb_lightning_scan", ul, ul.stride(0), lit.k_col, lit.q_col, lit.decay, lit.state, y, *who, *table, ncy, ndk, T, b.entries, nseg, lH, lD, lDv)
+                _call("mrs_hyb_rmsnorm", y, nv, lit.norm, yo, None, None, T, nv, 1, 1e-6, 0, 1, ul[:, lit.g_col:], ul.stride(0), 2)
+
+            def old_ret():
+                _call("mrs_hyb_decay_scan", uo, uo.stride(0), ret.decay, ret.state, y, *who, *seg, steps, cy, dk, T, b.entries, b.segments, lH, lDv, lD, lH)
+                _call("mrs_hyb_rmsnorm", y, nv, None, yo, None, None, T, nv, lH, 1e-6, 0, 1, uo[:, ret.gate_col:], uo.stride(0), 1)
+            pair(f"decayed_linear_attention_and_norm_vs_retention_and_norm_{label}", graphed(new_lit), graphed(old_ret),
+                 (b.entries * 8 * st + T * (4 * ul.shape[1] + 2 * nv),) * 2, (6.0 * T * st, 6.0 * T * st), segments=nseg)
+            # time mixing | gated linear attention: decays, recurrence, head norm, gate
+            n = tH * tD
+            st = n * tD
+            ut, ug, a1 = torch.randn(T, 4 * n, **f32) * 0.3, torch.randn(T, gla.w_in.shape[0], **f32) * 0.3, torch.randn(T, tmx.w1.shape[0], **f32)
+            zt, y, o2 = torch.randn(T, n, **f32), torch.empty(T, n, **f32), torch.empty(T, n, **bf)
+            table, nseg = scan_segments(b, tH, tD, tD)
+            ncy, ndk = (torch.empty(nseg, tH, tD, tD, **f32), torch.empty(nseg, tH, tD, **f32)) if nseg > b.entries else (None, None)
+
+            def new_tm():
+                if single:
+                    _call("mrs_hyb_bonus_step", ut, 4 * n, n, 2 * n, 3 * n, a1, a1.shape[1], tmx.w2, tmx.w0, tmx.bonus, tmx.norm, tmx.state, o2, b.seq_start, *who, T, b.entries, tH, tD, tD, 1e-6, 1)
+                    return
+                _call("mrs_hyb_gla_decays", zt, tmx.w0, T, n, 0.0)
+                _call("mrs_hyb_bonus_scan", ut, 4 * n, n, 2 * n, zt, tmx.bonus, tmx.state, y, *who, *table, ncy, ndk, T, b.entries, nseg, tH, tD, tD)
+                _call("mrs_hyb_head_norm_gate", y, tD, None, tmx.norm, 1, ut[:, 3 * n:], 4 * n, 2, o2, T, tH, tD, 1e-6, 1)
+
+            def old_gla():
+                if single:
+                    _call("mrs_hyb_gla_step", ug, ug.stride(0), gla.k_col, gla.q_col, gla.g_col, gla.a_col, gla.rank, gla.w_a2, gla.b_a, gla.norm, gla.state, o2, b.seq_start, *who, T,
+                          b.entries, tH, tD, tD, gla.q_mult, gla.inv_tau, 1e-6, 1)
+                    return
+                _call("mrs_hyb_gla_decays", zt, gla.b_a, T, n, gla.inv_tau)
+                _call("mrs_hyb_gla_scan", ug, ug.stride(0), gla.k_col, gla.q_col, zt, gla.state, y, *who, *table, ncy, ndk, T, b.entries, nseg, tH, tD, tD, gla.q_mult)
+                _call("mrs_hyb_head_norm_gate", y, tD, None, gla.norm, 0, ug[:, gla.g_col:], ug.stride(0), 2, o2, T, tH, tD, 1e-6, 1)
+            pair(f"time_mixing_recurrence_vs_gated_linear_attention_{label}", graphed(new_tm), graphed(old_gla), (b.entries * 8 * st + T * n * 22,) * 2, (6.0 * T * st, 6.0 * T * st), segments=nseg)
+            # operands: token shift into five mixes | short convolution over four times the width
+            h32, mix = torch.randn(T, W, **f32), torch.empty(5, T, W, **bf)
+            cv, cw, cst = torch.empty(T, 4 * W, **f32), torch.randn(4 * W, 4, **f32), torch.zeros(8, 4 * W, 3, **f32)
+            h4 = torch.randn(T, 4 * W, **f32)
+            t_new = graphed(lambda: _call("mrs_hyb_token_shift", h32, tmx.mu, tmx.last, mix, b.tok_seq, b.seq_start, *who, T, W, 5, 1))
+            t_old = graphed(lambda: _call("mrs_hyb_conv", h4, 4 * W, None, cw, None, cst, b.tok_seq, b.seq_start, *who, cv, T, b.entries, 4 * W, 4, 1))
+            pair(f"token_shift_five_mixes_vs_convolution_of_four_widths_{label}", t_new, t_old, (T * W * 14, T * W * 32))
+            # projections of time mixing: four products from four operands in one launch | one product of the same size
+            w4, u4 = tmx.w_in.view(4 * n, W), torch.empty(T, 4 * n, **f32)
+            t_new = graphed(lambda: _call("mrs_hyb_gemm_batched", mix, tmx.w_in, u4, T, n, W, W, W, 4 * n, 1, 4, T * W, n * W, n, 0))
+            t_old = graphed(lambda: nm.linear(mix[0], w4, out=u4))
+            pair(f"four_products_in_one_launch_vs_one_product_{label}", t_new, t_old, (8 * n * W,) * 2 if single else None, (8.0 * T * n * W,) * 2)
+            # row-wise
+            x, y1, y2, wv, ob = torch.randn(T, W, **f32), torch.randn(T, W, **f32), torch.randn(T, W, **f32), torch.randn(W, **f32), torch.empty(T, W, **bf)
+            t_new = graphed(lambda: _call("mrs_hyb_norm_pair_add_norm", x, W, y1, wv, y2, wv, T, W, 1e-6, 0.5, 1, wv, 0, ob, None, 1))
+
+            def old_join():
+                _call("mrs_hyb_norm_pair_add", x, W, y1, wv, y2, wv, T, W, 1e-6, 0.5, 1)
+                _call("mrs_hyb_rmsnorm", x, W, wv, ob, None, None, T, W, 1, 1e-6, 0, 1, None, 0, 0)
+            pair(f"normed_average_and_next_norm_in_one_launch_vs_two_{label}", t_new, graphed(old_join), (T * W * 18, T * W * 22))
+            t_new = graphed(lambda: _call("mrs_hyb_pass_norm", x, b.tokens, nm.embed, z["vocab"], 1.0, nm.step[1], wv, ob, None, T, W, 1e-6, 0, 1))
+            t_old = graphed(lambda: _call("mrs_hyb_rmsnorm", x, W, wv, ob, None, None, T, W, 1, 1e-6, 0, 1, None, 0, 0))
+            pair(f"pass_entry_and_norm_vs_norm_{label}", t_new, t_old, (T * W * 12, T * W * 6))
+            uq, uqo, q = torch.randn(T, att.w_qkv.shape[0], **f32), torch.randn(T, oat.w_qkv.shape[0], **f32), torch.empty(T, H * D, **bf)
+            t_new = graphed(lambda: _call("mrs_hyb_rope_half_cache", uq, uq.stride(0), att.v_col, att.qb, att.kb, att.vb, att.freq, att.trig_mult, b.tok_pos, b.slot_mapping, q, att.k_cache,
+                                          att.v_cache, T, H, G, D, Dv, D, bs, 1))
+            t_old = graphed(lambda: _call("mrs_hyb_qk_headnorm_rope_cache", uqo, uqo.stride(0), oat.q_norm, oat.k_norm, oat.freq, b.tok_pos, b.slot_mapping, q, oat.k_cache, oat.v_cache, T, H,
+                                          G, D, Dv, D // 2, bs, 1e-6, 1))
+            nqkv = H * D + G * (D + Dv)
+            pair(f"bias_rotary_page_write_vs_norm_rotary_page_write_{label}", t_new, t_old, (T * nqkv * 6, T * nqkv * 6))
+        for c_ in (att.k_cache, att.v_cache, oat.k_cache, oat.v_cache):
+            c_.normal_()
+        for label, ents, ch in (("prompt_2048", [(0, 2048)], 2048), ("prompt_2048_chunk_512", [(0, 2048)], 512), ("prompt_512_after_1536", [(1536, 512)], 2048), ("decode_batch8_ctx2048", [(2047, 1)] * 8, 2048),
+                                ("decode_batch1_ctx2048", [(2047, 1)], 2048)):
+            b = batch(ents)
+            T = b.rows
+            seg = (b.seg_entry, b.seg_row0, b.seg_len, b.segments, RaggedBatch.SEGMENT)
+            q, o, gate, sink = torch.randn(T, H * D, device=dev).to(torch.bfloat16), torch.empty(T, H * Dv, **bf), torch.randn(T, H, **f32), torch.randn(H, **f32)
+
+            def general(mx, gated):
+                _call("mrs_hyb_paged_attn_chunked", q, mx.k_cache, mx.v_cache, b.block_tables, b.tok_seq, b.tok_pos, o, T, H, G, D, Dv, bs, b.max_blocks, ch, scale, 1, *seg, 0.0, int(gated),
+                      sink if gated else None, gate if gated else None, H, 1, *nm.key_splits(b, H, Dv, ch))
+
+            def new_attn():
+                if T > b.entries:
+                    _call("mrs_hyb_attn_mfma_prompt", q, att.k_cache, att.v_cache, b.block_tables, b.tok_pos, *seg, None, None, 0, 0, o, T, H, G, D, Dv, nm.num_blocks, b.max_blocks, bs, 0, ch, scale)
+                else:
+                    general(att, False)
+            pairs = sum(p0 + i + 1 - (p0 + i) // ch * ch for p0, n in ents for i in range(n))
+            rows = sum(p0 + n - p0 // ch * ch for p0, n in ents)
+            pair("chunked_attention_vs_general_paged_kernel_with_sink_and_gate_" + label, graphed(new_attn, 5), graphed(lambda: general(oat, True), 5), (2 * (rows * G * (D + Dv) + T * H * (D + Dv)),) * 2,
+                 (2.0 * pairs * H * (D + Dv),) * 2)
+    print(json.dumps(line), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -1588,11 +1842,22 @@ def main():
                     help="instead of the default workload: a Kebisun layer list (latent attention with a rotated key part / window / sink / gate, gated linear attention; dense / routed GELU "
                          "feed-forwards) beside the package's closest model at equal size, and the like kernels of the two")
     ap.add_argument("--kebisun-models-only", action="store_true", help="--kebisun: without the like kernels (profiling runs)")
+    ap.add_argument("--zumuzen", choices=sorted(ZUMUZEN_SIZES), default=None,
+                    help="instead of the default workload: a Zumuzen layer list (recurrent block, chunked attention beside linear attention / time mixing, layers that run twice) beside the closest "
+                         "model of the package at equal size, and the kernels they have in common")
+    ap.add_argument("--zumuzen-models-only", action="store_true", help="--zumuzen: without the like kernels (profiling runs)")
     ap.add_argument("--gifopel", choices=sorted(GIFOPEL_SIZES), default=None,
                     help="instead of the default workload: a Gifopel layer list (matrix memory, chunked sink attention beside a delta rule, delta rule with channel decays; dense / routed "
                          "squared-ReLU feed-forwards; bf16) of the given size beside a state-space + windowed-attention + routed-experts list of the package at equal size, and the like "
                          "kernels of the two one by one")
     a = ap.parse_args()
+    if a.zumuzen:
+        import torch
+        dev = torch.device("cuda", 0)
+        torch.cuda.set_device(dev)
+        if a.steps == 256:
+            a.steps = 128
+        return zumuzen_leg(a, dev)
     if a.kebisun:
         import torch
         dev = torch.device("cuda", 0)

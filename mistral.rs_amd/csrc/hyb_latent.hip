@@ -7,7 +7,7 @@
 // Scores, maxima, exponentials, weights and all sums are f32: a score is an f32 sum of exact bf16 products; a weight enters its product as THREE bf16 terms that add up to the f32
 // number (8 + 8 + 8 significant bits, cut, not rounded), so the weighted sum too is an f32 sum of exact products.  Exponentials are taken in base two: scale and sink come
 // multiplied by log2(e).
-#include "common.cuh"
+#include "hyb_mfma.cuh"
 #include <float.h>
 
 namespace mrs {
@@ -20,30 +20,8 @@ static int ok_or(const char *what) {
   snprintf(g_err, sizeof g_err, "%s: launch failed", what);
   return 1;
 }
-typedef short bf16x8 __attribute__((ext_vector_type(8)));
-typedef float f32x16 __attribute__((ext_vector_type(16)));
-typedef float f32x4 __attribute__((ext_vector_type(4)));
+using namespace mrs::mfma;
 __device__ __forceinline__ float sigmoid_f(float v) { return 1.0f / (1.0f + expf(-v)); }
-__device__ __forceinline__ float exp2_f(float v) { return __builtin_amdgcn_exp2f(v); }
-constexpr float LOG2E = 1.4426950408889634f;
-
-// eight f32 weights as three bf16 operands whose sum is the weights: every term takes the top sixteen bits of what is left
-__device__ __forceinline__ void split3(const float *p, bf16x8 *out) {
-  unsigned w[3][4];
-#pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    float a = p[2 * j], b = p[2 * j + 1];
-#pragma unroll
-    for (int c = 0; c < 3; ++c) {
-      const unsigned ua = __float_as_uint(a) & 0xffff0000u, ub = __float_as_uint(b) & 0xffff0000u;
-      w[c][j] = (ua >> 16) | ub;
-      a -= __uint_as_float(ua);
-      b -= __uint_as_float(ub);
-    }
-  }
-#pragma unroll
-  for (int c = 0; c < 3; ++c) out[c] = __builtin_bit_cast(bf16x8, make_int4((int)w[c][0], (int)w[c][1], (int)w[c][2], (int)w[c][3]));
-}
 
 // ---------------------------------------------------------------------------------- prompt
 struct FlashArgs {

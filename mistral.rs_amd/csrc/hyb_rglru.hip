@@ -11,7 +11,7 @@
 //
 // Everything that enters the recurrence is f32.  bf16 weights: u enters its matrix-core products as THREE bf16 terms that add up to the f32 number, so a gate's logit is an f32 sum of
 // exact products.
-#include "common.cuh"
+#include "hyb_mfma.cuh"
 #include <float.h>
 
 namespace mrs {
@@ -24,8 +24,7 @@ static int ok_or(const char *what) {
   snprintf(g_err, sizeof g_err, "%s: launch failed", what);
   return 1;
 }
-typedef short bf16x8 __attribute__((ext_vector_type(8)));
-typedef float f32x16 __attribute__((ext_vector_type(16)));
+using namespace mrs::mfma;
 
 __device__ __forceinline__ float sigmoid_f(float v) { return 1.0f / (1.0f + expf(-v)); }
 __device__ __forceinline__ float softplus_f(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
@@ -100,20 +99,10 @@ template <class T> __global__ void __launch_bounds__(256) rglru_gates_kernel(Gat
     load_u(0, uv);
     wv[0] = load_w(wa, 0); wv[1] = load_w(wi, 0);
     for (int k0 = 0; k0 < part; k0 += GK) {
-      unsigned w[3][4];
+      bf16x8 ut[3];
+      split3(uv, ut);
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        float x = uv[2 * j], y = uv[2 * j + 1];
-#pragma unroll
-        for (int c = 0; c < 3; ++c) {   // the top sixteen bits of what is left, three times
-          const unsigned ux = __float_as_uint(x) & 0xffff0000u, uy = __float_as_uint(y) & 0xffff0000u;
-          w[c][j] = (ux >> 16) | uy;
-          x -= __uint_as_float(ux);
-          y -= __uint_as_float(uy);
-        }
-      }
-#pragma unroll
-      for (int c = 0; c < 3; ++c) *(int4 *)(Us + (c * GT + sr) * US + kc) = make_int4((int)w[c][0], (int)w[c][1], (int)w[c][2], (int)w[c][3]);
+      for (int c = 0; c < 3; ++c) *(int4 *)(Us + (c * GT + sr) * US + kc) = __builtin_bit_cast(int4, ut[c]);
 #pragma unroll
       for (int c = 0; c < 2; ++c) *(int4 *)(Ws + (c * GT + sr) * US + kc) = wv[c];
       __syncthreads();

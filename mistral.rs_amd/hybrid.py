@@ -82,6 +82,7 @@ _SIGS = {
     "mrs_hyb_latent_prep": [_vp] + [_i] * 5 + [_vp, _vp, _vp, _f] + [_vp] * 4 + [_f, _i, _i, _vp],
     "mrs_hyb_latent_query": [_vp] + [_i] * 6 + [_vp, _f, _vp, _vp, _vp, _i, _i, _vp],
     "mrs_hyb_latent_context": [_vp] * 4 + [_i] * 7 + [_vp],
+    "mrs_hyb_attn_mfma_prompt": [_vp] * 8 + [_i, _i, _vp, _vp, _i, _i, _vp] + [_i] * 10 + [_f, _vp],
     "mrs_hyb_latent_mfma_prompt": [_vp] * 8 + [_i, _i, _vp, _vp, _i, _vp] + [_i] * 8 + [_f, _vp],
     "mrs_hyb_latent_mfma_decode": [_vp] * 7 + [_i] * 8 + [_f, _vp],
     "mrs_hyb_latent_mfma_merge": [_vp] * 5 + [_i, _vp] + [_i] * 5 + [_vp],
@@ -117,6 +118,8 @@ def _last_error(name: str) -> str:
         return "mrs_hyb_recur_last_error"
     if name in _LINATTN:
         return "mrs_hyb_linattn_last_error"
+    if "attn_mfma" in name:
+        return "mrs_hyb_attn_mfma_last_error"
     if "rglru" in name:
         return "mrs_hyb_rglru_last_error"
     if "latent_mfma" in name:
@@ -942,6 +945,14 @@ class WindowAttention(_Module):
     def kv_bytes_per_token(self) -> int:
         return self.k_cache.element_size() * self.s.kv_heads * (self.s.dim + self.s.vdim)
 
+    USE_MFMA = os.environ.get("MRS_ATTN_MFMA", "1") != "0"
+
+    @property
+    def mfma_prompt(self) -> bool:
+        """the sizes that the matrix-core kernel's tiles cover (csrc/hyb_attn_mfma.hip); the general paged kernels serve the others and the all-f32 mode"""
+        s = self.s
+        return self.USE_MFMA and self.m.dt == 1 and s.dim % 8 == 0 and s.dim <= 256 and s.vdim % 8 == 0 and s.vdim <= 256 and s.keep_first == 0 and RaggedBatch.SEGMENT <= 64
+
     def forward(self, h, x, b: RaggedBatch, accumulate: bool = True, u=None):
         s, m = self.s, self.m
         T = b.rows
@@ -954,7 +965,11 @@ class WindowAttention(_Module):
             _call("mrs_hyb_qk_headnorm_rope_cache" if s.head_norm else "mrs_hyb_qk_norm_rope_cache", qkv, qkv.stride(0), self.q_norm, self.k_norm, self.freq, b.tok_pos,
                   b.slot_mapping, q, self.k_cache, self.v_cache, T, s.heads, s.kv_heads, s.dim, s.vdim, s.rotary.dims if s.rotary else 0, m.block_size, m.spec.eps, m.dt)
         o = torch.empty(T, s.heads * s.vdim, dtype=m.torch_dtype, device=m.device)
-        if s.chunk or s.sink or s.head_gate:
+        if b.seg_rows > 1 and self.mfma_prompt:   # steps with portions in bf16: the matrix cores
+            _call("mrs_hyb_attn_mfma_prompt", q, self.k_cache, self.v_cache, b.block_tables, b.tok_pos, b.seg_entry, b.seg_row0, b.seg_len, b.segments, RaggedBatch.SEGMENT, self.sink,
+                  qkv[:, self.gate_col:] if s.head_gate else None, qkv.stride(0), 0, o, T, s.heads, s.kv_heads, s.dim, s.vdim, m.num_blocks, b.max_blocks, m.block_size, s.window, s.chunk,
+                  s.scale)
+        elif s.chunk or s.sink or s.head_gate:
             if s.window or s.keep_first:
                 raise NotImplementedError("a learned sink / a per-head gate beside a sliding window")
             scratch, splits = m.key_splits(b, s.heads, s.vdim, s.chunk)   # single-row steps deal a long chunk's keys to several workgroups
