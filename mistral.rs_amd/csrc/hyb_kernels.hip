@@ -81,6 +81,39 @@ template <class T> __global__ void __launch_bounds__(256) rmsnorm_kernel(const f
   }
 }
 
+// The same for parts of at most 256 NC values without a gate in front: a row is read once, all its loads (and the weights') in flight, and waits in registers for its root mean square.
+template <class T, int NC> __global__ void __launch_bounds__(256) rmsnorm_row_kernel(const float *__restrict__ x, int ldx, const float *__restrict__ w, T *__restrict__ out,
+                                                                                     float *__restrict__ out32, float *__restrict__ rstd, int part, float eps, int one_plus, int ldo,
+                                                                                     const float *__restrict__ gate, int ldg, int gate_after) {
+  __shared__ float red[4];
+  const int t = blockIdx.x, g = blockIdx.y;
+  const float *xr = x + (size_t)t * ldx + (size_t)g * part;
+  const float *gr = gate ? gate + (size_t)t * ldg + (size_t)g * part : nullptr;
+  float v[NC], wv[NC], gv[NC], s = 0.f;
+#pragma unroll
+  for (int j = 0; j < NC; ++j) {
+    const int c = threadIdx.x + 256 * j, cc = c < part ? c : part - 1;
+    v[j] = xr[cc];
+    wv[j] = w ? w[(size_t)g * part + cc] : (one_plus ? 0.f : 1.0f);
+    gv[j] = gr ? gr[cc] : 0.f;
+  }
+#pragma unroll
+  for (int j = 0; j < NC; ++j)
+    if (threadIdx.x + 256 * j < part) s = fmaf(v[j], v[j], s);
+  s = block_sum_256(s, red);
+  const float inv = 1.0f / sqrtf(s / (float)part + eps);
+  if (rstd && threadIdx.x == 0) rstd[(size_t)t * gridDim.y + g] = inv;
+#pragma unroll
+  for (int j = 0; j < NC; ++j) {
+    const int c = threadIdx.x + 256 * j;
+    if (c >= part) break;
+    float y = v[j] * inv * (one_plus ? 1.0f + wv[j] : wv[j]);
+    if (gr) y *= gate_after == 2 ? sigmoid_f(gv[j]) : silu_f(gv[j]);
+    if (out) out[(size_t)t * ldo + (size_t)g * part + c] = from_f<T>(y);
+    if (out32) out32[(size_t)t * ldo + (size_t)g * part + c] = y;
+  }
+}
+
 // ---------------------------------------------------------------------------------- short causal convolution (+ SiLU) with carried taps
 // u [rows, ldu] (the channels start at column 0 of the pointer handed in), cw [C, taps] (the last column multiplies the current token), state [slots, C, taps - 1]
 // (oldest first).  An entry that starts at position 0 reads zeros instead of its slot.  in_bias (nullable, [C]): the bias of the product that made u -- the convolution
@@ -706,6 +739,158 @@ template <class T, int DVC, bool VEC> __global__ void __launch_bounds__(64) page
     if (d + 1 < a.Dv) out[d + 1] = from_f<T>(o[c][1] * inv * (gr ? sigmoid_f(gr[gs * (d + 1)]) : 1.0f));
   }
 }
+// Single rows of whole-vector sizes: one workgroup of four waves per (row, RC query heads of one key head, split); a wave takes every fourth pass of 64 keys.  A lane reads its key in
+// batches of sixteen 16-byte pieces, all of a batch in flight, and scores it against the RC heads; then a lane owns value pairs and walks the pass's keys, sixteen loads in
+// flight.  The waves' sums meet in LDS at the end.
+template <class T, int DVC, int RC> __global__ void __launch_bounds__(256) paged_decode_attn_kernel(AttnArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];  // q [RC][Dq] | p [4 waves][64][RC] | joined sums [RC][Dv]
+  __shared__ int rowbase[4][64];
+  __shared__ float wm[4][RC], wl[4][RC];
+  constexpr int PV = 16 / (int)sizeof(T), PB = 16;   // values per piece, pieces per batch
+  const int per_g = a.H / a.G, parts = (per_g + RC - 1) / RC;
+  const int t = blockIdx.x, g = blockIdx.y / parts, h0 = g * per_g + (blockIdx.y % parts) * RC, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int nh = (g + 1) * per_g - h0 < RC ? (g + 1) * per_g - h0 : RC, Dq = (a.D + 3) & ~3;
+  float *qs = lds, *ps = lds + RC * Dq + wave * 64 * RC, *js = lds + RC * Dq + 256 * RC;
+  const int s = a.tok_seq[t], i = a.tok_pos[t];
+  for (int e = tid; e < RC * a.D; e += 256) {
+    const int r = e / a.D, d = e - r * a.D;
+    qs[r * Dq + d] = r < nh ? to_f<T>(((const T *)a.q)[((size_t)t * a.H + h0 + r) * a.D + d]) : 0.f;
+  }
+  const int *bt = a.block_tables + (size_t)s * a.max_blocks;
+  int w_lo = a.window > 0 ? i - a.window + 1 : 0;
+  if (w_lo < 0) w_lo = 0;
+  if (a.chunk > 0) w_lo = (i / a.chunk) * a.chunk;
+  int n1 = a.keep_first < w_lo ? a.keep_first : w_lo;  // kept first tokens that the window does not already cover
+  if (n1 < 0 || a.chunk > 0) n1 = 0;
+  int total = n1 + (i - w_lo + 1), v_begin = 0;
+  const bool split = a.splits > 1;
+  if (split) {  // this workgroup's share of the passes
+    const int per = ((total + 63) / 64 + a.splits - 1) / a.splits;
+    v_begin = blockIdx.z * per * 64;
+    const int v_end = v_begin + per * 64;
+    total = total < v_end ? total : v_end;
+  }
+  float m[RC], l[RC], o[RC][DVC][2];
+#pragma unroll
+  for (int r = 0; r < RC; ++r) {
+    m[r] = -FLT_MAX; l[r] = 0.f;
+#pragma unroll
+    for (int c = 0; c < DVC; ++c) o[r][c][0] = o[r][c][1] = 0.f;
+  }
+  __syncthreads();
+  for (int v0 = v_begin + 64 * wave; v0 < total; v0 += 256) {
+    const int vi = v0 + lane, vc = vi < total ? vi : total - 1;   // lanes past the end read the last key and weigh nothing
+    const int base = (int)kv_row(a, bt, vc < n1 ? vc : w_lo + (vc - n1), g);
+    const T *kr = (const T *)a.k_cache + (size_t)base * a.D;
+    float sc[RC];
+#pragma unroll
+    for (int r = 0; r < RC; ++r) sc[r] = 0.f;
+    for (int d0 = 0; d0 < a.D; d0 += PB * PV) {
+      int4 piece[PB];
+#pragma unroll
+      for (int j = 0; j < PB; ++j) piece[j] = *(const int4 *)(kr + (d0 + j * PV < a.D ? d0 + j * PV : 0));
+#pragma unroll
+      for (int j = 0; j < PB; ++j) {
+        if (d0 + j * PV >= a.D) break;
+        float kv[PV];
+        const unsigned u[4] = {(unsigned)piece[j].x, (unsigned)piece[j].y, (unsigned)piece[j].z, (unsigned)piece[j].w};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          if (PV == 8) { kv[2 * e < PV ? 2 * e : 0] = __uint_as_float(u[e] << 16); kv[2 * e + 1 < PV ? 2 * e + 1 : 0] = __uint_as_float(u[e] & 0xffff0000u); }
+          else kv[e] = __uint_as_float(u[e]);
+        }
+#pragma unroll
+        for (int r = 0; r < RC; ++r) {
+          const float *q = qs + r * Dq + d0 + j * PV;
+#pragma unroll
+          for (int e = 0; e < PV; e += 4) {
+            const float4 q4 = *(const float4 *)(q + e);
+            sc[r] = fmaf(q4.x, kv[e], sc[r]); sc[r] = fmaf(q4.y, kv[e + 1], sc[r]); sc[r] = fmaf(q4.z, kv[e + 2], sc[r]); sc[r] = fmaf(q4.w, kv[e + 3], sc[r]);
+          }
+        }
+      }
+    }
+    MRS_WAVE_SYNC();  // the previous pass has read p and the row indices
+#pragma unroll
+    for (int r = 0; r < RC; ++r) {
+      const float sv = vi < total ? capped(sc[r] * a.scale, a.softcap) : -FLT_MAX;
+      const float mn = fmaxf(m[r], wave_max(sv)), alpha = expf(m[r] - mn), p = vi < total ? expf(sv - mn) : 0.f;
+      l[r] = l[r] * alpha + wave_sum(p);
+      m[r] = mn;
+      ps[lane * RC + r] = p;
+#pragma unroll
+      for (int c = 0; c < DVC; ++c) { o[r][c][0] *= alpha; o[r][c][1] *= alpha; }
+    }
+    rowbase[wave][lane] = base;
+    MRS_WAVE_SYNC();
+    const int cnt = total - v0 < 64 ? total - v0 : 64;
+#pragma unroll
+    for (int c = 0; c < DVC; ++c) {
+      const int d = 128 * c + 2 * lane;
+      const T *vb = (const T *)a.v_cache + (d < a.Dv ? d : 0);
+      for (int j0 = 0; j0 < cnt; j0 += 16) {
+        float x[16], y[16];
+#pragma unroll
+        for (int j = 0; j < 16; ++j) Ld<T>::v2(vb + (size_t)rowbase[wave][j0 + j] * a.ldv, x[j], y[j]);
+#pragma unroll
+        for (int j = 0; j < 16; ++j)
+#pragma unroll
+          for (int r = 0; r < RC; ++r) {
+            const float p = ps[(j0 + j) * RC + r];
+            o[r][c][0] = fmaf(p, x[j], o[r][c][0]);
+            o[r][c][1] = fmaf(p, y[j], o[r][c][1]);
+          }
+      }
+    }
+  }
+  // the waves' sums, one wave after the other
+  if (lane == 0)
+#pragma unroll
+    for (int r = 0; r < RC; ++r) { wm[wave][r] = m[r]; wl[wave][r] = l[r]; }
+  __syncthreads();
+  float M[RC], L[RC];
+#pragma unroll
+  for (int r = 0; r < RC; ++r) {
+    const bool sunk = a.sink && !split && r < nh;
+    M[r] = sunk ? sink_of(a, h0 + r) : -FLT_MAX;
+    L[r] = 0.f;
+    for (int w = 0; w < 4; ++w) M[r] = fmaxf(M[r], wm[w][r]);
+    if (sunk) L[r] = expf(sink_of(a, h0 + r) - M[r]);
+    for (int w = 0; w < 4; ++w) L[r] += wl[w][r] * expf(wm[w][r] - M[r]);
+    const float e = expf(m[r] - M[r]);
+#pragma unroll
+    for (int c = 0; c < DVC; ++c) { o[r][c][0] *= e; o[r][c][1] *= e; }
+  }
+  for (int w = 0; w < 4; ++w) {
+    if (wave == w)
+#pragma unroll
+      for (int r = 0; r < RC; ++r)
+#pragma unroll
+        for (int c = 0; c < DVC; ++c) {
+          const int d = 128 * c + 2 * lane;
+          if (d >= a.Dv) continue;
+          float *j = js + r * a.Dv + d;
+          j[0] = w ? j[0] + o[r][c][0] : o[r][c][0];
+          j[1] = w ? j[1] + o[r][c][1] : o[r][c][1];
+        }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int r = 0; r < RC; ++r) {
+    if (r >= nh) break;
+    const int h = h0 + r;
+    if (split) {
+      float *part = a.scratch + (((size_t)blockIdx.z * a.rows + t) * a.H + h) * (a.Dv + 2);
+      for (int d = tid; d < a.Dv; d += 256) part[d] = js[r * a.Dv + d];
+      if (tid == 0) { part[a.Dv] = M[r]; part[a.Dv + 1] = L[r]; }
+      continue;
+    }
+    const float inv = 1.0f / L[r];
+    T *out = (T *)a.out + ((size_t)t * a.H + h) * a.Dv;
+    const float *gr = gate_row(a, t, h);
+    for (int d = tid; d < a.Dv; d += 256) out[d] = from_f<T>(js[r * a.Dv + d] * inv * (gr ? sigmoid_f(gr[a.gate_per_head ? 0 : d]) : 1.0f));
+  }
+}
 // joins the splits of a row and head: M = max_s m_s (and 0 with the sink), L = sum_s l_s e^{m_s - M} (+ e^{-M}), out = sum_s o_s e^{m_s - M} / L (times sigmoid(gate))
 template <class T> __global__ void __launch_bounds__(64) attn_merge_kernel(AttnArgs a) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x, stride = a.Dv + 2;
@@ -1159,7 +1344,8 @@ template <class T> __global__ void __launch_bounds__(256) qkv_bias_temp_cache_ke
 }
 // ---------------------------------------------------------------------------------- layers that run again: what joins the stream in front of a pass, with the norm behind it
 // x += scale * table[token] (table null: not) + step (null: not), in this order; out = x / rms(x) * (w | 1 + w), out32 (nullable) the same in f32
-template <class T> __global__ void __launch_bounds__(256) pass_norm_kernel(float *__restrict__ x, const int *__restrict__ tokens, const T *__restrict__ table, int vocab, float scale,
+// (rows of at most 256 NC values: read once, all loads in flight; NC 0: any width, the row is read back)
+template <class T, int NC> __global__ void __launch_bounds__(256) pass_norm_kernel(float *__restrict__ x, const int *__restrict__ tokens, const T *__restrict__ table, int vocab, float scale,
                                                                            const float *__restrict__ step, const float *__restrict__ w, T *__restrict__ out, float *__restrict__ out32, int W,
                                                                            float eps, int one_plus) {
   __shared__ float red[4];
@@ -1172,6 +1358,34 @@ template <class T> __global__ void __launch_bounds__(256) pass_norm_kernel(float
     er = table + (size_t)id * W;
   }
   float s = 0.f;
+  if constexpr (NC > 0) {
+    float v[NC], ev[NC], sv[NC], wv[NC];
+#pragma unroll
+    for (int j = 0; j < NC; ++j) {
+      const int c = threadIdx.x + 256 * j, cc = c < W ? c : W - 1;
+      v[j] = xr[cc];
+      ev[j] = er ? to_f<T>(er[cc]) : 0.f;
+      sv[j] = step ? step[cc] : 0.f;
+      wv[j] = w[cc];
+    }
+#pragma unroll
+    for (int j = 0; j < NC; ++j) {
+      if (er) v[j] += ev[j] * scale;
+      if (step) v[j] += sv[j];
+      if (threadIdx.x + 256 * j < W) s = fmaf(v[j], v[j], s);
+    }
+    const float inv = 1.0f / sqrtf(block_sum_256(s, red) / (float)W + eps);
+#pragma unroll
+    for (int j = 0; j < NC; ++j) {
+      const int c = threadIdx.x + 256 * j;
+      if (c >= W) break;
+      const float y = v[j] * inv * (one_plus ? 1.0f + wv[j] : wv[j]);
+      xr[c] = v[j];
+      out[(size_t)t * W + c] = from_f<T>(y);
+      if (out32) out32[(size_t)t * W + c] = y;
+    }
+    return;
+  }
   for (int c = threadIdx.x; c < W; c += 256) {
     float v = xr[c];
     if (er) v += to_f<T>(er[c]) * scale;
@@ -1200,6 +1414,7 @@ struct RopeHalfArgs {
   int ld, v_col, H, G, D, Dv, rot, block_size;
   float trig_mult;
 };
+// (grid.y workgroups share a row's heads and values: a step of few rows would leave the chip idle)
 template <class T> __global__ void __launch_bounds__(256) rope_half_cache_kernel(RopeHalfArgs a) {
   extern __shared__ float trig[];  // cos [rot / 2] | sin [rot / 2]
   const int t = blockIdx.x, tid = threadIdx.x, half = a.rot >> 1, per = a.D - half, nq = a.H * a.D;
@@ -1215,8 +1430,8 @@ template <class T> __global__ void __launch_bounds__(256) rope_half_cache_kernel
   const long long slot = a.slot_mapping[t];
   const long long blk = slot / a.block_size;
   const int off = (int)(slot % a.block_size);
-  const int items = (a.H + (slot >= 0 ? a.G : 0)) * per;   // of a head: `half` pairs, then the D - rot values that pass
-  for (int e = tid; e < items; e += 256) {
+  const int items = (a.H + (slot >= 0 ? a.G : 0)) * per, stride = 256 * gridDim.y;   // of a head: `half` pairs, then the D - rot values that pass
+  for (int e = blockIdx.y * 256 + tid; e < items; e += stride) {
     const int h = e / per, i = e - h * per;
     const bool is_q = h < a.H;
     const int g = h - a.H;
@@ -1235,7 +1450,7 @@ template <class T> __global__ void __launch_bounds__(256) rope_half_cache_kernel
   }
   if (slot < 0) return;
   const float *v = row + a.v_col;
-  for (int e = tid; e < a.G * a.Dv; e += 256) {
+  for (int e = blockIdx.y * 256 + tid; e < a.G * a.Dv; e += stride) {
     const int g = e / a.Dv, d = e - g * a.Dv;
     ((T *)a.v_cache)[(((size_t)blk * a.G + g) * a.block_size + off) * a.Dv + d] = from_f<T>(v[e] + (a.vb ? a.vb[e] : 0.f));
   }
@@ -1448,6 +1663,15 @@ extern "C" int mrs_hyb_rmsnorm(const float *x, int ldx, const float *w, void *ou
   dim3 grid(rows, parts);
   const size_t lds = gate && !gate_after ? (size_t)(width / parts) * 4 : 0;
   if (lds > 60000) return fail("mrs_hyb_rmsnorm: a gated part above 15000 values");
+  const int part = width / parts;
+  if ((dtype == 1 || dtype == 2) && part <= 4096 && !(gate && !gate_after)) {
+#define MRS_RN(T, N) hipLaunchKernelGGL((rmsnorm_row_kernel<T, N>), grid, dim3(256), 0, S_(stream), x, ldx, w, (T *)out, out32, rstd, part, eps, one_plus, width, gate, ldg, gate_after)
+#define MRS_RNT(T) do { if (part <= 1024) MRS_RN(T, 4); else if (part <= 2048) MRS_RN(T, 8); else MRS_RN(T, 16); } while (0)
+    if (dtype == 1) MRS_RNT(mrs::bf16_t); else MRS_RNT(float);
+#undef MRS_RNT
+#undef MRS_RN
+    return ok_or("mrs_hyb_rmsnorm");
+  }
   if (dtype == 1) hipLaunchKernelGGL(rmsnorm_kernel<mrs::bf16_t>, grid, dim3(256), lds, S_(stream), x, ldx, w, (mrs::bf16_t *)out, out32, rstd, width / parts, eps, one_plus, width, gate, ldg, gate_after);
   else if (dtype == 2) hipLaunchKernelGGL(rmsnorm_kernel<float>, grid, dim3(256), lds, S_(stream), x, ldx, w, (float *)out, out32, rstd, width / parts, eps, one_plus, width, gate, ldg, gate_after);
   else return fail("mrs_hyb_rmsnorm: dtype");
@@ -1638,12 +1862,26 @@ static int attn_launch(const void *q, const void *k_cache, const void *v_cache, 
     a.splits = splits;
   }
   dim3 grid(rows, H, a.splits > 1 ? a.splits : 1);
+  const int per_g = H / G, rc = per_g <= 1 ? 1 : per_g <= 2 ? 2 : per_g <= 4 || c > 2 ? 4 : 8;   // query heads that share a workgroup's keys
+  const size_t lds_d = (size_t)(rc * ((D + 3) & ~3) + 256 * rc + rc * Dv) * 4;
+  const bool decode = vec && c <= 4 && lds_d <= 60000 && ((uintptr_t)q % 4) == 0 && (long long)G * ((per_g + rc - 1) / rc) <= 65535;
+  if (decode) {
+    dim3 gd(rows, G * ((per_g + rc - 1) / rc), grid.z);
+#define MRS_DEC__(T, C, R) hipLaunchKernelGGL((paged_decode_attn_kernel<T, C, R>), gd, dim3(256), lds_d, S_(stream), a)
+#define MRS_DEC_(T, C) do { if (rc == 1) MRS_DEC__(T, C, 1); else if (rc == 2) MRS_DEC__(T, C, 2); else if (rc == 4) MRS_DEC__(T, C, 4); else MRS_DEC__(T, C, 8); } while (0)
+#define MRS_DEC(T) do { if (c <= 1) MRS_DEC_(T, 1); else if (c <= 2) MRS_DEC_(T, 2); else if (rc == 1) MRS_DEC__(T, 4, 1); else if (rc == 2) MRS_DEC__(T, 4, 2); else MRS_DEC__(T, 4, 4); } while (0)
+    if (dtype == 1) MRS_DEC(mrs::bf16_t); else if (dtype == 2) MRS_DEC(float); else return fail("mrs_hyb_paged_window_attn: dtype");
+#undef MRS_DEC
+#undef MRS_DEC_
+#undef MRS_DEC__
+  } else {
 #define MRS_ATTN(T, C) do { if (vec) hipLaunchKernelGGL((paged_window_attn_kernel<T, C, true>), grid, dim3(64), lds, S_(stream), a); \
                             else hipLaunchKernelGGL((paged_window_attn_kernel<T, C, false>), grid, dim3(64), lds, S_(stream), a); } while (0)
   if (dtype == 1) { if (c <= 1) MRS_ATTN(mrs::bf16_t, 1); else if (c <= 2) MRS_ATTN(mrs::bf16_t, 2); else if (c <= 4) MRS_ATTN(mrs::bf16_t, 4); else MRS_ATTN(mrs::bf16_t, 8); }
   else if (dtype == 2) { if (c <= 1) MRS_ATTN(float, 1); else if (c <= 2) MRS_ATTN(float, 2); else if (c <= 4) MRS_ATTN(float, 4); else MRS_ATTN(float, 8); }
   else return fail("mrs_hyb_paged_window_attn: dtype");
 #undef MRS_ATTN
+  }
   if (a.splits > 1) {
     if (dtype == 1) hipLaunchKernelGGL(attn_merge_kernel<mrs::bf16_t>, dim3(rows, H), dim3(64), 0, S_(stream), a);
     else hipLaunchKernelGGL(attn_merge_kernel<float>, dim3(rows, H), dim3(64), 0, S_(stream), a);
@@ -1863,8 +2101,12 @@ extern "C" int mrs_hyb_pass_norm(float *x, const int *tokens, const void *table,
                                  float eps, int one_plus, int dtype, void *stream) {
   if (rows <= 0) return 0;
   if (!w || !out || (table && (!tokens || vocab <= 0))) return fail("mrs_hyb_pass_norm: a norm weight, an output and tokens beside a table");
-  if (dtype == 1) hipLaunchKernelGGL(pass_norm_kernel<mrs::bf16_t>, dim3(rows), dim3(256), 0, S_(stream), x, tokens, (const mrs::bf16_t *)table, vocab, scale, step, w, (mrs::bf16_t *)out, out32, W, eps, one_plus);
-  else if (dtype == 2) hipLaunchKernelGGL(pass_norm_kernel<float>, dim3(rows), dim3(256), 0, S_(stream), x, tokens, (const float *)table, vocab, scale, step, w, (float *)out, out32, W, eps, one_plus);
+#define MRS_PN(T, N) hipLaunchKernelGGL((pass_norm_kernel<T, N>), dim3(rows), dim3(256), 0, S_(stream), x, tokens, (const T *)table, vocab, scale, step, w, (T *)out, out32, W, eps, one_plus)
+#define MRS_PNT(T) do { if (W <= 1024) MRS_PN(T, 4); else if (W <= 2048) MRS_PN(T, 8); else if (W <= 4096) MRS_PN(T, 16); else MRS_PN(T, 0); } while (0)
+  if (dtype == 1) MRS_PNT(mrs::bf16_t);
+  else if (dtype == 2) MRS_PNT(float);
+#undef MRS_PNT
+#undef MRS_PN
   else return fail("mrs_hyb_pass_norm: dtype");
   return ok_or("mrs_hyb_pass_norm");
 }
@@ -1877,8 +2119,10 @@ extern "C" int mrs_hyb_rope_half_cache(const float *u, int ld, int v_col, const 
   if (v_col < 0 || ld < (H + G) * D || ld < v_col + G * Dv) return fail("mrs_hyb_rope_half_cache: rows shorter than q | k | v");
   if (rot > 8192) return fail("mrs_hyb_rope_half_cache: more than 8192 rotated dimensions");
   RopeHalfArgs a{u, qb, kb, vb, freq, tok_pos, slot_mapping, q_out, k_cache, v_cache, ld, v_col, H, G, D, Dv, rot, block_size, trig_mult};
-  if (dtype == 1) hipLaunchKernelGGL(rope_half_cache_kernel<mrs::bf16_t>, dim3(rows), dim3(256), (size_t)rot * 4, S_(stream), a);
-  else if (dtype == 2) hipLaunchKernelGGL(rope_half_cache_kernel<float>, dim3(rows), dim3(256), (size_t)rot * 4, S_(stream), a);
+  int share = rows >= 256 ? 1 : ((H + G) * (D - rot / 2) + 255) / 256;
+  share = share > 64 ? 64 : share;
+  if (dtype == 1) hipLaunchKernelGGL(rope_half_cache_kernel<mrs::bf16_t>, dim3(rows, share), dim3(256), (size_t)rot * 4, S_(stream), a);
+  else if (dtype == 2) hipLaunchKernelGGL(rope_half_cache_kernel<float>, dim3(rows, share), dim3(256), (size_t)rot * 4, S_(stream), a);
   else return fail("mrs_hyb_rope_half_cache: dtype");
   return ok_or("mrs_hyb_rope_half_cache");
 }

@@ -261,7 +261,7 @@ __global__ void __launch_bounds__(256) gla_carry_kernel(GlaArgs a) {
 // thread (y, x) owns the columns 4 x .. 4 x + 3 (VP = 4) or x (VP = 1) of the state rows y, y + Y, ..: it updates them in place and adds up its part of the read-out; the parts
 // meet in LDS, the head is divided by its root mean square, multiplied by the weight `norm` [Dv] and by silu(gate).
 // Bonus form: a1 is tanh of the row's values (rounded to T), decays exp(-exp(z)), the read-out before the update plus the row's own value through u, `norm` [H * Dv].
-// Head form: operands through SiLU, one decay, the read-out in f32 to out32.
+// Head form: operands through SiLU, one decay, the read-out in f32 to out32; grid.z workgroups of `span` columns each share a head.
 struct GlaStepArgs {
   const float *u;           // [rows, ldu]: v | k | q | gate [H * Dv] at g_col | a1 [rank] at a1_col
   const void *wa2;          // [H * D, rank] in T
@@ -274,6 +274,7 @@ struct GlaStepArgs {
   const float *a1;          // nullable: the decay projection's first step in rows of its own, [rows, rank], instead of columns of u
   const float *bonus, *head_decay;
   float *out32;
+  int span;
 };
 template <class T, int VP, int FORM> __global__ void __launch_bounds__(1024) gla_step_kernel(GlaStepArgs a) {
   extern __shared__ __attribute__((aligned(16))) float sm[];  // k [Dq] | q [Dq] | decay [Dq] | a1 [rank padded] | o [Dv padded] | parts [Y][X * VP]
@@ -305,9 +306,10 @@ template <class T, int VP, int FORM> __global__ void __launch_bounds__(1024) gla
   __syncthreads();
   const bool carried = a.seq_pos0[s] > 0;
   float *st = a.state + ((size_t)a.seq_slot[s] * a.H + h) * D * Dv;
-  const int cols = (Dv + VP - 1) / VP, X = cols < nthr ? cols : nthr, Y = nthr / X, x = tid % X, y = tid / X;
+  const int cf = FORM == FORM_HEAD ? blockIdx.z * a.span : 0, ce = FORM == FORM_HEAD && cf + a.span < Dv ? cf + a.span : Dv;   // this workgroup's columns
+  const int cols = (ce - cf + VP - 1) / VP, X = cols < nthr ? cols : nthr, Y = nthr / X, x = tid % X, y = tid / X;
   for (int cb = 0; cb < cols; cb += X) {
-    const int c = (cb + x) * VP;
+    const int c = cf + (cb + x) * VP;
     float o[VP], v[VP];
 #pragma unroll
     for (int j = 0; j < VP; ++j) o[j] = 0.f;
@@ -344,15 +346,15 @@ template <class T, int VP, int FORM> __global__ void __launch_bounds__(1024) gla
       for (int j = 0; j < VP; ++j) parts[(y * X + x) * VP + j] = o[j];
     __syncthreads();
     for (int e = tid; e < X * VP; e += nthr) {
-      if (cb * VP + e >= Dv) continue;
+      if (cf + cb * VP + e >= ce) continue;
       float sum = 0.f;
       for (int q = 0; q < Y; ++q) sum += parts[q * X * VP + e];
-      os[cb * VP + e] = sum;
+      os[cf + cb * VP + e] = sum;
     }
   }
   __syncthreads();
   if (FORM == FORM_HEAD) {
-    for (int d = tid; d < Dv; d += nthr) a.out32[((size_t)t * a.H + h) * Dv + d] = os[d];
+    for (int d = cf + tid; d < ce; d += nthr) a.out32[((size_t)t * a.H + h) * Dv + d] = os[d];
     return;
   }
   float ss = 0.f;
@@ -485,7 +487,7 @@ static int step_launch(int form, const GlaStepArgs &a, int rows, int entries, in
     return fail("mrs_hyb_gla_step: rows shorter than their columns");
   if (dtype != 1 && dtype != 2) return fail("mrs_hyb_gla_step: dtype");
   const bool v4 = Dv % 4 == 0 && ((uintptr_t)a.state % 16) == 0;
-  const int VP = v4 ? 4 : 1, cols = Dv / VP;
+  const int VP = v4 ? 4 : 1, cols = (form == FORM_HEAD ? (a.span < Dv ? a.span : Dv) : Dv) / VP;
   // threads: at most eight state rows each where a head has that many, whole waves
   long long want = (long long)cols * ((D + 7) / 8);
   int nthr = want > 1024 ? 1024 : (int)((want + 63) / 64 * 64);
@@ -493,7 +495,7 @@ static int step_launch(int form, const GlaStepArgs &a, int rows, int entries, in
   const int X = cols < nthr ? cols : nthr, Y = nthr / X;
   const size_t lds = (size_t)(3 * ((D + 3) & ~3) + ((a.rank + 3) & ~3) + ((Dv + 3) & ~3) + Y * X * VP) * 4;
   if (lds > 65536 - 128) return fail("mrs_hyb_gla_step: the head does not fit 64 KB of LDS");
-  dim3 grid(entries, H);
+  dim3 grid(entries, H, form == FORM_HEAD ? (Dv + a.span - 1) / a.span : 1);
 #define MRS_GLAS_(T, V_) do { if (form == FORM_CHANNEL) hipLaunchKernelGGL((gla_step_kernel<T, V_, FORM_CHANNEL>), grid, dim3(nthr), lds, S_(stream), a); \
                               else if (form == FORM_BONUS) hipLaunchKernelGGL((gla_step_kernel<T, V_, FORM_BONUS>), grid, dim3(nthr), lds, S_(stream), a); \
                               else hipLaunchKernelGGL((gla_step_kernel<T, V_, FORM_HEAD>), grid, dim3(nthr), lds, S_(stream), a); } while (0)
@@ -509,7 +511,7 @@ static int step_launch(int form, const GlaStepArgs &a, int rows, int entries, in
 extern "C" int mrs_hyb_gla_step(const float *u, int ldu, int k_col, int q_col, int g_col, int a1_col, int rank, const void *wa2, const float *zb, const float *norm, float *state,
                                 void *out, const int *seq_start, const int *seq_pos0, const int *seq_slot, int rows, int entries, int H, int D, int Dv, float q_mult, float inv_tau,
                                 float eps, int dtype, void *stream) {
-  const GlaStepArgs a{u, wa2, zb, norm, state, seq_start, seq_pos0, seq_slot, out, ldu, k_col, q_col, g_col, a1_col, rank, H, D, Dv, q_mult, inv_tau, eps, nullptr, nullptr, nullptr, nullptr};
+  const GlaStepArgs a{u, wa2, zb, norm, state, seq_start, seq_pos0, seq_slot, out, ldu, k_col, q_col, g_col, a1_col, rank, H, D, Dv, q_mult, inv_tau, eps, nullptr, nullptr, nullptr, nullptr, 0};
   return step_launch(FORM_CHANNEL, a, rows, entries, dtype, stream);
 }
 /* the same with a1 [rows, rank] in rows of its own (tanh is taken here), decays exp(-exp(W a1 + zb)), the bonus [H, D] and a norm weight of [H * Dv] */
@@ -517,14 +519,14 @@ extern "C" int mrs_hyb_bonus_step(const float *u, int ldu, int k_col, int q_col,
                                   const float *norm, float *state, void *out, const int *seq_start, const int *seq_pos0, const int *seq_slot, int rows, int entries, int H, int D,
                                   int Dv, float eps, int dtype, void *stream) {
   if (!a1 || !bonus) return fail("mrs_hyb_bonus_step: the decay projection's first step and the bonus are needed");
-  const GlaStepArgs a{u, wa2, zb, norm, state, seq_start, seq_pos0, seq_slot, out, ldu, k_col, q_col, g_col, 0, rank, H, D, Dv, 1.0f, 0.f, eps, a1, bonus, nullptr, nullptr};
+  const GlaStepArgs a{u, wa2, zb, norm, state, seq_start, seq_pos0, seq_slot, out, ldu, k_col, q_col, g_col, 0, rank, H, D, Dv, 1.0f, 0.f, eps, a1, bonus, nullptr, nullptr, 0};
   return step_launch(FORM_BONUS, a, rows, entries, dtype, stream);
 }
 /* single rows with one decay per head and SiLU operands: out (f32) [rows, H * Dv], no norm and no gate */
 extern "C" int mrs_hyb_lightning_step(const float *u, int ldu, int k_col, int q_col, const float *head_decay, float *state, float *out, const int *seq_start, const int *seq_pos0,
                                       const int *seq_slot, int rows, int entries, int H, int D, int Dv, void *stream) {
   if (!head_decay) return fail("mrs_hyb_lightning_step: the heads' decays are needed");
-  const GlaStepArgs a{u, nullptr, nullptr, nullptr, state, seq_start, seq_pos0, seq_slot, nullptr, ldu, k_col, q_col, 0, 0, 0, H, D, Dv, 1.0f, 0.f, 0.f, nullptr, nullptr, head_decay, out};
+  const GlaStepArgs a{u, nullptr, nullptr, nullptr, state, seq_start, seq_pos0, seq_slot, nullptr, ldu, k_col, q_col, 0, 0, 0, H, D, Dv, 1.0f, 0.f, 0.f, nullptr, nullptr, head_decay, out, 32};
   return step_launch(FORM_HEAD, a, rows, entries, 2, stream);
 }
 

@@ -486,13 +486,47 @@ template <class T> __global__ void __launch_bounds__(64) head_norm_gate_kernel(c
 
 // ---------------------------------------------------------------------------------- x (+)= c (y1 / rms(y1) w1 + y2 / rms(y2) w2)
 // then (nullable, with NEXT): the norm weight in front of the next sublayer; the updated row leaves normed as well, rounded (out) and in f32 (out32, nullable)
-template <class T, bool NEXT> __global__ void __launch_bounds__(256) norm_pair_add_kernel(float *__restrict__ x, int ldx, const float *__restrict__ y1, const float *__restrict__ w1,
+// (rows of at most 256 NC values: read once, all loads in flight; NC 0: any width)
+template <class T, bool NEXT, int NC> __global__ void __launch_bounds__(256) norm_pair_add_kernel(float *__restrict__ x, int ldx, const float *__restrict__ y1, const float *__restrict__ w1,
                                                             const float *__restrict__ y2, const float *__restrict__ w2, int W, float eps, float c, int accumulate,
                                                             const float *__restrict__ then, int one_plus, T *__restrict__ out, float *__restrict__ out32) {
   __shared__ float red[4];
   const int t = blockIdx.x;
   const float *a = y1 + (size_t)t * W, *b = y2 + (size_t)t * W;
   float s1 = 0.f, s2 = 0.f;
+  if constexpr (NC > 0) {
+    float av[NC], bv[NC], wa[NC], wb[NC], xv[NC], tv[NC], s3 = 0.f;
+    float *xr = x + (size_t)t * ldx;
+#pragma unroll
+    for (int j = 0; j < NC; ++j) {
+      const int k = threadIdx.x + 256 * j, kc = k < W ? k : W - 1;
+      av[j] = a[kc]; bv[j] = b[kc]; wa[j] = w1[kc]; wb[j] = w2[kc];
+      xv[j] = accumulate ? xr[kc] : 0.f;
+      tv[j] = NEXT ? then[kc] : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < NC; ++j)
+      if (threadIdx.x + 256 * j < W) { s1 = fmaf(av[j], av[j], s1); s2 = fmaf(bv[j], bv[j], s2); }
+    const float i1 = 1.0f / sqrtf(block_sum_256(s1, red) / (float)W + eps);
+    const float i2 = 1.0f / sqrtf(block_sum_256(s2, red) / (float)W + eps);
+#pragma unroll
+    for (int j = 0; j < NC; ++j) {
+      const float v = c * (av[j] * i1 * wa[j] + bv[j] * i2 * wb[j]);
+      xv[j] = accumulate ? xv[j] + v : v;
+      if (threadIdx.x + 256 * j < W) { xr[threadIdx.x + 256 * j] = xv[j]; s3 = fmaf(xv[j], xv[j], s3); }
+    }
+    if (!NEXT) return;
+    const float i3 = 1.0f / sqrtf(block_sum_256(s3, red) / (float)W + eps);
+#pragma unroll
+    for (int j = 0; j < NC; ++j) {
+      const int k = threadIdx.x + 256 * j;
+      if (k >= W) break;
+      const float v = xv[j] * i3 * (one_plus ? 1.0f + tv[j] : tv[j]);
+      out[(size_t)t * W + k] = from_f<T>(v);
+      if (out32) out32[(size_t)t * W + k] = v;
+    }
+    return;
+  }
   for (int k = threadIdx.x; k < W; k += 256) { s1 = fmaf(a[k], a[k], s1); s2 = fmaf(b[k], b[k], s2); }
   const float i1 = 1.0f / sqrtf(block_sum_256(s1, red) / (float)W + eps);
   const float i2 = 1.0f / sqrtf(block_sum_256(s2, red) / (float)W + eps);
@@ -651,10 +685,13 @@ extern "C" int mrs_hyb_head_norm_gate(const float *y, int ldp, const float *mexp
   return ok_or("mrs_hyb_head_norm_gate");
 }
 
+#define MRS_NPA(T, N, C_, ...) hipLaunchKernelGGL((norm_pair_add_kernel<T, N, C_>), dim3(rows), dim3(256), 0, S_(stream), x, ldx, y1, w1, y2, w2, W, eps, c, accumulate, __VA_ARGS__)
+#define MRS_NPAT(T, N, ...) do { if (W <= 1024) MRS_NPA(T, N, 4, __VA_ARGS__); else if (W <= 2048) MRS_NPA(T, N, 8, __VA_ARGS__); else if (W <= 4096) MRS_NPA(T, N, 16, __VA_ARGS__); \
+                                 else MRS_NPA(T, N, 0, __VA_ARGS__); } while (0)
 extern "C" int mrs_hyb_norm_pair_add(float *x, int ldx, const float *y1, const float *w1, const float *y2, const float *w2, int rows, int W, float eps, float c, int accumulate,
                                      void *stream) {
   if (rows <= 0) return 0;
-  hipLaunchKernelGGL((norm_pair_add_kernel<float, false>), dim3(rows), dim3(256), 0, S_(stream), x, ldx, y1, w1, y2, w2, W, eps, c, accumulate, nullptr, 0, nullptr, nullptr);
+  MRS_NPAT(float, false, nullptr, 0, nullptr, nullptr);
   return ok_or("mrs_hyb_norm_pair_add");
 }
 /* the same, and the norm in front of the next sublayer in the same launch: out (dtype) [rows, W] = x / rms(x) * (then | 1 + then) of the updated rows, out32 (nullable) in f32 */
@@ -662,11 +699,14 @@ extern "C" int mrs_hyb_norm_pair_add_norm(float *x, int ldx, const float *y1, co
                                           const float *then, int one_plus, void *out, float *out32, int dtype, void *stream) {
   if (rows <= 0) return 0;
   if (!then || !out) return fail("mrs_hyb_norm_pair_add_norm: the next norm's weight and an output are needed");
-  if (dtype == 1) hipLaunchKernelGGL((norm_pair_add_kernel<mrs::bf16_t, true>), dim3(rows), dim3(256), 0, S_(stream), x, ldx, y1, w1, y2, w2, W, eps, c, accumulate, then, one_plus, (mrs::bf16_t *)out, out32);
-  else if (dtype == 2) hipLaunchKernelGGL((norm_pair_add_kernel<float, true>), dim3(rows), dim3(256), 0, S_(stream), x, ldx, y1, w1, y2, w2, W, eps, c, accumulate, then, one_plus, (float *)out, out32);
+  if (dtype == 1) MRS_NPAT(mrs::bf16_t, true, then, one_plus, (mrs::bf16_t *)out, out32);
+  else if (dtype == 2) MRS_NPAT(float, true, then, one_plus, (float *)out, out32);
   else return fail("mrs_hyb_norm_pair_add_norm: dtype");
   return ok_or("mrs_hyb_norm_pair_add_norm");
 }
+
+#undef MRS_NPAT
+#undef MRS_NPA
 
 extern "C" int mrs_hyb_round_cols(const float *u, int ldu, void *out, int rows, int n, int dtype, void *stream) {
   const size_t total = (size_t)rows * n;

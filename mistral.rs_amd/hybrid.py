@@ -2153,7 +2153,7 @@ class HybridDecoder:
         return (out, out32) if want32 else out
 
     KEY_SPLIT_ROWS = 128   # steps of single rows up to this many rows split their keys
-    KEYS_PER_SPLIT = 256   # at least this many keys (of the longest table in the batch) per workgroup
+    KEYS_PER_SPLIT = 256   # about this many keys (of the longest table in the batch) per workgroup: one pass of 64 per wave
     KEY_SPLITS = 32
 
     def key_splits(self, b: RaggedBatch, heads: int, vdim: int, most_keys: int = 0):
@@ -2162,7 +2162,7 @@ class HybridDecoder:
         if b.seg_rows != 1 or b.rows > self.KEY_SPLIT_ROWS:
             return None, 0
         keys = b.max_blocks * self.block_size
-        splits = min(self.KEY_SPLITS, (min(keys, most_keys) if most_keys > 0 else keys) // self.KEYS_PER_SPLIT)
+        splits = min(self.KEY_SPLITS, -(-(min(keys, most_keys) if most_keys > 0 else keys) // self.KEYS_PER_SPLIT))
         if splits < 2:
             return None, 0
         return torch.empty(splits, b.rows, heads, vdim + 2, dtype=torch.float32, device=self.device), splits
