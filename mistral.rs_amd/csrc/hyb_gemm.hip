@@ -6,7 +6,8 @@
 //     are sorted by group, group g owns rows [bounds[g], bounds[g + 1]) and the weight slab W + g * wstride (mixture-of-experts layers: one launch for all experts,
 //     the bounds are read on the device, tiles past a group's rows leave).
 //   * gemv_rows_kernel: M <= 8 rows (decode steps): one wave per output column streams the weight row with 16-byte loads, f32 accumulation per activation row,
-//     butterfly sum.  Grouped form: every activation row has its own weight slab (row_group[m]).
+//     butterfly sum.  Grouped form: every activation row has its own weight slab (row_group[m]).  Three bf16 rows and more run on the matrix cores (gemv_mfma_kernel): on the vector
+//     ALU eight rows cost two and a half times one.
 // f32 results only: the consumers (residual sum, norms, recurrences, routers) are f32 anyway; what a consumer feeds into the next product it rounds itself, once.
 #include "common.cuh"
 
@@ -447,6 +448,90 @@ template <class T, int MR, int IN, int EP = EP_NONE> __global__ void __launch_bo
   }
 }
 
+// A few bf16 rows on the matrix cores: one workgroup per sixteen output columns (of a gated weight: sixteen gate and sixteen up columns), its waves share K in runs of 128.  The weights
+// are the A operand (lane (i, g): column i, values 8 g .. of a run of 32), the activation rows the B operand, padded to sixteen; a run's eight loads of weights stay in flight while the
+// one before multiplies.  The waves' sums meet in LDS.
+template <int NW, int EP> __global__ void __launch_bounds__(64 * NW) gemv_mfma_kernel(GemvArgs a) {
+  constexpr bool GLU = EP == EP_GLU_SILU || EP == EP_GLU_GELU;
+  constexpr int RUN = 128, NF = RUN / 32;
+  typedef float f32x4 __attribute__((ext_vector_type(4)));
+  __shared__ float part[GLU ? 2 : 1][NW][16][17];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, i = lane & 15, g = lane >> 4, n0 = blockIdx.x * 16;
+  const bf16_t *W = (const bf16_t *)a.W + (size_t)blockIdx.z * (a.batch > 0 ? a.wstride : 0);
+  const bf16_t *A = (const bf16_t *)a.A + (size_t)blockIdx.z * a.a_bstride;
+  const bf16_t *wr = W + (size_t)(n0 + i < a.N ? n0 + i : a.N - 1) * a.ldw, *wu = wr + (size_t)(GLU ? a.N : 0) * a.ldw;
+  const bf16_t *ar = A + (size_t)(i < a.M ? i : a.M - 1) * a.lda;   // (rows past M repeat the last one: their columns of the result are not stored)
+  f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f}, up = acc;
+  int4 w0[NF], w1[GLU ? NF : 1], x[NF];
+  auto fetch = [&](int k0) {
+#pragma unroll
+    for (int f = 0; f < NF; ++f) {
+      const int k = k0 + 32 * f + 8 * g;
+      w0[f] = x[f] = make_int4(0, 0, 0, 0);
+      if (GLU) w1[GLU ? f : 0] = w0[f];
+      if (k < a.K) {
+        w0[f] = ld16nt_a4(wr + k);
+        if (GLU) w1[GLU ? f : 0] = ld16nt_a4(wu + k);
+        x[f] = *(const int4 *)(ar + k);
+      }
+    }
+  };
+  if (wave * RUN < a.K) fetch(wave * RUN);
+  for (int k0 = wave * RUN; k0 < a.K; k0 += NW * RUN) {
+    bf16x8 wf[NF], uf[GLU ? NF : 1], xf[NF];
+#pragma unroll
+    for (int f = 0; f < NF; ++f) {
+      wf[f] = __builtin_bit_cast(bf16x8, w0[f]);
+      if (GLU) uf[GLU ? f : 0] = __builtin_bit_cast(bf16x8, w1[GLU ? f : 0]);
+      xf[f] = __builtin_bit_cast(bf16x8, x[f]);
+    }
+    if (k0 + NW * RUN < a.K) fetch(k0 + NW * RUN);
+#pragma unroll
+    for (int f = 0; f < NF; ++f) {
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[f], xf[f], acc, 0, 0, 0);
+      if (GLU) up = __builtin_amdgcn_mfma_f32_16x16x32_bf16(uf[GLU ? f : 0], xf[f], up, 0, 0, 0);
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {   // register r: column 4 g + r, row i
+    part[0][wave][i][4 * g + r] = acc[r];
+    if (GLU) part[GLU ? 1 : 0][wave][i][4 * g + r] = up[r];
+  }
+  __syncthreads();
+  if (tid >= 256) return;
+  const int m = tid >> 4, n = tid & 15;
+  if (m >= a.M || n0 + n >= a.N) return;
+  float s = 0.f, u = 0.f;
+#pragma unroll
+  for (int w = 0; w < NW; ++w) {
+    s += part[0][w][m][n];
+    if (GLU) u += part[GLU ? 1 : 0][w][m][n];
+  }
+  s *= a.alpha;
+  if (EP != EP_NONE) s = ep_act(EP, s);
+  if (GLU) s *= u;
+  const size_t idx = (size_t)blockIdx.z * a.c_bstride + (size_t)m * a.ldc + n0 + n;
+  if (a.c_is_T) ((bf16_t *)a.C)[idx] = from_f<bf16_t>(s);
+  else a.C[idx] = a.accumulate ? a.C[idx] + s : s;
+}
+// rows from which the matrix cores take over from the row kernel (below, the products of a streamed weight hide behind its loads)
+constexpr int MFMA_ROWS = 3;
+static bool gemv_mfma(const GemvArgs &a, int dtype, int in_mode, int ep, hipStream_t s) {
+  if (dtype != 1 || in_mode != IN_PLAIN || a.row_group || !a.vec_ok || a.M < MFMA_ROWS || a.M > 16) return false;
+  const dim3 grid((a.N + 15) / 16, 1, a.batch > 0 ? a.batch : 1);
+  const bool wide = (long long)grid.x * grid.z < 1024;   // few columns: more waves per workgroup keep the memory system busy
+#define MRS_GM(EP_) do { if (wide) hipLaunchKernelGGL((gemv_mfma_kernel<8, EP_>), grid, dim3(512), 0, s, a); else hipLaunchKernelGGL((gemv_mfma_kernel<4, EP_>), grid, dim3(256), 0, s, a); } while (0)
+  switch (ep) {
+    case EP_NONE: MRS_GM(EP_NONE); break;
+    case EP_RELU_SQ: MRS_GM(EP_RELU_SQ); break;
+    case EP_GELU: MRS_GM(EP_GELU); break;
+    case EP_GLU_SILU: MRS_GM(EP_GLU_SILU); break;
+    default: MRS_GM(EP_GLU_GELU); break;
+  }
+#undef MRS_GM
+  return true;
+}
+
 static thread_local char g_err[256];
 static int fail(const char *m) { snprintf(g_err, sizeof g_err, "%s", m); return 1; }
 
@@ -505,6 +590,7 @@ extern "C" int mrs_hyb_gemm_batched(const void *A, const void *W, void *C, int M
   if (batch > 65535) return fail("mrs_hyb_gemm_batched: more than 65535 products in one batch");
   dim3 grid((N + 3) / 4, 1, batch > 0 ? batch : 1);
   hipStream_t s = (hipStream_t)stream;
+  if (gemv_mfma(a, dtype, IN_PLAIN, EP_NONE, s)) return hipGetLastError() == hipSuccess ? 0 : fail("mrs_hyb_gemm_batched: launch failed");
 #define MRS_GEMVB(T) do { if (M <= 1) hipLaunchKernelGGL((gemv_rows_kernel<T, 1, IN_PLAIN>), grid, dim3(256), 0, s, a); else if (M <= 2) hipLaunchKernelGGL((gemv_rows_kernel<T, 2, IN_PLAIN>), grid, dim3(256), 0, s, a); \
                           else if (M <= 4) hipLaunchKernelGGL((gemv_rows_kernel<T, 4, IN_PLAIN>), grid, dim3(256), 0, s, a); else hipLaunchKernelGGL((gemv_rows_kernel<T, 8, IN_PLAIN>), grid, dim3(256), 0, s, a); } while (0)
   if (dtype == 1) MRS_GEMVB(mrs::bf16_t); else MRS_GEMVB(float);
@@ -527,6 +613,7 @@ static int gemv_launch(const void *A, const void *W, float *C, int M, int N, int
               (!in_bias || ((uintptr_t)in_bias % 16) == 0)) ? 1 : 0, src_row, src_scale, src_div, in_bias, p0, p1, 0, 0, 0, 0, alpha};
   dim3 grid((N + 3) / 4, row_group ? M : 1);
   hipStream_t s = (hipStream_t)stream;
+  if (gemv_mfma(a, dtype, in_mode, EP_NONE, s)) return hipGetLastError() == hipSuccess ? 0 : fail("mrs_hyb_gemv: launch failed");
 #define MRS_GEMV_(T, MR, IN) hipLaunchKernelGGL((gemv_rows_kernel<T, MR, IN>), grid, dim3(256), 0, s, a)
 #define MRS_GEMV(T, MR) do { if (in_mode == 0) MRS_GEMV_(T, MR, IN_PLAIN); else if (in_mode == 1) MRS_GEMV_(T, MR, IN_GLU); else if (in_mode == 2) MRS_GEMV_(T, MR, IN_SCALED); \
                              else if (in_mode == 3) MRS_GEMV_(T, MR, IN_GLU_CLAMP); else if (in_mode == 4) MRS_GEMV_(T, MR, IN_BIAS_XIELU); else MRS_GEMV_(T, MR, IN_RELU_SQ); } while (0)
@@ -574,6 +661,7 @@ extern "C" int mrs_hyb_gemv_ep(const void *A, const void *W, void *C, int M, int
              0.f, 0.f, 0, 0, 0, 1, 1.0f};
   dim3 grid((N + 3) / 4, row_group ? M : 1);
   hipStream_t s = (hipStream_t)stream;
+  if (gemv_mfma(a, dtype, in_mode, ep, s)) return hipGetLastError() == hipSuccess ? 0 : fail("mrs_hyb_gemv_ep: launch failed");
 #define MRS_GEP_(T, MR, IN, EP) hipLaunchKernelGGL((gemv_rows_kernel<T, MR, IN, EP>), grid, dim3(256), 0, s, a)
 #define MRS_GEP1(T, IN) do { if (ep == 1) MRS_GEP_(T, 1, IN, EP_RELU_SQ); else MRS_GEP_(T, 1, IN, EP_GELU); } while (0)
 #define MRS_GEPM(T, MR) do { if (ep == 1) MRS_GEP_(T, MR, IN_PLAIN, EP_RELU_SQ); else if (ep == 2) MRS_GEP_(T, MR, IN_PLAIN, EP_GELU); \

@@ -746,7 +746,7 @@ def test_sharp_attention_needs_the_chunk_the_sink_the_ramp_and_the_biases(dev, d
             edit_w(x)
         return rel(logits_of(c, f64(x), t), want)
     left = lambda c, i: c["layers"][i]["mixer"]["left"]
-    far = {"chunk": changed(lambda c: left(c, 0)["mask"].update(size=25)), "chunk_b": changed(lambda c: left(c, 1)["mask"].update(size=16)),
+    far = {"chunk": changed(lambda c: left(c, 0)["mask"].update(size=25)), "chunk_b": changed(lambda c: left(c, 1)["mask"].update(size=9)),
            "ramp": changed(lambda c: left(c, 0)["rot"].pop("scaling")), "sink": changed(None, lambda x: x["l0.mix.left.sink"].fill_(-1e4)),
            "bias": changed(None, lambda x: x["l0.mix.left.k.b"].zero_()), "v_bias": changed(None, lambda x: x["l1.mix.left.v.b"].zero_()), "bonus": changed(None, lambda x: x["l0.mix.right.u"].zero_()),
            "shift": changed(None, lambda x: x["l0.mix.right.mu.k"].zero_()), "step": changed(None, lambda x: x["loop.step"].copy_(x["loop.step"].flip(0))),
