@@ -87,6 +87,26 @@ const char *mrs_hyb_latent_mfma_last_error();
 int mrs_hyb_latent_mfma_prompt(const void *q, const void *k, const void *vt, const int *tables, const int *tok_pos, const int *seg_entry, const int *seg_row0, const int *seg_len, int segments, int seg_rows, const float *sink, const float *gate, int ldg, void *out, int rows, int H, int DK, int Dv, int n_rows, int max_blocks, int block_size, int window, float scale, void *stream);
 int mrs_hyb_latent_mfma_decode(const void *q, const void *cache, const int *block_tables, const int *tok_seq, const int *tok_pos, float *part, float *ml, int rows, int H, int R, int E, int block_size, int max_blocks, int window, int splits, float scale, void *stream);
 int mrs_hyb_latent_mfma_merge(const float *part, const float *ml, const float *sink, const void *w_uv, const float *gate, int ldg, void *out, int rows, int H, int R, int Dv, int splits, void *stream);
+/* ---- hyb_kernels.hip: passes through layers that run several times, half-split rotary with biases */
+int mrs_hyb_pass_norm(float *x, const int *tokens, const void *table, int vocab, float scale, const float *step, const float *w, void *out, float *out32, int rows, int W, float eps, int one_plus, int dtype, void *stream);
+int mrs_hyb_rope_half_cache(const float *u, int ld, int v_col, const float *qb, const float *kb, const float *vb, const float *freq, float trig_mult, const int *tok_pos, const long long *slot_mapping, void *q_out, void *k_cache, void *v_cache, int rows, int H, int G, int D, int Dv, int rot, int block_size, int dtype, void *stream);
+/* ---- hyb_recur.hip / hyb_gemm.hip: normed average with the next norm, products that join with a factor */
+int mrs_hyb_norm_pair_add_norm(float *x, int ldx, const float *y1, const float *w1, const float *y2, const float *w2, int rows, int W, float eps, float c, int accumulate, const float *then, int one_plus, void *out, float *out32, int dtype, void *stream);
+int mrs_hyb_gemm_scaled(const void *A, const void *W, float *C, int M, int N, int K, int lda, int ldw, int ldc, int dtype, int accumulate, float alpha, void *stream);
+/* ---- hyb_linattn.hip: one decay per head with SiLU operands, time mixing */
+int mrs_hyb_lightning_scan(const float *u, int ldu, int k_col, int q_col, const float *head_decay, float *state, float *out, const int *seq_pos0, const int *seq_slot, const int *seg_entry, const int *seg_row0, const int *seg_len, const int *ent_seg0, float *carry, float *decay, int rows, int entries, int segments, int H, int D, int Dv, void *stream);
+int mrs_hyb_lightning_step(const float *u, int ldu, int k_col, int q_col, const float *head_decay, float *state, float *out, const int *seq_start, const int *seq_pos0, const int *seq_slot, int rows, int entries, int H, int D, int Dv, void *stream);
+int mrs_hyb_bonus_scan(const float *u, int ldu, int k_col, int q_col, const float *dec, const float *bonus, float *state, float *out, const int *seq_pos0, const int *seq_slot, const int *seg_entry, const int *seg_row0, const int *seg_len, const int *ent_seg0, float *carry, float *decay, int rows, int entries, int segments, int H, int D, int Dv, void *stream);
+int mrs_hyb_bonus_step(const float *u, int ldu, int k_col, int q_col, int g_col, const float *a1, int rank, const void *wa2, const float *zb, const float *bonus, const float *norm, float *state, void *out, const int *seq_start, const int *seq_pos0, const int *seq_slot, int rows, int entries, int H, int D, int Dv, float eps, int dtype, void *stream);
+int mrs_hyb_token_shift(const float *h, const float *mu, float *state, void *out, const int *tok_seq, const int *seq_start, const int *seq_pos0, const int *seq_slot, int rows, int W, int n, int dtype, void *stream);
+int mrs_hyb_tanh_round(const float *x, void *out, int rows, int cols, int dtype, void *stream);
+/* ---- hyb_rglru.hip: real-gated linear recurrent unit */
+const char *mrs_hyb_rglru_last_error();
+int mrs_hyb_rglru_scan(const float *u, const void *wa, const void *wi, const float *ba, const float *bi, const float *lam, const float *y, int ldy, const float *yb, float *state, float *local, float *prod, float *start, void *out, const int *seq_pos0, const int *seq_slot, const int *seg_row0, const int *seg_len, const int *ent_seg0, int rows, int entries, int segments, int seg_rows, int C, int blocks, int dtype, void *stream);
+int mrs_hyb_rglru_step(const float *u, const void *wa, const void *wi, const float *ba, const float *bi, const float *lam, const float *y, int ldy, const float *yb, float *state, void *out, const int *seq_start, const int *seq_pos0, const int *seq_slot, int rows, int entries, int C, int blocks, int dtype, void *stream);
+/* ---- hyb_attn_mfma.hip: paged attention of portions on the matrix cores (bf16) */
+const char *mrs_hyb_attn_mfma_last_error();
+int mrs_hyb_attn_mfma_prompt(const void *q, const void *k_cache, const void *v_cache, const int *tables, const int *tok_pos, const int *seg_entry, const int *seg_row0, const int *seg_len, int segments, int seg_rows, const float *sink, const float *gate, int ldg, int gate_each, void *out, int rows, int H, int G, int D, int Dv, int num_blocks, int max_blocks, int block_size, int window, int chunk, float scale, void *stream);
 void *mrs_state_pool_create(size_t num_slots);
 void mrs_state_pool_destroy(void *h);
 size_t mrs_state_pool_capacity(void *h);

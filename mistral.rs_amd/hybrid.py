@@ -1,10 +1,12 @@
 """Layer-list ("hybrid") decoders served in their checkpoint dtype: every layer is `x += mixer(norm(x))` then optionally `x += feed_forward(norm(x))` (or both sublayers
 reading two norms of the same x: `parallel_sublayers`), the mixer being one of the registered kinds (`MIXERS`: state-space-duality recurrence, paged softmax attention with a
 sliding window / position chunks / kept first tokens / a learned sink, paged sigmoid attention with a distance bias and mixed head scores, sink attention with convolved
-projections, retention, latent attention, the gated delta rule, gated linear attention, a matrix memory with exponential gates, two mixers side by side), the feed-forward one of
+projections, retention, latent attention, the gated delta rule, gated linear attention, decayed linear attention with SiLU operands, time mixing, a real-gated linear recurrent unit, a matrix
+memory with exponential gates, two mixers side by side), the feed-forward one of
 `FEED_FORWARDS` (sigmoid-routed experts with a gated shared expert, softmax-routed clamped-GLU experts, routed squared-ReLU or GELU experts, dense xIELU, SiLU-GLU and GELU-GLU
 layers).  The norms are RMS norms (plain or one-plus weights) before every sublayer, layer norms with bias before AND after every sublayer (`HybridSpec.norm`, `post_norms`), or
-layer norms behind the sublayers only (`join_norms`).  The Gekilix, Sobunex, Setopel, Gifopel and Kebisun architectures (config.json `"architecture"`) are such lists.
+layer norms behind the sublayers only (`join_norms`).  Layers may run several times with the same weights (`LayerSpec.weights_of`, `enter`).  The Gekilix, Sobunex, Setopel, Gifopel,
+Kebisun and Zumuzen architectures (config.json `"architecture"`) are such lists.
 
 The step function is `HybridDecoder.forward_batch(batch)`: ONE ragged batch -- prompt portions of any length next to single decoded tokens -- through the HIP kernels of
 csrc/hyb_*.hip (C ABI, this process's current stream; PyTorch owns buffers and the stream, nothing else).  What the sequences carry between
