@@ -1575,11 +1575,11 @@ def zumuzen_leg(a, dev):
     scale, ff = D ** -0.5, GluSpec(z["ff"])
     yarn = {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}
     decays = [1.0 - 2.0 ** (-5 - h % 8) for h in range(lH)]
-    both = ParallelSpec("attention", AttentionSpec(H, G, D, Dv, scale, 0, 0, RotarySpec(D, 500000.0, None, "half"), False, chunk=z["chunk"], bias=True), "lightning",
+    both = ParallelSpec("attention", AttentionSpec(H, G, D, Dv, scale, 0, 0, RotarySpec(D, 1000000.0, None, "half"), False, chunk=z["chunk"], bias=True), "lightning",
                         LightningSpec(lH, lD, lDv, decays))
-    both2 = ParallelSpec("attention", AttentionSpec(H, G, D, D, scale, 0, 0, RotarySpec(D // 2, 250000.0, yarn, "half"), False, chunk=z["chunk"], sink=True, bias=True, values_are_keys=True),
+    both2 = ParallelSpec("attention", AttentionSpec(H, G, D, D, scale, 0, 0, RotarySpec(D // 2, 100000.0, yarn, "half"), False, chunk=z["chunk"], sink=True, bias=True, values_are_keys=True),
                          "time_mix", TimeMixSpec(tH, tD), (0.75, 1.25))
-    oattn = AttentionSpec(H, G, D, Dv, scale, 0, 0, RotarySpec(D // 2, 500000.0), True, chunk=z["chunk"], head_norm=True, sink=True, head_gate=True)
+    oattn = AttentionSpec(H, G, D, Dv, scale, 0, 0, RotarySpec(D // 2, 1000000.0), True, chunk=z["chunk"], head_norm=True, sink=True, head_gate=True)
     new = [LayerSpec("rglru", RgLruSpec(C, z["blocks"], z["conv"]), ff, "l0.")]
     old = [LayerSpec("mamba2", Mamba2Spec(C // 64, 64, 16, 1, z["conv"], 1), ff, "l0.")]
     for t in range(2):   # two passes with the same weights

@@ -359,7 +359,7 @@ def sees(chunk=0, window=0):
 @pytest.mark.gpu
 @pytest.mark.parametrize("view", sorted(VIEWS))
 @pytest.mark.parametrize("form", ["matrix_cores", "general_bf16", "general_f32"])
-@pytest.mark.parametrize("H,G,D,Dv,bs", [(4, 2, 16, 24, 8), (3, 1, 96, 192, 12), (2, 2, 200, 256, 16), (6, 2, 128, 128, 32), (5, 5, 8, 8, 5)])
+@pytest.mark.parametrize("H,G,D,Dv,bs", [(4, 2, 16, 24, 8), (3, 1, 88, 184, 12), (2, 2, 200, 256, 16), (6, 2, 128, 128, 32), (5, 5, 8, 8, 5)])
 def test_paged_attention_over_portions_and_single_rows(dev, H, G, D, Dv, bs, form, view):
     """portions (down to one row) and single rows of several sequences over shuffled pages; one key per sequence stands out, one lies just outside what most rows see, so that a key too
     many or too few is an error of the size of the values; learned sinks and a gate per head"""
@@ -620,7 +620,7 @@ def test_time_mixing_recurrence_over_portions_single_rows_and_reused_slots(dev, 
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("dt", [2, 1], ids=["f32", "bf16"])
-@pytest.mark.parametrize("C,blocks", [(48, 3), (40, 1), (128, 2), (7, 7), (15, 3), (260, 2), (192, 1), (1, 1), (1024, 4)])
+@pytest.mark.parametrize("C,blocks", [(48, 3), (40, 1), (144, 2), (7, 7), (15, 3), (260, 2), (192, 1), (1, 1), (1024, 4)])
 def test_gated_recurrent_unit_over_portions_single_rows_and_reused_slots(dev, C, blocks, dt):
     """gates of channel parts of many sizes, segments and their carry, the GELU branch; log a from nearly zero to far below: states that keep and states that forget"""
     from mistralrs_amd.hybrid import _call
